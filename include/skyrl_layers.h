@@ -1,0 +1,126 @@
+/*
+ * skyrl_layers.h — C ABI of libskyrl_layers.so: the decoder-layer mechanisms of the hybrid decoders
+ * (inference_engines/hybrid.py) on MI355X (gfx950). A library of its own, so that serving such a
+ * model compiles these kernels only. Conventions (status codes, dtype codes, stream order, no
+ * allocation, skyrl_last_error()) are those of skyrl_hip.h.
+ *
+ * `dtype` is the element type T of activations and weights: SKYRL_BF16, or SKYRL_F32 for a model run
+ * wholly in 32-bit. The residual stream, norms, rotary angles, attention scores and weights, gates
+ * and recurrent state are f32 for either.
+ */
+#ifndef SKYRL_LAYERS_H
+#define SKYRL_LAYERS_H
+
+#include "skyrl_hip.h"
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+/* ---- norms, activations, logits -------------------------------------------------------------
+ *   skyrl_add_norm  hidden f32 [n, H] += delta T [n, H] (may be NULL) and += step T [H] (may be
+ *                   NULL: one vector for every row); out T [n, H] = norm(hidden) * weight T [H].
+ *                   kind 0: layer norm without bias (mean taken off, variance = mean squared
+ *                   deviation), 1: RMS norm; eps inside the root. H <= 8192.
+ *   skyrl_gate_mul  out T [n, I] = act(gate) * up of gate_up T [n, 2I] (gate | up);
+ *                   act 0: silu, 1: gelu in its tanh form. The product is f32, rounded once.
+ *   skyrl_softcap   out f32 = cap * tanh(x / cap) over count elements of x T (cap <= 0: a copy). */
+#define SKYRL_NORM_LAYER 0
+#define SKYRL_NORM_RMS 1
+#define SKYRL_ACT_SILU 0
+#define SKYRL_ACT_GELU_TANH 1
+int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, int32_t n, int32_t H,
+                   float eps, int32_t kind, void* out, int32_t dtype, void* stream);
+int skyrl_gate_mul(const void* gate_up, int64_t n, int32_t I, int32_t act, void* out, int32_t dtype, void* stream);
+int skyrl_softcap(const void* x, float* out, int64_t count, float cap, int32_t dtype, void* stream);
+
+/* ---- latent attention over a paged latent cache ----------------------------------------------
+ * A layer run's cache is T [num_blocks, 16, row]: per token the normed latent (rank), the rotated key
+ * part all heads share (rot_dim), zero padding up to row = a multiple of 32. slot = block * 16 +
+ * offset. Token t of a step belongs to row bt_row[t] of block_tables i32 [*, bt_stride] and attends
+ * to the cached positions [max(0, positions[t] - window + 1), positions[t]] (window <= 0: all).
+ *   skyrl_latent_write   proj T [T, proj_stride]: q (heads x (dim + rot_dim)) | latent (rank) | key
+ *                        part (rot_dim). Rotates the q parts in place (interleaved pairs), writes the
+ *                        RMS-normed latent (weight T [rank]) and the rotated key part into the cache
+ *                        at slots[t] (< 0: no write). cos_sin f32 [max_pos, rot_dim] = cos | sin
+ *                        halves, one entry per pair, amplitude included.
+ *   skyrl_latent_attend  one query row per token in the latent space: qa T [heads, T, rank] is the
+ *                        unrotated query times the key up-projection, q_rot points at the rotated part
+ *                        of head 0 of token 0 (token stride q_stride, head stride q_head); out
+ *                        T [heads, T, rank] = softmax(scale * (qa.c + q_rot.k_rot)) c. nparts waves
+ *                        share a token's keys (MFMA form, bf16); part_min >= 16 keys, a multiple of
+ *                        16, per wave; nparts > 1 needs skyrl_latent_attend_workspace_bytes. f32, and
+ *                        shapes outside the MFMA form (skyrl_latent_attend_mfma == 0), take a plain
+ *                        kernel and ignore nparts.
+ *   skyrl_latent_gather  prompt form, step 1: copies for each of nseg segments the cached rows of
+ *                        positions [seg_first, seg_first + seg_count) (seg i32 [nseg, 4]: block-table
+ *                        row, first position, count, first packed row) to latent T [rows, rank] and
+ *                        k_rot T [rows, rot_dim].
+ *   skyrl_latent_prefill prompt form, step 2 (bf16): per head keys k_nope [rows, k_stride] (head h at
+ *                        h * dim) | k_rot, values transposed v_t [heads * vdim, vt_stride] over packed
+ *                        rows; one workgroup per (tile, head), tiles i32 [ntiles, 8]: first token,
+ *                        token count (<= 128), position of the first token, first packed row of its
+ *                        segment, position of that row, 0, 0, 0. A segment's packed rows are a multiple
+ *                        of 64 (skyrl_latent_gather zeroes the padding rows). out T [T, out_stride], head h at
+ *                        h * vdim. dim + rot_dim <= 256, vdim <= 256, vt_stride % 64 == 0. */
+int skyrl_latent_write(void* proj, int64_t proj_stride, int32_t T, int32_t heads, int32_t dim, int32_t rot_dim,
+                       int32_t rank, const void* norm_weight, float eps, const int64_t* positions,
+                       const int64_t* slots, const float* cos_sin, void* cache, int32_t row, int32_t dtype,
+                       void* stream);
+int skyrl_latent_attend_mfma(int32_t rank, int32_t rot_dim, int32_t row, int32_t dtype);
+size_t skyrl_latent_attend_workspace_bytes(int32_t T, int32_t heads, int32_t rank, int32_t nparts);
+int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_stride, int64_t q_head, const void* cache,
+                        int32_t row, const int32_t* block_tables, int64_t bt_stride, const int32_t* bt_row,
+                        const int64_t* positions, int32_t T, int32_t heads, int32_t rank, int32_t rot_dim,
+                        float scale, int32_t window, int32_t part_min, int32_t nparts, void* out, void* workspace,
+                        int32_t dtype, void* stream);
+int skyrl_latent_gather(const void* cache, int32_t row, const int32_t* block_tables, int64_t bt_stride,
+                        const int32_t* seg, int32_t nseg, int32_t max_count, int32_t rank, int32_t rot_dim,
+                        void* latent, void* k_rot, int32_t dtype, void* stream);
+int skyrl_latent_prefill(const void* q, int64_t q_stride, const void* k_nope, int64_t k_stride, const void* k_rot,
+                         const void* v_t, int64_t vt_stride, const int32_t* tiles, int32_t ntiles, int32_t heads,
+                         int32_t dim, int32_t rot_dim, int32_t vdim, float scale, int32_t window, void* out,
+                         int64_t out_stride, void* stream);
+
+/* ---- gated delta rule ------------------------------------------------------------------------
+ * proj T [T, proj_stride]: q (kv_heads x dim) | k (kv_heads x dim) | v (heads x vdim) | output gate
+ * (heads x vdim) | beta (heads) | decay (heads). q, k and v pass a causal convolution over time
+ * (conv_w T [2 kv_heads dim + heads vdim, taps], last tap on the current token) and silu; q and k
+ * become unit vectors, q times dim^-1/2. Per head: S <- g S; u = sigmoid(beta) (v - S^T k); S <- S +
+ * k u^T; o = S^T q with g = exp(-exp(A_log) softplus(decay + dt_bias)); out = rms_norm(o) * norm_w *
+ * silu(output gate).
+ * State per row: S f32 [rows, heads, dim, vpad], vpad = vdim up to a multiple of 4, and the last
+ * `taps` inputs of the convolutions, T [rows, taps, channels], the input of position p at p % taps. A
+ * sequence that starts at position 0 starts from zero, whatever the row holds.
+ * Sequences: tokens [cu[s], cu[s+1]) of row rows[s] (< 0: skipped, nothing written), their positions
+ * consecutive from positions[cu[s]].
+ *   skyrl_delta_scan       token by token, the state in registers: decode steps and short portions.
+ *                          save_conv 1 also stores the convolution inputs and needs every sequence to
+ *                          have one token; otherwise skyrl_delta_save follows.
+ *   skyrl_delta_save       stores the last inputs of every sequence.
+ *   skyrl_delta_conv       prompt form, step 1: qk f32 [T, 2, kv_heads, dim] (unit vectors), v f32
+ *                          [T, heads, vdim], lg f32 [T, heads] (log decay), beta f32 [T, heads].
+ *   skyrl_delta_chunk      step 2, one workgroup per (chunk, head): chunk i32 [nchunks, 4] (first
+ *                          token, tokens <= 64, sequence, 0). Solves the chunk's own triangular system
+ *                          and writes W f32 [nchunks, heads, 64, dim], U f32 [nchunks, heads, 64,
+ *                          vpad], P f32 [nchunks, heads, 64, 64] and G f32 [nchunks, heads, 64]
+ *                          (summed log decays).
+ *   skyrl_delta_chain      step 3, sequential over a sequence's chunks (seq_chunks i32 [nseq + 1]):
+ *                          reads and writes S, o f32 [T, heads, vdim].
+ *   skyrl_delta_out        step 4: out T from o. */
+typedef struct skyrl_delta_shape {
+    int32_t heads, kv_heads, dim, vdim, taps;
+    float eps; /* of the output norm */
+} skyrl_delta_shape;
+int skyrl_delta_scan(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride, const void* conv_w,
+                     const float* a_log, const float* dt_bias, const void* norm_w, const int32_t* cu,
+                     const int32_t* rows, const int64_t* positions, int32_t nseq, float* state, void* conv_state,
+                     int32_t save_conv, void* out, int64_t out_stride, int32_t dtype, void* stream);
+int skyrl_delta_save(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride, const int32_t* cu,
+                     const int32_t* rows, const int64_t* positions, int32_t nseq, void* conv_state, int32_t dtype,
+                     void* stream);
+
+#ifdef __cplusplus
+}
+#endif
+#endif /* SKYRL_LAYERS_H */

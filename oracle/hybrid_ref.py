@@ -1,0 +1,191 @@
+"""Plain CPU restatement of the hybrid decoder (latent attention + gated delta rule layers), one
+function per mechanism, whole sequences at a time, in the dtype of its weights (float64 in the tests).
+Test infrastructure only: nothing under skyrl_amd/ imports it and it shares no code with it.
+
+`w` maps tensor names to CPU tensors; `cfg` is the parsed config.json.
+"""
+
+from __future__ import annotations
+
+import math
+
+import torch
+
+
+def layer_norm(x, w, eps):
+    d = x - x.mean(-1, keepdim=True)
+    return d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * w
+
+
+def rms_norm(x, w, eps):
+    return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w
+
+
+def rotary_frequencies(rot):
+    """(frequencies [dims/2], amplitude of cos and sin); YaRN interpolation when rot has 'scaling'."""
+    D, base = rot["dims"], rot["base"]
+    f = [base ** (-2.0 * i / D) for i in range(D // 2)]
+    sc = rot.get("scaling")
+    if not sc:
+        return f, 1.0
+
+    def dim_of(turns):
+        return D * math.log(sc["original"] / (2 * math.pi * turns)) / (2 * math.log(base))
+
+    lo = max(math.floor(dim_of(sc["fast"])), 0)
+    hi = min(math.ceil(dim_of(sc["slow"])), D - 1)
+    out = []
+    for i, fi in enumerate(f):
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        out.append(fi / sc["factor"] * ramp + fi * (1 - ramp))
+    return out, 0.1 * math.log(sc["factor"]) + 1.0
+
+
+def rotate_pairs(x, positions, rot):
+    """Interleaved rotary of the first rot.dims of x [T, ..., D]."""
+    f, amp = rotary_frequencies(rot)
+    y = x.clone()
+    for i, fi in enumerate(f):
+        a = positions.to(torch.float64) * fi
+        c, s = (torch.cos(a) * amp).to(x.dtype), (torch.sin(a) * amp).to(x.dtype)
+        shape = (-1,) + (1,) * (x.dim() - 2)
+        c, s = c.view(shape), s.view(shape)
+        u, v = x[..., 2 * i], x[..., 2 * i + 1]
+        y[..., 2 * i] = u * c - v * s
+        y[..., 2 * i + 1] = v * c + u * s
+    return y
+
+
+def window_attention(q, k, v, scale, size):
+    """q, k [T, H, D], v [T, H, V]; position i sees j with 0 <= i - j < size (None: every j <= i)."""
+    T = q.shape[0]
+    s = torch.einsum("ihd,jhd->hij", q, k) * scale
+    i = torch.arange(T)
+    d = i[:, None] - i[None]
+    see = d >= 0
+    if size is not None:
+        see &= d < size
+    s = s.masked_fill(~see, float("-inf"))
+    return torch.einsum("hij,jhv->ihv", torch.softmax(s, -1), v)
+
+
+def latent_attention(h, w, p, m, eps):
+    T = h.shape[0]
+    H, D, R, V, C = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+    pos = torch.arange(T)
+    q = (h @ w[p + "q"].T).view(T, H, D + R)
+    down = h @ w[p + "dkv"].T
+    c = rms_norm(down[:, :C], w[p + "dkv.norm"], eps)
+    qr = rotate_pairs(q[..., D:], pos, m["rot"])
+    kr = rotate_pairs(down[:, C:], pos, m["rot"])
+    k = (c @ w[p + "uk"].T).view(T, H, D)
+    v = (c @ w[p + "uv"].T).view(T, H, V)
+    q = torch.cat([q[..., :D], qr], -1)
+    k = torch.cat([k, kr[:, None].expand(T, H, R)], -1)
+    mask = m.get("mask")
+    o = window_attention(q, k, v, m["scale"], mask["size"] if mask else None)
+    return o.reshape(T, H * V) @ w[p + "o"].T
+
+
+def silu(x):
+    return x * torch.sigmoid(x)
+
+
+def short_conv(x, w):
+    """Causal per-channel convolution of x [T, C] with w [C, taps], the last tap on the current token."""
+    y = torch.zeros_like(x)
+    taps = w.shape[1]
+    for t in range(x.shape[0]):
+        for j in range(taps):
+            s = t - (taps - 1) + j
+            if s >= 0:
+                y[t] += x[s] * w[:, j]
+    return y
+
+
+def unit(x):
+    return x / torch.sqrt((x * x).sum(-1, keepdim=True) + 1e-6)
+
+
+def delta_gates(h, w, p):
+    """(beta, decay g), each [T, heads]."""
+    beta = torch.sigmoid(h @ w[p + "b"].T)
+    z = h @ w[p + "a"].T + w[p + "dt_bias"]
+    softplus = torch.where(z > 0, z, torch.zeros_like(z)) + torch.log1p(torch.exp(-z.abs()))
+    return beta, torch.exp(-torch.exp(w[p + "A_log"]) * softplus)
+
+
+def delta_recurrence(q, k, v, beta, g, state=None):
+    """q, k [T, H, D], v [T, H, V], beta, g [T, H] -> outputs [T, H, V] and the final state [H, D, V]."""
+    T, H, D = q.shape
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype) if state is None else state.clone()
+    out = torch.zeros_like(v)
+    for t in range(T):
+        for h in range(H):
+            s = S[h] * g[t, h]
+            u = beta[t, h] * (v[t, h] - s.T @ k[t, h])
+            s = s + torch.outer(k[t, h], u)
+            out[t, h] = s.T @ q[t, h]
+            S[h] = s
+    return out, S
+
+
+def delta_mixer(h, w, p, m, eps):
+    T = h.shape[0]
+    H, K, D, V = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q = silu(short_conv(h @ w[p + "q"].T, w[p + "q.conv"])).view(T, K, D)
+    k = silu(short_conv(h @ w[p + "k"].T, w[p + "k.conv"])).view(T, K, D)
+    v = silu(short_conv(h @ w[p + "v"].T, w[p + "v.conv"])).view(T, H, V)
+    group = torch.tensor([hh // (H // K) for hh in range(H)])
+    q, k = (unit(q) * D ** -0.5)[:, group], unit(k)[:, group]
+    beta, g = delta_gates(h, w, p)
+    o, _ = delta_recurrence(q, k, v, beta, g)
+    o = rms_norm(o, w[p + "norm"], eps) * silu(h @ w[p + "g"].T).view(T, H, V)
+    return o.reshape(T, H * V) @ w[p + "o"].T
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1 + torch.tanh(math.sqrt(2 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def dense_ff(h, w, p):
+    return (gelu_tanh(h @ w[p + "gate"].T) * (h @ w[p + "up"].T)) @ w[p + "down"].T
+
+
+def layer(x, w, i, entry, eps):
+    p = f"l{i}."
+    h = layer_norm(x, w[p + "norm1"], eps)
+    mixer = {"latent_attention": latent_attention, "delta": delta_mixer}[entry["type"]]
+    x = x + mixer(h, w, p + "mix.", entry["mixer"], eps)
+    if entry.get("mlp"):
+        x = x + dense_ff(layer_norm(x, w[p + "norm2"], eps), w, p + "mlp.")
+    return x
+
+
+def layer_runs(cfg):
+    """[(layer, pass or None)]: None outside the loop; pass t's step vector is added before its first layer."""
+    n, lp = len(cfg["layers"]), cfg.get("loop")
+    if not lp:
+        return [(i, None) for i in range(n)]
+    a, b = lp["start"], lp["stop"]
+    runs = [(i, None) for i in range(a)]
+    for t in range(lp["times"]):
+        runs += [(i, t if i == a else None) for i in range(a, b)]
+    return runs + [(i, None) for i in range(b, n)]
+
+
+def forward(tokens, w, cfg):
+    """Logits [T, vocab] and the residual after every layer run [runs, T, width]."""
+    eps = cfg["norm"]["eps"]
+    x = w["embed"][torch.as_tensor(tokens)]
+    trail = []
+    for i, t in layer_runs(cfg):
+        if t is not None:
+            x = x + w["loop.step"][t]
+        x = layer(x, w, i, cfg["layers"][i], eps)
+        trail.append(x)
+    logits = layer_norm(x, w["final.norm"], eps) @ w["head"].T
+    cap = cfg.get("logit_softcap")
+    if cap:
+        logits = cap * torch.tanh(logits / cap)
+    return logits, torch.stack(trail)

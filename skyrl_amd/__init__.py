@@ -17,7 +17,8 @@ def native_library_path() -> str:
 
 
 def require_native():
-    """Load the HIP library (raises ImportError if it was not built)."""
+    """Load the HIP libraries (raises ImportError if one was not built)."""
     from . import _ffi
 
+    _ffi.load_layers()
     return _ffi.load()

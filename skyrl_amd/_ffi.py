@@ -19,7 +19,9 @@ import threading
 
 import torch  # noqa: F401  (must precede the CDLL load, see module docstring)
 
-LIB_PATH = os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib", "libskyrl_hip.so")
+LIB_DIR = os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib")
+LIB_PATH = os.path.join(LIB_DIR, "libskyrl_hip.so")
+LAYERS_PATH = os.path.join(LIB_DIR, "libskyrl_layers.so")
 
 F32, BF16, I64, I32, U8 = 0, 1, 2, 3, 4
 M_FINAL_LOSS, M_POLICY_LOSS, M_ENTROPY, M_KL, M_CLIP_RATIO, M_MASK_SUM = 0, 1, 2, 3, 4, 5
@@ -214,6 +216,38 @@ SIGNATURES = {
     "skyrl_silu_mul": (_INT, [_P, _I64, _I32, _P, _P]),
 }
 
+
+class DeltaShape(ctypes.Structure):
+    """Mirror of ``skyrl_delta_shape`` (include/skyrl_layers.h)."""
+
+    _fields_ = [
+        ("heads", ctypes.c_int32),
+        ("kv_heads", ctypes.c_int32),
+        ("dim", ctypes.c_int32),
+        ("vdim", ctypes.c_int32),
+        ("taps", ctypes.c_int32),
+        ("eps", ctypes.c_float),
+    ]
+
+
+# the exported surface of include/skyrl_layers.h, in a library of its own (libskyrl_layers.so)
+_DS = ctypes.POINTER(DeltaShape)
+LAYERS_SIGNATURES = {
+    "skyrl_add_norm": (_INT, [_P, _P, _P, _P, _I32, _I32, _F, _I32, _P, _I32, _P]),
+    "skyrl_gate_mul": (_INT, [_P, _I64, _I32, _I32, _P, _I32, _P]),
+    "skyrl_softcap": (_INT, [_P, _P, _I64, _F, _I32, _P]),
+    "skyrl_latent_write": (_INT, [_P, _I64, _I32, _I32, _I32, _I32, _I32, _P, _F, _P, _P, _P, _P, _I32, _I32, _P]),
+    "skyrl_latent_attend_mfma": (_INT, [_I32, _I32, _I32, _I32]),
+    "skyrl_latent_attend_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
+    "skyrl_latent_attend": (_INT, [_P, _P, _I64, _I64, _P, _I32, _P, _I64, _P, _P, _I32, _I32, _I32, _I32, _F, _I32,
+                                   _I32, _I32, _P, _P, _I32, _P]),
+    "skyrl_latent_gather": (_INT, [_P, _I32, _P, _I64, _P, _I32, _I32, _I32, _I32, _P, _P, _I32, _P]),
+    "skyrl_latent_prefill": (_INT, [_P, _I64, _P, _I64, _P, _P, _I64, _P, _I32, _I32, _I32, _I32, _I32, _F, _I32, _P,
+                                    _I64, _P]),
+    "skyrl_delta_scan": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I32, _P, _I64, _I32, _P]),
+    "skyrl_delta_save": (_INT, [_DS, _P, _I64, _P, _P, _P, _I32, _P, _I32, _P]),
+}
+
 # entry points with a per-call variant form (name + "_ex": the same arguments, then the variant)
 EX_FORMS = ("skyrl_grpo_advantage", "skyrl_ppo_loss_fwd", "skyrl_grpo_ppo_loss_fwd", "skyrl_ppo_loss_bwd",
             "skyrl_ppo_loss_finish", "skyrl_logprob_fwd", "skyrl_logprob_bwd", "skyrl_lmhead_gemm",
@@ -260,39 +294,54 @@ def current_variant():
 
 
 _lock = threading.Lock()
-_lib = None
+_libs: dict = {}
 
 
 def lib_available() -> bool:
     return os.path.exists(LIB_PATH)
 
 
-def load() -> ctypes.CDLL:
-    """Load the library once and bind every signature. Raises if it is missing."""
-    global _lib
-    if _lib is not None:
-        return _lib
+def _open(path: str, signatures: dict) -> ctypes.CDLL:
+    lib = _libs.get(path)
+    if lib is not None:
+        return lib
     with _lock:
-        if _lib is not None:
-            return _lib
-        if not os.path.exists(LIB_PATH):
+        if path in _libs:
+            return _libs[path]
+        if not os.path.exists(path):
             raise ImportError(
-                f"skyrl_amd HIP library not built: {LIB_PATH} is missing. "
+                f"skyrl_amd HIP library not built: {path} is missing. "
                 "Run `python -c 'import __graft_entry__ as g; g.build()'` (make -C skyrl_amd/csrc)."
             )
-        lib = ctypes.CDLL(LIB_PATH, mode=ctypes.RTLD_LOCAL)
-        for name, (res, args) in SIGNATURES.items():
+        lib = ctypes.CDLL(path, mode=ctypes.RTLD_LOCAL)
+        for name, (res, args) in signatures.items():
             fn = getattr(lib, name)
             fn.restype = res
             fn.argtypes = args
-        _lib = lib
+        _libs[path] = lib
         return lib
+
+
+def load() -> ctypes.CDLL:
+    """Load libskyrl_hip.so once and bind every signature. Raises if it is missing."""
+    return _open(LIB_PATH, SIGNATURES)
+
+
+def load_layers() -> ctypes.CDLL:
+    """libskyrl_layers.so, likewise."""
+    lib = _open(LAYERS_PATH, LAYERS_SIGNATURES)
+    lib.skyrl_last_error.restype = ctypes.c_char_p
+    return lib
+
+
+def _lib_of(name: str) -> ctypes.CDLL:
+    return load_layers() if name in LAYERS_SIGNATURES else load()
 
 
 def call(name: str, *args) -> int:
     """Invoke a status-returning entry point; raise SkyrlHipError on a non-zero status. Under an
     active ``variant(...)`` an entry point with an _ex form runs that form with the variant."""
-    lib = load()
+    lib = _lib_of(name)
     v = _VARIANT.get()
     if v is not None and name in EX_FORMS:
         rc = getattr(lib, name + "_ex")(*args, ctypes.byref(v))
@@ -309,4 +358,4 @@ def query(name: str, *args):
     v = _VARIANT.get()
     if v is not None and name in EX_FORMS:
         return getattr(load(), name + "_ex")(*args, ctypes.byref(v))
-    return getattr(load(), name)(*args)
+    return getattr(_lib_of(name), name)(*args)

@@ -11,8 +11,10 @@ request returns the tokens generated so far with stop_reason "abort").
 Layers:
   * EngineCore — scheduler: waiting/running queues, block allocation with recompute
     preemption, stop conditions. Pure host logic over a runner interface (CPU-testable).
-  * ModelRunner — builds the device inputs of one scheduled batch, runs PagedDecoder
-    (prefill or decode) and the HIP sampler (skyrl_sample), returns tokens/logprobs.
+    For a model that serves portions (HybridDecoder) a step mixes portions of prompts with
+    decoded tokens under one token budget; `run_portions` is the same step with given tokens.
+  * ModelRunner — builds the device inputs of one scheduled batch, runs the decoder (prefill,
+    decode or portions) and the HIP sampler (skyrl_sample), returns tokens/logprobs.
   * AMDInferenceEngine — the async InferenceEngineInterface: generate/sample, abort,
     sleep/wake_up, weight updates (WeightUpdateRequest + receiver, or named tensors).
 
@@ -126,6 +128,7 @@ class Request:
     state: int = WAITING
     row: int = -1  # persistent batch row while running (the runner's per-row device state)
     num_cached: int = 0  # leading tokens whose K/V came from the prefix cache at admission
+    num_computed: int = 0  # leading tokens the cache or state holds (models that serve portions)
     block_hashes: List[int] = field(default_factory=list)
     finish_reason: Optional[str] = None
     on_finish: Optional[Callable[["Request"], None]] = None
@@ -133,6 +136,13 @@ class Request:
     @property
     def num_tokens(self) -> int:
         return len(self.prompt) + len(self.out_tokens)
+
+    def tokens(self, start: int, end: int) -> List[int]:
+        """Tokens [start, end) of prompt + output."""
+        p = len(self.prompt)
+        if end <= p:
+            return self.prompt[start:end]
+        return self.prompt[start:] + self.out_tokens[max(0, start - p):end - p]
 
 
 class BlockAllocator:
@@ -218,11 +228,12 @@ def block_hashes(tokens: Sequence[int], nblocks: int) -> List[int]:
 
 @dataclass
 class ScheduledBatch:
-    kind: str                       # "prefill" | "decode"
+    kind: str                       # "prefill" | "decode" | "portions"
     requests: List[Request]
     # per request: (temperature, top_k, top_p, min_p), sampler key, mask-stop flag
     keys: np.ndarray                # int64 [n]: (key << 20) | response position
     suppress: List[Tuple[int, ...]]  # stop ids to mask (min_tokens not reached), per request
+    counts: Optional[List[int]] = None  # portions: tokens each request runs, from its num_computed on
 
 
 def _blocks_needed(num_tokens: int) -> int:
@@ -234,7 +245,10 @@ class EngineCore:
 
     def __init__(self, runner, num_blocks: int, max_num_seqs: int = 512, max_model_len: int = 4096,
                  max_prefill_tokens: int = 32768, eos_token_id: Optional[int] = None, seed: int = 0,
-                 detokenize: Optional[Callable[[List[int]], str]] = None, enable_prefix_caching: bool = False):
+                 detokenize: Optional[Callable[[List[int]], str]] = None, enable_prefix_caching: bool = False,
+                 portions: bool = False):
+        # portions: a step mixes decoded tokens with portions of prompts, max_prefill_tokens in all
+        self.portions = portions
         self.runner = runner
         self.detokenize = detokenize  # stop strings are matched on the decoded tail of the output
         self.allocator = BlockAllocator(num_blocks, enable_caching=enable_prefix_caching)
@@ -374,6 +388,7 @@ class EngineCore:
             self.allocator.free(victim.blocks)
             victim.blocks = []
             self._release_row(victim)
+            victim.num_computed = 0
             victim.state = WAITING
             self.waiting.appendleft(victim)
             self.num_preemptions += 1
@@ -400,6 +415,8 @@ class EngineCore:
     def step(self) -> List[Request]:
         """Run one prefill or decode step; returns the requests that finished in it."""
         self.num_steps += 1
+        if self.portions:
+            return self._step_portions()
         batch = self._schedule_prefill()
         kind = "prefill"
         if not batch:
@@ -418,6 +435,12 @@ class EngineCore:
             for r in batch:  # the full blocks this prefill computed are now shareable
                 for i in range(r.num_cached // BLOCK_SIZE, len(r.block_hashes)):
                     self.allocator.register(r.blocks[i], r.block_hashes[i])
+        finished = self._append(batch, tokens, logprobs)
+        self._account(kind, t0, t1, t2)
+        return finished
+
+    def _append(self, batch: List[Request], tokens: np.ndarray, logprobs: np.ndarray) -> List[Request]:
+        """Take a step's samples; returns the requests they finished."""
         finished: List[Request] = []
         for r, t, lp in zip(batch, tokens.tolist(), logprobs.tolist()):
             r.out_tokens.append(t)
@@ -429,11 +452,101 @@ class EngineCore:
         if finished:
             done = {id(r) for r in finished}
             self.running = [r for r in self.running if id(r) not in done]
+        return finished
+
+    def _account(self, kind: str, t0: float, t1: float, t2: float) -> None:
         st = self.stats
         st[kind + "_steps"] += 1
         st[kind + "_exec_s"] += t2 - t1
         st[kind + "_host_s"] += (t1 - t0) + (time.perf_counter() - t2)
+
+    # ---------------------------------------------------------------- portions
+    def _schedule_portions(self) -> List[Tuple[Request, int]]:
+        """(request, tokens to run) of one step: every request that decodes gets its token; what is left
+        of the budget continues prompts, oldest first, then admits waiting requests (FIFO) while rows
+        and blocks last."""
+        self._ensure_decode_blocks()
+        work = [(r, 1) for r in self.running if r.num_tokens - r.num_computed == 1]
+        budget = max(1, self.max_prefill_tokens) - len(work)
+        for r in self.running:
+            left = r.num_tokens - r.num_computed
+            if left > 1 and budget > 0:
+                work.append((r, min(left, budget)))
+                budget -= work[-1][1]
+        while self.waiting and budget > 0 and len(self.running) < self.max_num_seqs:
+            r = self.waiting[0]
+            need = _blocks_needed(r.num_tokens + 1)
+            if need > self.allocator.num_free:
+                break
+            self.waiting.popleft()
+            r.blocks = self.allocator.allocate(need)
+            self._admit(r)
+            self.running.append(r)
+            work.append((r, min(r.num_tokens, budget)))
+            budget -= work[-1][1]
+        return work
+
+    def _admit(self, r: Request) -> None:
+        r.row = heapq.heappop(self._free_rows)
+        r.num_computed = 0
+        r.state = RUNNING
+
+    def _batch_of(self, work: List[Tuple[Request, int]]) -> ScheduledBatch:
+        reqs = [r for r, _ in work]
+        keys, sup = self._keys_and_masks(reqs)
+        decode = all(n == 1 and r.num_computed == r.num_tokens - 1 for r, n in work)
+        return ScheduledBatch("decode" if decode else "portions", reqs, keys, sup, [n for _, n in work])
+
+    def _step_portions(self) -> List[Request]:
+        t0 = time.perf_counter()
+        work = self._schedule_portions()
+        if not work:
+            return []
+        batch = self._batch_of(work)
+        t1 = time.perf_counter()
+        tokens, logprobs = self.runner.execute(batch)  # of the requests whose last token this step ran
+        t2 = time.perf_counter()
+        for r, n in work:
+            r.num_computed += n
+        finished = self._append([r for r, _ in work if r.num_computed == r.num_tokens], tokens, logprobs)
+        self._account(batch.kind, t0, t1, t2)
         return finished
+
+    def open_request(self) -> Request:
+        """A request whose tokens arrive through run_portions: it holds a row, and blocks as its tokens
+        need them, until close_request."""
+        if not self._free_rows:
+            raise RuntimeError("no free batch row")
+        r = Request(rid=next(self._rid), prompt=[], params=RequestParams(), key=0)
+        self._admit(r)
+        return r
+
+    def run_portions(self, entries: Sequence[Tuple[Request, Sequence[int], Sequence[int]]]):
+        """One step over given tokens: entries of (open request, its next tokens, places among them whose
+        logits are asked for). Returns the logits [wanted, vocab] in the order of the entries, None if
+        none are wanted. Nothing is sampled."""
+        if not self.portions:
+            raise RuntimeError("this model does not serve portions")
+        work, want = [], []
+        for i, (r, toks, places) in enumerate(entries):
+            if r.state != RUNNING or not toks:
+                raise ValueError("run_portions: a finished request or an empty portion")
+            n = r.num_tokens + len(toks)
+            if n > self.max_model_len:
+                raise ValueError(f"{n} tokens exceed max_model_len={self.max_model_len}")
+            r.prompt.extend(int(t) for t in toks)
+            r.blocks.extend(self.allocator.allocate(_blocks_needed(n) - len(r.blocks)))
+            work.append((r, len(toks)))
+            want += [(i, int(p)) for p in places]
+        logits = self.runner.portion_logits(self._batch_of(work), want)
+        for r, n in work:
+            r.num_computed += n
+        self.num_steps += 1
+        return logits
+
+    def close_request(self, r: Request) -> None:
+        """Give back an open request's row and blocks."""
+        self._finish(r, "stop")
 
     def _stop_reason(self, r: Request, tok: int) -> Optional[str]:
         p = r.params
@@ -485,7 +598,8 @@ class ModelRunner:
             fused_lmhead = "auto"
         if fused_lmhead not in ("auto", "always", "off"):
             raise ValueError(f"fused_lmhead must be 'auto', 'always' or 'off', got {fused_lmhead!r}")
-        fits = model.spec.hidden_size % 64 == 0 and str(getattr(model, "dtype", "")) == "torch.bfloat16"
+        fits = (model.plain_lm_head and model.spec.hidden_size % 64 == 0
+                and str(getattr(model, "dtype", "")) == "torch.bfloat16")
         self.fused_lmhead = fused_lmhead if fits else "off"
         self.fused_steps = 0  # decode/prefill steps sampled by the fused kernel
         self._last_nb = 0
@@ -512,10 +626,16 @@ class ModelRunner:
         self.d_i64 = torch.zeros((3, R), dtype=torch.int64, device=self.device)
         self.d_i32 = torch.zeros((R, self.max_blocks), dtype=torch.int32, device=self.device)
         self.d_ctx = torch.ones(R, dtype=torch.int32, device=self.device)
+        if model.portions:  # decode steps also name each row's state row (-1: idle)
+            self.h_rows = torch.full((R,), -1, dtype=torch.int32, pin_memory=pin)
+            self.n_rows = self.h_rows.numpy()
+            self.d_rows = torch.full((R,), -1, dtype=torch.int32, device=self.device)
+            self.d_iota = torch.arange(R + 1, dtype=torch.int32, device=self.device)
         self.d_keys = torch.zeros(R, dtype=torch.int64, device=self.device)
         self.tokens = torch.empty(R, dtype=torch.int32, device=self.device)
         self.lps = torch.empty(R, dtype=torch.float32, device=self.device)
         self.h_out = torch.zeros((2, R), dtype=torch.float64, pin_memory=pin)
+        self._staged = torch.cuda.Event() if pin and self.device.type == "cuda" else None
         self._nblk = np.zeros(R, dtype=np.int64)  # table entries already staged per row
         self._graphs: Dict[int, Tuple[Any, Any]] = {}
         self._pool = None
@@ -530,10 +650,7 @@ class ModelRunner:
 
     def ensure_cache(self, num_blocks: int):
         if self.cache is None:
-            from .model import PagedKVCache
-
-            s = self.model.spec
-            self.cache = PagedKVCache(s.num_layers, num_blocks, s.num_kv_heads, s.head_dim, self.device)
+            self.cache = self.model.make_cache(num_blocks, self.max_num_seqs)
             self._graphs.clear()
 
     def drop_graphs(self):
@@ -550,13 +667,14 @@ class ModelRunner:
 
         nparts = max_ctx = None
         if fixed:  # graph: the wave count is baked into the launch (the split adapts on device)
-            from . import kernels
-
-            max_ctx = self.model.max_model_len
-            nparts = kernels.choose_nparts(nb, self.model.spec.num_kv_heads, max_ctx)
-        return StepInputs(tokens=self.d_i64[0, :nb], positions=self.d_i64[1, :nb], slots=self.d_i64[2, :nb],
-                          block_tables=self.d_i32[:nb], context_lens=self.d_ctx[:nb], max_ctx=max_ctx or 0,
-                          nparts=nparts)
+            max_ctx, nparts = self.model.decode_split(nb)
+        inp = StepInputs(tokens=self.d_i64[0, :nb], positions=self.d_i64[1, :nb], slots=self.d_i64[2, :nb],
+                         block_tables=self.d_i32[:nb], context_lens=self.d_ctx[:nb], max_ctx=max_ctx or 0,
+                         nparts=nparts)
+        if self.model.portions:
+            inp.rows, inp.cu, inp.bt_row = self.d_rows[:nb], self.d_iota[:nb + 1], self.d_iota[:nb]
+            inp.one_token, inp.n_short, inp.short_tokens = True, nb, nb
+        return inp
 
     def _forward_hidden(self, inp):
         return self.model.forward_decode(inp, self.cache)
@@ -566,20 +684,18 @@ class ModelRunner:
         if g is not None:
             return g
         torch = self.torch
-        from . import kernels
-
-        s = self.model.spec
-        need = 0  # pre-size the merge workspace for every bucket: a graph must never see it move
-        for b in self.buckets:
-            nparts = kernels.choose_nparts(b, s.num_kv_heads, self.model.max_model_len)
-            need = max(need, _decode_ws_bytes(b, s.num_heads, s.head_dim, nparts))
-        self.model.workspace.get(need)
+        self.model.reserve(self.buckets)
         inp = self._decode_inputs(nb, fixed=True)
         side = torch.cuda.Stream(self.device)
         side.wait_stream(torch.cuda.current_stream(self.device))
+        if self.model.portions:  # the warm-up must not advance a recurrent state
+            self.d_rows.fill_(-1)
+            side.wait_stream(torch.cuda.current_stream(self.device))
         with torch.cuda.stream(side):
             self._forward_hidden(inp)  # warm-up outside capture (library handles, workspaces)
         torch.cuda.current_stream(self.device).wait_stream(side)
+        if self.model.portions:
+            self.d_rows.copy_(self.h_rows)
         if self._pool is None:
             self._pool = torch.cuda.graph_pool_handle()
         graph = torch.cuda.CUDAGraph()
@@ -589,6 +705,8 @@ class ModelRunner:
         return self._graphs[nb]
 
     def _stage_decode(self, reqs: List["Request"], nb: int) -> None:
+        if self._staged is not None:  # a step that fetched nothing may still be reading the pinned buffers
+            self._staged.synchronize()
         n_i64, n_i32, n_ctx = self.n_i64, self.n_i32, self.n_ctx
         n_i64[:, :nb] = 0
         n_i64[2, :nb] = -1
@@ -596,13 +714,15 @@ class ModelRunner:
         rows = np.fromiter((r.row for r in reqs), dtype=np.int64, count=len(reqs))
         L = np.fromiter((r.num_tokens for r in reqs), dtype=np.int64, count=len(reqs))
         for r in reqs:  # table rows: only newly allocated blocks are staged
+            if r.num_tokens == 1:  # a request that starts with a decode step: the row's table is another's
+                self._nblk[r.row] = 0
             k = self._nblk[r.row]
             if len(r.blocks) != k:
                 if len(r.blocks) < k:
                     k = 0
                 n_i32[r.row, k:len(r.blocks)] = r.blocks[k:]
                 self._nblk[r.row] = len(r.blocks)
-        n_i64[0, rows] = np.fromiter((r.out_tokens[-1] for r in reqs), dtype=np.int64, count=len(reqs))
+        n_i64[0, rows] = np.fromiter(((r.out_tokens or r.prompt)[-1] for r in reqs), dtype=np.int64, count=len(reqs))
         pos = L - 1
         n_i64[1, rows] = pos
         n_i64[2, rows] = n_i32[rows, pos // BLOCK_SIZE].astype(np.int64) * BLOCK_SIZE + pos % BLOCK_SIZE
@@ -610,6 +730,73 @@ class ModelRunner:
         self.d_i64[:, :nb].copy_(self.h_i64[:, :nb], non_blocking=True)
         self.d_i32[:nb].copy_(self.h_i32[:nb], non_blocking=True)
         self.d_ctx[:nb].copy_(self.h_ctx[:nb], non_blocking=True)
+        if self.model.portions:
+            self.n_rows[:nb] = -1
+            self.n_rows[rows] = rows
+            self.d_rows[:nb].copy_(self.h_rows[:nb], non_blocking=True)
+        if self._staged is not None:
+            self._staged.record(self.torch.cuda.current_stream(self.device))
+
+    # ---------------------------------------------------------------- portion inputs
+    def _portion_inputs(self, batch: ScheduledBatch, want: Sequence[Tuple[int, int]]):
+        """StepInputs of a portions step; want: (request index, place in its portion) per returned row.
+        Short portions come first (HybridDecoder.is_short), so that each form's tokens are a range."""
+        from .model import StepInputs
+
+        order = sorted(range(len(batch.requests)), key=lambda i: not self.model.is_short(batch.counts[i]))
+        reqs, lens = [batch.requests[i] for i in order], [batch.counts[i] for i in order]
+        starts = [r.num_computed for r in reqs]
+        n_short = sum(1 for n in lens if self.model.is_short(n))
+        n, T = len(reqs), sum(lens)
+        first = np.concatenate([[0], np.cumsum(lens)]).astype(np.int64)
+        place = {i: first[k] for k, i in enumerate(order)}
+        i64 = np.empty((3, T), dtype=np.int64)
+        width = max(len(r.blocks) for r in reqs)
+        tables = np.zeros((n, width), dtype=np.int32)
+        for k, (r, s, L) in enumerate(zip(reqs, starts, lens)):
+            a, b = first[k], first[k + 1]
+            i64[0, a:b] = r.tokens(s, s + L)
+            i64[1, a:b] = np.arange(s, s + L)
+            i64[2, a:b] = _slots(r.blocks, s, s + L)
+            tables[k, :len(r.blocks)] = r.blocks
+            self._nblk[r.row] = 0  # a decode step restages the row's table
+        wanted = np.fromiter((place[i] + p for i, p in want), dtype=np.int64, count=len(want))
+        d64 = self._h2d(np.concatenate([i64.reshape(-1), wanted]))
+        plan = self.model.plan(lens, starts, n_short)
+        parts = [first.astype(np.int32), np.fromiter((r.row for r in reqs), dtype=np.int32, count=n),
+                 np.repeat(np.arange(n, dtype=np.int32), lens), tables.reshape(-1)]
+        arrays = [] if plan is None else [(key, f) for key, p in plan.items() for f in range(len(p))
+                                          if isinstance(p[f], np.ndarray)]
+        parts += [plan[key][f].reshape(-1) for key, f in arrays]
+        offs = np.cumsum([0] + [(p.size + 3) // 4 * 4 for p in parts])  # 16-byte aligned pieces
+        flat = np.zeros(offs[-1], dtype=np.int32)
+        for p, o in zip(parts, offs):
+            flat[o:o + p.size] = p
+        d32 = self._h2d(flat)
+        piece = lambda k: d32[offs[k]:offs[k] + parts[k].size]  # noqa: E731
+        dplan = None
+        if plan is not None:
+            dplan = {key: list(p) for key, p in plan.items()}
+            for k, (key, f) in enumerate(arrays):
+                dplan[key][f] = piece(4 + k).view(plan[key][f].shape)
+        return StepInputs(tokens=d64[:T], positions=d64[T:2 * T], slots=d64[2 * T:3 * T], want=d64[3 * T:],
+                          block_tables=piece(3).view(n, width), max_ctx=max(s + L for s, L in zip(starts, lens)),
+                          seq_lens=lens, cached_lens=starts, rows=piece(1), cu=piece(0), bt_row=piece(2),
+                          n_short=n_short, short_tokens=sum(lens[:n_short]), plan=dplan)
+
+    def _run_portions(self, batch: ScheduledBatch, want: Sequence[Tuple[int, int]]):
+        return self.model.forward_portions(self._portion_inputs(batch, want), self.cache)
+
+    def portion_logits(self, batch: ScheduledBatch, want: Sequence[Tuple[int, int]]):
+        """Run one step; logits of the wanted (request index, place) tokens, or None."""
+        if batch.kind == "decode":
+            hidden = self._run_decode(batch.requests)
+            if not want:
+                return None
+            idx = np.fromiter((batch.requests[i].row for i, _ in want), dtype=np.int64, count=len(want))
+            return self.model.logits(hidden.index_select(0, self._h2d(idx)))
+        hidden = self._run_portions(batch, want)
+        return self.model.logits(hidden) if want else None
 
     # ---------------------------------------------------------------- execute
     def execute(self, batch: ScheduledBatch):
@@ -630,7 +817,15 @@ class ModelRunner:
 
         reqs = batch.requests
         n = len(reqs)
-        if batch.kind == "prefill":
+        if batch.kind == "portions":
+            done = [i for i, (r, c) in enumerate(zip(reqs, batch.counts)) if r.num_computed + c == r.num_tokens]
+            hidden = self._run_portions(batch, [(i, batch.counts[i] - 1) for i in done])
+            if not done:
+                return np.empty(0, dtype=np.int64), np.empty(0, dtype=np.float32)
+            batch = ScheduledBatch("portions", [reqs[i] for i in done], batch.keys[done],
+                                   [batch.suppress[i] for i in done])
+            rows = np.arange(len(done))
+        elif batch.kind == "prefill":
             cached = [r.num_cached for r in reqs]  # prefix-cache hits: only the suffix is computed
             seqs = [(r.prompt + r.out_tokens)[c:] for r, c in zip(reqs, cached)]
             lens = [len(s) for s in seqs]
@@ -653,19 +848,23 @@ class ModelRunner:
                 self._nblk[r.row] = 0  # (re)admitted row: restage its whole table
             rows = np.arange(n)
         else:
-            hi = 1 + max(r.row for r in reqs)
-            nb = next(b for b in self.buckets if b >= hi)
-            self._stage_decode(reqs, nb)
-            self._last_nb = nb
-            if self.use_graphs:
-                graph, hidden = self._graph(nb)
-                graph.replay()
-            else:
-                inp = self._decode_inputs(nb, fixed=False)
-                inp.max_ctx = int(max(r.num_tokens for r in reqs))
-                hidden = self._forward_hidden(inp)
+            hidden = self._run_decode(reqs)
             rows = np.fromiter((r.row for r in reqs), dtype=np.int64, count=n)
         return self._sample(hidden, batch, rows)
+
+    def _run_decode(self, reqs: List["Request"]):
+        """Hidden states [nb, H] of one decode step, indexed by batch row."""
+        hi = 1 + max(r.row for r in reqs)
+        nb = next(b for b in self.buckets if b >= hi)
+        self._stage_decode(reqs, nb)
+        self._last_nb = nb
+        if self.use_graphs:
+            graph, hidden = self._graph(nb)
+            graph.replay()
+            return hidden
+        inp = self._decode_inputs(nb, fixed=False)
+        inp.max_ctx = int(max(r.num_tokens for r in reqs))
+        return self._forward_hidden(inp)
 
     def _fused_ok(self, groups, batch: ScheduledBatch) -> bool:
         if self.fused_lmhead == "off" or len(groups) != 1 or any(batch.suppress):
@@ -679,7 +878,7 @@ class ModelRunner:
         # where the fused kernel measured faster (256 x 256 tiles waste MFMA work on mid-size
         # batches). Greedy: 143 vs 128 us at 64 rows, 143 vs 175 at 8, 248 vs 292 at 512. T > 0
         # (cross-tile row bar): 314 vs 319 us at 512 rows, 198 vs 188 at 256, so only full tiles.
-        nb = len(batch.requests) if batch.kind == "prefill" else self._last_nb
+        nb = self._last_nb if batch.kind == "decode" else len(batch.requests)
         if temp == 0.0:
             return unfiltered and (nb >= 192 or nb <= 16)
         return unfiltered and nb >= 480
@@ -720,7 +919,8 @@ class ModelRunner:
                 lg, ky = logits.index_select(0, idx), self.d_keys.index_select(0, idx)
                 to = torch.empty(len(grows), dtype=torch.int32, device=self.device)
                 lo = torch.empty(len(grows), dtype=torch.float32, device=self.device)
-            _ffi.call("skyrl_sample", _ptr(lg), _ffi.BF16, lg.stride(0), lg.shape[0], V, float(temp), int(top_k),
+            dt = _ffi.F32 if lg.dtype == torch.float32 else _ffi.BF16
+            _ffi.call("skyrl_sample", _ptr(lg), dt, lg.stride(0), lg.shape[0], V, float(temp), int(top_k),
                       float(top_p), float(min_p), self.seed & 0xFFFFFFFFFFFFFFFF, _ptr(ky), 0, _ptr(to), _ptr(lo),
                       _ptr(self._sampler_ws), st)
             if len(groups) != 1:
@@ -777,12 +977,6 @@ class ModelRunner:
         return o[0, rows].astype(np.int64), o[1, rows].astype(np.float32)
 
 
-def _decode_ws_bytes(nseq: int, nh: int, head_dim: int, nparts: int) -> int:
-    from .. import _ffi
-
-    return int(_ffi.query("skyrl_paged_decode_workspace_bytes", nseq, nh, head_dim, nparts))
-
-
 def _slots(blocks: List[int], start: int, end: int) -> np.ndarray:
     p = np.arange(start, end, dtype=np.int64)
     b = np.asarray(blocks, dtype=np.int64)
@@ -792,7 +986,7 @@ def _slots(blocks: List[int], start: int, end: int) -> np.ndarray:
 class AMDInferenceEngine(InferenceEngineInterface):
     """One rollout engine on one GPU (tp = pp = dp = 1), asyncio-driven.
 
-    `model` is a PagedDecoder; `num_blocks` sizes the KV cache (default: ``kv_cache_fraction``
+    `model` is a PagedDecoder or a HybridDecoder; `num_blocks` sizes the KV cache (default: ``kv_cache_fraction``
     of the free HBM after weights). Decoding runs in a background task while any request is
     unfinished; each step is one prefill or decode batch of every running request."""
 
@@ -805,12 +999,11 @@ class AMDInferenceEngine(InferenceEngineInterface):
         if num_blocks is None:
             import torch
 
-            from .model import PagedKVCache
-
             free, _ = torch.cuda.mem_get_info(model.device)
-            s = model.spec
-            num_blocks = int(free * kv_cache_fraction) // PagedKVCache.bytes_per_block(
-                s.num_layers, s.num_kv_heads, s.head_dim)
+            room = int(free * kv_cache_fraction) - max_num_seqs * model.row_bytes()
+            num_blocks = room // model.block_bytes()
+            if num_blocks < 1:
+                raise ValueError("max_num_seqs state rows leave no memory for cache blocks")
         self.num_blocks = num_blocks
         self.runner = runner if runner is not None else ModelRunner(model, num_blocks, max_num_seqs, seed,
                                                                          use_graphs=use_graphs,
@@ -821,7 +1014,9 @@ class AMDInferenceEngine(InferenceEngineInterface):
                                eos_token_id=model.spec.eos_token_id, seed=seed,
                                detokenize=(lambda ids: tokenizer.decode(ids, skip_special_tokens=True))
                                if tokenizer is not None else None,
-                               enable_prefix_caching=enable_prefix_caching)
+                               enable_prefix_caching=(enable_prefix_caching
+                                                      and getattr(model, "prefix_cacheable", True)),
+                               portions=getattr(model, "portions", False))
         self._task: Optional[asyncio.Task] = None
         self._futures: Dict[int, asyncio.Future] = {}
         self._receiver = None

@@ -1,0 +1,251 @@
+"""Hybrid decoder: a list of layers, each with its own kind of mixer (paged attention or recurrent
+state) and feed-forward, part of which may run several times with the same weights.
+
+Dovidra is such a design: latent attention under a sliding window beside gated delta rule layers,
+bias-free layer norms before each half, tanh-form GELU gates, a looped range of layers that adds one
+learned vector per pass, and a tanh cap on the logits. The model is what config.json lists; the
+mechanisms are mixers.py.
+
+The residual stream is f32. One pass of the HIP norm kernel adds the previous half-layer's output and
+(at the start of a loop pass) its vector, stores the stream and writes the next product's input.
+
+HybridDecoder has PagedDecoder's interface (model.py), so the engine's scheduler, runner, sampler and
+weight updates serve it unchanged; besides, it takes portions: a step may continue several prompts
+and decode others at the same time (`forward_portions`).
+"""
+
+from __future__ import annotations
+
+from dataclasses import dataclass
+from typing import Any, Dict, Iterable, Iterator, List, Optional, Tuple
+
+import torch
+import torch.nn.functional as F
+
+from . import kernels
+from . import layer_kernels as lk
+from .mixers import FEEDFORWARDS, MIXERS, PROMPT_MIN, Weights, prompt_plan
+from .model import StepInputs
+
+DEFAULT_MAX_MODEL_LEN = 32768
+
+
+@dataclass
+class LayerRun:
+    layer: int
+    step: Optional[int] = None  # the pass whose vector is added before this layer (first layer of a pass)
+
+
+@dataclass
+class HybridSpec:
+    """What the engine reads of a model, and the layer order."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    logit_softcap: Optional[float]
+    layers: List[Dict[str, Any]]
+    runs: List[LayerRun]
+    loop_times: int
+    max_position_embeddings: int
+    eos_token_id: Optional[int] = None
+    tie_word_embeddings: bool = False
+    initializer_range: float = 0.02
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.runs)
+
+    @classmethod
+    def from_config(cls, cfg: Dict[str, Any]) -> "HybridSpec":
+        layers = cfg["layers"]
+        for e in layers:
+            if e["type"] not in MIXERS:
+                raise ValueError(f"unknown layer type {e['type']!r} (known: {sorted(MIXERS)})")
+            if e.get("mlp") and e["mlp"]["kind"] not in FEEDFORWARDS:
+                raise ValueError(f"unknown feed-forward {e['mlp']['kind']!r} (known: {sorted(FEEDFORWARDS)})")
+        n, loop = len(layers), cfg.get("loop")
+        runs, times = [], 0
+        if loop:
+            a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+            if not 0 <= a <= b <= n or times < 0:
+                raise ValueError(f"loop {loop} does not fit {n} layers")
+            runs += [LayerRun(i) for i in range(a)]
+            for t in range(times):
+                runs += [LayerRun(i, t if i == a else None) for i in range(a, b)]
+            runs += [LayerRun(i) for i in range(b, n)]
+        else:
+            runs = [LayerRun(i) for i in range(n)]
+        eos = cfg.get("eos_token_id")
+        return cls(vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]), norm_eps=float(cfg["norm"]["eps"]),
+                   logit_softcap=float(cfg["logit_softcap"]) if cfg.get("logit_softcap") else None, layers=layers,
+                   runs=runs, loop_times=times,
+                   max_position_embeddings=int(cfg.get("max_position_embeddings") or DEFAULT_MAX_MODEL_LEN),
+                   eos_token_id=None if eos is None else int(eos))
+
+
+class HybridCache:
+    """Cache or state of every layer run: a looped layer has one per pass. Paged runs share the
+    sequences' block tables; recurrent runs are indexed by the request's persistent batch row."""
+
+    def __init__(self, model: "HybridDecoder", num_blocks: int, num_rows: int):
+        self.num_blocks, self.num_rows = num_blocks, num_rows
+        self.runs = [model.layers[r.layer]["mixer"].make_state(num_blocks, num_rows, model.device)
+                     for r in model.spec.runs]
+
+
+class HybridDecoder:
+    """Weights + forward of a hybrid decoder over a HybridCache."""
+
+    portions = True         # serves steps that mix prompt portions with decoded tokens
+    plain_lm_head = False   # logits are more than hidden . head^T (cap, f32)
+
+    def __init__(self, config: Dict[str, Any], device, dtype: torch.dtype = torch.bfloat16,
+                 seed: Optional[int] = 0, max_model_len: Optional[int] = None):
+        if dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError("dtype must be bfloat16 or float32")
+        self.config = config
+        self.spec = HybridSpec.from_config(config)
+        self.device, self.dtype = torch.device(device), dtype
+        self.max_model_len = max_model_len or self.spec.max_position_embeddings
+        self.workspace = kernels.DecodeWorkspace(self.device)          # decode steps: captured graphs hold it
+        self.portion_workspace = kernels.DecodeWorkspace(self.device)  # eager portion steps: free to grow
+        self._alloc(seed)
+
+    # recurrent state cannot be shared by prefix
+    @property
+    def prefix_cacheable(self) -> bool:
+        return all(MIXERS[self.spec.layers[r.layer]["type"]].paged for r in self.spec.runs)
+
+    # ---------------------------------------------------------------- weights
+    def _alloc(self, seed: Optional[int]):
+        s = self.spec
+        w = Weights(self.device, self.dtype, seed, s.initializer_range)
+        H = s.hidden_size
+        self.embed = w.matrix(s.vocab_size, H)
+        self.layers: List[Dict[str, Any]] = []
+        for e in s.layers:
+            mlp = e.get("mlp")
+            self.layers.append({
+                "norm1": w.ones(H),
+                "mixer": MIXERS[e["type"]](e["mixer"], H, s.norm_eps, self.max_model_len, w),
+                "norm2": w.ones(H) if mlp else None,
+                "mlp": FEEDFORWARDS[mlp["kind"]](mlp, H, w) if mlp else None,
+            })
+        self.loop_step = w.matrix(s.loop_times, H) if s.loop_times else None
+        self.norm = w.ones(H)
+        self.lm_head = w.matrix(s.vocab_size, H)
+
+    def _param_views(self) -> Dict[str, torch.Tensor]:
+        """Checkpoint name -> view into the (fused) storage."""
+        out = {"embed": self.embed, "final.norm": self.norm, "head": self.lm_head}
+        if self.loop_step is not None:
+            out["loop.step"] = self.loop_step
+        for i, L in enumerate(self.layers):
+            p = f"l{i}."
+            out[p + "norm1"] = L["norm1"]
+            for name, t in L["mixer"].params():
+                out[p + "mix." + name] = t
+            if L["mlp"] is not None:
+                out[p + "norm2"] = L["norm2"]
+                for name, t in L["mlp"].params():
+                    out[p + "mlp." + name] = t
+        return out
+
+    def hf_named_tensors(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        yield from self._param_views().items()
+
+    def load_weights(self, named: Iterable[Tuple[str, torch.Tensor]]) -> int:
+        """Copy named tensors into place (any subset; unknown names and wrong shapes raise)."""
+        views = self._param_views()
+        n = 0
+        with torch.no_grad():
+            for name, t in named:
+                dst = views.get(name)
+                if dst is None:
+                    raise KeyError(f"unknown parameter {name!r}")
+                if tuple(t.shape) != tuple(dst.shape):
+                    raise ValueError(f"{name}: shape {tuple(t.shape)} != {tuple(dst.shape)}")
+                dst.copy_(t, non_blocking=True)
+                n += 1
+            for L in self.layers:
+                L["mixer"].refresh()
+        return n
+
+    def num_params(self) -> int:
+        return sum(int(t.numel()) for t in self._param_views().values())
+
+    def release(self):
+        self.embed = self.lm_head = self.norm = self.loop_step = None
+        self.layers = []
+
+    # ---------------------------------------------------------------- cache and plans
+    def make_cache(self, num_blocks: int, num_rows: int) -> HybridCache:
+        return HybridCache(self, num_blocks, num_rows)
+
+    def block_bytes(self) -> int:
+        return max(1, sum(self.layers[r.layer]["mixer"].block_bytes() for r in self.spec.runs))
+
+    def row_bytes(self) -> int:
+        return sum(self.layers[r.layer]["mixer"].row_bytes() for r in self.spec.runs)
+
+    def decode_split(self, nb: int) -> Tuple[int, Optional[int]]:
+        """(max_ctx, nparts) of a captured decode step: each mixer splits by its own window."""
+        return self.max_model_len, None
+
+    def reserve(self, token_counts: Iterable[int]) -> None:
+        """Size the merge workspace for these step sizes, so that a captured graph never sees it move."""
+        need = 0
+        for n in token_counts:
+            for L in self.layers:
+                need = max(need, L["mixer"].workspace_bytes(n, self.max_model_len))
+        if need:
+            self.workspace.get(need)
+
+    @staticmethod
+    def is_short(tokens: int) -> bool:
+        """Whether a portion takes the per-token forms; the runner orders a step's short portions first."""
+        return tokens < PROMPT_MIN
+
+    def plan(self, seq_lens: List[int], starts: List[int], n_short: int):
+        """Host plan of the prompt forms: {window: (seg, tiles, rows, longest)} as numpy arrays."""
+        if n_short == len(seq_lens) or self.dtype != torch.bfloat16:
+            return None
+        first = sum(seq_lens[:n_short])
+        return {w: prompt_plan(seq_lens, starts, n_short, first, w)
+                for w in {L["mixer"].window for L in self.layers if L["mixer"].paged}}
+
+    # ---------------------------------------------------------------- forward
+    def _run_layers(self, inp: StepInputs, cache: HybridCache, want: Optional[torch.Tensor], trail=None):
+        """Final-norm output of the wanted tokens (None: all). `trail` collects the residual after every
+        layer run (inspection)."""
+        eps = self.spec.norm_eps
+        h = F.embedding(inp.tokens, self.embed).float()
+        x = torch.empty(h.shape, dtype=self.dtype, device=self.device)
+        delta = None
+        ws = self.workspace if inp.one_token else self.portion_workspace
+        for r, state in zip(self.spec.runs, cache.runs):
+            L = self.layers[r.layer]
+            step = None if r.step is None else self.loop_step[r.step]
+            lk.add_norm(delta, h, L["norm1"], eps, step=step, out=x)
+            delta = L["mixer"].forward(x, inp, state, ws)
+            if L["mlp"] is not None:
+                lk.add_norm(delta, h, L["norm2"], eps, out=x)
+                delta = L["mlp"].forward(x)
+            if trail is not None:
+                trail.append(h + delta.float())
+        if want is None:
+            return lk.add_norm(delta, h, self.norm, eps, out=x)
+        return lk.add_norm(None if delta is None else delta[want], h[want], self.norm, eps)
+
+    def forward_decode(self, inp: StepInputs, cache: HybridCache) -> torch.Tensor:
+        """One token per row: final hidden states [n, H]."""
+        return self._run_layers(inp, cache, None)
+
+    def forward_portions(self, inp: StepInputs, cache: HybridCache, trail=None) -> torch.Tensor:
+        """A step of portions: final hidden states of the tokens `inp.want` lists."""
+        return self._run_layers(inp, cache, inp.want, trail)
+
+    def logits(self, hidden: torch.Tensor) -> torch.Tensor:
+        """f32 [n, V]."""
+        return lk.softcap(F.linear(hidden, self.lm_head), self.spec.logit_softcap)

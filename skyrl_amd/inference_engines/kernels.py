@@ -108,6 +108,10 @@ class DecodeWorkspace:
         return self.buf
 
 
+def decode_workspace_bytes(nseq: int, nh: int, head_dim: int, nparts: int) -> int:
+    return int(_ffi.query("skyrl_paged_decode_workspace_bytes", nseq, nh, head_dim, nparts))
+
+
 def paged_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor,
                  context_lens: torch.Tensor, max_ctx: int, scale: float, out: Optional[torch.Tensor] = None,
                  workspace: Optional[DecodeWorkspace] = None, nparts: Optional[int] = None,
@@ -138,7 +142,7 @@ def paged_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
     nparts = nparts or choose_nparts(n, nkv, max_ctx)
     ws = None
     if nparts > 1:
-        nbytes = _ffi.query("skyrl_paged_decode_workspace_bytes", n, nh, D, nparts)
+        nbytes = decode_workspace_bytes(n, nh, D, nparts)
         ws = (workspace or DecodeWorkspace(dev)).get(nbytes)
     _ffi.call("skyrl_paged_decode", _ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
               block_tables.stride(0), _ptr(context_lens), n, nh, nkv, D, float(scale), part_min, nparts, _ptr(out),

@@ -1,0 +1,244 @@
+"""Host launchers of the hybrid decoders' layer kernels (include/skyrl_layers.h).
+
+Shapes, dtypes and strides are checked here before every launch, as in kernels.py; there is no CPU
+fallback."""
+
+from __future__ import annotations
+
+import ctypes
+from typing import Optional
+
+import torch
+
+from .. import _ffi
+from ..ops import _ptr, _require_gpu, _stream
+
+NORMS = {"layer": 0, "rms": 1}
+ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+_DTYPES = {torch.bfloat16: _ffi.BF16, torch.float32: _ffi.F32}
+
+
+def _code(t: torch.Tensor) -> int:
+    code = _DTYPES.get(t.dtype)
+    if code is None:
+        raise TypeError(f"activations must be bfloat16 or float32, got {t.dtype}")
+    return code
+
+
+def _check(t: Optional[torch.Tensor], name: str, dtype, shape=None, contiguous: bool = True):
+    if t is None:
+        return
+    if t.dtype != dtype:
+        raise TypeError(f"{name} must be {dtype}, got {t.dtype}")
+    if shape is not None and tuple(t.shape) != tuple(shape):
+        raise ValueError(f"{name} must be {tuple(shape)}, got {tuple(t.shape)}")
+    if contiguous and not t.is_contiguous():
+        raise ValueError(f"{name} must be contiguous")
+
+
+def add_norm(delta: Optional[torch.Tensor], hidden: torch.Tensor, weight: torch.Tensor, eps: float,
+             kind: str = "layer", step: Optional[torch.Tensor] = None,
+             out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """hidden (f32, in place) += delta and += step (one vector for every row), then the norm."""
+    dev = _require_gpu(hidden, weight, delta, step, out)
+    n, H = hidden.shape
+    _check(hidden, "hidden", torch.float32)
+    _check(weight, "weight", weight.dtype, (H,))
+    _check(delta, "delta", weight.dtype, (n, H))
+    _check(step, "step", weight.dtype, (H,))
+    if out is None:
+        out = torch.empty((n, H), dtype=weight.dtype, device=dev)
+    _check(out, "out", weight.dtype, (n, H))
+    _ffi.call("skyrl_add_norm", _ptr(delta), _ptr(hidden), _ptr(step), _ptr(weight), n, H, float(eps), NORMS[kind],
+              _ptr(out), _code(weight), _stream(dev))
+    return out
+
+
+def gate_mul(gate_up: torch.Tensor, act: str) -> torch.Tensor:
+    """act(gate) * up of the fused [n, 2I] projection."""
+    dev = _require_gpu(gate_up)
+    n, I2 = gate_up.shape
+    _check(gate_up, "gate_up", gate_up.dtype)
+    out = torch.empty((n, I2 // 2), dtype=gate_up.dtype, device=dev)
+    _ffi.call("skyrl_gate_mul", _ptr(gate_up), n, I2 // 2, ACTIVATIONS[act], _ptr(out), _code(gate_up), _stream(dev))
+    return out
+
+
+def softcap(x: torch.Tensor, cap: Optional[float]) -> torch.Tensor:
+    """f32 cap * tanh(x / cap); a plain f32 copy without a cap."""
+    dev = _require_gpu(x)
+    _check(x, "x", x.dtype)
+    out = torch.empty(x.shape, dtype=torch.float32, device=dev)
+    _ffi.call("skyrl_softcap", _ptr(x), _ptr(out), x.numel(), float(cap or 0.0), _code(x), _stream(dev))
+    return out
+
+
+# ---------------------------------------------------------------- latent attention
+def latent_row(rank: int, rot_dim: int) -> int:
+    """Elements of one cached token: latent | rotated key part | padding to a multiple of 32."""
+    return (rank + rot_dim + 31) // 32 * 32
+
+
+def _check_cache(cache: torch.Tensor, rank: int, rot_dim: int, dtype):
+    if cache.dim() != 3 or cache.shape[1] != 16 or cache.shape[2] != latent_row(rank, rot_dim):
+        raise ValueError("cache must be [blocks, 16, latent_row(rank, rot_dim)]")
+    _check(cache, "cache", dtype)
+
+
+def _check_table(block_tables, bt_row, positions, T):
+    if block_tables.dtype != torch.int32 or block_tables.dim() != 2 or block_tables.stride(1) != 1:
+        raise ValueError("block_tables must be int32 [n, blocks] with unit column stride")
+    _check(bt_row, "bt_row", torch.int32, (T,))
+    _check(positions, "positions", torch.int64, (T,))
+
+
+def latent_write(proj, heads, dim, rot_dim, rank, norm_weight, eps, positions, slots, cos_sin, cache) -> None:
+    """Rotate the q parts of ``proj`` in place; write the normed latent and the rotated key part."""
+    dev = _require_gpu(proj, norm_weight, positions, slots, cos_sin, cache)
+    T = proj.shape[0]
+    width = heads * (dim + rot_dim) + rank + rot_dim
+    if proj.dim() != 2 or proj.shape[1] != width or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, {width}] with unit column stride")
+    _check(norm_weight, "norm_weight", proj.dtype, (rank,))
+    _check(positions, "positions", torch.int64, (T,))
+    _check(slots, "slots", torch.int64, (T,))
+    if cos_sin.dim() != 2 or cos_sin.shape[1] != rot_dim:
+        raise ValueError("cos_sin must be [max_pos, rot_dim]")
+    _check(cos_sin, "cos_sin", torch.float32)
+    _check_cache(cache, rank, rot_dim, proj.dtype)
+    _ffi.call("skyrl_latent_write", _ptr(proj), proj.stride(0), T, heads, dim, rot_dim, rank, _ptr(norm_weight),
+              float(eps), _ptr(positions), _ptr(slots), _ptr(cos_sin), _ptr(cache), cache.shape[2], _code(proj),
+              _stream(dev))
+
+
+def latent_attend(qa, q_rot, cache, rank, rot_dim, block_tables, bt_row, positions, scale, window, nparts=1,
+                  part_min=64, workspace=None) -> torch.Tensor:
+    """Latent-space attention, one query row per token. qa [heads, T, rank]; q_rot [T, heads, rot_dim]
+    (any token and head stride); returns [heads, T, rank]."""
+    dev = _require_gpu(qa, q_rot, cache, block_tables, bt_row, positions)
+    heads, T, R = qa.shape
+    _check(qa, "qa", cache.dtype, (heads, T, rank))
+    if q_rot.dtype != qa.dtype or tuple(q_rot.shape) != (T, heads, rot_dim) or (rot_dim > 1 and q_rot.stride(2) != 1):
+        raise ValueError("q_rot must be [T, heads, rot_dim] with unit last stride")
+    _check_cache(cache, rank, rot_dim, qa.dtype)
+    _check_table(block_tables, bt_row, positions, T)
+    out = torch.empty_like(qa)
+    ws = None
+    if nparts > 1 and mfma_attend(rank, rot_dim, qa.dtype):
+        need = _ffi.query("skyrl_latent_attend_workspace_bytes", T, heads, rank, nparts)
+        ws = workspace.get(need) if workspace is not None else torch.empty(need, dtype=torch.uint8, device=dev)
+    else:
+        nparts = 1
+    _ffi.call("skyrl_latent_attend", _ptr(qa), _ptr(q_rot), q_rot.stride(0), q_rot.stride(1), _ptr(cache),
+              cache.shape[2], _ptr(block_tables), block_tables.stride(0), _ptr(bt_row), _ptr(positions), T, heads,
+              rank, rot_dim, float(scale), int(window or 0), part_min, nparts, _ptr(out), _ptr(ws), _code(qa),
+              _stream(dev))
+    return out
+
+
+def mfma_attend(rank: int, rot_dim: int, dtype) -> bool:
+    return bool(_ffi.query("skyrl_latent_attend_mfma", rank, rot_dim, latent_row(rank, rot_dim), _DTYPES[dtype]))
+
+
+def latent_gather(cache, rank, rot_dim, block_tables, seg, nrows: int, max_count: int):
+    """Packed (latent [nrows, rank], k_rot [nrows, rot_dim]) of the segments ``seg`` int32 [n, 4]: block-table
+    row, first position, count, first packed row. nrows covers every segment rounded up to 64."""
+    dev = _require_gpu(cache, block_tables, seg)
+    _check_cache(cache, rank, rot_dim, cache.dtype)
+    _check(seg, "seg", torch.int32, (seg.shape[0], 4))
+    latent = torch.empty((nrows, rank), dtype=cache.dtype, device=dev)
+    k_rot = torch.empty((nrows, rot_dim), dtype=cache.dtype, device=dev)
+    _ffi.call("skyrl_latent_gather", _ptr(cache), cache.shape[2], _ptr(block_tables), block_tables.stride(0),
+              _ptr(seg), seg.shape[0], max_count, rank, rot_dim, _ptr(latent), _ptr(k_rot), _code(cache),
+              _stream(dev))
+    return latent, k_rot
+
+
+def latent_prefill(q, k_nope, k_rot, v_t, tiles, heads, dim, rot_dim, vdim, scale, window, out) -> torch.Tensor:
+    """Windowed attention of prompt tiles over packed keys. q [T, >= heads * (dim + rot_dim)]; k_nope
+    [rows, heads * dim]; k_rot [rows, rot_dim]; v_t [heads * vdim, rows]; out [T, heads * vdim]."""
+    dev = _require_gpu(q, k_nope, k_rot, v_t, tiles, out)
+    rows = k_nope.shape[0]
+    for t, name in ((q, "q"), (k_nope, "k_nope"), (k_rot, "k_rot"), (v_t, "v_t"), (out, "out")):
+        if t.dtype != torch.bfloat16 or t.dim() != 2 or t.stride(1) != 1:
+            raise ValueError(f"{name} must be bf16, 2-D, with unit column stride")
+    if q.shape[1] < heads * (dim + rot_dim) or k_nope.shape[1] != heads * dim or out.shape[1] != heads * vdim \
+            or out.shape[0] != q.shape[0]:
+        raise ValueError("latent_prefill: q / k_nope / out widths do not match the heads")
+    _check(k_rot, "k_rot", torch.bfloat16, (rows, rot_dim))
+    if v_t.shape != (heads * vdim, rows) or rows % 64:
+        raise ValueError("v_t must be [heads * vdim, rows] with rows a multiple of 64")
+    _check(tiles, "tiles", torch.int32, (tiles.shape[0], 8))
+    _ffi.call("skyrl_latent_prefill", _ptr(q), q.stride(0), _ptr(k_nope), k_nope.stride(0), _ptr(k_rot), _ptr(v_t),
+              v_t.stride(0), _ptr(tiles), tiles.shape[0], heads, dim, rot_dim, vdim, float(scale), int(window or 0),
+              _ptr(out), out.stride(0), _stream(dev))
+    return out
+
+
+def prefill_fits(dim: int, rot_dim: int, vdim: int, dtype) -> bool:
+    return dtype == torch.bfloat16 and 0 < dim and dim + rot_dim <= 256 and vdim <= 256
+
+
+# ---------------------------------------------------------------- gated delta rule
+def delta_shape(heads, kv_heads, dim, vdim, taps, eps) -> _ffi.DeltaShape:
+    return _ffi.DeltaShape(heads, kv_heads, dim, vdim, taps, eps)
+
+
+def delta_channels(sh) -> int:
+    """Channels of the short convolutions: q | k | v."""
+    return 2 * sh.kv_heads * sh.dim + sh.heads * sh.vdim
+
+
+def delta_width(sh) -> int:
+    """Columns of the fused projection: q | k | v | output gate | beta | decay."""
+    return delta_channels(sh) + sh.heads * sh.vdim + 2 * sh.heads
+
+
+def delta_vpad(sh) -> int:
+    return (sh.vdim + 3) // 4 * 4
+
+
+def _check_delta(sh, proj, cu, rows, positions, conv_state, state=None):
+    T = proj.shape[0]
+    if proj.dim() != 2 or proj.shape[1] != delta_width(sh) or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, {delta_width(sh)}] with unit column stride")
+    n = rows.shape[0]
+    _check(rows, "rows", torch.int32, (n,))
+    _check(cu, "cu", torch.int32, (n + 1,))
+    _check(positions, "positions", torch.int64, (T,))
+    if conv_state.dim() != 3 or tuple(conv_state.shape[1:]) != (sh.taps, delta_channels(sh)):
+        raise ValueError("conv_state must be [rows, taps, channels]")
+    _check(conv_state, "conv_state", proj.dtype)
+    if state is not None:
+        _check(state, "state", torch.float32, (conv_state.shape[0], sh.heads, sh.dim, delta_vpad(sh)))
+    return n
+
+
+def _check_delta_weights(sh, dtype, conv_w, a_log, dt_bias, norm_w=None):
+    _check(conv_w, "conv_w", dtype, (delta_channels(sh), sh.taps))
+    _check(a_log, "a_log", torch.float32, (sh.heads,))
+    _check(dt_bias, "dt_bias", torch.float32, (sh.heads,))
+    _check(norm_w, "norm_w", dtype, (sh.vdim,))
+
+
+def delta_scan(sh, proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, state, conv_state, save_conv,
+               out) -> torch.Tensor:
+    """Token by token over each sequence's tokens [cu[s], cu[s + 1]); state and (save_conv: one token per
+    sequence) convolution inputs updated in place."""
+    dev = _require_gpu(proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, state, conv_state, out)
+    n = _check_delta(sh, proj, cu, rows, positions, conv_state, state)
+    _check_delta_weights(sh, proj.dtype, conv_w, a_log, dt_bias, norm_w)
+    if out.dtype != proj.dtype or out.shape != (proj.shape[0], sh.heads * sh.vdim) or out.stride(1) != 1:
+        raise ValueError("out must be [T, heads * vdim]")
+    _ffi.call("skyrl_delta_scan", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(conv_w), _ptr(a_log),
+              _ptr(dt_bias), _ptr(norm_w), _ptr(cu), _ptr(rows), _ptr(positions), n, _ptr(state), _ptr(conv_state),
+              int(save_conv), _ptr(out), out.stride(0), _code(proj), _stream(dev))
+    return out
+
+
+def delta_save(sh, proj, cu, rows, positions, conv_state) -> None:
+    """Store the last inputs of each sequence's convolutions."""
+    dev = _require_gpu(proj, cu, rows, positions, conv_state)
+    n = _check_delta(sh, proj, cu, rows, positions, conv_state)
+    _ffi.call("skyrl_delta_save", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(cu), _ptr(rows),
+              _ptr(positions), n, _ptr(conv_state), _code(proj), _stream(dev))

@@ -111,10 +111,23 @@ class StepInputs:
     # prefill only: tokens computed per sequence (host) and the cached prefix each starts after
     seq_lens: Optional[List[int]] = None
     cached_lens: Optional[List[int]] = None
+    # models that serve portions (hybrid.py), decode steps included
+    rows: Optional[torch.Tensor] = None    # int32 [n]: state row per sequence, -1: idle
+    cu: Optional[torch.Tensor] = None      # int32 [n + 1]: first token of each sequence
+    bt_row: Optional[torch.Tensor] = None  # int32 [T]: each token's row of block_tables
+    one_token: bool = False                # every sequence has exactly one token
+    n_short: int = 0                       # leading sequences that take the per-token forms
+    short_tokens: int = 0                  # and their tokens
+    plan: Optional[Dict] = None            # prompt forms of the others (HybridDecoder.plan), on the device
+    want: Optional[torch.Tensor] = None    # int64 [k]: tokens whose hidden states are returned
 
 
 class PagedDecoder:
     """Weights + forward of a Qwen2/Llama decoder over a paged KV cache."""
+
+    portions = False         # a step is a prefill or a decode
+    plain_lm_head = True     # logits = hidden . lm_head^T (the sampler may run in that product's epilogue)
+    prefix_cacheable = True  # a block's K/V depend on the token prefix alone
 
     def __init__(self, hf_config, device, dtype: torch.dtype = torch.bfloat16, seed: Optional[int] = 0,
                  max_model_len: Optional[int] = None):
@@ -125,7 +138,8 @@ class PagedDecoder:
         self.max_model_len = min(max_model_len or s.max_position_embeddings, s.max_position_embeddings)
         self.scale = 1.0 / math.sqrt(s.head_dim)
         self.cos_sin = rope_cos_sin(hf_config, self.max_model_len, dtype).to(self.device)
-        self.workspace = kernels.DecodeWorkspace(self.device)
+        self.workspace = kernels.DecodeWorkspace(self.device)          # decode steps: captured graphs hold it
+        self.prefill_workspace = kernels.DecodeWorkspace(self.device)  # eager prefills: free to grow
         self._alloc(seed)
 
     # ---------------------------------------------------------------- weights
@@ -210,6 +224,30 @@ class PagedDecoder:
         """Drop the weights (sleep level 2 discards them, vllm_engine.py sleep())."""
         self.embed = self.lm_head = self.norm = None
         self.layers = []
+
+    # ---------------------------------------------------------------- cache
+    def make_cache(self, num_blocks: int, num_rows: int) -> PagedKVCache:
+        s = self.spec
+        return PagedKVCache(s.num_layers, num_blocks, s.num_kv_heads, s.head_dim, self.device)
+
+    def block_bytes(self) -> int:
+        s = self.spec
+        return PagedKVCache.bytes_per_block(s.num_layers, s.num_kv_heads, s.head_dim)
+
+    def row_bytes(self) -> int:
+        return 0
+
+    def decode_split(self, nb: int) -> Tuple[int, Optional[int]]:
+        """(max_ctx, nparts) baked into a captured decode step of nb rows."""
+        return self.max_model_len, kernels.choose_nparts(nb, self.spec.num_kv_heads, self.max_model_len)
+
+    def reserve(self, token_counts: Iterable[int]) -> None:
+        """Size the merge workspace for these decode batches: a captured graph must never see it move."""
+        s = self.spec
+        need = 0
+        for n in token_counts:
+            need = max(need, kernels.decode_workspace_bytes(n, s.num_heads, s.head_dim, self.decode_split(n)[1]))
+        self.workspace.get(need)
 
     # ---------------------------------------------------------------- forward
     def _run_layers(self, h: torch.Tensor, attention) -> torch.Tensor:
@@ -297,7 +335,7 @@ class PagedDecoder:
                 of = self._sdpa(q, k_out, qkv, T, pad_idx, rep)
                 o.index_copy_(0, tok_full, of.transpose(1, 2).reshape(-1, nhd)[valid])
             op = kernels.paged_decode(q.index_select(0, tok_part), cache.k[li], cache.v[li], bt, ctx, max_ctx,
-                                      self.scale, workspace=self.workspace)
+                                      self.scale, workspace=self.prefill_workspace)
             o.index_copy_(0, tok_part, op.view(-1, nhd))
             return o
 
