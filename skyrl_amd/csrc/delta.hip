@@ -6,6 +6,17 @@
 // of the state. Convolution, unit norms, gates, recurrence, output norm and output gate are one pass.
 // Both products with the state are taken before the update, S^T k and S^T q, in one sweep:
 // o = (g S + k u^T)^T q = g S^T q + (k . q) u.
+//
+// Prompt form (conv, chunk, chain, out): chunks of 64 tokens. Unrolling the recurrence over a chunk
+// with G_i the summed log decays up to token i gives
+//   u_i = beta_i (v_i - e^{G_i} S0^T k_i - sum_{j<i} e^{G_i - G_j} (k_i . k_j) u_j),
+// i.e. (I + A) U = diag(beta) V - diag(beta e^G) K S0 with A_ij = beta_i e^{G_i - G_j} k_i . k_j below
+// the diagonal. delta_chunk solves it for both right-hand sides, all chunks at once: U0 = (I + A)^-1
+// diag(beta) V and W = (I + A)^-1 diag(beta e^G) K, and forms P_ij = e^{G_i - G_j} q_i . k_j (j <= i).
+// delta_chain then walks a sequence's chunks with a 16-column slice of S per workgroup:
+//   U = U0 - W S,   O = diag(e^G) Q S + P U,   S <- e^{G_n} S + K^T diag(e^{G_n - G}) U.
+// Everything is f32, the products on the f32 matrix instructions (v_mfma_f32_16x16x4_f32): a lane's
+// four consecutive k values of a 16-step feed four instructions, the same permutation of k on both sides.
 #include "elem.h"
 
 namespace skyrl {
@@ -13,11 +24,17 @@ namespace {
 
 constexpr int kNT = 256;
 constexpr int kMaxTaps = 64;
+constexpr int kC = 64;       // tokens per chunk
+constexpr int kWindow = 8;   // convolution taps held in registers by the prompt form
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 struct Dims {
     int H, K, D, V, taps;
     float eps;
     __host__ __device__ int vpad() const { return (V + 3) / 4 * 4; }
+    __host__ __device__ int d16() const { return (D + 15) / 16 * 16; }
+    __host__ __device__ int v16() const { return (V + 15) / 16 * 16; }
     __host__ __device__ int channels() const { return 2 * K * D + H * V; }
 };
 
@@ -192,6 +209,373 @@ __global__ __launch_bounds__(kNT) void delta_save_kernel(Dims d, const T* __rest
         conv_state[((int64_t)row * d.taps + (pos0 + t - t0) % d.taps) * n + ch] = proj[(int64_t)t * stride + ch];
 }
 
+// ---- prompt form ------------------------------------------------------------------------------
+struct SeqRef {
+    const int32_t* chunk;  // [nchunks, 4]: first token, tokens, sequence, 0
+    const int32_t* cu;
+    const int32_t* rows;
+    const int64_t* positions;
+};
+
+// Convolution, silu, unit norms and gates. grid (nchunks, K + ceil(H V / 256)): the first K groups are the
+// key heads (q and k), the others 256 value channels each; gates with group 0.
+template <typename T>
+__global__ __launch_bounds__(kNT) void delta_conv_kernel(Dims d, SeqRef sq, const T* __restrict__ proj, int64_t stride,
+                                                         const T* __restrict__ conv_w, const float* __restrict__ a_log,
+                                                         const float* __restrict__ dt_bias,
+                                                         const T* __restrict__ conv_state, float* __restrict__ qk,
+                                                         float* __restrict__ vout, float* __restrict__ lg,
+                                                         float* __restrict__ beta) {
+    extern __shared__ float smem[];  // [16][2 D] of the key heads
+    const int32_t* ck = sq.chunk + 4 * blockIdx.x;
+    const int t0 = ck[0], n = ck[1], seq = ck[2];
+    const int sfirst = sq.cu[seq];
+    const int pos0 = (int)sq.positions[sfirst] + (t0 - sfirst);
+    const int ch_all = d.channels(), D = d.D, D16 = d.d16();
+    const T* ring = conv_state + (int64_t)sq.rows[seq] * d.taps * ch_all;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const bool keys = (int)blockIdx.y < d.K;
+    const int kh = blockIdx.y;
+    if (blockIdx.y == 0) {
+        for (int e = tid; e < n * d.H; e += kNT) {
+            const int i = e / d.H, h = e - i * d.H;
+            const T* p = proj + (int64_t)(t0 + i) * stride + ch_all + d.H * d.V;
+            beta[(int64_t)(t0 + i) * d.H + h] = sigmoidf_(ld(p + h));
+            lg[(int64_t)(t0 + i) * d.H + h] = -expf(a_log[h]) * softplusf_(ld(p + d.H + h) + dt_bias[h]);
+        }
+    }
+    // input of channel ch at local token i (negative: before the chunk, from the portion or the stored inputs)
+    auto input = [&](int ch, int i) -> float {
+        if (pos0 + i < 0) return 0.f;
+        if (t0 + i >= sfirst) return ld(proj + (int64_t)(t0 + i) * stride + ch);
+        return ld(ring + (int64_t)((pos0 + i) % d.taps) * ch_all + ch);
+    };
+    const int nch = keys ? 2 * D : min(kNT, d.H * d.V - ((int)blockIdx.y - d.K) * kNT);
+    for (int i0 = 0; i0 < n; i0 += 16) {
+        const int m = min(16, n - i0);
+        for (int e = tid; e < nch; e += kNT) {
+            const int ch = !keys ? 2 * d.K * D + ((int)blockIdx.y - d.K) * kNT + e
+                                 : e < D ? kh * D + e : (d.K + kh) * D + (e - D);
+            float x[kWindow], w[kWindow];
+            const bool held = d.taps <= kWindow;
+            if (held) {
+#pragma unroll
+                for (int j = 0; j < kWindow; ++j) {
+                    const int tap = j - (kWindow - d.taps);
+                    w[j] = tap >= 0 ? ld(conv_w + (int64_t)ch * d.taps + tap) : 0.f;
+                    x[j] = (j > 0 && tap > 0) ? input(ch, i0 - kWindow + j) : 0.f;
+                }
+            }
+            for (int i = 0; i < m; ++i) {
+                float y = 0.f;
+                if (held) {
+#pragma unroll
+                    for (int j = 0; j < kWindow - 1; ++j) x[j] = x[j + 1];
+                    x[kWindow - 1] = ld(proj + (int64_t)(t0 + i0 + i) * stride + ch);
+#pragma unroll
+                    for (int j = 0; j < kWindow; ++j) y += x[j] * w[j];
+                } else {
+                    for (int j = 0; j < d.taps; ++j)
+                        y += input(ch, i0 + i - (d.taps - 1) + j) * ld(conv_w + (int64_t)ch * d.taps + j);
+                }
+                y = siluf_(y);
+                if (keys) smem[i * 2 * D + e] = y;
+                else vout[(int64_t)(t0 + i0 + i) * d.H * d.V + ((int)blockIdx.y - d.K) * kNT + e] = y;
+            }
+        }
+        if (!keys) continue;
+        __syncthreads();
+        for (int e = wave; e < 2 * m; e += kNT / kWave) {
+            const int i = e >> 1, which = e & 1;
+            const float* src = smem + i * 2 * D + which * D;
+            float ss = 0.f;
+            for (int k = lane; k < D; k += kWave) ss += src[k] * src[k];
+            float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
+            if (which == 0) r *= 1.f / sqrtf((float)D);
+            float* dst = qk + (((int64_t)(t0 + i0 + i) * 2 + which) * d.K + kh) * D16;
+            for (int k = lane; k < D16; k += kWave) dst[k] = k < D ? src[k] * r : 0.f;
+        }
+        __syncthreads();
+    }
+}
+
+// One workgroup per (chunk, head).
+__global__ __launch_bounds__(kNT) void delta_chunk_kernel(Dims d, const int32_t* __restrict__ chunk,
+                                                          const float* __restrict__ qk, const float* __restrict__ v,
+                                                          const float* __restrict__ lg, const float* __restrict__ beta,
+                                                          float* __restrict__ W, float* __restrict__ U,
+                                                          float* __restrict__ P, float* __restrict__ G) {
+    constexpr int LD = kC + 4;
+    __shared__ __attribute__((aligned(16))) float s_k[kC * LD];  // a 64-wide slab of K; then A
+    __shared__ __attribute__((aligned(16))) float s_q[kC * LD];
+    __shared__ float s_g[kC], s_b[kC];
+    const int h = blockIdx.x % d.H, ci = blockIdx.x / d.H;
+    const int32_t* ck = chunk + 4 * ci;
+    const int t0 = ck[0], n = ck[1];
+    const int kh = h / (d.H / d.K), D16 = d.d16(), V16 = d.v16();
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int64_t ch = (int64_t)ci * d.H + h;
+    if (wave == 0) {  // inclusive sums of the log decays
+        float x = lane < n ? lg[(int64_t)(t0 + lane) * d.H + h] : 0.f;
+#pragma unroll
+        for (int o = 1; o < kWave; o <<= 1) {
+            const float y = __shfl_up(x, o, kWave);
+            if (lane >= o) x += y;
+        }
+        s_g[lane] = x;
+        s_b[lane] = lane < n ? beta[(int64_t)(t0 + lane) * d.H + h] : 0.f;
+        G[ch * kC + lane] = x;
+    }
+    f32x4 akk[4], aqk[4];  // rows 16 wave .., column blocks 0 .. wave
+#pragma unroll
+    for (int b = 0; b < 4; ++b) akk[b] = aqk[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int d0 = 0; d0 < D16; d0 += kC) {
+        const int w4 = min(kC, D16 - d0) / 4;
+        __syncthreads();
+        for (int e = tid; e < kC * w4; e += kNT) {
+            const int i = e / w4, x = (e - i * w4) * 4;
+            float4 kv = make_float4(0.f, 0.f, 0.f, 0.f), qv = kv;
+            if (i < n) {
+                const float* src = qk + ((int64_t)(t0 + i) * 2 * d.K + kh) * D16 + d0 + x;
+                qv = ld4(src);
+                kv = ld4(src + (int64_t)d.K * D16);
+            }
+            st4(&s_k[i * LD + x], kv);
+            st4(&s_q[i * LD + x], qv);
+        }
+        __syncthreads();
+        for (int s = 0; s < w4 / 4; ++s) {
+            const float4 ak = ld4(&s_k[(16 * wave + c) * LD + 16 * s + 4 * g]);
+            const float4 aq = ld4(&s_q[(16 * wave + c) * LD + 16 * s + 4 * g]);
+#pragma unroll
+            for (int b = 0; b < 4; ++b) {
+                if (b <= wave) {
+                    const float4 bk = ld4(&s_k[(16 * b + c) * LD + 16 * s + 4 * g]);
+                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.x, bk.x, akk[b], 0, 0, 0);
+                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.x, bk.x, aqk[b], 0, 0, 0);
+                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.y, bk.y, akk[b], 0, 0, 0);
+                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.y, bk.y, aqk[b], 0, 0, 0);
+                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.z, bk.z, akk[b], 0, 0, 0);
+                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.z, bk.z, aqk[b], 0, 0, 0);
+                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.w, bk.w, akk[b], 0, 0, 0);
+                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.w, bk.w, aqk[b], 0, 0, 0);
+                }
+            }
+        }
+    }
+    __syncthreads();
+    float* s_a = s_k;
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int r = 16 * wave + 4 * g + i, cc = 16 * b + c;
+            const float dec = cc <= r ? expf(s_g[r] - s_g[cc]) : 0.f;
+            s_a[r * LD + cc] = cc < r ? s_b[r] * dec * akk[b][i] : 0.f;
+            P[(ch * kC + r) * kC + cc] = dec * aqk[b][i];
+        }
+    }
+    __syncthreads();
+    // forward substitution, one right-hand-side column per thread: W's D16 columns, then U's V16
+    for (int col = tid; col < D16 + V16; col += kNT) {
+        const bool isw = col < D16;
+        const int cc = isw ? col : col - D16;
+        float x[kC];
+#pragma unroll
+        for (int i = 0; i < kC; ++i) {
+            float r = 0.f;
+            if (i < n) {
+                if (isw) r = s_b[i] * expf(s_g[i]) * qk[(((int64_t)(t0 + i) * 2 + 1) * d.K + kh) * D16 + cc];
+                else if (cc < d.V) r = s_b[i] * v[((int64_t)(t0 + i) * d.H + h) * d.V + cc];
+            }
+            x[i] = r;
+        }
+#pragma unroll
+        for (int i = 1; i < kC; ++i) {
+            float r = x[i];
+#pragma unroll
+            for (int j4 = 0; j4 < (i + 3) / 4; ++j4) {
+                const float4 a = ld4(&s_a[i * LD + 4 * j4]);  // zero at and above the diagonal
+                r -= a.x * x[4 * j4];
+                if (4 * j4 + 1 < i) r -= a.y * x[4 * j4 + 1];
+                if (4 * j4 + 2 < i) r -= a.z * x[4 * j4 + 2];
+                if (4 * j4 + 3 < i) r -= a.w * x[4 * j4 + 3];
+            }
+            x[i] = r;
+        }
+        float* dst = isw ? W + ch * kC * D16 + cc : U + ch * kC * V16 + cc;
+        const int ld_ = isw ? D16 : V16;
+#pragma unroll
+        for (int i = 0; i < kC; ++i) dst[(int64_t)i * ld_] = x[i];
+    }
+}
+
+// One workgroup per (sequence, head, 16 columns of S). NS: 16-wide steps of dim; DT = ceil(NS / 4) 16-row
+// tiles of S per wave.
+template <int NS>
+__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_chain_kernel(
+    Dims d, SeqRef sq, const int32_t* __restrict__ seq_chunks, int seq0, const float* __restrict__ qk,
+    const float* __restrict__ W, const float* __restrict__ U, const float* __restrict__ P, const float* __restrict__ G,
+    float* __restrict__ state, float* __restrict__ o) {
+    constexpr int LS = NS * 16 + 4, LU = kC + 4, DT = (NS + 3) / 4;
+    __shared__ __attribute__((aligned(16))) float s_s[16 * LS];      // S^T slice
+    __shared__ __attribute__((aligned(16))) float s_u[2][16 * LU];   // U^T and its decayed copy
+    const int V16 = d.v16(), D16 = d.d16(), VP = d.vpad(), nt = V16 / 16;
+    const int vt = blockIdx.x % nt, h = (blockIdx.x / nt) % d.H, si = blockIdx.x / (nt * d.H);
+    const int seq = seq0 + si, row = sq.rows[seq];
+    if (row < 0) return;
+    const int64_t pos0 = sq.positions[sq.cu[seq]];
+    const int kh = h / (d.H / d.K);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int ns = D16 / 16;
+    float* st_ = state + ((int64_t)row * d.H + h) * d.D * VP;
+    const int vcol = 16 * vt + c;
+
+    // this wave's rows of S: tiles wave, wave + 4, ...; element i: dim 16 tile + 4 g + i, column c
+    f32x4 S[DT];
+#pragma unroll
+    for (int k = 0; k < DT; ++k) {
+        const int tile = wave + 4 * k;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int dd = 16 * tile + 4 * g + i;
+            S[k][i] = (pos0 > 0 && dd < d.D && vcol < VP) ? st_[(int64_t)dd * VP + vcol] : 0.f;
+        }
+        if (tile < ns) *reinterpret_cast<f32x4*>(&s_s[c * LS + 16 * tile + 4 * g]) = S[k];
+    }
+    struct Tile {
+        float4 w[NS], q[NS], p[4];
+        float kk[DT][16];
+        float u0[4], gr[4], gl;
+    };
+    auto load = [&](int ci, Tile& t) {
+        const int32_t* ck = sq.chunk + 4 * ci;
+        const int t0 = ck[0], n = ck[1];
+        const int64_t ch = (int64_t)ci * d.H + h;
+        const int r = 16 * wave + c, rq = t0 + min(r, n - 1);
+        const float* wp = W + (ch * kC + r) * D16 + 4 * g;
+        const float* qp = qk + ((int64_t)rq * 2 * d.K + kh) * D16 + 4 * g;
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+            if (s < ns) {
+                t.w[s] = ld4(wp + 16 * s);
+                t.q[s] = ld4(qp + 16 * s);
+            }
+        }
+        const float* pp = P + (ch * kC + r) * kC + 4 * g;
+#pragma unroll
+        for (int s = 0; s < 4; ++s) t.p[s] = ld4(pp + 16 * s);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int rr = 16 * wave + 4 * g + i;
+            t.u0[i] = U[(ch * kC + rr) * V16 + vcol];
+            t.gr[i] = G[ch * kC + rr];
+        }
+        t.gl = G[ch * kC + kC - 1];
+#pragma unroll
+        for (int k = 0; k < DT; ++k) {
+            const int tile = wave + 4 * k;
+            if (tile < ns) {
+#pragma unroll
+                for (int j = 0; j < 16; ++j) {  // token 16 (j / 4) + 4 g + j % 4, dim 16 tile + c
+                    const int tok = t0 + min(16 * (j >> 2) + 4 * g + (j & 3), n - 1);
+                    t.kk[k][j] = qk[(((int64_t)tok * 2 + 1) * d.K + kh) * D16 + 16 * tile + c];
+                }
+            }
+        }
+    };
+    auto mma4 = [](const float4& a, const float4& b, f32x4 acc) {
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, acc, 0, 0, 0);
+        return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
+    };
+    auto run = [&](int ci, const Tile& t) {
+        const int32_t* ck = sq.chunk + 4 * ci;
+        const int t0 = ck[0], n = ck[1];
+        __syncthreads();  // S^T of the previous chunk is in LDS
+        f32x4 aw = {0.f, 0.f, 0.f, 0.f}, ao = aw;
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+            if (s < ns) {
+                const float4 b = ld4(&s_s[c * LS + 16 * s + 4 * g]);
+                aw = mma4(t.w[s], b, aw);
+                ao = mma4(t.q[s], b, ao);
+            }
+        }
+        float4 u, ud;
+        float* up = &u.x;
+        float* dp = &ud.x;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            up[i] = t.u0[i] - aw[i];
+            dp[i] = up[i] * expf(t.gl - t.gr[i]);
+            ao[i] *= expf(t.gr[i]);
+        }
+        st4(&s_u[0][c * LU + 16 * wave + 4 * g], u);
+        st4(&s_u[1][c * LU + 16 * wave + 4 * g], ud);
+        __syncthreads();
+        const float decay = expf(t.gl);
+#pragma unroll
+        for (int k = 0; k < DT; ++k) S[k] = S[k] * decay;
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            ao = mma4(t.p[s], ld4(&s_u[0][c * LU + 16 * s + 4 * g]), ao);
+            const float4 b = ld4(&s_u[1][c * LU + 16 * s + 4 * g]);
+#pragma unroll
+            for (int k = 0; k < DT; ++k)
+                if (wave + 4 * k < ns)
+                    S[k] = mma4(make_float4(t.kk[k][4 * s], t.kk[k][4 * s + 1], t.kk[k][4 * s + 2], t.kk[k][4 * s + 3]),
+                                b, S[k]);
+        }
+#pragma unroll
+        for (int k = 0; k < DT; ++k)
+            if (wave + 4 * k < ns) *reinterpret_cast<f32x4*>(&s_s[c * LS + 16 * (wave + 4 * k) + 4 * g]) = S[k];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int r = 16 * wave + 4 * g + i;
+            if (r < n && vcol < d.V) o[((int64_t)(t0 + r) * d.H + h) * d.V + vcol] = ao[i];
+        }
+    };
+    const int c0 = seq_chunks[si], c1 = seq_chunks[si + 1];
+    Tile ta, tb;
+    if (c0 < c1) load(c0, ta);
+    for (int ci = c0; ci < c1; ci += 2) {
+        if (ci + 1 < c1) load(ci + 1, tb);
+        run(ci, ta);
+        if (ci + 1 < c1) {
+            if (ci + 2 < c1) load(ci + 2, ta);
+            run(ci + 1, tb);
+        }
+    }
+#pragma unroll
+    for (int k = 0; k < DT; ++k)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int dd = 16 * (wave + 4 * k) + 4 * g + i;
+            if (dd < d.D && vcol < VP) st_[(int64_t)dd * VP + vcol] = S[k][i];
+        }
+}
+
+// Output norm and gate: one wave per (token, head) of tokens [first, T).
+template <typename T>
+__global__ __launch_bounds__(kNT) void delta_out_kernel(Dims d, const float* __restrict__ o, const T* __restrict__ proj,
+                                                        int64_t stride, const T* __restrict__ norm_w, int first,
+                                                        int64_t items, T* __restrict__ out, int64_t out_stride) {
+    const int lane = threadIdx.x & 63;
+    const int64_t e = (int64_t)blockIdx.x * (kNT / kWave) + (threadIdx.x >> 6);
+    if (e >= items) return;
+    const int64_t t = first + e / d.H;
+    const int h = (int)(e % d.H);
+    const float* src = o + (t * d.H + h) * d.V;
+    const T* gate = proj + t * stride + d.channels() + h * d.V;
+    float ss = 0.f;
+    for (int i = lane; i < d.V; i += kWave) ss += src[i] * src[i];
+    const float r = 1.f / sqrtf(wave_sum(ss) / (float)d.V + d.eps);
+    for (int i = lane; i < d.V; i += kWave)
+        st(out + t * out_stride + h * d.V + i, src[i] * r * ld(norm_w + i) * siluf_(ld(gate + i)));
+}
+
 int scan_rows_per_thread(const Dims& d) {
     const int RG = kNT / (d.vpad() / 4);
     return (d.D + RG - 1) / RG;
@@ -264,4 +648,84 @@ extern "C" int skyrl_delta_save(const skyrl_delta_shape* shape, const void* proj
                            reinterpret_cast<T*>(conv_state));
     })
     return check_launch("delta_save_kernel");
+}
+
+extern "C" int skyrl_delta_conv(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride,
+                                const void* conv_w, const float* a_log, const float* dt_bias, const int32_t* chunk,
+                                int32_t nchunks, const int32_t* cu, const int32_t* rows, const int64_t* positions,
+                                const void* conv_state, float* qk, float* v, float* lg, float* beta, int32_t dtype,
+                                void* stream) {
+    SKYRL_REQUIRE_T(dtype, "delta_conv");
+    const char* bad = bad_shape(shape);
+    SKYRL_REQUIRE(!bad, bad);
+    const Dims d = dims_of(shape);
+    SKYRL_REQUIRE(nchunks >= 0 && proj_stride >= proj_width(d), "delta_conv: bad sizes");
+    if (nchunks == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(proj && conv_w && a_log && dt_bias && chunk && cu && rows && positions && conv_state && qk && v && lg &&
+                      beta,
+                  "delta_conv: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        hipLaunchKernelGGL((delta_conv_kernel<T>), dim3(nchunks, d.K + (d.H * d.V + kNT - 1) / kNT), dim3(kNT),
+                           16 * 2 * d.D * sizeof(float), as_stream(stream), d, SeqRef{chunk, cu, rows, positions},
+                           reinterpret_cast<const T*>(proj), proj_stride, reinterpret_cast<const T*>(conv_w), a_log,
+                           dt_bias, reinterpret_cast<const T*>(conv_state), qk, v, lg, beta);
+    })
+    return check_launch("delta_conv_kernel");
+}
+
+extern "C" int skyrl_delta_chunk(const skyrl_delta_shape* shape, const int32_t* chunk, int32_t nchunks,
+                                 const float* qk, const float* v, const float* lg, const float* beta, float* W,
+                                 float* U, float* P, float* G, void* stream) {
+    const char* bad = bad_shape(shape);
+    SKYRL_REQUIRE(!bad, bad);
+    const Dims d = dims_of(shape);
+    SKYRL_REQUIRE(nchunks >= 0 && (int64_t)nchunks * d.H < (1 << 30), "delta_chunk: bad sizes");
+    if (nchunks == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(chunk && qk && v && lg && beta && W && U && P && G, "delta_chunk: null pointer");
+    hipLaunchKernelGGL(delta_chunk_kernel, dim3(nchunks * d.H), dim3(kNT), 0, as_stream(stream), d, chunk, qk, v, lg,
+                       beta, W, U, P, G);
+    return check_launch("delta_chunk_kernel");
+}
+
+#define LAUNCH_CHAIN(NS)                                                                                          \
+    hipLaunchKernelGGL((delta_chain_kernel<NS>), dim3((unsigned)nseq * d.H * (d.v16() / 16)), dim3(kNT), 0,       \
+                       as_stream(stream), d, SeqRef{chunk, cu, rows, positions}, seq_chunks, seq0, qk, W, U, P, G, \
+                       state, o)
+
+extern "C" int skyrl_delta_chain(const skyrl_delta_shape* shape, const int32_t* chunk, const int32_t* seq_chunks,
+                                 int32_t seq0, int32_t nseq, const int32_t* cu, const int32_t* rows,
+                                 const int64_t* positions, const float* qk, const float* W, const float* U,
+                                 const float* P, const float* G, float* state, float* o, void* stream) {
+    const char* bad = bad_shape(shape);
+    SKYRL_REQUIRE(!bad, bad);
+    const Dims d = dims_of(shape);
+    SKYRL_REQUIRE(d.D <= 256, "delta_chain: dim must be at most 256");
+    SKYRL_REQUIRE(nseq >= 0 && seq0 >= 0 && (int64_t)nseq * d.H * (d.v16() / 16) < (1 << 30), "delta_chain: bad sizes");
+    if (nseq == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(chunk && seq_chunks && cu && rows && positions && qk && W && U && P && G && state && o,
+                  "delta_chain: null pointer");
+    if (d.D <= 64) LAUNCH_CHAIN(4);
+    else if (d.D <= 128) LAUNCH_CHAIN(8);
+    else LAUNCH_CHAIN(16);
+    return check_launch("delta_chain_kernel");
+}
+
+extern "C" int skyrl_delta_out(const skyrl_delta_shape* shape, const float* o, const void* proj, int64_t proj_stride,
+                               const void* norm_w, int32_t first, int32_t T_, void* out, int64_t out_stride,
+                               int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "delta_out");
+    const char* bad = bad_shape(shape);
+    SKYRL_REQUIRE(!bad, bad);
+    const Dims d = dims_of(shape);
+    SKYRL_REQUIRE(first >= 0 && T_ >= first && proj_stride >= proj_width(d) && out_stride >= (int64_t)d.H * d.V,
+                  "delta_out: bad sizes");
+    const int64_t items = (int64_t)(T_ - first) * d.H;
+    if (items == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(o && proj && norm_w && out, "delta_out: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)((items + 3) / 4)), dim3(kNT), 0, as_stream(stream), d,
+                           o, reinterpret_cast<const T*>(proj), proj_stride, reinterpret_cast<const T*>(norm_w), first,
+                           items, reinterpret_cast<T*>(out), out_stride);
+    })
+    return check_launch("delta_out_kernel");
 }

@@ -24,7 +24,7 @@ import torch.nn.functional as F
 
 from . import kernels
 from . import layer_kernels as lk
-from .mixers import FEEDFORWARDS, MIXERS, PROMPT_MIN, Weights, prompt_plan
+from .mixers import FEEDFORWARDS, MIXERS, PROMPT_MIN, Weights, chunk_plan, prompt_plan
 from .model import StepInputs
 
 DEFAULT_MAX_MODEL_LEN = 32768
@@ -208,12 +208,15 @@ class HybridDecoder:
         return tokens < PROMPT_MIN
 
     def plan(self, seq_lens: List[int], starts: List[int], n_short: int):
-        """Host plan of the prompt forms: {window: (seg, tiles, rows, longest)} as numpy arrays."""
-        if n_short == len(seq_lens) or self.dtype != torch.bfloat16:
+        """Host plan of the prompt forms, numpy arrays: {window: (seg, tiles, rows, longest)} of the paged
+        mixers' windows and {"chunks": (chunk, seq_chunks)} of the recurrent ones."""
+        if n_short == len(seq_lens):
             return None
         first = sum(seq_lens[:n_short])
-        return {w: prompt_plan(seq_lens, starts, n_short, first, w)
-                for w in {L["mixer"].window for L in self.layers if L["mixer"].paged}}
+        plan = {"chunks": chunk_plan(seq_lens, n_short, first)}
+        for w in {L["mixer"].window for L in self.layers if L["mixer"].paged}:
+            plan[w] = prompt_plan(seq_lens, starts, n_short, first, w)
+        return plan
 
     # ---------------------------------------------------------------- forward
     def _run_layers(self, inp: StepInputs, cache: HybridCache, want: Optional[torch.Tensor], trail=None):

@@ -242,3 +242,43 @@ def delta_save(sh, proj, cu, rows, positions, conv_state) -> None:
     n = _check_delta(sh, proj, cu, rows, positions, conv_state)
     _ffi.call("skyrl_delta_save", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(cu), _ptr(rows),
               _ptr(positions), n, _ptr(conv_state), _code(proj), _stream(dev))
+
+
+CHUNK = 64  # tokens per chunk of the prompt form
+
+
+def delta_prompt_fits(sh) -> bool:
+    return sh.dim <= 256
+
+
+def delta_prompt(sh, proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, state, conv_state, chunk, seq_chunks,
+                 first_seq: int, first_token: int, out) -> torch.Tensor:
+    """Chunked form over the sequences from first_seq on, whose tokens are [first_token, T): chunk int32
+    [n, 4] and seq_chunks int32 [sequences + 1] (mixers.chunk_plan). `state` is updated in place; the
+    convolution inputs are delta_save's."""
+    dev = _require_gpu(proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, state, conv_state, chunk,
+                       seq_chunks, out)
+    n = _check_delta(sh, proj, cu, rows, positions, conv_state, state)
+    _check_delta_weights(sh, proj.dtype, conv_w, a_log, dt_bias, norm_w)
+    T, nc, nseq = proj.shape[0], chunk.shape[0], n - first_seq
+    _check(chunk, "chunk", torch.int32, (nc, 4))
+    _check(seq_chunks, "seq_chunks", torch.int32, (nseq + 1,))
+    if out.dtype != proj.dtype or out.shape != (T, sh.heads * sh.vdim) or out.stride(1) != 1:
+        raise ValueError("out must be [T, heads * vdim]")
+    d16, v16 = (sh.dim + 15) // 16 * 16, (sh.vdim + 15) // 16 * 16
+    f32 = lambda *shape: torch.empty(shape, dtype=torch.float32, device=dev)  # noqa: E731
+    qk, v = f32(T, 2, sh.kv_heads, d16), f32(T, sh.heads, sh.vdim)
+    lg, beta = f32(T, sh.heads), f32(T, sh.heads)
+    W, U = f32(nc, sh.heads, CHUNK, d16), f32(nc, sh.heads, CHUNK, v16)
+    P, G = f32(nc, sh.heads, CHUNK, CHUNK), f32(nc, sh.heads, CHUNK)
+    o, st, ref = f32(T, sh.heads, sh.vdim), _stream(dev), ctypes.byref(sh)
+    _ffi.call("skyrl_delta_conv", ref, _ptr(proj), proj.stride(0), _ptr(conv_w), _ptr(a_log), _ptr(dt_bias),
+              _ptr(chunk), nc, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(conv_state), _ptr(qk), _ptr(v), _ptr(lg),
+              _ptr(beta), _code(proj), st)
+    _ffi.call("skyrl_delta_chunk", ref, _ptr(chunk), nc, _ptr(qk), _ptr(v), _ptr(lg), _ptr(beta), _ptr(W), _ptr(U),
+              _ptr(P), _ptr(G), st)
+    _ffi.call("skyrl_delta_chain", ref, _ptr(chunk), _ptr(seq_chunks), first_seq, nseq, _ptr(cu), _ptr(rows),
+              _ptr(positions), _ptr(qk), _ptr(W), _ptr(U), _ptr(P), _ptr(G), _ptr(state), _ptr(o), st)
+    _ffi.call("skyrl_delta_out", ref, _ptr(o), _ptr(proj), proj.stride(0), _ptr(norm_w), first_token, T, _ptr(out),
+              out.stride(0), _code(proj), st)
+    return out

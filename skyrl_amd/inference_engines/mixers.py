@@ -105,6 +105,18 @@ def prompt_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_to
             longest)
 
 
+def chunk_plan(seq_lens: List[int], first_seq: int, first_token: int):
+    """Host plan of the chunked recurrence of sequences first_seq..: (chunk int32 [n, 4], seq_chunks int32
+    [sequences + 1])."""
+    chunk, ends, tok = [], [0], first_token
+    for i in range(first_seq, len(seq_lens)):
+        for a in range(0, seq_lens[i], lk.CHUNK):
+            chunk.append((tok + a, min(lk.CHUNK, seq_lens[i] - a), i, 0))
+        ends.append(len(chunk))
+        tok += seq_lens[i]
+    return np.asarray(chunk, dtype=np.int32).reshape(-1, 4), np.asarray(ends, dtype=np.int32)
+
+
 class LatentAttention:
     """Attention over low-rank latents shared by all heads, with a rotated key part beside them and
     an optional sliding window. Caches [blocks, 16, row]: per token the normed latent | the rotated key
@@ -255,8 +267,16 @@ class GatedDelta:
         S, ring = state
         proj = F.linear(x, self.wproj)
         out = torch.empty((x.shape[0], self.heads * self.vdim), dtype=self.dtype, device=x.device)
-        lk.delta_scan(self.shape, proj, self.conv, self.a_log, self.dt_bias, self.norm, inp.cu, inp.rows,
-                      inp.positions, S, ring, inp.one_token, out)
+        args = (self.conv, self.a_log, self.dt_bias, self.norm)
+        n = inp.rows.shape[0]
+        k = inp.n_short if inp.plan is not None and lk.delta_prompt_fits(self.shape) else n
+        if k:
+            lk.delta_scan(self.shape, proj, *args, inp.cu[:k + 1], inp.rows[:k], inp.positions, S, ring,
+                          inp.one_token, out)
+        if k < n:
+            chunk, seq_chunks = inp.plan["chunks"]
+            lk.delta_prompt(self.shape, proj, *args, inp.cu, inp.rows, inp.positions, S, ring, chunk, seq_chunks, k,
+                            inp.short_tokens, out)
         if not inp.one_token:
             lk.delta_save(self.shape, proj, inp.cu, inp.rows, inp.positions, ring)
         return F.linear(out, self.wo)
