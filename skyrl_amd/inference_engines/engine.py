@@ -531,6 +531,8 @@ class EngineCore:
         for i, (r, toks, places) in enumerate(entries):
             if r.state != RUNNING or not toks:
                 raise ValueError("run_portions: a finished request or an empty portion")
+            if any(not 0 <= p < len(toks) for p in places):
+                raise ValueError(f"run_portions: wanted places {list(places)} outside a portion of {len(toks)} tokens")
             n = r.num_tokens + len(toks)
             if n > self.max_model_len:
                 raise ValueError(f"{n} tokens exceed max_model_len={self.max_model_len}")
@@ -723,6 +725,8 @@ class ModelRunner:
                 n_i32[r.row, k:len(r.blocks)] = r.blocks[k:]
                 self._nblk[r.row] = len(r.blocks)
         n_i64[0, rows] = np.fromiter(((r.out_tokens or r.prompt)[-1] for r in reqs), dtype=np.int64, count=len(reqs))
+        if self.model.portions and (n_i64[0, rows].min() < 0 or n_i64[0, rows].max() >= self.model.spec.vocab_size):
+            raise ValueError(f"token ids must be in [0, {self.model.spec.vocab_size})")
         pos = L - 1
         n_i64[1, rows] = pos
         n_i64[2, rows] = n_i32[rows, pos // BLOCK_SIZE].astype(np.int64) * BLOCK_SIZE + pos % BLOCK_SIZE
@@ -760,6 +764,8 @@ class ModelRunner:
             i64[2, a:b] = _slots(r.blocks, s, s + L)
             tables[k, :len(r.blocks)] = r.blocks
             self._nblk[r.row] = 0  # a decode step restages the row's table
+        if i64[0].min() < 0 or i64[0].max() >= self.model.spec.vocab_size:
+            raise ValueError(f"token ids must be in [0, {self.model.spec.vocab_size})")
         wanted = np.fromiter((place[i] + p for i, p in want), dtype=np.int64, count=len(want))
         d64 = self._h2d(np.concatenate([i64.reshape(-1), wanted]))
         plan = self.model.plan(lens, starts, n_short)

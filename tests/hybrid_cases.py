@@ -1,0 +1,95 @@
+"""Small hybrid-decoder configurations and weights for the tests, made from a seed."""
+
+import math
+
+import torch
+
+
+def latent(heads=3, dim=20, rot_dim=12, vdim=28, kv_rank=40, window=37, scale=None, base=5000.0, scaling=True):
+    rot = {"base": base, "dims": rot_dim}
+    if scaling:
+        rot["scaling"] = {"factor": 4.0, "original": 64, "fast": 8.0, "slow": 0.5}
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "rot": rot,
+         "scale": scale or 1.3 / math.sqrt(dim + rot_dim)}
+    if window:
+        m["mask"] = {"size": window}
+    return {"type": "latent_attention", "mixer": m}
+
+
+def delta(heads=4, kv_heads=2, dim=24, vdim=36, conv=3):
+    return {"type": "delta", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def config(layers, width=72, vocab=211, ff=100, loop=None, softcap=9.0, eps=3e-5, no_mlp=()):
+    layers = [dict(e, mlp=None if i in no_mlp else {"kind": "dense", "ff": ff}) for i, e in enumerate(layers)]
+    cfg = {"architecture": "Dovidra", "layers": layers, "norm": {"eps": eps}, "vocab": vocab, "width": width}
+    if loop:
+        cfg["loop"] = dict(zip(("start", "stop", "times"), loop))
+    if softcap:
+        cfg["logit_softcap"] = softcap
+    return cfg
+
+
+CONFIGS = {
+    # odd sizes, two windows, a loop over both kinds
+    "odd": config([delta(), latent(), latent(heads=5, dim=18, rot_dim=6, vdim=11, kv_rank=33, window=16),
+                   delta(heads=3, kv_heads=3, dim=18, vdim=10, conv=5)], loop=(1, 3, 3)),
+    # no loop, no cap, layers without a feed-forward, no window, no rotary scaling
+    "plain": config([latent(window=None, scaling=False), delta(heads=2, kv_heads=1, dim=64, vdim=64, conv=4),
+                     latent(window=1)], width=128, softcap=None, no_mlp=(0, 2)),
+    # loop from the first to the last layer, once; shapes the matrix kernels take exactly
+    "once": config([latent(heads=16, dim=32, rot_dim=32, vdim=32, kv_rank=96, window=50),
+                    delta(heads=4, kv_heads=4, dim=32, vdim=48, conv=1)], width=96, ff=64, loop=(0, 2, 1)),
+    # only recurrent layers, wide convolution
+    "recurrent": config([delta(heads=6, kv_heads=3, dim=16, vdim=16, conv=9), delta(conv=2)], width=64,
+                        loop=(1, 2, 2), no_mlp=(1,)),
+}
+
+
+def make_weights(cfg, seed=0):
+    """bf16 tensors by checkpoint name. Decays span short and long memory, norms and gates are not 1."""
+    g = torch.Generator().manual_seed(seed)
+    W = cfg["width"]
+    w = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        w[name] = torch.randn(rows, cols, generator=g) * gain / math.sqrt(cols)
+
+    def vec(name, n, mean=1.0, std=0.2):
+        w[name] = mean + std * torch.randn(n, generator=g)
+
+    w["embed"] = torch.randn(cfg["vocab"], W, generator=g)
+    if cfg.get("loop"):
+        w["loop.step"] = torch.randn(cfg["loop"]["times"], W, generator=g)
+    for i, e in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        vec(p + "norm1", W)
+        q = p + "mix."
+        if e["type"] == "latent_attention":
+            H, C = m["heads"], m["kv_rank"]
+            mat(q + "q", H * (m["dim"] + m["rot_dim"]), W, 2.0)
+            mat(q + "dkv", C + m["rot_dim"], W, 1.5)
+            vec(q + "dkv.norm", C)
+            mat(q + "uk", H * m["dim"], C)
+            mat(q + "uv", H * m["vdim"], C)
+            mat(q + "o", W, H * m["vdim"])
+        else:
+            H, K = m["heads"], m["kv_heads"]
+            for n, rows in (("q", K * m["dim"]), ("k", K * m["dim"]), ("v", H * m["vdim"])):
+                mat(q + n, rows, W)
+                w[q + n + ".conv"] = torch.randn(rows, m["conv"], generator=g) / math.sqrt(m["conv"])
+            mat(q + "b", H, W)
+            mat(q + "a", H, W)
+            vec(q + "A_log", H, -2.0, 1.5)
+            vec(q + "dt_bias", H, 0.0, 1.0)
+            vec(q + "norm", m["vdim"])
+            mat(q + "g", H * m["vdim"], W)
+            mat(q + "o", W, H * m["vdim"], 1.5)
+        if e.get("mlp"):
+            vec(p + "norm2", W)
+            mat(p + "mlp.gate", e["mlp"]["ff"], W)
+            mat(p + "mlp.up", e["mlp"]["ff"], W)
+            mat(p + "mlp.down", W, e["mlp"]["ff"])
+    vec("final.norm", W)
+    mat("head", cfg["vocab"], W, 3.0)
+    return {k: v.to(torch.bfloat16) for k, v in w.items()}

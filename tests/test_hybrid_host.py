@@ -1,0 +1,242 @@
+"""Hybrid decoder host logic on the CPU: configuration and layer order, weight names, rotary tables,
+portion plans, the portion scheduler over a fake runner, and the runner's portion inputs."""
+
+import json
+
+import numpy as np
+import pytest
+import torch
+
+from hybrid_cases import CONFIGS, config, delta, latent, make_weights
+from oracle import hybrid_ref as ref
+from skyrl_amd.inference_engines import mixers
+from skyrl_amd.inference_engines.engine import BLOCK_SIZE, EngineCore, ModelRunner, RequestParams
+from skyrl_amd.inference_engines.hybrid import HybridDecoder, HybridSpec
+from skyrl_amd.inference_engines.registry import build_decoder, decoder_factory, load_decoder
+from test_engine_host import V, FakeRunner, next_token, reference_output, run_all
+
+
+def test_layer_order_with_and_without_loops():
+    order = lambda cfg: [(r.layer, r.step) for r in HybridSpec.from_config(cfg).runs]  # noqa: E731
+    for cfg in CONFIGS.values():
+        assert order(cfg) == ref.layer_runs(cfg)
+    assert order(CONFIGS["odd"]) == [(0, None), (1, 0), (2, None), (1, 1), (2, None), (1, 2), (2, None), (3, None)]
+    with pytest.raises(ValueError):
+        HybridSpec.from_config(config([delta()], loop=(0, 2, 1)))
+    with pytest.raises(ValueError):
+        HybridSpec.from_config(config([dict(delta(), type="unknown")]))
+
+
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
+def test_weight_names_round_trip(dtype):
+    for name, cfg in CONFIGS.items():
+        m = HybridDecoder(cfg, "cpu", dtype=dtype, seed=None, max_model_len=64)
+        w = make_weights(cfg)
+        assert m.load_weights(w.items()) == len(w)
+        ours = dict(m.hf_named_tensors())
+        assert sorted(ours) == sorted(w)
+        for k in w:
+            assert torch.equal(ours[k].float(), w[k].float()), (name, k)
+        assert m.num_params() == sum(t.numel() for t in w.values())
+        for L in m.layers:  # derived tensors follow the weights
+            if isinstance(L["mixer"], mixers.LatentAttention):
+                x = L["mixer"]
+                assert torch.equal(x.wuv_t, x.wuv.view(x.heads, x.vdim, x.rank).transpose(1, 2))
+        with pytest.raises(KeyError):
+            m.load_weights([("l9.norm1", w["final.norm"])])
+        with pytest.raises(ValueError):
+            m.load_weights([("final.norm", torch.zeros(3))])
+
+
+def test_checkpoint_folder_and_registry(tmp_path):
+    from safetensors.torch import save_file
+
+    cfg, w = CONFIGS["odd"], make_weights(CONFIGS["odd"], 3)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file(w, str(tmp_path / "model.safetensors"))
+    m = load_decoder(str(tmp_path), "cpu", max_model_len=64)
+    assert isinstance(m, HybridDecoder) and torch.equal(dict(m.hf_named_tensors())["l1.mix.uv"], w["l1.mix.uv"])
+    assert not m.prefix_cacheable and build_decoder(config([latent()]), "cpu", max_model_len=8).prefix_cacheable
+    del w["l0.mix.norm"]
+    save_file(w, str(tmp_path / "model.safetensors"))
+    with pytest.raises(ValueError, match="l0.mix.norm"):
+        load_decoder(str(tmp_path), "cpu", max_model_len=64)
+    for bad in ({"architecture": "Nothing"}, {"model_type": "nothing"}, {}):
+        with pytest.raises(ValueError):
+            decoder_factory(bad)
+
+
+@pytest.mark.parametrize("rot", [
+    {"base": 10000.0, "dims": 8}, {"base": 500.0, "dims": 12, "scaling": {"factor": 4.0, "original": 64, "fast": 8.0, "slow": 0.5}},
+    {"base": 1e6, "dims": 64, "scaling": {"factor": 40.0, "original": 4096, "fast": 32.0, "slow": 1.0}},
+    {"base": 20.0, "dims": 4, "scaling": {"factor": 2.0, "original": 7, "fast": 1.0, "slow": 1.0}},  # lo == hi
+    {"base": 10.0, "dims": 2, "scaling": {"factor": 1.0, "original": 9, "fast": 3.0, "slow": 2.0}}])
+def test_rotary_table(rot):
+    n = 200
+    t = mixers.rotary_table(rot, n).double()
+    x = torch.randn(n, rot["dims"], generator=torch.Generator().manual_seed(0), dtype=torch.float64)
+    y = ref.rotate_pairs(x, torch.arange(n), rot)
+    c, s = t[:, :rot["dims"] // 2], t[:, rot["dims"] // 2:]
+    u, v = x[:, 0::2], x[:, 1::2]
+    torch.testing.assert_close(torch.stack([u * c - v * s, v * c + u * s], -1).reshape(n, -1), y, atol=1e-5, rtol=1e-5)
+
+
+def test_sizes_outside_the_design_are_refused():
+    for bad in (dict(rot_dim=7), dict(rot_dim=12)):
+        e = latent(**bad)
+        e["mixer"]["rot"]["dims"] = 7 if bad["rot_dim"] == 7 else 10
+        with pytest.raises(ValueError):
+            HybridDecoder(config([e]), "cpu", seed=None, max_model_len=8)
+    with pytest.raises(ValueError):
+        HybridDecoder(config([delta(heads=3, kv_heads=2)]), "cpu", seed=None, max_model_len=8)
+    with pytest.raises(ValueError):
+        HybridDecoder(config([delta()]), "cpu", dtype=torch.float16)
+
+
+@pytest.mark.parametrize("window", [1, 16, 37, 100, None])
+def test_prompt_plan_covers_every_visible_key(window):
+    lens, starts = [1, 3, 40, 200, 129], [9, 0, 5, 0, 333]
+    seg, tiles, rows, longest = mixers.prompt_plan(lens, starts, 2, 4, window)
+    assert len(seg) == 3 and longest == seg[:, 2].max() and rows % 64 == 0
+    tok, used = 4, 0
+    for (row, lo, n, r0), i in zip(seg, range(2, 5)):
+        first = max(0, starts[i] - window + 1) if window else 0
+        assert row == i and lo % BLOCK_SIZE == 0 and first - BLOCK_SIZE < lo <= first
+        assert lo + n == starts[i] + lens[i] and r0 == used and r0 % 64 == 0
+        used += (n + 63) // 64 * 64
+        mine = [t for t in tiles if t[3] == r0 and t[4] == lo]
+        covered = []
+        for t in mine:
+            assert 0 < t[1] <= mixers.PREFILL_TILE and t[2] - starts[i] == t[0] - tok
+            covered += range(t[0], t[0] + t[1])
+        assert covered == list(range(tok, tok + lens[i]))
+        tok += lens[i]
+    assert used == rows
+    chunk, ends = mixers.chunk_plan(lens, 2, 4)
+    assert ends.tolist() == [0, 1, 5, 8] and chunk[:, 1].tolist() == [40, 64, 64, 64, 8, 64, 64, 1]
+    assert chunk[:, 2].tolist() == [2, 3, 3, 3, 3, 4, 4, 4] and chunk[1, 0] == 44
+
+
+class PortionRunner(FakeRunner):
+    """Checks that every request's tokens are run once, in order, and answers from its whole history."""
+
+    def __init__(self, num_blocks, budget):
+        super().__init__(num_blocks)
+        self.budget, self.seen = budget, {}
+
+    def execute(self, batch):
+        self.batches.append((batch.kind, len(batch.requests)))
+        rows = [r.row for r in batch.requests]
+        assert len(set(rows)) == len(rows) and min(rows) >= 0
+        decodes = sum(c == 1 for c in batch.counts)
+        assert sum(batch.counts) <= max(self.budget, decodes)
+        owners = {}
+        out = []
+        for r, c, sup in zip(batch.requests, batch.counts, batch.suppress):
+            assert c >= 1 and r.num_computed + c <= r.num_tokens <= len(r.blocks) * BLOCK_SIZE
+            for b in r.blocks:
+                assert owners.setdefault(b, r.rid) == r.rid
+            hist = self.seen.setdefault(r.rid, [])
+            del hist[r.num_computed:]  # a preempted request starts over
+            assert len(hist) == r.num_computed
+            hist += r.tokens(r.num_computed, r.num_computed + c)
+            if r.num_computed + c == r.num_tokens:
+                out.append(next_token(hist, sup))
+        if batch.kind == "decode":
+            assert len(out) == len(batch.requests)
+        return np.array(out, dtype=np.int64), np.zeros(len(out), dtype=np.float32)
+
+
+@pytest.mark.parametrize("num_blocks,budget", [(400, 64), (400, 5), (12, 16), (12, 1)])
+def test_portion_scheduler_outputs_independent_of_budget_and_pressure(num_blocks, budget):
+    rng = np.random.default_rng(1)
+    runner = PortionRunner(num_blocks, budget)
+    core = EngineCore(runner, num_blocks, max_num_seqs=6, max_model_len=200, max_prefill_tokens=budget, eos_token_id=3,
+                      portions=True)
+    reqs, expect = [], []
+    for _ in range(12):
+        prompt = rng.integers(0, V, size=int(rng.integers(1, 40))).tolist()
+        params = RequestParams(max_tokens=int(rng.integers(1, 40)), min_tokens=int(rng.integers(0, 3)), stop_token_ids=(5,))
+        reqs.append(core.add_request(prompt, params))
+        expect.append(reference_output(prompt, params, eos=3))
+    run_all(core)
+    for r, (toks, reason) in zip(reqs, expect):
+        assert r.out_tokens == toks and r.finish_reason == reason
+    assert core.allocator.num_free == num_blocks and len(core._free_rows) == 6
+    kinds = {k for k, _ in runner.batches}
+    assert kinds == {"portions", "decode"}
+    if (num_blocks, budget) == (12, 16):
+        assert core.num_preemptions > 0
+
+
+def test_decodes_are_not_held_up_by_a_long_prompt():
+    runner = PortionRunner(100, 16)
+    core = EngineCore(runner, 100, max_num_seqs=4, max_model_len=800, max_prefill_tokens=16, portions=True)
+    a = core.add_request([1, 2], RequestParams(max_tokens=50))
+    core.step()
+    core.add_request(list(range(90)), RequestParams(max_tokens=5))
+    before = len(a.out_tokens)
+    for _ in range(4):
+        core.step()
+    assert len(a.out_tokens) == before + 4
+
+
+def test_run_portions_admission_and_limits():
+    class LogitRunner:
+        def portion_logits(self, batch, want):
+            self.last = (batch.kind, list(batch.counts), list(want))
+            return "logits" if want else None
+
+    r = LogitRunner()
+    core = EngineCore(r, 4, max_num_seqs=2, max_model_len=64, portions=True)
+    a, b = core.open_request(), core.open_request()
+    with pytest.raises(RuntimeError, match="row"):
+        core.open_request()
+    assert core.run_portions([(a, [1] * 16, [3]), (b, [2], [])]) == "logits"
+    assert r.last == ("portions", [16, 1], [(0, 3)]) and len(a.blocks) == 1 and len(b.blocks) == 1
+    assert core.run_portions([(a, [5], [])]) is None and r.last[0] == "decode" and len(a.blocks) == 2
+    core.run_portions([(b, [1, 2], [1])])
+    assert r.last == ("portions", [2], [(0, 1)]) and b.num_computed == 3
+    with pytest.raises(RuntimeError, match="blocks"):
+        core.run_portions([(b, [1] * 40, [])])
+    core.close_request(a)
+    c = core.open_request()
+    assert c.row == 0 and core.allocator.num_free == 3
+    with pytest.raises(ValueError):
+        core.run_portions([(a, [1], [])])
+    with pytest.raises(ValueError):
+        core.run_portions([(c, [1] * 65, [])])
+    with pytest.raises(ValueError, match="places"):
+        core.run_portions([(c, [1] * 5, [5])])
+
+
+def test_portion_inputs_order_and_contents():
+    """Short portions first, slots through the block tables, wanted places mapped to the new order."""
+    m = HybridDecoder(CONFIGS["odd"], "cpu", seed=None, max_model_len=256)
+    runner = ModelRunner(m, num_blocks=40, max_num_seqs=4)
+    runner._h2d = torch.from_numpy
+    core = EngineCore(runner, 40, max_num_seqs=4, max_model_len=256, portions=True)
+    got = {}
+    m.forward_portions = lambda inp, cache: got.setdefault("inp", inp)
+    m.logits = lambda hidden: hidden
+    m.forward_decode = lambda inp, cache: got.setdefault("dec", inp)
+    runner.use_graphs = False
+    a, b = core.open_request(), core.open_request()
+    core.run_portions([(a, list(range(100, 140)), [0, 39]), (b, [7, 8], [1])])
+    inp = got["inp"]
+    assert inp.n_short == 1 and inp.short_tokens == 2 and inp.seq_lens == [2, 40] and inp.cu.tolist() == [0, 2, 42]
+    assert inp.tokens.tolist() == [7, 8] + list(range(100, 140)) and inp.rows.tolist() == [b.row, a.row]
+    assert inp.want.tolist() == [2, 41, 1] and inp.bt_row.tolist() == [0, 0] + [1] * 40
+    assert inp.slots[2 + 17].item() == a.blocks[1] * BLOCK_SIZE + 1 and inp.positions[41].item() == 39
+    assert inp.block_tables[1, :3].tolist() == a.blocks
+    assert set(inp.plan) == {"chunks", 37, 16} and inp.plan[37][0].tolist() == [[1, 0, 40, 0]]
+    for bad in ([CONFIGS["odd"]["vocab"]], [-1, 3]):
+        b.prompt.extend(bad * 2)
+        with pytest.raises(ValueError, match="token ids"):
+            runner._portion_inputs(core._batch_of([(b, len(bad) * 2)]), [])
+        del b.prompt[2:]
+    # a decode step of one request leaves the other's row idle
+    core.run_portions([(b, [9], [])])
+    dec = got["dec"]
+    assert dec.one_token and dec.rows.tolist() == [-1, b.row] and dec.tokens.tolist() == [0, 9]
+    assert dec.slots.tolist() == [-1, b.blocks[0] * BLOCK_SIZE + 2]
