@@ -47,9 +47,9 @@ int skyrl_softcap(const void* x, float* out, int64_t count, float cap, int32_t d
  *   skyrl_latent_attend  one query row per token in the latent space: qa T [heads, T, rank] is the
  *                        unrotated query times the key up-projection, q_rot points at the rotated part
  *                        of head 0 of token 0 (token stride q_stride, head stride q_head); out
- *                        T [heads, T, rank] = softmax(scale * (qa.c + q_rot.k_rot)) c. nparts waves
- *                        share a token's keys (MFMA form, bf16); part_min >= 16 keys, a multiple of
- *                        16, per wave; nparts > 1 needs skyrl_latent_attend_workspace_bytes. f32, and
+ *                        T [heads, T, rank] = softmax(scale * (qa.c + q_rot.k_rot)) c. nparts
+ *                        workgroups share a token's keys (MFMA form, bf16); part_min >= 16 keys, a
+ *                        multiple of 16, per workgroup; nparts > 1 needs skyrl_latent_attend_workspace_bytes. f32, and
  *                        shapes outside the MFMA form (skyrl_latent_attend_mfma == 0), take a plain
  *                        kernel and ignore nparts.
  *   skyrl_latent_gather  prompt form, step 1: copies for each of nseg segments the cached rows of

@@ -39,26 +39,38 @@ struct Dims {
 };
 
 // silu(causal convolution) of channel ch at token t of a sequence whose first token is t0 at position p0;
-// inputs before t0 come from the stored ones (the input of position p at p % taps).
+// inputs before t0 come from the stored ones (the input of position p at p % taps; r = pos % taps). Up to
+// kWindow taps every load is in flight at once.
 template <typename T>
 __device__ __forceinline__ float conv_silu(const T* __restrict__ proj, int64_t stride, const T* __restrict__ w,
                                            const T* __restrict__ ring, int channels, int taps, int ch, int t, int t0,
-                                           int pos) {
+                                           int pos, int r) {
     float y = 0.f;
-    for (int j = 0; j < taps; ++j) {
-        const int back = taps - 1 - j;
-        const int p = pos - back;
-        if (p < 0) continue;
-        const int tt = t - back;
-        const float x = tt >= t0 ? ld(proj + (int64_t)tt * stride + ch) : ld(ring + (int64_t)(p % taps) * channels + ch);
-        y += x * ld(w + (int64_t)ch * taps + j);
+    auto input = [&](int back) -> float {
+        if (t - back >= t0) return ld(proj + (int64_t)(t - back) * stride + ch);
+        const int slot = r - back < 0 ? r - back + taps : r - back;
+        return ld(ring + (int64_t)slot * channels + ch);
+    };
+    if (taps <= kWindow) {
+        float x[kWindow], f[kWindow];
+#pragma unroll
+        for (int back = 0; back < kWindow; ++back) {
+            const bool on = back < taps && back <= pos;
+            x[back] = on ? input(back) : 0.f;
+            f[back] = on ? ld(w + (int64_t)ch * taps + taps - 1 - back) : 0.f;
+        }
+#pragma unroll
+        for (int back = 0; back < kWindow; ++back) y += x[back] * f[back];
+    } else {
+        for (int back = 0; back < taps && back <= pos; ++back)
+            y += input(back) * ld(w + (int64_t)ch * taps + taps - 1 - back);
     }
     return siluf_(y);
 }
 
-// RPT: state rows per thread. Thread (cg, rg) holds columns 4 cg .. 4 cg + 3 of rows rg, rg + RG, ...
-template <typename T, int RPT>
-__global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __restrict__ proj, int64_t stride,
+// NT threads, RPT state rows per thread: thread (cg, rg) holds columns 4 cg .. 4 cg + 3 of rows rg, rg + RG, ...
+template <typename T, int NT, int RPT>
+__global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void delta_scan_kernel(Dims d, const T* __restrict__ proj, int64_t stride,
                                                          const T* __restrict__ conv_w, const float* __restrict__ a_log,
                                                          const float* __restrict__ dt_bias,
                                                          const T* __restrict__ norm_w, const int32_t* __restrict__ cu,
@@ -72,7 +84,7 @@ __global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __rest
     if (row < 0) return;
     const int t0 = cu[s], t1 = cu[s + 1];
     if (t0 >= t1) return;
-    const int D = d.D, V = d.V, VP = d.vpad(), NC = VP / 4, RG = kNT / NC;
+    const int D = d.D, V = d.V, VP = d.vpad(), NC = VP / 4, RG = NT / NC;
     const int ch_all = d.channels();
     const int kh = h / (d.H / d.K);
     float* s_q = smem;             // D
@@ -84,6 +96,8 @@ __global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __rest
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int cg = tid % NC, rg = tid / NC;
     const bool act = rg < RG;
+    const bool fold = NC <= kWave && (NC & (NC - 1)) == 0;  // a wave holds whole row groups
+    const int nrec = fold ? NT / kWave : RG;
     const int64_t pos0 = positions[t0];
     T* ring = conv_state + (int64_t)row * d.taps * ch_all;
     float* st_ = state + ((int64_t)row * d.H + h) * D * VP;
@@ -95,18 +109,20 @@ __global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __rest
         if (act && r < D && pos0 > 0) v = ld4(st_ + (int64_t)r * VP + 4 * cg);
         S[i][0] = v.x; S[i][1] = v.y; S[i][2] = v.z; S[i][3] = v.w;
     }
-    const float neg_rate = -expf(a_log[h]);
+    const float neg_rate = -expf(a_log[h]), dt = dt_bias[h];
     const float qscale = 1.f / sqrtf((float)D);
     const int qoff = kh * D, koff = (d.K + kh) * D, voff = 2 * d.K * D + h * V;
     const int goff = ch_all + h * V, boff = ch_all + d.H * V + h, aoff = boff + d.H;
     for (int t = t0; t < t1; ++t) {
         const int pos = (int)pos0 + (t - t0);
         const T* p = proj + (int64_t)t * stride;
-        for (int e = tid; e < 2 * D + VP; e += kNT) {
+        const int slot = pos % d.taps;
+        const float b_raw = ld(p + boff), a_raw = ld(p + aoff);
+        for (int e = tid; e < 2 * D + VP; e += NT) {
             float y = 0.f;
             if (e < 2 * D + V) {
                 const int ch = e < D ? qoff + e : e < 2 * D ? koff + e - D : voff + e - 2 * D;
-                y = conv_silu(proj, stride, conv_w, ring, ch_all, d.taps, ch, t, t0, pos);
+                y = conv_silu(proj, stride, conv_w, ring, ch_all, d.taps, ch, t, t0, pos, slot);
             }
             smem[e] = y;  // s_q | s_k | s_v are contiguous
         }
@@ -122,8 +138,8 @@ __global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __rest
         __syncthreads();
         const float rq = qscale / sqrtf(s_n[0] + 1e-6f), rk = 1.f / sqrtf(s_n[1] + 1e-6f);
         const float kq = s_n[2] * rq * rk;
-        const float beta = sigmoidf_(ld(p + boff));
-        const float g = expf(neg_rate * softplusf_(ld(p + aoff) + dt_bias[h]));
+        const float beta = sigmoidf_(b_raw);
+        const float g = expf(neg_rate * softplusf_(a_raw + dt));
         float a[4] = {0.f, 0.f, 0.f, 0.f}, b[4] = {0.f, 0.f, 0.f, 0.f};
         if (act) {
 #pragma unroll
@@ -138,13 +154,24 @@ __global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __rest
                     }
                 }
             }
-            st4(s_red + (rg * 2) * VP + 4 * cg, make_float4(a[0], a[1], a[2], a[3]));
-            st4(s_red + (rg * 2 + 1) * VP + 4 * cg, make_float4(b[0], b[1], b[2], b[3]));
+            if (fold)  // the wave's own row groups first
+                for (int o = NC; o < kWave; o <<= 1) {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        a[j] += __shfl_xor(a[j], o, kWave);
+                        b[j] += __shfl_xor(b[j], o, kWave);
+                    }
+                }
+            if (!fold || lane < NC) {
+                const int rec = fold ? wave : rg;
+                st4(s_red + (rec * 2) * VP + 4 * cg, make_float4(a[0], a[1], a[2], a[3]));
+                st4(s_red + (rec * 2 + 1) * VP + 4 * cg, make_float4(b[0], b[1], b[2], b[3]));
+            }
         }
         __syncthreads();
         if (act) {
             float4 A = make_float4(0.f, 0.f, 0.f, 0.f), B = A;
-            for (int r = 0; r < RG; ++r) {
+            for (int r = 0; r < nrec; ++r) {
                 const float4 x = ld4(s_red + (r * 2) * VP + 4 * cg), y = ld4(s_red + (r * 2 + 1) * VP + 4 * cg);
                 A.x += x.x; A.y += x.y; A.z += x.z; A.w += x.w;
                 B.x += y.x; B.y += y.y; B.z += y.z; B.w += y.w;
@@ -184,9 +211,9 @@ __global__ __launch_bounds__(kNT) void delta_scan_kernel(Dims d, const T* __rest
     if (save_conv) {  // one token: its slot is not among those the convolutions read
         const T* p = proj + (int64_t)t0 * stride;
         T* dst = ring + (int64_t)(pos0 % d.taps) * ch_all;
-        for (int e = tid; e < V; e += kNT) dst[voff + e] = p[voff + e];
+        for (int e = tid; e < V; e += NT) dst[voff + e] = p[voff + e];
         if (h % (d.H / d.K) == 0)
-            for (int e = tid; e < D; e += kNT) {
+            for (int e = tid; e < D; e += NT) {
                 dst[qoff + e] = p[qoff + e];
                 dst[koff + e] = p[koff + e];
             }
@@ -251,36 +278,43 @@ __global__ __launch_bounds__(kNT) void delta_conv_kernel(Dims d, SeqRef sq, cons
         return ld(ring + (int64_t)((pos0 + i) % d.taps) * ch_all + ch);
     };
     const int nch = keys ? 2 * D : min(kNT, d.H * d.V - ((int)blockIdx.y - d.K) * kNT);
-    for (int i0 = 0; i0 < n; i0 += 16) {
-        const int m = min(16, n - i0);
+    const bool held = d.taps <= kWindow, carry = nch <= kNT;  // carry: one channel per thread, inputs stay in registers
+    constexpr int kSub = 16, kBack = kWindow - 1;
+    float x[kBack + kSub];
+    for (int i0 = 0; i0 < n; i0 += kSub) {
+        const int m = min(kSub, n - i0);
         for (int e = tid; e < nch; e += kNT) {
             const int ch = !keys ? 2 * d.K * D + ((int)blockIdx.y - d.K) * kNT + e
                                  : e < D ? kh * D + e : (d.K + kh) * D + (e - D);
-            float x[kWindow], w[kWindow];
-            const bool held = d.taps <= kWindow;
+            float w[kWindow];
             if (held) {
+                if (carry && i0 > 0) {
 #pragma unroll
-                for (int j = 0; j < kWindow; ++j) {
-                    const int tap = j - (kWindow - d.taps);
-                    w[j] = tap >= 0 ? ld(conv_w + (int64_t)ch * d.taps + tap) : 0.f;
-                    x[j] = (j > 0 && tap > 0) ? input(ch, i0 - kWindow + j) : 0.f;
+                    for (int j = 0; j < kBack; ++j) x[j] = x[j + kSub];
+                } else {
+#pragma unroll
+                    for (int j = 0; j < kBack; ++j) x[j] = j >= kWindow - d.taps ? input(ch, i0 - kBack + j) : 0.f;
                 }
+#pragma unroll
+                for (int j = 0; j < kSub; ++j)
+                    x[kBack + j] = ld(proj + (int64_t)(t0 + min(i0 + j, n - 1)) * stride + ch);
+#pragma unroll
+                for (int j = 0; j < kWindow; ++j)
+                    w[j] = j >= kWindow - d.taps ? ld(conv_w + (int64_t)ch * d.taps + j - (kWindow - d.taps)) : 0.f;
             }
-            for (int i = 0; i < m; ++i) {
+#pragma unroll
+            for (int i = 0; i < kSub; ++i) {
                 float y = 0.f;
                 if (held) {
 #pragma unroll
-                    for (int j = 0; j < kWindow - 1; ++j) x[j] = x[j + 1];
-                    x[kWindow - 1] = ld(proj + (int64_t)(t0 + i0 + i) * stride + ch);
-#pragma unroll
-                    for (int j = 0; j < kWindow; ++j) y += x[j] * w[j];
-                } else {
+                    for (int j = 0; j < kWindow; ++j) y += x[i + j] * w[j];
+                } else if (i < m) {
                     for (int j = 0; j < d.taps; ++j)
                         y += input(ch, i0 + i - (d.taps - 1) + j) * ld(conv_w + (int64_t)ch * d.taps + j);
                 }
                 y = siluf_(y);
                 if (keys) smem[i * 2 * D + e] = y;
-                else vout[(int64_t)(t0 + i0 + i) * d.H * d.V + ((int)blockIdx.y - d.K) * kNT + e] = y;
+                else if (i < m) vout[(int64_t)(t0 + i0 + i) * d.H * d.V + ((int)blockIdx.y - d.K) * kNT + e] = y;
             }
         }
         if (!keys) continue;
@@ -299,7 +333,18 @@ __global__ __launch_bounds__(kNT) void delta_conv_kernel(Dims d, SeqRef sq, cons
     }
 }
 
-// One workgroup per (chunk, head).
+__device__ __forceinline__ f32x4 mma4(const float4& a, const float4& b, f32x4 acc) {
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, acc, 0, 0, 0);
+    return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
+}
+__device__ __forceinline__ float4 as_float4(const f32x4& v) { return make_float4(v[0], v[1], v[2], v[3]); }
+
+// One workgroup per (chunk, head). The 64 x 64 system is solved in 16 x 16 blocks: each wave inverts one
+// diagonal block by substitution, the blocks below follow diagonal by diagonal from
+// T_rb = -T_rr sum_k A_rk T_kb, and T then multiplies both right-hand sides. A 16 x 16 result's registers
+// (rows 4 g + i, column c) are the next product's right operand as they are.
 __global__ __launch_bounds__(kNT) void delta_chunk_kernel(Dims d, const int32_t* __restrict__ chunk,
                                                           const float* __restrict__ qk, const float* __restrict__ v,
                                                           const float* __restrict__ lg, const float* __restrict__ beta,
@@ -307,95 +352,79 @@ __global__ __launch_bounds__(kNT) void delta_chunk_kernel(Dims d, const int32_t*
                                                           float* __restrict__ P, float* __restrict__ G) {
     constexpr int LD = kC + 4;
     __shared__ __attribute__((aligned(16))) float s_k[kC * LD];  // a 64-wide slab of K; then A
-    __shared__ __attribute__((aligned(16))) float s_q[kC * LD];
-    __shared__ float s_g[kC], s_b[kC];
+    __shared__ __attribute__((aligned(16))) float s_q[kC * LD];  // a slab of Q; then T = (I + A)^-1
+    __shared__ __attribute__((aligned(16))) float s_g[kC], s_b[kC], s_w[kC];
     const int h = blockIdx.x % d.H, ci = blockIdx.x / d.H;
     const int32_t* ck = chunk + 4 * ci;
     const int t0 = ck[0], n = ck[1];
     const int kh = h / (d.H / d.K), D16 = d.d16(), V16 = d.v16();
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
     const int64_t ch = (int64_t)ci * d.H + h;
-    if (wave == 0) {  // inclusive sums of the log decays
+    if (wave == 0) {  // inclusive sums of the log decays; tokens past the chunk's end have beta 0 and decay 1
         float x = lane < n ? lg[(int64_t)(t0 + lane) * d.H + h] : 0.f;
 #pragma unroll
         for (int o = 1; o < kWave; o <<= 1) {
             const float y = __shfl_up(x, o, kWave);
             if (lane >= o) x += y;
         }
+        const float be = lane < n ? beta[(int64_t)(t0 + lane) * d.H + h] : 0.f;
         s_g[lane] = x;
-        s_b[lane] = lane < n ? beta[(int64_t)(t0 + lane) * d.H + h] : 0.f;
+        s_b[lane] = be;
+        s_w[lane] = be * expf(x);
         G[ch * kC + lane] = x;
     }
-    f32x4 akk[4], aqk[4];  // rows 16 wave .., column blocks 0 .. wave
+    // K K^T and Q K^T on the ten blocks at and below the diagonal: 20 block products, five per wave
+    f32x4 acc[5];
+    int br[5], bc[5];
 #pragma unroll
-    for (int b = 0; b < 4; ++b) akk[b] = aqk[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < 5; ++k) {
+        acc[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+        const int item = (wave + 4 * k) % 10;  // (0,0) (1,0) (1,1) (2,0) ...
+        br[k] = item >= 6 ? 3 : item >= 3 ? 2 : item >= 1 ? 1 : 0;
+        bc[k] = item - br[k] * (br[k] + 1) / 2;
+    }
     for (int d0 = 0; d0 < D16; d0 += kC) {
         const int w4 = min(kC, D16 - d0) / 4;
         __syncthreads();
         for (int e = tid; e < kC * w4; e += kNT) {
             const int i = e / w4, x = (e - i * w4) * 4;
-            float4 kv = make_float4(0.f, 0.f, 0.f, 0.f), qv = kv;
-            if (i < n) {
-                const float* src = qk + ((int64_t)(t0 + i) * 2 * d.K + kh) * D16 + d0 + x;
-                qv = ld4(src);
-                kv = ld4(src + (int64_t)d.K * D16);
-            }
+            const float* src = qk + ((int64_t)(t0 + min(i, n - 1)) * 2 * d.K + kh) * D16 + d0 + x;
+            float4 qv = ld4(src), kv = ld4(src + (int64_t)d.K * D16);
             st4(&s_k[i * LD + x], kv);
             st4(&s_q[i * LD + x], qv);
         }
         __syncthreads();
         for (int s = 0; s < w4 / 4; ++s) {
-            const float4 ak = ld4(&s_k[(16 * wave + c) * LD + 16 * s + 4 * g]);
-            const float4 aq = ld4(&s_q[(16 * wave + c) * LD + 16 * s + 4 * g]);
 #pragma unroll
-            for (int b = 0; b < 4; ++b) {
-                if (b <= wave) {
-                    const float4 bk = ld4(&s_k[(16 * b + c) * LD + 16 * s + 4 * g]);
-                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.x, bk.x, akk[b], 0, 0, 0);
-                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.x, bk.x, aqk[b], 0, 0, 0);
-                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.y, bk.y, akk[b], 0, 0, 0);
-                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.y, bk.y, aqk[b], 0, 0, 0);
-                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.z, bk.z, akk[b], 0, 0, 0);
-                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.z, bk.z, aqk[b], 0, 0, 0);
-                    akk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(ak.w, bk.w, akk[b], 0, 0, 0);
-                    aqk[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(aq.w, bk.w, aqk[b], 0, 0, 0);
-                }
+            for (int k = 0; k < 5; ++k) {
+                const float* left = wave + 4 * k < 10 ? s_k : s_q;
+                acc[k] = mma4(ld4(&left[(16 * br[k] + c) * LD + 16 * s + 4 * g]),
+                              ld4(&s_k[(16 * bc[k] + c) * LD + 16 * s + 4 * g]), acc[k]);
             }
         }
     }
     __syncthreads();
-    float* s_a = s_k;
+    float *s_a = s_k, *s_t = s_q;
 #pragma unroll
-    for (int b = 0; b < 4; ++b) {
+    for (int k = 0; k < 5; ++k) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            const int r = 16 * wave + 4 * g + i, cc = 16 * b + c;
+            const int r = 16 * br[k] + 4 * g + i, cc = 16 * bc[k] + c;
             const float dec = cc <= r ? expf(s_g[r] - s_g[cc]) : 0.f;
-            s_a[r * LD + cc] = cc < r ? s_b[r] * dec * akk[b][i] : 0.f;
-            P[(ch * kC + r) * kC + cc] = dec * aqk[b][i];
+            if (wave + 4 * k < 10) s_a[r * LD + cc] = cc < r ? s_b[r] * dec * acc[k][i] : 0.f;
+            else P[(ch * kC + r) * kC + cc] = dec * acc[k][i];
         }
     }
     __syncthreads();
-    // forward substitution, one right-hand-side column per thread: W's D16 columns, then U's V16
-    for (int col = tid; col < D16 + V16; col += kNT) {
-        const bool isw = col < D16;
-        const int cc = isw ? col : col - D16;
-        float x[kC];
+    {  // diagonal block `wave`: column c of its inverse
+        float x[16];
 #pragma unroll
-        for (int i = 0; i < kC; ++i) {
-            float r = 0.f;
-            if (i < n) {
-                if (isw) r = s_b[i] * expf(s_g[i]) * qk[(((int64_t)(t0 + i) * 2 + 1) * d.K + kh) * D16 + cc];
-                else if (cc < d.V) r = s_b[i] * v[((int64_t)(t0 + i) * d.H + h) * d.V + cc];
-            }
-            x[i] = r;
-        }
-#pragma unroll
-        for (int i = 1; i < kC; ++i) {
-            float r = x[i];
+        for (int i = 0; i < 16; ++i) {
+            float r = i == c ? 1.f : 0.f;
 #pragma unroll
             for (int j4 = 0; j4 < (i + 3) / 4; ++j4) {
-                const float4 a = ld4(&s_a[i * LD + 4 * j4]);  // zero at and above the diagonal
+                const float4 a = ld4(&s_a[(16 * wave + i) * LD + 16 * wave + 4 * j4]);
                 r -= a.x * x[4 * j4];
                 if (4 * j4 + 1 < i) r -= a.y * x[4 * j4 + 1];
                 if (4 * j4 + 2 < i) r -= a.z * x[4 * j4 + 2];
@@ -403,10 +432,56 @@ __global__ __launch_bounds__(kNT) void delta_chunk_kernel(Dims d, const int32_t*
             }
             x[i] = r;
         }
-        float* dst = isw ? W + ch * kC * D16 + cc : U + ch * kC * V16 + cc;
-        const int ld_ = isw ? D16 : V16;
+        if (g == 0) {
 #pragma unroll
-        for (int i = 0; i < kC; ++i) dst[(int64_t)i * ld_] = x[i];
+            for (int i = 0; i < 16; ++i) s_t[(16 * wave + i) * LD + 16 * wave + c] = x[i];
+        }
+    }
+#pragma unroll
+    for (int lev = 1; lev < 4; ++lev) {
+        __syncthreads();
+        if (wave + lev < 4) {
+            const int b = wave, r = wave + lev;
+            f32x4 m = {0.f, 0.f, 0.f, 0.f}, tt = m;
+            for (int k = b; k < r; ++k) {
+                const float* tk = &s_t[(16 * k + 4 * g) * LD + 16 * b + c];
+                m = mma4(ld4(&s_a[(16 * r + c) * LD + 16 * k + 4 * g]),
+                         make_float4(tk[0], tk[LD], tk[2 * LD], tk[3 * LD]), m);
+            }
+            tt = mma4(ld4(&s_t[(16 * r + c) * LD + 16 * r + 4 * g]), as_float4(m), tt);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) s_t[(16 * r + 4 * g + i) * LD + 16 * b + c] = -tt[i];
+        }
+    }
+    __syncthreads();
+    // T times [diag(beta e^G) K | diag(beta) V], 16 columns at a time
+    const int nw = D16 / 16, ntile = nw + V16 / 16;
+    for (int tile = wave; tile < ntile; tile += 4) {
+        const bool isw = tile < nw;
+        const int cc = 16 * (isw ? tile : tile - nw) + c;
+        const float* src = isw ? qk + ((int64_t)t0 * 2 + 1) * d.K * D16 + (int64_t)kh * D16 + cc
+                               : v + ((int64_t)t0 * d.H + h) * d.V + min(cc, d.V - 1);
+        const int64_t step = isw ? (int64_t)2 * d.K * D16 : (int64_t)d.H * d.V;
+        float x[16];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) x[j] = src[min(16 * (j >> 2) + 4 * g + (j & 3), n - 1) * step];
+        f32x4 o[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            const float4 sc = ld4((isw ? s_w : s_b) + 16 * s + 4 * g);
+            const float4 bv = make_float4(x[4 * s] * sc.x, x[4 * s + 1] * sc.y, x[4 * s + 2] * sc.z, x[4 * s + 3] * sc.w);
+#pragma unroll
+            for (int r = s; r < 4; ++r) o[r] = mma4(ld4(&s_t[(16 * r + c) * LD + 16 * s + 4 * g]), bv, o[r]);
+        }
+        float* dst = isw ? W + ch * kC * D16 + cc : U + ch * kC * V16 + cc;
+        const int ldd = isw ? D16 : V16;
+        const bool pad = !isw && cc >= d.V;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) dst[(int64_t)(16 * r + 4 * g + i) * ldd] = pad ? 0.f : o[r][i];
     }
 }
 
@@ -414,19 +489,23 @@ __global__ __launch_bounds__(kNT) void delta_chunk_kernel(Dims d, const int32_t*
 // tiles of S per wave.
 template <int NS>
 __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_chain_kernel(
-    Dims d, SeqRef sq, const int32_t* __restrict__ seq_chunks, int seq0, const float* __restrict__ qk,
+    Dims d, SeqRef sq, const int32_t* __restrict__ seq_chunks, int seq0, int nseq, const float* __restrict__ qk,
     const float* __restrict__ W, const float* __restrict__ U, const float* __restrict__ P, const float* __restrict__ G,
     float* __restrict__ state, float* __restrict__ o) {
     constexpr int LS = NS * 16 + 4, LU = kC + 4, DT = (NS + 3) / 4;
     __shared__ __attribute__((aligned(16))) float s_s[16 * LS];      // S^T slice
     __shared__ __attribute__((aligned(16))) float s_u[2][16 * LU];   // U^T and its decayed copy
     const int V16 = d.v16(), D16 = d.d16(), VP = d.vpad(), nt = V16 / 16;
-    const int vt = blockIdx.x % nt, h = (blockIdx.x / nt) % d.H, si = blockIdx.x / (nt * d.H);
+    // the slices of one (sequence, head) read the same W, Q, K and P: consecutive on one XCD
+    const int xcd = blockIdx.x % 8, slot = blockIdx.x / 8, grp = slot / nt * 8 + xcd;
+    if (grp >= nseq * d.H) return;
+    const int vt = slot % nt, h = grp % d.H, si = grp / d.H;
     const int seq = seq0 + si, row = sq.rows[seq];
     if (row < 0) return;
     const int64_t pos0 = sq.positions[sq.cu[seq]];
     const int kh = h / (d.H / d.K);
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
     const int ns = D16 / 16;
     float* st_ = state + ((int64_t)row * d.H + h) * d.D * VP;
     const int vcol = 16 * vt + c;
@@ -464,7 +543,8 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
         }
         const float* pp = P + (ch * kC + r) * kC + 4 * g;
 #pragma unroll
-        for (int s = 0; s < 4; ++s) t.p[s] = ld4(pp + 16 * s);
+        for (int s = 0; s < 4; ++s)
+            if (s <= wave) t.p[s] = ld4(pp + 16 * s);  // P is lower triangular
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int rr = 16 * wave + 4 * g + i;
@@ -483,12 +563,6 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
                 }
             }
         }
-    };
-    auto mma4 = [](const float4& a, const float4& b, f32x4 acc) {
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, acc, 0, 0, 0);
-        return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
     };
     auto run = [&](int ci, const Tile& t) {
         const int32_t* ck = sq.chunk + 4 * ci;
@@ -520,7 +594,7 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
         for (int k = 0; k < DT; ++k) S[k] = S[k] * decay;
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
-            ao = mma4(t.p[s], ld4(&s_u[0][c * LU + 16 * s + 4 * g]), ao);
+            if (s <= wave) ao = mma4(t.p[s], ld4(&s_u[0][c * LU + 16 * s + 4 * g]), ao);
             const float4 b = ld4(&s_u[1][c * LU + 16 * s + 4 * g]);
 #pragma unroll
             for (int k = 0; k < DT; ++k)
@@ -557,12 +631,44 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
         }
 }
 
-// Output norm and gate: one wave per (token, head) of tokens [first, T).
-template <typename T>
+// Output norm and gate of tokens [first, T). LG lanes share a (token, head), four values a lane (VEC: vdim
+// a multiple of 4, at most 4 LG); otherwise a wave takes one and strides over vdim.
+template <typename T, bool VEC>
 __global__ __launch_bounds__(kNT) void delta_out_kernel(Dims d, const float* __restrict__ o, const T* __restrict__ proj,
-                                                        int64_t stride, const T* __restrict__ norm_w, int first,
+                                                        int64_t stride, const T* __restrict__ norm_w, int first, int LG,
                                                         int64_t items, T* __restrict__ out, int64_t out_stride) {
     const int lane = threadIdx.x & 63;
+    if constexpr (VEC) {
+        const int per = kNT / LG, sub = threadIdx.x % LG, i = 4 * sub;
+        constexpr int kIt = 4;
+        const int64_t e0 = (int64_t)blockIdx.x * per * kIt + threadIdx.x / LG;
+        float4 x[kIt], gt[kIt];
+#pragma unroll
+        for (int k = 0; k < kIt; ++k) {
+            const int64_t e = min(e0 + (int64_t)k * per, items - 1), t = first + e / d.H;
+            const int h = (int)(e % d.H), ii = min(i, d.V - 4);
+            x[k] = ld4(o + (t * d.H + h) * d.V + ii);
+            const T* gp = proj + t * stride + d.channels() + h * d.V + ii;
+            gt[k] = make_float4(ld(gp), ld(gp + 1), ld(gp + 2), ld(gp + 3));
+        }
+        const int ii = min(i, d.V - 4);
+        const float4 w = make_float4(ld(norm_w + ii), ld(norm_w + ii + 1), ld(norm_w + ii + 2), ld(norm_w + ii + 3));
+#pragma unroll
+        for (int k = 0; k < kIt; ++k) {
+            float ss = i < d.V ? x[k].x * x[k].x + x[k].y * x[k].y + x[k].z * x[k].z + x[k].w * x[k].w : 0.f;
+            for (int q = 1; q < LG; q <<= 1) ss += __shfl_xor(ss, q, kWave);
+            const float r = 1.f / sqrtf(ss / (float)d.V + d.eps);
+            const int64_t e = e0 + (int64_t)k * per;
+            if (e < items && i < d.V) {
+                T* dst = out + (first + e / d.H) * out_stride + (e % d.H) * d.V + i;
+                st(dst, x[k].x * r * w.x * siluf_(gt[k].x));
+                st(dst + 1, x[k].y * r * w.y * siluf_(gt[k].y));
+                st(dst + 2, x[k].z * r * w.z * siluf_(gt[k].z));
+                st(dst + 3, x[k].w * r * w.w * siluf_(gt[k].w));
+            }
+        }
+        return;
+    }
     const int64_t e = (int64_t)blockIdx.x * (kNT / kWave) + (threadIdx.x >> 6);
     if (e >= items) return;
     const int64_t t = first + e / d.H;
@@ -576,8 +682,8 @@ __global__ __launch_bounds__(kNT) void delta_out_kernel(Dims d, const float* __r
         st(out + t * out_stride + h * d.V + i, src[i] * r * ld(norm_w + i) * siluf_(ld(gate + i)));
 }
 
-int scan_rows_per_thread(const Dims& d) {
-    const int RG = kNT / (d.vpad() / 4);
+int scan_rows_per_thread(const Dims& d, int nt) {
+    const int RG = nt / (d.vpad() / 4);
     return (d.D + RG - 1) / RG;
 }
 
@@ -598,8 +704,8 @@ int64_t proj_width(const Dims& d) { return d.channels() + (int64_t)d.H * d.V + 2
 
 using namespace skyrl;
 
-#define LAUNCH_SCAN(R)                                                                                             \
-    hipLaunchKernelGGL((delta_scan_kernel<T, R>), dim3(d.H, nseq), dim3(kNT), lds, as_stream(stream), d,           \
+#define LAUNCH_SCAN(NT, R)                                                                                         \
+    hipLaunchKernelGGL((delta_scan_kernel<T, NT, R>), dim3(d.H, nseq), dim3(NT), lds, as_stream(stream), d,        \
                        reinterpret_cast<const T*>(proj), proj_stride, reinterpret_cast<const T*>(conv_w), a_log,   \
                        dt_bias, reinterpret_cast<const T*>(norm_w), cu, rows, positions, state,                    \
                        reinterpret_cast<T*>(conv_state), save_conv, reinterpret_cast<T*>(out), out_stride)
@@ -619,15 +725,16 @@ extern "C" int skyrl_delta_scan(const skyrl_delta_shape* shape, const void* proj
     if (nseq == 0) return SKYRL_OK;
     SKYRL_REQUIRE(proj && conv_w && a_log && dt_bias && norm_w && cu && rows && positions && state && conv_state && out,
                   "delta_scan: null pointer");
-    const int RG = kNT / (d.vpad() / 4), rpt = scan_rows_per_thread(d);
-    SKYRL_REQUIRE(rpt <= 64, "delta_scan: dim * vdim too large for one workgroup's registers (at most 65536)");
+    const int nt = scan_rows_per_thread(d, 256) <= 8 ? 256 : scan_rows_per_thread(d, 512) <= 8 ? 512 : 1024;
+    const int rpt = scan_rows_per_thread(d, nt), RG = nt / (d.vpad() / 4);
+    SKYRL_REQUIRE(rpt <= 16, "delta_scan: dim * vdim too large for one workgroup's registers (at most 65536)");
     const size_t lds = (size_t)(2 * d.D + 2 * d.vpad() + 2 * RG * d.vpad() + 4) * sizeof(float);
     SKYRL_DISPATCH_T(dtype, {
-        if (rpt <= 4) LAUNCH_SCAN(4);
-        else if (rpt <= 8) LAUNCH_SCAN(8);
-        else if (rpt <= 16) LAUNCH_SCAN(16);
-        else if (rpt <= 32) LAUNCH_SCAN(32);
-        else LAUNCH_SCAN(64);
+        if (nt == 256 && rpt <= 4) LAUNCH_SCAN(256, 4);
+        else if (nt == 256) LAUNCH_SCAN(256, 8);
+        else if (nt == 512) LAUNCH_SCAN(512, 8);
+        else if (rpt <= 8) LAUNCH_SCAN(1024, 8);
+        else LAUNCH_SCAN(1024, 16);
     })
     return check_launch("delta_scan_kernel");
 }
@@ -688,8 +795,10 @@ extern "C" int skyrl_delta_chunk(const skyrl_delta_shape* shape, const int32_t* 
 }
 
 #define LAUNCH_CHAIN(NS)                                                                                          \
-    hipLaunchKernelGGL((delta_chain_kernel<NS>), dim3((unsigned)nseq * d.H * (d.v16() / 16)), dim3(kNT), 0,       \
-                       as_stream(stream), d, SeqRef{chunk, cu, rows, positions}, seq_chunks, seq0, qk, W, U, P, G, \
+    hipLaunchKernelGGL((delta_chain_kernel<NS>), dim3((unsigned)(nseq * d.H + 7) / 8 * 8 * (d.v16() / 16)),       \
+                       dim3(kNT), 0,                                                                              \
+                       as_stream(stream), d, SeqRef{chunk, cu, rows, positions}, seq_chunks, seq0, nseq, qk, W, U, \
+                       P, G,                                                                                      \
                        state, o)
 
 extern "C" int skyrl_delta_chain(const skyrl_delta_shape* shape, const int32_t* chunk, const int32_t* seq_chunks,
@@ -723,9 +832,19 @@ extern "C" int skyrl_delta_out(const skyrl_delta_shape* shape, const float* o, c
     if (items == 0) return SKYRL_OK;
     SKYRL_REQUIRE(o && proj && norm_w && out, "delta_out: null pointer");
     SKYRL_DISPATCH_T(dtype, {
-        hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)((items + 3) / 4)), dim3(kNT), 0, as_stream(stream), d,
-                           o, reinterpret_cast<const T*>(proj), proj_stride, reinterpret_cast<const T*>(norm_w), first,
-                           items, reinterpret_cast<T*>(out), out_stride);
+        int LG = 1;
+        while (4 * LG < d.V) LG <<= 1;
+        const T* p = reinterpret_cast<const T*>(proj);
+        const T* w = reinterpret_cast<const T*>(norm_w);
+        T* dst = reinterpret_cast<T*>(out);
+        if (d.V % 4 == 0 && LG <= kWave) {
+            const int64_t per = (int64_t)kNT / LG * 4;
+            hipLaunchKernelGGL((delta_out_kernel<T, true>), dim3((unsigned)((items + per - 1) / per)), dim3(kNT), 0,
+                               as_stream(stream), d, o, p, proj_stride, w, first, LG, items, dst, out_stride);
+        } else {
+            hipLaunchKernelGGL((delta_out_kernel<T, false>), dim3((unsigned)((items + 3) / 4)), dim3(kNT), 0,
+                               as_stream(stream), d, o, p, proj_stride, w, first, LG, items, dst, out_stride);
+        }
     })
     return check_launch("delta_out_kernel");
 }

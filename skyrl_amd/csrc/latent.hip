@@ -6,10 +6,11 @@
 // Decode form (latent_attend): the up-projections are moved to the query and the output, so that all
 // heads share one key row [c | kr] and one value row c: q_n . (W_uk c) = (W_uk^T q_n) . c, and the sum
 // over keys of p_j W_uv c_j = W_uv (sum p_j c_j). The cache is streamed once for up to 16 heads.
-// One wave takes a share of a token's pages: per 16-token page, S^T[token x head] = K[16 x row] .
-// Q^T[row x 16] (mfma_f32_16x16x32_bf16, K straight from HBM to registers, the next page's loads in
-// flight), online softmax per lane, and O^T[rank x head] += C^T[rank x 16] . P^T[16 x head]. C^T needs
-// four tokens of one dimension per lane, so the page also goes through a wave-private LDS tile.
+// A workgroup takes a share of a token's pages, four pages (64 keys) at a time: each wave scores one
+// page, S^T[token x head] = K[16 x row] . Q^T[row x 16] (mfma_f32_16x16x32_bf16, K straight from HBM to
+// registers, the next tile's loads in flight), the latents also go to LDS, and after an exchange of
+// maxima and weights each wave sums a quarter of the rank over all 64 keys, O^T[rank x head] +=
+// C^T[rank x keys] . P^T[keys x head], C^T by transposing LDS reads.
 //
 // Prompt form (latent_gather + two library products + latent_prefill): a long portion pays the
 // up-projection once per key instead of once per query, and the scores cost dim + rot_dim instead of
@@ -130,7 +131,8 @@ __global__ __launch_bounds__(kNT) void latent_attend_plain_kernel(
     }
 }
 
-// Pages [p0, p0 + np) of a token's context cut into shares of `per` pages; parts = number of shares.
+// Pages [p0, p0 + np) of a token's context cut into shares of `per` pages, a multiple of the workgroup's
+// four; parts = number of shares.
 struct PageSplit {
     int p0, per, parts, np;
 };
@@ -138,24 +140,36 @@ __device__ __forceinline__ PageSplit page_split(int lo, int pos, int part_min, i
     PageSplit s;
     s.p0 = lo / kBS;
     s.np = pos / kBS - s.p0 + 1;
-    const int per = (s.np + nparts - 1) / nparts;
-    s.per = max(per, part_min / kBS);
+    const int per = max((s.np + nparts - 1) / nparts, part_min / kBS);
+    s.per = (per + 3) / 4 * 4;
     s.parts = (s.np + s.per - 1) / s.per;
     return s;
 }
 
+// Transposing LDS read: within each group of 16 lanes, lane 4 k + q supplies the address of row k's
+// elements 4 q .. 4 q + 3, and lane i receives element i of the four rows.
+__device__ __forceinline__ s16x4 lds_read_tr(const uint16_t* p) {
+    typedef __attribute__((address_space(3))) s16x4* lds_ptr;
+    return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)p);
+}
+
 // ---- decode form, MFMA ------------------------------------------------------------------------
-// grid (nparts, ceil(heads / 16), tokens), one wave each. NV: 16-wide tiles of the rank, NK: 32-wide
-// steps of the cache row; EXACT when both equal the shape's own.
+// grid (nparts, ceil(heads / 16), tokens), four waves. A tile is four pages, one per wave for the scores;
+// for the values each wave takes a quarter of the rank over all 64 keys. NV: 16-wide tiles of the rank,
+// NK: 32-wide steps of the cache row; EXACT when both equal the shape's own.
 template <int NV, int NK, bool EXACT>
-__global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 4))) void latent_attend_mfma_kernel(
+__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) void latent_attend_mfma_kernel(
     const uint16_t* __restrict__ qa, const uint16_t* __restrict__ q_rot, int64_t q_stride, int64_t q_head,
     const uint16_t* __restrict__ cache, int row, const int32_t* __restrict__ tables, int64_t bt_stride,
     const int32_t* __restrict__ bt_row, const int64_t* __restrict__ positions, int ntok, int heads, int rank, int rot,
     float scale_log2, int window, int part_min, int nparts, uint16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml) {
-    constexpr int LDR = NV * 16 + 8;  // padded LDS row: the four token groups fall into distinct banks
-    __shared__ __attribute__((aligned(16))) uint16_t s_c[kBS * LDR];
+    constexpr int LDR = NV * 16 + 16;  // padded LDS row: sixteen rows' 32-byte pieces fall into distinct banks
+    constexpr int LDP = 64 + 8, NW = NV / 4, LDQ = NK * 32 + 8;
+    constexpr int kTile = 64 * LDR > 16 * LDQ ? 64 * LDR : 16 * LDQ;
+    __shared__ __attribute__((aligned(16))) uint16_t s_c[kTile];  // first the query, then the latent tile
+    __shared__ __attribute__((aligned(16))) uint16_t s_p[16 * LDP];
+    __shared__ float s_m[4][16];
     const int t = blockIdx.z;
     const int pos = (int)positions[t];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
@@ -164,152 +178,163 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 4))) void
     if (part >= sp.parts) return;
     const int nk = EXACT ? NK : row / 32;
     const int nv = EXACT ? NV : (rank + 15) / 16;
-    const int lane = threadIdx.x, c = lane & 15, g = lane >> 4;
-    const int h = blockIdx.y * 16 + c;
-    const bool hv = h < heads;
-
-    s16x8 qf[NK];
-    {
-        const uint16_t* qrow = qa + ((int64_t)(hv ? h : 0) * ntok + t) * rank;
-        const uint16_t* rrow = q_rot + (int64_t)t * q_stride + (int64_t)(hv ? h : 0) * q_head;
-        const bool vec = rank % 8 == 0;
-#pragma unroll
-        for (int s = 0; s < NK; ++s) {
-            const int d = 32 * s + 8 * g;
-            s16x8 f = {0, 0, 0, 0, 0, 0, 0, 0};
-            if (hv && (EXACT || s < nk)) {
-                if (vec && d + 8 <= rank) {
-                    f = *reinterpret_cast<const s16x8*>(qrow + d);
-                } else {
-#pragma unroll
-                    for (int j = 0; j < 8; ++j) {
-                        const int dd = d + j;
-                        if (dd < rank) f[j] = (short)qrow[dd];
-                        else if (dd < rank + rot) f[j] = (short)rrow[dd - rank];
-                    }
-                }
-            }
-            qf[s] = f;
-        }
-    }
-    f32x4 o[NV];
-#pragma unroll
-    for (int n = 0; n < NV; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
-    float m = -INFINITY, l = 0.f;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
+    const int h0 = blockIdx.y * 16;
 
     const int first = sp.p0 + part * sp.per;
     const int np = min(sp.per, sp.np - part * sp.per);
     const int32_t* bt = tables + (int64_t)bt_row[t] * bt_stride + first;
-    int tbl = lane < np ? bt[lane] : 0;
     const uint16_t* kbase = cache + (int64_t)c * row + 8 * g;
-    auto load_page = [&](int j, s16x8 (&kf)[NK]) {
-        const int64_t blk = __builtin_amdgcn_readlane(tbl, j & 63);
-        const uint16_t* p = kbase + blk * kBS * row;
+    s16x8 kf[NK];
+    auto load_page = [&](int j) {
+        if (j < np) {
+            const uint16_t* p = kbase + (int64_t)bt[j] * kBS * row;
 #pragma unroll
-        for (int s = 0; s < NK; ++s)
-            if (EXACT || s < nk) kf[s] = *reinterpret_cast<const s16x8*>(p + 32 * s);
+            for (int s = 0; s < NK; ++s)
+                if (EXACT || s < nk) kf[s] = *reinterpret_cast<const s16x8*>(p + 32 * s);
+        } else {
+#pragma unroll
+            for (int s = 0; s < NK; ++s) kf[s] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+        }
     };
-    auto step = [&](int j, const s16x8 (&kf)[NK]) {
+    load_page(wave);
+
+    // the query rows of this head group, [latent | rotated | 0], through LDS into MFMA operands
+    const bool vec = rank % 8 == 0;
+    for (int e = tid; e < 16 * NK * 4; e += kNT) {
+        const int hh = e / (NK * 4), d = (e - hh * (NK * 4)) * 8, h = h0 + hh;
+        s16x8 f = {0, 0, 0, 0, 0, 0, 0, 0};
+        if (h < heads && d < row) {
+            const uint16_t* qrow = qa + ((int64_t)h * ntok + t) * rank;
+            const uint16_t* rrow = q_rot + (int64_t)t * q_stride + (int64_t)h * q_head;
+            if (vec && d + 8 <= rank) {
+                f = *reinterpret_cast<const s16x8*>(qrow + d);
+            } else {
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    const int dd = d + j;
+                    f[j] = (short)(dd < rank ? qrow[dd] : dd < rank + rot ? rrow[dd - rank] : (uint16_t)0);
+                }
+            }
+        }
+        *reinterpret_cast<s16x8*>(&s_c[hh * LDQ + d]) = f;
+    }
+    __syncthreads();
+    s16x8 qf[NK];
+#pragma unroll
+    for (int s = 0; s < NK; ++s) qf[s] = *reinterpret_cast<const s16x8*>(&s_c[c * LDQ + 32 * s + 8 * g]);
+
+    f32x4 o[NW];
+#pragma unroll
+    for (int n = 0; n < NW; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;
+    for (int j0 = 0; j0 < np; j0 += 4) {
+        const int tb = (first + j0 + wave) * kBS;  // this wave's page
+        const bool edge = j0 + wave >= np || tb < lo || tb + kBS - 1 > pos;
+        if (edge) {  // a masked slot may hold anything: 0 * NaN must not reach the sums
+            const bool ok = j0 + wave < np && tb + c >= lo && tb + c <= pos;
+#pragma unroll
+            for (int s = 0; s < NK; ++s)
+                if (!ok) kf[s] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+        }
+        __syncthreads();  // the query operands, or the previous tile, are consumed
         f32x4 sacc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < NK; ++s) {
             if (EXACT || s < nk) {
-                if (32 * s < NV * 16)  // the latent part of the page, for the value side
-                    *reinterpret_cast<s16x8*>(&s_c[c * LDR + 32 * s + 8 * g]) = kf[s];
+                if (32 * s < NV * 16)
+                    *reinterpret_cast<s16x8*>(&s_c[(16 * wave + c) * LDR + 32 * s + 8 * g]) = kf[s];
                 sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sacc, 0, 0, 0);
             }
         }
-        const int tb = (first + j) * kBS;
-        const bool edge = tb < lo || tb + kBS - 1 > pos;  // the page holds masked tokens
+        load_page(j0 + 4 + wave);
+        // sacc[i]: score of token tb + 4 g + i and head c
         float sv[4], bm = -INFINITY;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int tok = tb + 4 * g + i;
-            sv[i] = (!edge || (tok >= lo && tok <= pos)) ? sacc[i] * scale_log2 : -INFINITY;
+            sv[i] = (!edge || (j0 + wave < np && tok >= lo && tok <= pos)) ? sacc[i] * scale_log2 : -INFINITY;
             bm = fmaxf(bm, sv[i]);
         }
         bm = fmaxf(bm, __shfl_xor(bm, 16, kWave));
         bm = fmaxf(bm, __shfl_xor(bm, 32, kWave));
-        const float mn = fmaxf(m, bm);
-        const float alpha = fast_exp2(m - mn);  // first page: m = -inf, 0
+        if (g == 0) s_m[wave][c] = bm;
+        __syncthreads();
+        const float mn = fmaxf(fmaxf(m, fmaxf(s_m[0][c], s_m[1][c])), fmaxf(s_m[2][c], s_m[3][c]));
+        const float alpha = fast_exp2(m - mn);  // first tile: m = -inf, 0; every tile holds a visible key
         float p[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) p[i] = fast_exp2(sv[i] - mn);
         l = l * alpha + ((p[0] + p[1]) + (p[2] + p[3]));
         m = mn;
-        const uint32_t p01 = pack_bf16x2(p[0], p[1]), p23 = pack_bf16x2(p[2], p[3]);
-        const s16x4 pf = {(short)(p01 & 0xffff), (short)(p01 >> 16), (short)(p23 & 0xffff), (short)(p23 >> 16)};
-        __syncthreads();  // one wave: orders the LDS tile's writes before its reads
-#pragma unroll
-        for (int n = 0; n < NV; ++n) {
-            if (EXACT || n < nv) {
-                s16x4 vf;
-#pragma unroll
-                for (int i = 0; i < 4; ++i) vf[i] = (short)s_c[(4 * g + i) * LDR + 16 * n + c];
-                if (edge) {  // a masked slot may hold anything: 0 * NaN must not reach the sum
-#pragma unroll
-                    for (int i = 0; i < 4; ++i)
-                        if (!(tb + 4 * g + i >= lo && tb + 4 * g + i <= pos)) vf[i] = 0;
-                }
-                o[n] = o[n] * alpha;
-                o[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pf, o[n], 0, 0, 0);
-            }
-        }
+        *reinterpret_cast<uint2*>(&s_p[c * LDP + 16 * wave + 4 * g]) =
+            make_uint2(pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3]));
         __syncthreads();
-    };
-    s16x8 ka[NK], kb[NK];
-    load_page(0, ka);
-    for (int j = 0; j < np; j += 2) {
-        if (j + 1 < np) load_page(j + 1, kb);
-        step(j, ka);
-        if (j + 1 < np) {
-            if (j + 2 < np) {
-                if (((j + 2) & 63) == 0) tbl = (j + 2 + lane < np) ? bt[j + 2 + lane] : 0;
-                load_page(j + 2, ka);
+        s16x8 pf[2];
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            const s16x4 a = *reinterpret_cast<const s16x4*>(&s_p[c * LDP + 32 * kk + 4 * g]);
+            const s16x4 b = *reinterpret_cast<const s16x4*>(&s_p[c * LDP + 32 * kk + 16 + 4 * g]);
+            pf[kk] = s16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+        }
+#pragma unroll
+        for (int n = 0; n < NW; ++n) {
+            const int tile = wave * NW + n;
+            if (EXACT || tile < nv) {
+                o[n] = o[n] * alpha;
+#pragma unroll
+                for (int kk = 0; kk < 2; ++kk) {
+                    const uint16_t* vp = &s_c[(32 * kk + 4 * g + (c >> 2)) * LDR + 16 * tile + 4 * (c & 3)];
+                    const s16x4 a = lds_read_tr(vp), b = lds_read_tr(vp + 16 * LDR);
+                    const s16x8 vf = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+                    o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[kk], o[n], 0, 0, 0);
+                }
             }
-            step(j + 1, kb);
         }
     }
     l += __shfl_xor(l, 16, kWave);
     l += __shfl_xor(l, 32, kWave);
-    if (!hv) return;
+    if (g == 0) s_m[wave][c] = l;
+    __syncthreads();
+    l = (s_m[0][c] + s_m[1][c]) + (s_m[2][c] + s_m[3][c]);
+    const int h = h0 + c;
+    if (h >= heads) return;
     if (sp.parts == 1) {
         const float inv = 1.f / l;
         uint16_t* orow = out + ((int64_t)h * ntok + t) * rank;
 #pragma unroll
-        for (int n = 0; n < NV; ++n) {
-            if (EXACT || n < nv) {
-                const int d = 16 * n + 4 * g;
-                if (EXACT || (rank % 4 == 0 && d + 4 <= rank)) {
-                    *reinterpret_cast<uint2*>(orow + d) =
-                        make_uint2(pack_bf16x2(o[n][0] * inv, o[n][1] * inv), pack_bf16x2(o[n][2] * inv, o[n][3] * inv));
-                } else {
+        for (int n = 0; n < NW; ++n) {
+            const int d = 16 * (wave * NW + n) + 4 * g;
+            if (EXACT || (rank % 4 == 0 && d + 4 <= rank)) {
+                *reinterpret_cast<uint2*>(orow + d) =
+                    make_uint2(pack_bf16x2(o[n][0] * inv, o[n][1] * inv), pack_bf16x2(o[n][2] * inv, o[n][3] * inv));
+            } else {
 #pragma unroll
-                    for (int i = 0; i < 4; ++i)
-                        if (d + i < rank) orow[d + i] = f32_to_bf16(o[n][i] * inv);
-                }
+                for (int i = 0; i < 4; ++i)
+                    if (d + i < rank) orow[d + i] = f32_to_bf16(o[n][i] * inv);
             }
         }
     } else {
         const int64_t rec = ((int64_t)t * heads + h) * nparts + part;
         float* wo = ws_o + rec * (((rank + 15) / 16) * 16);
 #pragma unroll
-        for (int n = 0; n < NV; ++n)
-            if (EXACT || n < nv) *reinterpret_cast<f32x4*>(wo + 16 * n + 4 * g) = o[n];
-        if (g == 0) {
+        for (int n = 0; n < NW; ++n)
+            if (EXACT || wave * NW + n < nv) *reinterpret_cast<f32x4*>(wo + 16 * (wave * NW + n) + 4 * g) = o[n];
+        if (wave == 0 && g == 0) {
             ws_ml[rec * 2] = m;
             ws_ml[rec * 2 + 1] = l;
         }
     }
 }
 
-// Merge of the shares of one (token, head): grid (heads, tokens).
-__global__ __launch_bounds__(kNT) void latent_merge_kernel(const float* __restrict__ ws_o,
-                                                           const float* __restrict__ ws_ml,
-                                                           const int64_t* __restrict__ positions, int ntok, int heads,
-                                                           int rank, int window, int part_min, int nparts,
-                                                           uint16_t* __restrict__ out) {
-    const int h = blockIdx.x, t = blockIdx.y;
+// Merge of the shares of one (token, head): grid (heads, tokens), one wave per 256 dimensions.
+__global__ __launch_bounds__(kWave * 2) void latent_merge_kernel(const float* __restrict__ ws_o,
+                                                                 const float* __restrict__ ws_ml,
+                                                                 const int64_t* __restrict__ positions, int ntok,
+                                                                 int heads, int rank, int window, int part_min,
+                                                                 int nparts, uint16_t* __restrict__ out) {
+    const int h = blockIdx.x, t = blockIdx.y, lane = threadIdx.x & 63;
     const int pos = (int)positions[t];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
     const PageSplit sp = page_split(lo, pos, part_min, nparts);
@@ -317,15 +342,27 @@ __global__ __launch_bounds__(kNT) void latent_merge_kernel(const float* __restri
     const int64_t rec = ((int64_t)t * heads + h) * nparts;
     const int rp = ((rank + 15) / 16) * 16;
     float M = -INFINITY;
-    for (int p = 0; p < sp.parts; ++p) M = fmaxf(M, ws_ml[(rec + p) * 2]);
-    for (int d = threadIdx.x; d < rank; d += kNT) {
-        float L = 0.f, acc = 0.f;
+    for (int p = lane; p < sp.parts; p += kWave) M = fmaxf(M, ws_ml[(rec + p) * 2]);
+    M = wave_max(M);
+    float L = 0.f;
+    for (int p = lane; p < sp.parts; p += kWave) L += fast_exp2(ws_ml[(rec + p) * 2] - M) * ws_ml[(rec + p) * 2 + 1];
+    const float inv = 1.f / wave_sum(L);
+    uint16_t* orow = out + ((int64_t)h * ntok + t) * rank;
+    for (int d = threadIdx.x * 4; d < rp; d += kWave * 8) {
+        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 4
         for (int p = 0; p < sp.parts; ++p) {
-            const float w = fast_exp2(ws_ml[(rec + p) * 2] - M);
-            L += w * ws_ml[(rec + p) * 2 + 1];
-            acc += w * ws_o[(rec + p) * rp + d];
+            const float w = fast_exp2(ws_ml[(rec + p) * 2] - M) * inv;
+            const float4 x = ld4(ws_o + (rec + p) * rp + d);
+            acc.x += w * x.x; acc.y += w * x.y; acc.z += w * x.z; acc.w += w * x.w;
         }
-        out[((int64_t)h * ntok + t) * rank + d] = f32_to_bf16(acc / L);
+        if (rank % 4 == 0 && d + 4 <= rank) {
+            st4(orow + d, acc);
+        } else {
+            const float v[4] = {acc.x, acc.y, acc.z, acc.w};
+            for (int i = 0; i < 4; ++i)
+                if (d + i < rank) orow[d + i] = f32_to_bf16(v[i]);
+        }
     }
 }
 
@@ -374,10 +411,10 @@ __global__ __launch_bounds__(kNT) void latent_gather_kernel(const T* __restrict_
 constexpr int kKT = 64;   // keys per LDS tile
 
 // 8 consecutive elements starting at column d of a key row assembled from [nope | rot | 0].
-__device__ __forceinline__ s16x8 key_chunk(const uint16_t* nope, const uint16_t* rotp, int d, int dim, int rot,
-                                           bool vec) {
+template <bool VEC>
+__device__ __forceinline__ s16x8 key_chunk(const uint16_t* nope, const uint16_t* rotp, int d, int dim, int rot) {
     s16x8 f = {0, 0, 0, 0, 0, 0, 0, 0};
-    if (vec) {
+    if constexpr (VEC) {
         if (d < dim) f = *reinterpret_cast<const s16x8*>(nope + d);
         else if (d < dim + rot) f = *reinterpret_cast<const s16x8*>(rotp + (d - dim));
         return f;
@@ -385,126 +422,118 @@ __device__ __forceinline__ s16x8 key_chunk(const uint16_t* nope, const uint16_t*
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
         const int dd = d + j;
-        if (dd < dim) f[j] = (short)nope[dd];
-        else if (dd < dim + rot) f[j] = (short)rotp[dd - dim];
+        f[j] = (short)(dd < dim ? nope[dd] : dd < dim + rot ? rotp[dd - dim] : (uint16_t)0);
     }
     return f;
 }
 
-template <int NK, int NV>
-__global__ __launch_bounds__(kNT) void latent_prefill_kernel(
+// QT: 16-query tiles per wave, 128 queries per workgroup. VEC: every row piece is 16-byte aligned.
+template <int NK, int NV, int QT, bool VEC>
+__global__ __launch_bounds__(512 / QT) __attribute__((amdgpu_waves_per_eu(2))) void latent_prefill_kernel(
     const uint16_t* __restrict__ q, int64_t q_stride, const uint16_t* __restrict__ k_nope, int64_t k_stride,
     const uint16_t* __restrict__ k_rot, const uint16_t* __restrict__ v_t, int64_t vt_stride,
     const int32_t* __restrict__ tiles, int heads, int dim, int rot, int vdim, float scale_log2, int window,
     uint16_t* __restrict__ out, int64_t out_stride) {
+    constexpr int NT = 512 / QT, QW = 16 * QT;
     constexpr int LDK = NK * 32 + 8, LDV = kKT + 8;
-    constexpr int KCH = NK * 4;                           // 16-byte chunks per key row
-    constexpr int KPT = (kKT * KCH + kNT - 1) / kNT;      // per thread
-    constexpr int VPT = (NV * 16 * (kKT / 8) + kNT - 1) / kNT;
+    constexpr int TPK = NT / kKT, KPT = NK * 4 / TPK;     // threads per key row, 16-byte chunks per thread
+    constexpr int VPT = NV * 16 * (kKT / 8) / NT, VROWS = NT / 8;
     __shared__ __attribute__((aligned(16))) uint16_t s_k[kKT * LDK];
     __shared__ __attribute__((aligned(16))) uint16_t s_v[NV * 16 * LDV];
     const int h = blockIdx.x % heads;  // one head's tiles stay on one XCD when heads is a multiple of 8
     const int32_t* tl = tiles + 8 * (blockIdx.x / heads);
     const int tok0 = tl[0], ntok = tl[1], pos0 = tl[2], seg_row = tl[3], seg_pos = tl[4];
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, g = lane >> 4;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = lane & 15, g = lane >> 4;
     const int dk = dim + rot;
-    const int nk = (dk + 31) / 32, nv = (vdim + 15) / 16;
-    const bool kvec = dim % 8 == 0 && rot % 8 == 0 && k_stride % 8 == 0;
-    const bool qvec = kvec && q_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(q) & 15) == 0;
     const int w = window > 0 ? window : 0x3fffffff;
 
-    // this wave's queries: 32 * wave + 16 qq + c
-    s16x8 qf[2][NK];
-    int qpos[2];
+    // this wave's queries: QW * wave + 16 qq + c
+    s16x8 qf[QT][NK];
+    int qpos[QT];
 #pragma unroll
-    for (int qq = 0; qq < 2; ++qq) {
-        const int qi = 32 * wave + 16 * qq + c;
+    for (int qq = 0; qq < QT; ++qq) {
+        const int qi = QW * wave + 16 * qq + c;
         const bool ok = qi < ntok;
         qpos[qq] = pos0 + qi;
         const uint16_t* qr = q + (int64_t)(tok0 + (ok ? qi : 0)) * q_stride + (int64_t)h * dk;
 #pragma unroll
         for (int s = 0; s < NK; ++s) {
             s16x8 f = {0, 0, 0, 0, 0, 0, 0, 0};
-            if (s < nk && ok) f = key_chunk(qr, qr + dim, 32 * s + 8 * g, dim, rot, qvec);
+            if (ok) f = key_chunk<VEC>(qr, qr + dim, 32 * s + 8 * g, dim, rot);
             qf[qq][s] = f;
         }
     }
-    f32x4 o[NV][2];
+    f32x4 o[NV][QT];
 #pragma unroll
-    for (int n = 0; n < NV; ++n) o[n][0] = o[n][1] = f32x4{0.f, 0.f, 0.f, 0.f};
-    float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
+    for (int n = 0; n < NV; ++n)
+#pragma unroll
+        for (int qq = 0; qq < QT; ++qq) o[n][qq] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float m[QT], l[QT];
+#pragma unroll
+    for (int qq = 0; qq < QT; ++qq) {
+        m[qq] = -INFINITY;
+        l[qq] = 0.f;
+    }
 
     const int lo = max(0, pos0 - w + 1);
     const int j0 = (lo - seg_pos) / kKT, j1 = (pos0 + ntok - 1 - seg_pos) / kKT;
-    const int wq0 = pos0 + 32 * wave;                                // the wave's first query
-    const int wq1 = min(wq0 + 31, pos0 + ntok - 1);                  // and its last
+    const int wq0 = pos0 + QW * wave;                                // the wave's first query
+    const int wq1 = min(wq0 + QW - 1, pos0 + ntok - 1);                  // and its last
     s16x8 kr[KPT], vr[VPT];
+    const int ktok = threadIdx.x / TPK, kd = (threadIdx.x % TPK) * 8;   // key row and first column of this thread
+    const int vd = threadIdx.x >> 3, vtok = (threadIdx.x & 7) * 8;      // value row and first key
     auto fetch = [&](int j) {
         const int64_t r0 = seg_row + (int64_t)j * kKT;
+        const uint16_t* kp = k_nope + (r0 + ktok) * k_stride + (int64_t)h * dim;
+        const uint16_t* rp = k_rot + (r0 + ktok) * rot;
 #pragma unroll
-        for (int i = 0; i < KPT; ++i) {
-            const int e = threadIdx.x + i * kNT;
-            const int tk = e / KCH, d = (e - tk * KCH) * 8;
-            if (tk < kKT && d < nk * 32)
-                kr[i] = key_chunk(k_nope + (r0 + tk) * k_stride + (int64_t)h * dim, k_rot + (r0 + tk) * rot, d, dim,
-                                  rot, kvec);
-        }
+        for (int i = 0; i < KPT; ++i) kr[i] = key_chunk<VEC>(kp, rp, kd + 8 * TPK * i, dim, rot);
+        const uint16_t* vp = v_t + ((int64_t)h * vdim + vd) * vt_stride + r0 + vtok;
 #pragma unroll
         for (int i = 0; i < VPT; ++i) {
-            const int e = threadIdx.x + i * kNT;
-            const int d = e >> 3, tk = (e & 7) * 8;
-            if (d < vdim) vr[i] = *reinterpret_cast<const s16x8*>(v_t + ((int64_t)h * vdim + d) * vt_stride + r0 + tk);
-            else vr[i] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+            vr[i] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
+            if (vd + VROWS * i < vdim) vr[i] = *reinterpret_cast<const s16x8*>(vp + (int64_t)VROWS * i * vt_stride);
         }
     };
     fetch(j0);
     for (int j = j0; j <= j1; ++j) {
         __syncthreads();  // the previous tile is consumed
 #pragma unroll
-        for (int i = 0; i < KPT; ++i) {
-            const int e = threadIdx.x + i * kNT;
-            const int tk = e / KCH, d = (e - tk * KCH) * 8;
-            if (tk < kKT && d < nk * 32) *reinterpret_cast<s16x8*>(&s_k[tk * LDK + d]) = kr[i];
-        }
+        for (int i = 0; i < KPT; ++i) *reinterpret_cast<s16x8*>(&s_k[ktok * LDK + kd + 8 * TPK * i]) = kr[i];
 #pragma unroll
-        for (int i = 0; i < VPT; ++i) {
-            const int e = threadIdx.x + i * kNT;
-            const int d = e >> 3, tk = (e & 7) * 8;
-            if (d < NV * 16) *reinterpret_cast<s16x8*>(&s_v[d * LDV + tk]) = vr[i];
-        }
+        for (int i = 0; i < VPT; ++i) *reinterpret_cast<s16x8*>(&s_v[(vd + VROWS * i) * LDV + vtok]) = vr[i];
         __syncthreads();
         if (j < j1) fetch(j + 1);
         const int kp0 = seg_pos + j * kKT, kp1 = kp0 + kKT - 1;
         if (kp0 > wq1 || kp1 < wq0 - w + 1 || wq0 > wq1) continue;  // no key of this tile for this wave
-        const bool edge = kp1 > wq0 || kp0 < wq1 - w + 1 || wq1 != wq0 + 31;
-        f32x4 sc[4][2];
+        const bool edge = kp1 > wq0 || kp0 < wq1 - w + 1 || wq1 != wq0 + QW - 1;
+        f32x4 sc[4][QT];
 #pragma unroll
-        for (int tt = 0; tt < 4; ++tt) sc[tt][0] = sc[tt][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int tt = 0; tt < 4; ++tt)
+#pragma unroll
+            for (int qq = 0; qq < QT; ++qq) sc[tt][qq] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < NK; ++s) {
-            if (s < nk) {
 #pragma unroll
-                for (int tt = 0; tt < 4; ++tt) {
-                    const s16x8 kf = *reinterpret_cast<const s16x8*>(&s_k[(16 * tt + c) * LDK + 32 * s + 8 * g]);
-                    sc[tt][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[0][s], sc[tt][0], 0, 0, 0);
-                    sc[tt][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[1][s], sc[tt][1], 0, 0, 0);
-                }
+            for (int tt = 0; tt < 4; ++tt) {
+                const s16x8 kf = *reinterpret_cast<const s16x8*>(&s_k[(16 * tt + c) * LDK + 32 * s + 8 * g]);
+#pragma unroll
+                for (int qq = 0; qq < QT; ++qq)
+                    sc[tt][qq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[qq][s], sc[tt][qq], 0, 0, 0);
             }
         }
-        s16x8 pf[2][2];  // [query tile][32-key step]
-        float alpha[2];
+        s16x8 pf[QT][2];  // [query tile][32-key step]
+        float alpha[QT];
 #pragma unroll
-        for (int qq = 0; qq < 2; ++qq) {
+        for (int qq = 0; qq < QT; ++qq) {
             float bm = -INFINITY;
+            const unsigned dist = qpos[qq] - kp0 - 4 * g;  // to the lane's first key
 #pragma unroll
             for (int tt = 0; tt < 4; ++tt)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     float v = sc[tt][qq][i] * scale_log2;
-                    if (edge) {
-                        const int d = qpos[qq] - (kp0 + 16 * tt + 4 * g + i);
-                        if (d < 0 || d >= w) v = -INFINITY;
-                    }
+                    if (edge && dist - (16 * tt + i) >= (unsigned)w) v = -INFINITY;  // after the query, or too far back
                     sc[tt][qq][i] = v;
                     bm = fmaxf(bm, v);
                 }
@@ -535,27 +564,26 @@ __global__ __launch_bounds__(kNT) void latent_prefill_kernel(
         }
 #pragma unroll
         for (int n = 0; n < NV; ++n) {
-            if (n < nv) {
-                o[n][0] = o[n][0] * alpha[0];
-                o[n][1] = o[n][1] * alpha[1];
 #pragma unroll
-                for (int kk = 0; kk < 2; ++kk) {
-                    const uint16_t* vp = &s_v[(16 * n + c) * LDV + 32 * kk + 4 * g];
-                    const s16x4 v0 = *reinterpret_cast<const s16x4*>(vp);
-                    const s16x4 v1 = *reinterpret_cast<const s16x4*>(vp + 16);
-                    const s16x8 vf = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-                    o[n][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[0][kk], o[n][0], 0, 0, 0);
-                    o[n][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[1][kk], o[n][1], 0, 0, 0);
-                }
+            for (int qq = 0; qq < QT; ++qq) o[n][qq] = o[n][qq] * alpha[qq];
+#pragma unroll
+            for (int kk = 0; kk < 2; ++kk) {
+                const uint16_t* vp = &s_v[(16 * n + c) * LDV + 32 * kk + 4 * g];
+                const s16x4 v0 = *reinterpret_cast<const s16x4*>(vp);
+                const s16x4 v1 = *reinterpret_cast<const s16x4*>(vp + 16);
+                const s16x8 vf = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+#pragma unroll
+                for (int qq = 0; qq < QT; ++qq)
+                    o[n][qq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[qq][kk], o[n][qq], 0, 0, 0);
             }
         }
     }
 #pragma unroll
-    for (int qq = 0; qq < 2; ++qq) {
+    for (int qq = 0; qq < QT; ++qq) {
         float s = l[qq];
         s += __shfl_xor(s, 16, kWave);
         s += __shfl_xor(s, 32, kWave);
-        const int qi = 32 * wave + 16 * qq + c;
+        const int qi = QW * wave + 16 * qq + c;
         if (qi >= ntok) continue;
         const float inv = 1.f / s;
         uint16_t* orow = out + (int64_t)(tok0 + qi) * out_stride + (int64_t)h * vdim;
@@ -613,7 +641,7 @@ extern "C" size_t skyrl_latent_attend_workspace_bytes(int32_t T_, int32_t heads,
 }
 
 #define LAUNCH_ATTEND(NV, NK, EX)                                                                                     \
-    hipLaunchKernelGGL((latent_attend_mfma_kernel<NV, NK, EX>), dim3(nparts, (heads + 15) / 16, T_), dim3(64), 0, s,  \
+    hipLaunchKernelGGL((latent_attend_mfma_kernel<NV, NK, EX>), dim3(nparts, (heads + 15) / 16, T_), dim3(kNT), 0, s,  \
                        q_, r_, q_stride, q_head, c_, row, block_tables, bt_stride, bt_row, positions, T_, heads, rank, \
                        rot_dim, scale * kLog2e, window, part_min, nparts, o_, ws_o, ws_ml)
 
@@ -657,7 +685,7 @@ extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_
     else LAUNCH_ATTEND(32, 20, false);
     int rc = check_launch("latent_attend_mfma_kernel");
     if (rc != SKYRL_OK || nparts == 1) return rc;
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(heads, T_), dim3(kNT), 0, s, ws_o, ws_ml, positions, T_, heads, rank,
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(heads, T_), dim3(kWave * 2), 0, s, ws_o, ws_ml, positions, T_, heads, rank,
                        window, part_min, nparts, o_);
     return check_launch("latent_merge_kernel");
 }
@@ -679,8 +707,11 @@ extern "C" int skyrl_latent_gather(const void* cache, int32_t row, const int32_t
     return check_launch("latent_gather_kernel");
 }
 
-#define LAUNCH_PREFILL(NK, NV)                                                                                        \
-    hipLaunchKernelGGL((latent_prefill_kernel<NK, NV>), dim3((unsigned)ntiles * heads), dim3(kNT), 0,                 \
+#define LAUNCH_PREFILL(NK, NV, QT)                                                                                    \
+    if (vec) LAUNCH_PREFILL_(NK, NV, QT, true);                                                                       \
+    else LAUNCH_PREFILL_(NK, NV, QT, false)
+#define LAUNCH_PREFILL_(NK, NV, QT, VEC)                                                                              \
+    hipLaunchKernelGGL((latent_prefill_kernel<NK, NV, QT, VEC>), dim3((unsigned)ntiles * heads), dim3(512 / QT), 0,   \
                        as_stream(stream), reinterpret_cast<const uint16_t*>(q), q_stride,                             \
                        reinterpret_cast<const uint16_t*>(k_nope), k_stride, reinterpret_cast<const uint16_t*>(k_rot), \
                        reinterpret_cast<const uint16_t*>(v_t), vt_stride, tiles, heads, dim, rot_dim, vdim,           \
@@ -699,10 +730,15 @@ extern "C" int skyrl_latent_prefill(const void* q, int64_t q_stride, const void*
     SKYRL_REQUIRE(q && k_nope && k_rot && v_t && tiles && out, "latent_prefill: null pointer");
     SKYRL_REQUIRE(aligned16(k_nope) && aligned16(k_rot) && aligned16(v_t), "latent_prefill: 16-byte alignment");
     const int nk = (dim + rot_dim + 31) / 32, nv = (vdim + 15) / 16;
-    if (nk <= 2 && nv <= 8) LAUNCH_PREFILL(2, 8);
-    else if (nk <= 4 && nv <= 8) LAUNCH_PREFILL(4, 8);
-    else if (nk <= 6 && nv <= 8) LAUNCH_PREFILL(6, 8);
-    else if (nk <= 6) LAUNCH_PREFILL(6, 16);
-    else LAUNCH_PREFILL(8, 16);
+    const bool vec = dim % 8 == 0 && rot_dim % 8 == 0 && k_stride % 8 == 0 && q_stride % 8 == 0 && aligned16(q);
+    if (nk <= 2 && nv <= 8) {
+        LAUNCH_PREFILL(2, 8, 2);
+    } else if (nk <= 4 && nv <= 8) {
+        LAUNCH_PREFILL(4, 8, 2);
+    } else if (nk <= 6 && nv <= 8) {
+        LAUNCH_PREFILL(6, 8, 2);
+    } else {
+        LAUNCH_PREFILL(8, 16, 1);
+    }
     return check_launch("latent_prefill_kernel");
 }

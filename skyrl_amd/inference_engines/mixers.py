@@ -27,6 +27,7 @@ BLOCK_SIZE = kernels.BLOCK_SIZE
 # From this many tokens on a portion takes the prompt forms (keys expanded once per key, chunked
 # recurrence) instead of one query row or one recurrence step per token.
 PROMPT_MIN = 32
+ATTEND_WORKGROUPS = 512  # of the decode attention: two per CU
 PREFILL_TILE = 128  # queries per workgroup of the prompt attention
 
 
@@ -170,7 +171,7 @@ class LatentAttention:
     # ---- decode split
     def nparts(self, tokens: int, max_ctx: int) -> int:
         ctx = min(max_ctx, self.window + BLOCK_SIZE) if self.window else max_ctx
-        return kernels.choose_nparts(tokens, (self.heads + 15) // 16, ctx)
+        return kernels.choose_nparts(tokens, (self.heads + 15) // 16, ctx, target_waves=ATTEND_WORKGROUPS)
 
     def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
         from .. import _ffi
