@@ -101,11 +101,12 @@ int skyrl_latent_prefill(const void* q, int64_t q_stride, const void* k_nope, in
  *   Prompt form, for portions of many tokens, in chunks of 64: chunk i32 [nchunks, 4] (first token,
  *   tokens <= 64, sequence, 0), chunks of one sequence consecutive and in order, cut from its first
  *   token on; d16, v16 = dim, vdim up to a multiple of 16. dim <= 256.
- *   skyrl_delta_conv       1: qk f32 [T, 2, kv_heads, d16] (unit vectors, q scaled), v f32
- *                          [T, heads, vdim], lg f32 [T, heads] (log decay), beta f32 [T, heads], at the
+ *   skyrl_delta_conv       1: qk f32 [T, 2, kv_heads, d16] (unit vectors, q scaled), kt f32
+ *                          [nchunks, kv_heads, d16, 64] (k transposed), v f32 [T, heads, vdim], lg f32 [T, heads] (log decay), beta f32 [T, heads], at the
  *                          chunks' tokens.
  *   skyrl_delta_chunk      2: each chunk's own triangular system: W f32 [nchunks, heads, 64, d16],
- *                          U f32 [nchunks, heads, 64, v16], P f32 [nchunks, heads, 64, 64], G f32
+ *                          U f32 [nchunks, heads, v16, 64] (transposed), P f32 [nchunks, heads, 64, 64] (its
+ *                          blocks below and on the diagonal), G f32
  *                          [nchunks, heads, 64] (summed log decays).
  *   skyrl_delta_chain      3: sequential over the chunks seq_chunks[i] .. seq_chunks[i + 1] - 1 of sequence
  *                          seq0 + i: reads and writes S, o f32 [T, heads, vdim]. skyrl_delta_save stores
@@ -125,13 +126,13 @@ int skyrl_delta_save(const skyrl_delta_shape* shape, const void* proj, int64_t p
 int skyrl_delta_conv(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride, const void* conv_w,
                      const float* a_log, const float* dt_bias, const int32_t* chunk, int32_t nchunks,
                      const int32_t* cu, const int32_t* rows, const int64_t* positions, const void* conv_state,
-                     float* qk, float* v, float* lg, float* beta, int32_t dtype, void* stream);
+                     float* qk, float* kt, float* v, float* lg, float* beta, int32_t dtype, void* stream);
 int skyrl_delta_chunk(const skyrl_delta_shape* shape, const int32_t* chunk, int32_t nchunks, const float* qk,
                       const float* v, const float* lg, const float* beta, float* W, float* U, float* P, float* G,
                       void* stream);
 int skyrl_delta_chain(const skyrl_delta_shape* shape, const int32_t* chunk, const int32_t* seq_chunks, int32_t seq0,
                       int32_t nseq, const int32_t* cu, const int32_t* rows, const int64_t* positions, const float* qk,
-                      const float* W, const float* U, const float* P, const float* G, float* state, float* o,
+                      const float* kt, const float* W, const float* U, const float* P, const float* G, float* state, float* o,
                       void* stream);
 int skyrl_delta_out(const skyrl_delta_shape* shape, const float* o, const void* proj, int64_t proj_stride,
                     const void* norm_w, int32_t first, int32_t T, void* out, int64_t out_stride, int32_t dtype,

@@ -246,9 +246,9 @@ LAYERS_SIGNATURES = {
                                     _I64, _P]),
     "skyrl_delta_scan": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I32, _P, _I64, _I32, _P]),
     "skyrl_delta_save": (_INT, [_DS, _P, _I64, _P, _P, _P, _I32, _P, _I32, _P]),
-    "skyrl_delta_conv": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P]),
+    "skyrl_delta_conv": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P]),
     "skyrl_delta_chunk": (_INT, [_DS, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P]),
-    "skyrl_delta_chain": (_INT, [_DS, _P, _P, _I32, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P]),
+    "skyrl_delta_chain": (_INT, [_DS, _P, _P, _I32, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P]),
     "skyrl_delta_out": (_INT, [_DS, _P, _P, _I64, _P, _I32, _I32, _P, _I64, _I32, _P]),
 }
 

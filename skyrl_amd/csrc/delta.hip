@@ -118,6 +118,7 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void de
         const T* p = proj + (int64_t)t * stride;
         const int slot = pos % d.taps;
         const float b_raw = ld(p + boff), a_raw = ld(p + aoff);
+        const float gate = tid < V ? ld(p + goff + tid) : 0.f, nw = tid < V ? ld(norm_w + tid) : 0.f;
         for (int e = tid; e < 2 * D + VP; e += NT) {
             float y = 0.f;
             if (e < 2 * D + V) {
@@ -193,13 +194,14 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void de
                     make_float4(g * B.x + kq * u[0], g * B.y + kq * u[1], g * B.z + kq * u[2], g * B.w + kq * u[3]));
         }
         __syncthreads();
-        if (wave == 0) {
+        if (wave * kWave < V) {
             float x = 0.f;
             for (int i = lane; i < V; i += kWave) x += s_o[i] * s_o[i];
             x = wave_sum(x);
             const float r = 1.f / sqrtf(x / (float)V + d.eps);
-            for (int i = lane; i < V; i += kWave)
-                st(out + (int64_t)t * out_stride + h * V + i, s_o[i] * r * ld(norm_w + i) * siluf_(ld(p + goff + i)));
+            T* dst = out + (int64_t)t * out_stride + h * V;
+            if (tid < V) st(dst + tid, s_o[tid] * r * nw * siluf_(gate));
+            for (int i = tid + NT; i < V; i += NT) st(dst + i, s_o[i] * r * ld(norm_w + i) * siluf_(ld(p + goff + i)));
         }
         // s_q/s_k/s_v are rewritten only after every thread passed the barrier above; s_o not before the next two
     }
@@ -251,7 +253,7 @@ __global__ __launch_bounds__(kNT) void delta_conv_kernel(Dims d, SeqRef sq, cons
                                                          const T* __restrict__ conv_w, const float* __restrict__ a_log,
                                                          const float* __restrict__ dt_bias,
                                                          const T* __restrict__ conv_state, float* __restrict__ qk,
-                                                         float* __restrict__ vout, float* __restrict__ lg,
+                                                         float* __restrict__ kt, float* __restrict__ vout, float* __restrict__ lg,
                                                          float* __restrict__ beta) {
     extern __shared__ float smem[];  // [16][2 D] of the key heads
     const int32_t* ck = sq.chunk + 4 * blockIdx.x;
@@ -321,16 +323,34 @@ __global__ __launch_bounds__(kNT) void delta_conv_kernel(Dims d, SeqRef sq, cons
         __syncthreads();
         for (int e = wave; e < 2 * m; e += kNT / kWave) {
             const int i = e >> 1, which = e & 1;
-            const float* src = smem + i * 2 * D + which * D;
+            float* src = smem + i * 2 * D + which * D;
             float ss = 0.f;
             for (int k = lane; k < D; k += kWave) ss += src[k] * src[k];
             float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
             if (which == 0) r *= 1.f / sqrtf((float)D);
             float* dst = qk + (((int64_t)(t0 + i0 + i) * 2 + which) * d.K + kh) * D16;
-            for (int k = lane; k < D16; k += kWave) dst[k] = k < D ? src[k] * r : 0.f;
+            for (int k = lane; k < D16; k += kWave) {
+                const float y = k < D ? src[k] * r : 0.f;
+                dst[k] = y;
+                if (which && k < D) src[k] = y;
+            }
+        }
+        __syncthreads();
+        float* tr = kt + (((int64_t)blockIdx.x * d.K + kh) * D16) * kC + i0;  // K^T, zero past the chunk's end
+        for (int e = tid; e < D16 * 4; e += kNT) {
+            const int k = e >> 2, i = (e & 3) * 4;
+            float y[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) y[j] = (k < D && i + j < m) ? smem[(i + j) * 2 * D + D + k] : 0.f;
+            st4(tr + (int64_t)k * kC + i, make_float4(y[0], y[1], y[2], y[3]));
         }
         __syncthreads();
     }
+    if (keys)
+        for (int i0 = (n + kSub - 1) / kSub * kSub; i0 < kC; i0 += kSub)
+            for (int e = tid; e < D16 * 4; e += kNT)
+                st4(kt + (((int64_t)blockIdx.x * d.K + kh) * D16 + (e >> 2)) * kC + i0 + (e & 3) * 4,
+                    make_float4(0.f, 0.f, 0.f, 0.f));
 }
 
 __device__ __forceinline__ f32x4 mma4(const float4& a, const float4& b, f32x4 acc) {
@@ -475,27 +495,33 @@ __global__ __launch_bounds__(kNT) void delta_chunk_kernel(Dims d, const int32_t*
 #pragma unroll
             for (int r = s; r < 4; ++r) o[r] = mma4(ld4(&s_t[(16 * r + c) * LD + 16 * s + 4 * g]), bv, o[r]);
         }
-        float* dst = isw ? W + ch * kC * D16 + cc : U + ch * kC * V16 + cc;
-        const int ldd = isw ? D16 : V16;
-        const bool pad = !isw && cc >= d.V;
+        if (isw) {
+            float* dst = W + ch * kC * D16 + cc;
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
+            for (int r = 0; r < 4; ++r)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) dst[(int64_t)(16 * r + 4 * g + i) * ldd] = pad ? 0.f : o[r][i];
+                for (int i = 0; i < 4; ++i) dst[(16 * r + 4 * g + i) * D16] = o[r][i];
+        } else {  // U^T
+            float* dst = U + (ch * V16 + cc) * kC + 4 * g;
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                st4(dst + 16 * r, cc < d.V ? as_float4(o[r]) : make_float4(0.f, 0.f, 0.f, 0.f));
+        }
     }
 }
 
-// One workgroup per (sequence, head, 16 columns of S). NS: 16-wide steps of dim; DT = ceil(NS / 4) 16-row
-// tiles of S per wave.
-template <int NS>
-__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_chain_kernel(
+// One workgroup per (sequence, head, 16 columns of S). NS: 16-wide steps of dim (EXACT: dim = 16 NS); DT
+// 16-row tiles of S per wave. What a phase has consumed is loaded for the next chunk at once, into the
+// same registers: W and Q during the second phase, K^T and P during the next chunk's first.
+template <int NS, bool EXACT>
+__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 8 ? 2 : 1))) void delta_chain_kernel(
     Dims d, SeqRef sq, const int32_t* __restrict__ seq_chunks, int seq0, int nseq, const float* __restrict__ qk,
-    const float* __restrict__ W, const float* __restrict__ U, const float* __restrict__ P, const float* __restrict__ G,
-    float* __restrict__ state, float* __restrict__ o) {
+    const float* __restrict__ kt, const float* __restrict__ W, const float* __restrict__ U, const float* __restrict__ P,
+    const float* __restrict__ G, float* __restrict__ state, float* __restrict__ o) {
     constexpr int LS = NS * 16 + 4, LU = kC + 4, DT = (NS + 3) / 4;
     __shared__ __attribute__((aligned(16))) float s_s[16 * LS];      // S^T slice
     __shared__ __attribute__((aligned(16))) float s_u[2][16 * LU];   // U^T and its decayed copy
-    const int V16 = d.v16(), D16 = d.d16(), VP = d.vpad(), nt = V16 / 16;
+    const int V16 = d.v16(), D16 = EXACT ? NS * 16 : d.d16(), VP = d.vpad(), nt = V16 / 16;
     // the slices of one (sequence, head) read the same W, Q, K and P: consecutive on one XCD
     const int xcd = blockIdx.x % 8, slot = blockIdx.x / 8, grp = slot / nt * 8 + xcd;
     if (grp >= nseq * d.H) return;
@@ -506,7 +532,7 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     const int kh = h / (d.H / d.K);
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c = lane & 15, g = lane >> 4;
-    const int ns = D16 / 16;
+    const int ns = EXACT ? NS : D16 / 16;
     float* st_ = state + ((int64_t)row * d.H + h) * d.D * VP;
     const int vcol = 16 * vt + c;
 
@@ -520,106 +546,94 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
             const int dd = 16 * tile + 4 * g + i;
             S[k][i] = (pos0 > 0 && dd < d.D && vcol < VP) ? st_[(int64_t)dd * VP + vcol] : 0.f;
         }
-        if (tile < ns) *reinterpret_cast<f32x4*>(&s_s[c * LS + 16 * tile + 4 * g]) = S[k];
+        if (EXACT || tile < ns) *reinterpret_cast<f32x4*>(&s_s[c * LS + 16 * tile + 4 * g]) = S[k];
     }
-    struct Tile {
-        float4 w[NS], q[NS], p[4];
-        float kk[DT][16];
-        float u0[4], gr[4], gl;
-    };
-    auto load = [&](int ci, Tile& t) {
-        const int32_t* ck = sq.chunk + 4 * ci;
-        const int t0 = ck[0], n = ck[1];
-        const int64_t ch = (int64_t)ci * d.H + h;
-        const int r = 16 * wave + c, rq = t0 + min(r, n - 1);
-        const float* wp = W + (ch * kC + r) * D16 + 4 * g;
-        const float* qp = qk + ((int64_t)rq * 2 * d.K + kh) * D16 + 4 * g;
+    const int c0 = seq_chunks[si], c1 = seq_chunks[si + 1];
+    const int woff = (16 * wave + c) * D16 + 4 * g, poff = (16 * wave + c) * kC + 4 * g;
+    const int koff = (16 * wave + c) * kC + 4 * g, goff = 16 * wave + 4 * g, uoff = vcol * kC + goff;
+    const int qstep = 2 * d.K * D16, ostep = d.H * d.V;
+    float4 w[NS], q[NS], p[4], kk[DT][4], u0, gr;
+    float gl;
+    auto load_first = [&](int ci, int t0, int n) {
+        const float* wp = W + ((int64_t)ci * d.H + h) * kC * D16;
+        const float* qp = qk + ((int64_t)t0 * 2 * d.K + kh) * D16;
+        const int qoff = min(16 * wave + c, n - 1) * qstep + 4 * g;
 #pragma unroll
         for (int s = 0; s < NS; ++s) {
-            if (s < ns) {
-                t.w[s] = ld4(wp + 16 * s);
-                t.q[s] = ld4(qp + 16 * s);
+            if (EXACT || s < ns) {
+                w[s] = ld4(wp + woff + 16 * s);
+                q[s] = ld4(qp + qoff + 16 * s);
             }
         }
-        const float* pp = P + (ch * kC + r) * kC + 4 * g;
+        const float* gp = G + ((int64_t)ci * d.H + h) * kC;
+        u0 = ld4(U + ((int64_t)ci * d.H + h) * V16 * kC + uoff);
+        gr = ld4(gp + goff);
+        gl = gp[kC - 1];
+    };
+    auto load_second = [&](int ci) {
+        const float* pp = P + ((int64_t)ci * d.H + h) * kC * kC;
+        const float* kp = kt + ((int64_t)ci * d.K + kh) * D16 * kC;
 #pragma unroll
-        for (int s = 0; s < 4; ++s)
-            if (s <= wave) t.p[s] = ld4(pp + 16 * s);  // P is lower triangular
+        for (int s = 0; s < 4; ++s) {
+            if (s <= wave) p[s] = ld4(pp + poff + 16 * s);  // P is lower triangular
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int rr = 16 * wave + 4 * g + i;
-            t.u0[i] = U[(ch * kC + rr) * V16 + vcol];
-            t.gr[i] = G[ch * kC + rr];
-        }
-        t.gl = G[ch * kC + kC - 1];
-#pragma unroll
-        for (int k = 0; k < DT; ++k) {
-            const int tile = wave + 4 * k;
-            if (tile < ns) {
-#pragma unroll
-                for (int j = 0; j < 16; ++j) {  // token 16 (j / 4) + 4 g + j % 4, dim 16 tile + c
-                    const int tok = t0 + min(16 * (j >> 2) + 4 * g + (j & 3), n - 1);
-                    t.kk[k][j] = qk[(((int64_t)tok * 2 + 1) * d.K + kh) * D16 + 16 * tile + c];
-                }
-            }
+            for (int k = 0; k < DT; ++k)
+                if (EXACT || wave + 4 * k < ns) kk[k][s] = ld4(kp + koff + 64 * k * kC + 16 * s);
         }
     };
-    auto run = [&](int ci, const Tile& t) {
-        const int32_t* ck = sq.chunk + 4 * ci;
-        const int t0 = ck[0], n = ck[1];
+    int t0 = 0, n = 0;
+    if (c0 < c1) {
+        t0 = sq.chunk[4 * c0];
+        n = sq.chunk[4 * c0 + 1];
+        load_first(c0, t0, n);
+    }
+    for (int ci = c0; ci < c1; ++ci) {
+        load_second(ci);
         __syncthreads();  // S^T of the previous chunk is in LDS
         f32x4 aw = {0.f, 0.f, 0.f, 0.f}, ao = aw;
 #pragma unroll
         for (int s = 0; s < NS; ++s) {
-            if (s < ns) {
+            if (EXACT || s < ns) {
                 const float4 b = ld4(&s_s[c * LS + 16 * s + 4 * g]);
-                aw = mma4(t.w[s], b, aw);
-                ao = mma4(t.q[s], b, ao);
+                aw = mma4(w[s], b, aw);
+                ao = mma4(q[s], b, ao);
             }
         }
-        float4 u, ud;
-        float* up = &u.x;
-        float* dp = &ud.x;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            up[i] = t.u0[i] - aw[i];
-            dp[i] = up[i] * expf(t.gl - t.gr[i]);
-            ao[i] *= expf(t.gr[i]);
-        }
-        st4(&s_u[0][c * LU + 16 * wave + 4 * g], u);
-        st4(&s_u[1][c * LU + 16 * wave + 4 * g], ud);
+        const float4 u = make_float4(u0.x - aw[0], u0.y - aw[1], u0.z - aw[2], u0.w - aw[3]);
+        const float4 ud = make_float4(u.x * expf(gl - gr.x), u.y * expf(gl - gr.y), u.z * expf(gl - gr.z),
+                                      u.w * expf(gl - gr.w));
+        ao[0] *= expf(gr.x);
+        ao[1] *= expf(gr.y);
+        ao[2] *= expf(gr.z);
+        ao[3] *= expf(gr.w);
+        const float decay = expf(gl);
+        st4(&s_u[0][c * LU + goff], u);
+        st4(&s_u[1][c * LU + goff], ud);
         __syncthreads();
-        const float decay = expf(t.gl);
+        const int tc = t0, nc = n;
+        if (ci + 1 < c1) {
+            t0 = sq.chunk[4 * ci + 4];
+            n = sq.chunk[4 * ci + 5];
+            load_first(ci + 1, t0, n);
+        }
 #pragma unroll
         for (int k = 0; k < DT; ++k) S[k] = S[k] * decay;
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
-            if (s <= wave) ao = mma4(t.p[s], ld4(&s_u[0][c * LU + 16 * s + 4 * g]), ao);
             const float4 b = ld4(&s_u[1][c * LU + 16 * s + 4 * g]);
+            if (s <= wave) ao = mma4(p[s], ld4(&s_u[0][c * LU + 16 * s + 4 * g]), ao);
 #pragma unroll
             for (int k = 0; k < DT; ++k)
-                if (wave + 4 * k < ns)
-                    S[k] = mma4(make_float4(t.kk[k][4 * s], t.kk[k][4 * s + 1], t.kk[k][4 * s + 2], t.kk[k][4 * s + 3]),
-                                b, S[k]);
+                if (EXACT || wave + 4 * k < ns) S[k] = mma4(kk[k][s], b, S[k]);
         }
 #pragma unroll
         for (int k = 0; k < DT; ++k)
-            if (wave + 4 * k < ns) *reinterpret_cast<f32x4*>(&s_s[c * LS + 16 * (wave + 4 * k) + 4 * g]) = S[k];
+            if (EXACT || wave + 4 * k < ns) *reinterpret_cast<f32x4*>(&s_s[c * LS + 16 * (wave + 4 * k) + 4 * g]) = S[k];
+        float* op = o + ((int64_t)tc * d.H + h) * d.V;
+        if (vcol < d.V) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int r = 16 * wave + 4 * g + i;
-            if (r < n && vcol < d.V) o[((int64_t)(t0 + r) * d.H + h) * d.V + vcol] = ao[i];
-        }
-    };
-    const int c0 = seq_chunks[si], c1 = seq_chunks[si + 1];
-    Tile ta, tb;
-    if (c0 < c1) load(c0, ta);
-    for (int ci = c0; ci < c1; ci += 2) {
-        if (ci + 1 < c1) load(ci + 1, tb);
-        run(ci, ta);
-        if (ci + 1 < c1) {
-            if (ci + 2 < c1) load(ci + 2, ta);
-            run(ci + 1, tb);
+            for (int i = 0; i < 4; ++i)
+                if (goff + i < nc) op[(goff + i) * ostep + vcol] = ao[i];
         }
     }
 #pragma unroll
@@ -760,22 +774,22 @@ extern "C" int skyrl_delta_save(const skyrl_delta_shape* shape, const void* proj
 extern "C" int skyrl_delta_conv(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride,
                                 const void* conv_w, const float* a_log, const float* dt_bias, const int32_t* chunk,
                                 int32_t nchunks, const int32_t* cu, const int32_t* rows, const int64_t* positions,
-                                const void* conv_state, float* qk, float* v, float* lg, float* beta, int32_t dtype,
-                                void* stream) {
+                                const void* conv_state, float* qk, float* kt, float* v, float* lg, float* beta,
+                                int32_t dtype, void* stream) {
     SKYRL_REQUIRE_T(dtype, "delta_conv");
     const char* bad = bad_shape(shape);
     SKYRL_REQUIRE(!bad, bad);
     const Dims d = dims_of(shape);
     SKYRL_REQUIRE(nchunks >= 0 && proj_stride >= proj_width(d), "delta_conv: bad sizes");
     if (nchunks == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(proj && conv_w && a_log && dt_bias && chunk && cu && rows && positions && conv_state && qk && v && lg &&
-                      beta,
+    SKYRL_REQUIRE(proj && conv_w && a_log && dt_bias && chunk && cu && rows && positions && conv_state && qk && kt && v &&
+                      lg && beta,
                   "delta_conv: null pointer");
     SKYRL_DISPATCH_T(dtype, {
         hipLaunchKernelGGL((delta_conv_kernel<T>), dim3(nchunks, d.K + (d.H * d.V + kNT - 1) / kNT), dim3(kNT),
                            16 * 2 * d.D * sizeof(float), as_stream(stream), d, SeqRef{chunk, cu, rows, positions},
                            reinterpret_cast<const T*>(proj), proj_stride, reinterpret_cast<const T*>(conv_w), a_log,
-                           dt_bias, reinterpret_cast<const T*>(conv_state), qk, v, lg, beta);
+                           dt_bias, reinterpret_cast<const T*>(conv_state), qk, kt, v, lg, beta);
     })
     return check_launch("delta_conv_kernel");
 }
@@ -794,28 +808,28 @@ extern "C" int skyrl_delta_chunk(const skyrl_delta_shape* shape, const int32_t* 
     return check_launch("delta_chunk_kernel");
 }
 
-#define LAUNCH_CHAIN(NS)                                                                                          \
-    hipLaunchKernelGGL((delta_chain_kernel<NS>), dim3((unsigned)(nseq * d.H + 7) / 8 * 8 * (d.v16() / 16)),       \
-                       dim3(kNT), 0,                                                                              \
-                       as_stream(stream), d, SeqRef{chunk, cu, rows, positions}, seq_chunks, seq0, nseq, qk, W, U, \
-                       P, G,                                                                                      \
-                       state, o)
+#define LAUNCH_CHAIN(NS, EXACT)                                                                                 \
+    hipLaunchKernelGGL((delta_chain_kernel<NS, EXACT>),                                                           \
+                       dim3((unsigned)(nseq * d.H + 7) / 8 * 8 * (d.v16() / 16)), dim3(kNT), 0, as_stream(stream), \
+                       d, SeqRef{chunk, cu, rows, positions}, seq_chunks, seq0, nseq, qk, kt, W, U, P, G, state, o)
 
 extern "C" int skyrl_delta_chain(const skyrl_delta_shape* shape, const int32_t* chunk, const int32_t* seq_chunks,
                                  int32_t seq0, int32_t nseq, const int32_t* cu, const int32_t* rows,
-                                 const int64_t* positions, const float* qk, const float* W, const float* U,
-                                 const float* P, const float* G, float* state, float* o, void* stream) {
+                                 const int64_t* positions, const float* qk, const float* kt, const float* W,
+                                 const float* U, const float* P, const float* G, float* state, float* o, void* stream) {
     const char* bad = bad_shape(shape);
     SKYRL_REQUIRE(!bad, bad);
     const Dims d = dims_of(shape);
     SKYRL_REQUIRE(d.D <= 256, "delta_chain: dim must be at most 256");
     SKYRL_REQUIRE(nseq >= 0 && seq0 >= 0 && (int64_t)nseq * d.H * (d.v16() / 16) < (1 << 30), "delta_chain: bad sizes");
     if (nseq == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(chunk && seq_chunks && cu && rows && positions && qk && W && U && P && G && state && o,
+    SKYRL_REQUIRE(chunk && seq_chunks && cu && rows && positions && qk && kt && W && U && P && G && state && o,
                   "delta_chain: null pointer");
-    if (d.D <= 64) LAUNCH_CHAIN(4);
-    else if (d.D <= 128) LAUNCH_CHAIN(8);
-    else LAUNCH_CHAIN(16);
+    if (d.D == 64) LAUNCH_CHAIN(4, true);
+    else if (d.D < 64) LAUNCH_CHAIN(4, false);
+    else if (d.D == 128) LAUNCH_CHAIN(8, true);
+    else if (d.D < 128) LAUNCH_CHAIN(8, false);
+    else LAUNCH_CHAIN(16, false);
     return check_launch("delta_chain_kernel");
 }
 

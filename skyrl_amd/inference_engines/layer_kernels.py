@@ -269,16 +269,17 @@ def delta_prompt(sh, proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, 
     f32 = lambda *shape: torch.empty(shape, dtype=torch.float32, device=dev)  # noqa: E731
     qk, v = f32(T, 2, sh.kv_heads, d16), f32(T, sh.heads, sh.vdim)
     lg, beta = f32(T, sh.heads), f32(T, sh.heads)
-    W, U = f32(nc, sh.heads, CHUNK, d16), f32(nc, sh.heads, CHUNK, v16)
+    kt = f32(nc, sh.kv_heads, d16, CHUNK)
+    W, U = f32(nc, sh.heads, CHUNK, d16), f32(nc, sh.heads, v16, CHUNK)
     P, G = f32(nc, sh.heads, CHUNK, CHUNK), f32(nc, sh.heads, CHUNK)
     o, st, ref = f32(T, sh.heads, sh.vdim), _stream(dev), ctypes.byref(sh)
     _ffi.call("skyrl_delta_conv", ref, _ptr(proj), proj.stride(0), _ptr(conv_w), _ptr(a_log), _ptr(dt_bias),
-              _ptr(chunk), nc, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(conv_state), _ptr(qk), _ptr(v), _ptr(lg),
+              _ptr(chunk), nc, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(conv_state), _ptr(qk), _ptr(kt), _ptr(v), _ptr(lg),
               _ptr(beta), _code(proj), st)
     _ffi.call("skyrl_delta_chunk", ref, _ptr(chunk), nc, _ptr(qk), _ptr(v), _ptr(lg), _ptr(beta), _ptr(W), _ptr(U),
               _ptr(P), _ptr(G), st)
     _ffi.call("skyrl_delta_chain", ref, _ptr(chunk), _ptr(seq_chunks), first_seq, nseq, _ptr(cu), _ptr(rows),
-              _ptr(positions), _ptr(qk), _ptr(W), _ptr(U), _ptr(P), _ptr(G), _ptr(state), _ptr(o), st)
+              _ptr(positions), _ptr(qk), _ptr(kt), _ptr(W), _ptr(U), _ptr(P), _ptr(G), _ptr(state), _ptr(o), st)
     _ffi.call("skyrl_delta_out", ref, _ptr(o), _ptr(proj), proj.stride(0), _ptr(norm_w), first_token, T, _ptr(out),
               out.stride(0), _code(proj), st)
     return out
