@@ -8,8 +8,7 @@
 // over keys of p_j W_uv c_j = W_uv (sum p_j c_j). The cache is streamed once for up to 16 heads.
 // A workgroup takes a share of a token's pages, four pages (64 keys) at a time: each wave scores one
 // page, S^T[token x head] = K[16 x row] . Q^T[row x 16] (mfma_f32_16x16x32_bf16, K straight from HBM to
-// registers, the next tile's loads in flight), the latents also go to LDS, and after an exchange of
-// maxima and weights each wave sums a quarter of the rank over all 64 keys, O^T[rank x head] +=
+// registers, the next tile's loads in flight), scores and latents go to LDS, and each wave sums a quarter of the rank over all 64 keys, O^T[rank x head] +=
 // C^T[rank x keys] . P^T[keys x head], C^T by transposing LDS reads.
 //
 // Prompt form (latent_gather + two library products + latent_prefill): a long portion pays the
@@ -165,11 +164,10 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     float scale_log2, int window, int part_min, int nparts, uint16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml) {
     constexpr int LDR = NV * 16 + 16;  // padded LDS row: sixteen rows' 32-byte pieces fall into distinct banks
-    constexpr int LDP = 64 + 8, NW = NV / 4, LDQ = NK * 32 + 8;
+    constexpr int LDS_ = 64 + 4, NW = NV / 4, LDQ = NK * 32 + 8;
     constexpr int kTile = 64 * LDR > 16 * LDQ ? 64 * LDR : 16 * LDQ;
     __shared__ __attribute__((aligned(16))) uint16_t s_c[kTile];  // first the query, then the latent tile
-    __shared__ __attribute__((aligned(16))) uint16_t s_p[16 * LDP];
-    __shared__ float s_m[4][16];
+    __shared__ __attribute__((aligned(16))) float s_s[16 * LDS_];  // scores [head][key of the tile]
     const int t = blockIdx.z;
     const int pos = (int)positions[t];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
@@ -186,18 +184,22 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     const int np = min(sp.per, sp.np - part * sp.per);
     const int32_t* bt = tables + (int64_t)bt_row[t] * bt_stride + first;
     const uint16_t* kbase = cache + (int64_t)c * row + 8 * g;
-    s16x8 kf[NK];
-    auto load_page = [&](int j) {
-        if (j < np) {
-            const uint16_t* p = kbase + (int64_t)bt[j] * kBS * row;
-#pragma unroll
-            for (int s = 0; s < NK; ++s)
-                if (EXACT || s < nk) kf[s] = *reinterpret_cast<const s16x8*>(p + 32 * s);
-        } else {
-#pragma unroll
-            for (int s = 0; s < NK; ++s) kf[s] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
-        }
+    s16x8 kf[NK];  // this wave's page of the current tile, then of the next
+    // Pages come in windows of 64, whose block ids a wave holds by lane (no table load ahead of a page's).
+    // Loads are unconditional, the last page again past the end: a branch around them would turn every
+    // wait into one for all loads in flight.
+    int tbl = 0, npw = 0;
+    auto window_at = [&](int w0) {
+        npw = min(64, np - w0);
+        tbl = bt[w0 + min(lane, npw - 1)];
     };
+    auto load_page = [&](int j) {
+        const uint16_t* p = kbase + (int64_t)__builtin_amdgcn_readlane(tbl, min(j, npw - 1)) * kBS * row;
+#pragma unroll
+        for (int s = 0; s < NK; ++s)
+            if (EXACT || s < nk) kf[s] = *reinterpret_cast<const s16x8*>(p + 32 * s);
+    };
+    window_at(0);
     load_page(wave);
 
     // the query rows of this head group, [latent | rotated | 0], through LDS into MFMA operands
@@ -214,7 +216,9 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     const int dd = d + j;
-                    f[j] = (short)(dd < rank ? qrow[dd] : dd < rank + rot ? rrow[dd - rank] : (uint16_t)0);
+                    const uint16_t* src = dd < rank ? qrow + dd : dd < rank + rot ? rrow + (dd - rank) : qrow;
+                    const uint16_t x = *src;
+                    f[j] = (short)(dd < rank + rot ? x : 0);
                 }
             }
         }
@@ -229,75 +233,94 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
 #pragma unroll
     for (int n = 0; n < NW; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.f;
-    for (int j0 = 0; j0 < np; j0 += 4) {
-        const int tb = (first + j0 + wave) * kBS;  // this wave's page
-        const bool edge = j0 + wave >= np || tb < lo || tb + kBS - 1 > pos;
+    auto tile = [&](int w0, int j0) {
+        const int tb = (first + w0 + j0 + wave) * kBS;  // this wave's page
+        const bool edge = j0 + wave >= npw || tb < lo || tb + kBS - 1 > pos;
         if (edge) {  // a masked slot may hold anything: 0 * NaN must not reach the sums
-            const bool ok = j0 + wave < np && tb + c >= lo && tb + c <= pos;
+            const bool ok = j0 + wave < npw && tb + c >= lo && tb + c <= pos;
 #pragma unroll
             for (int s = 0; s < NK; ++s)
                 if (!ok) kf[s] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
         }
-        __syncthreads();  // the query operands, or the previous tile, are consumed
-        f32x4 sacc = {0.f, 0.f, 0.f, 0.f};
+        f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = sa;
 #pragma unroll
         for (int s = 0; s < NK; ++s) {
             if (EXACT || s < nk) {
-                if (32 * s < NV * 16)
-                    *reinterpret_cast<s16x8*>(&s_c[(16 * wave + c) * LDR + 32 * s + 8 * g]) = kf[s];
-                sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sacc, 0, 0, 0);
+                if (s & 1) sb = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sb, 0, 0, 0);
+                else sa = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sa, 0, 0, 0);
             }
         }
-        load_page(j0 + 4 + wave);
-        // sacc[i]: score of token tb + 4 g + i and head c
-        float sv[4], bm = -INFINITY;
+        __syncthreads();  // the query operands, or the previous tile, are consumed
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int tok = tb + 4 * g + i;
-            sv[i] = (!edge || (j0 + wave < np && tok >= lo && tok <= pos)) ? sacc[i] * scale_log2 : -INFINITY;
-            bm = fmaxf(bm, sv[i]);
+        for (int s = 0; s < NK; ++s)
+            if ((EXACT || s < nk) && 32 * s < NV * 16)
+                *reinterpret_cast<s16x8*>(&s_c[(16 * wave + c) * LDR + 32 * s + 8 * g]) = kf[s];
+        f32x4 sv = (sa + sb) * scale_log2;  // token tb + 4 g + i, head c
+        if (edge) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int tok = tb + 4 * g + i;
+                if (!(j0 + wave < npw && tok >= lo && tok <= pos)) sv[i] = -INFINITY;
+            }
         }
+        *reinterpret_cast<f32x4*>(&s_s[c * LDS_ + 16 * wave + 4 * g]) = sv;
+        load_page(j0 + 4 + wave);
+        __syncthreads();
+        // every wave: weights of all 64 keys, the lane's own 16 in the order of the MFMA operand
+        f32x4 x[4];
+#pragma unroll
+        for (int w = 0; w < 4; ++w) x[w] = *reinterpret_cast<const f32x4*>(&s_s[c * LDS_ + 16 * w + 4 * g]);
+        float bm = -INFINITY;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) bm = fmaxf(bm, fmaxf(fmaxf(x[w][0], x[w][1]), fmaxf(x[w][2], x[w][3])));
         bm = fmaxf(bm, __shfl_xor(bm, 16, kWave));
         bm = fmaxf(bm, __shfl_xor(bm, 32, kWave));
-        if (g == 0) s_m[wave][c] = bm;
-        __syncthreads();
-        const float mn = fmaxf(fmaxf(m, fmaxf(s_m[0][c], s_m[1][c])), fmaxf(s_m[2][c], s_m[3][c]));
-        const float alpha = fast_exp2(m - mn);  // first tile: m = -inf, 0; every tile holds a visible key
-        float p[4];
-#pragma unroll
-        for (int i = 0; i < 4; ++i) p[i] = fast_exp2(sv[i] - mn);
-        l = l * alpha + ((p[0] + p[1]) + (p[2] + p[3]));
-        m = mn;
-        *reinterpret_cast<uint2*>(&s_p[c * LDP + 16 * wave + 4 * g]) =
-            make_uint2(pack_bf16x2(p[0], p[1]), pack_bf16x2(p[2], p[3]));
-        __syncthreads();
+        const float mn = fmaxf(m, bm);
+        const float alpha = fast_exp2(m - mn);  // first tile: m = -inf, 0; every share starts with a visible key
+        float sum = 0.f;
         s16x8 pf[2];
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
-            const s16x4 a = *reinterpret_cast<const s16x4*>(&s_p[c * LDP + 32 * kk + 4 * g]);
-            const s16x4 b = *reinterpret_cast<const s16x4*>(&s_p[c * LDP + 32 * kk + 16 + 4 * g]);
-            pf[kk] = s16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+            uint32_t pk[4];
+#pragma unroll
+            for (int b = 0; b < 2; ++b) {
+                float p[4];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    p[i] = fast_exp2(x[2 * kk + b][i] - mn);
+                    sum += p[i];
+                }
+                pk[2 * b] = pack_bf16x2(p[0], p[1]);
+                pk[2 * b + 1] = pack_bf16x2(p[2], p[3]);
+            }
+            pf[kk] = __builtin_bit_cast(s16x8, make_uint4(pk[0], pk[1], pk[2], pk[3]));
         }
+        l = l * alpha + sum;
+        m = mn;
 #pragma unroll
         for (int n = 0; n < NW; ++n) {
-            const int tile = wave * NW + n;
-            if (EXACT || tile < nv) {
+            const int vt = wave * NW + n;
+            if (EXACT || vt < nv) {
                 o[n] = o[n] * alpha;
 #pragma unroll
                 for (int kk = 0; kk < 2; ++kk) {
-                    const uint16_t* vp = &s_c[(32 * kk + 4 * g + (c >> 2)) * LDR + 16 * tile + 4 * (c & 3)];
+                    const uint16_t* vp = &s_c[(32 * kk + 4 * g + (c >> 2)) * LDR + 16 * vt + 4 * (c & 3)];
                     const s16x4 a = lds_read_tr(vp), b = lds_read_tr(vp + 16 * LDR);
                     const s16x8 vf = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
                     o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[kk], o[n], 0, 0, 0);
                 }
             }
         }
+    };
+    for (int w0 = 0; w0 < np; w0 += 64) {
+        if (w0 > 0) {
+            window_at(w0);
+            load_page(wave);
+        }
+        for (int j0 = 0; j0 < npw; j0 += 4) tile(w0, j0);
     }
-    l += __shfl_xor(l, 16, kWave);
+    l += __shfl_xor(l, 16, kWave);  // the sum over all keys, the same in every wave
     l += __shfl_xor(l, 32, kWave);
-    if (g == 0) s_m[wave][c] = l;
-    __syncthreads();
-    l = (s_m[0][c] + s_m[1][c]) + (s_m[2][c] + s_m[3][c]);
     const int h = h0 + c;
     if (h >= heads) return;
     if (sp.parts == 1) {

@@ -27,7 +27,7 @@ BLOCK_SIZE = kernels.BLOCK_SIZE
 # From this many tokens on a portion takes the prompt forms (keys expanded once per key, chunked
 # recurrence) instead of one query row or one recurrence step per token.
 PROMPT_MIN = 32
-ATTEND_WORKGROUPS = 512  # of the decode attention: two per CU
+ATTEND_WORKGROUPS = 256  # of the decode attention: one per CU (more split finer than they overlap)
 PREFILL_TILE = 128  # queries per workgroup of the prompt attention
 
 

@@ -11,8 +11,8 @@ from skyrl_amd import _ffi
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def header_functions():
-    src = open(os.path.join(ROOT, "include", "skyrl_hip.h")).read()
+def header_functions(name="skyrl_hip.h"):
+    src = open(os.path.join(ROOT, "include", name)).read()
     src = re.sub(r"/\*.*?\*/", "", src, flags=re.S)
     return sorted(set(re.findall(r"^\s*(?:const\s+)?\w+\*?\s+\*?(skyrl_\w+)\s*\(", src, flags=re.M)))
 
@@ -30,6 +30,35 @@ def test_library_exports_every_declared_symbol():
 
 def test_ffi_signatures_cover_header():
     assert sorted(_ffi.SIGNATURES) == header_functions()
+
+
+def test_layers_library_matches_its_header():
+    """libskyrl_layers.so exports what include/skyrl_layers.h declares, and is bound name by name."""
+    names = header_functions("skyrl_layers.h")
+    assert "skyrl_latent_attend" in names and "skyrl_delta_scan" in names and sorted(_ffi.LAYERS_SIGNATURES) == names
+    lib = _ffi.load_layers()
+    assert not [n for n in names if not hasattr(lib, n)]
+    assert not set(names) & set(header_functions())
+
+
+def test_layers_entries_validate_on_host():
+    p, sh = ctypes.c_void_p(16), _ffi.DeltaShape(3, 2, 8, 8, 4, 1e-5)
+    for name, args, msg in (
+            ("skyrl_add_norm", (None, p, None, p, 1, 9000, 1e-5, 0, p, _ffi.BF16, None), "H must be"),
+            ("skyrl_add_norm", (None, p, None, p, 1, 64, 1e-5, 0, p, _ffi.I64, None), "dtype"),
+            ("skyrl_gate_mul", (p, 1, 8, 7, p, _ffi.F32, None), "activation"),
+            ("skyrl_latent_write", (p, 10, 1, 1, 4, 4, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "proj_stride"),
+            ("skyrl_latent_write", (p, 100, 1, 1, 4, 4, 40, p, 1e-5, p, p, p, p, 40, _ffi.F32, None), "multiple of 32"),
+            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 8, 1, p, p, _ffi.BF16, None),
+             "part_min"),
+            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 64, 2, p, None, _ffi.BF16, None),
+             "workspace"),
+            ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 65, p, 1, 1, 16, 16, 16, 1.0, 0, p, 16, None), "vt_stride"),
+            ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 64, p, 1, 1, 250, 16, 16, 1.0, 0, p, 16, None), "256"),
+            ("skyrl_delta_scan", (ctypes.byref(sh), p, 100, p, p, p, p, p, p, p, 1, p, p, 1, p, 24, _ffi.F32, None),
+             "multiple of kv_heads")):
+        with pytest.raises(_ffi.SkyrlHipError, match=msg):
+            _ffi.call(name, *args)
 
 
 def test_abi_version_and_error_path():

@@ -542,3 +542,38 @@ def test_larger_layers_bf16():
     s = TraceSession(m, 512)
     for i, cuts in enumerate(([200], [100, 20, 40] + [1] * 40)):
         model_close(feed(s, f"r{i}", toks, cuts), want, torch.bfloat16)
+
+
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_trace_program_and_command_line(tmp_path, dtype, capsys, monkeypatch):
+    """A checkpoint folder through the trace replay program (steps on stdin, logits as files) and through
+    the generation command line: the same greedy tokens."""
+    import io
+    import json
+
+    import numpy as np
+    from safetensors.torch import save_file
+
+    from skyrl_amd.inference_engines import __main__ as cli
+    from skyrl_amd.inference_engines import trace
+
+    cfg = CONFIGS["odd"]
+    w = make_weights(cfg, 4)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file(w, str(tmp_path / "model.safetensors"))
+    toks = tokens_of(cfg, 45, 6)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": toks[:40], "want": [39]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": toks[40:42], "want": []},
+                                     {"id": "b", "tokens": toks[:1], "want": [0]}], "end": ["b"]},
+             {"step": 2, "entries": [{"id": "a", "tokens": toks[42:], "want": [2, 0]}], "end": ["a"]}]
+    monkeypatch.setattr("sys.stdin", io.StringIO("\n".join(map(json.dumps, steps)) + "\n"))
+    assert trace.main(["--model", str(tmp_path), "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "128"]) == 0
+    assert capsys.readouterr().out.split("\n")[:3] == ["done 0", "done 1", "done 2"]
+    want, _ = ref.forward(toks, {k: v.double() for k, v in w.items()}, cfg)
+    for step, rows in ((0, [39]), (1, [0]), (2, [44, 42])):
+        got = np.fromfile(str(tmp_path / f"{step}.f32"), dtype="<f4").reshape(len(rows), cfg["vocab"])
+        model_close(torch.from_numpy(got), want[rows], getattr(torch, dtype))
+    assert cli.main(["--model", str(tmp_path), "--dtype", dtype, "--prompt-ids", ",".join(map(str, toks)), "--temperature",
+                     "0", "--max-tokens", "3", "--num-blocks", "20", "--max-model-len", "256"]) == 0
+    ids = json.loads(capsys.readouterr().out.strip().splitlines()[-1])["response_ids"]
+    assert len(ids) == 3 and float(want[44].max() - want[44, ids[0]]) < (1e-3 if dtype == "float32" else 0.3)

@@ -240,3 +240,13 @@ def test_portion_inputs_order_and_contents():
     dec = got["dec"]
     assert dec.one_token and dec.rows.tolist() == [-1, b.row] and dec.tokens.tolist() == [0, 9]
     assert dec.slots.tolist() == [-1, b.blocks[0] * BLOCK_SIZE + 2]
+
+
+def test_command_line_arguments():
+    from skyrl_amd.inference_engines import __main__ as cli
+    from skyrl_amd.inference_engines import trace
+
+    a = cli.parse(["--model", "m", "--prompt-ids", "1,2", "--prompt-ids", "3", "--temperature", "0"])
+    assert a.prompt_ids == ["1,2", "3"] and a.temperature == 0 and a.dtype == "bfloat16"
+    with pytest.raises(SystemExit):
+        trace.main(["--model", "m", "--dtype", "float16", "--out", "o", "--max-tokens", "64"])
