@@ -153,11 +153,12 @@ __device__ __forceinline__ s16x4 lds_read_tr(const uint16_t* p) {
 }
 
 // ---- decode form, MFMA ------------------------------------------------------------------------
-// grid (nparts, ceil(heads / 16), tokens), four waves. A tile is four pages, one per wave for the scores;
-// for the values each wave takes a quarter of the rank over all 64 keys. NV: 16-wide tiles of the rank,
+// grid (nparts, ceil(heads / (16 HG)), tokens), four waves per group of 16 heads. A tile is four pages, one
+// per wave of a group for the scores; for the values each wave takes a quarter of the rank over all 64
+// keys. With HG = 2 two head groups share the tile in LDS and its HBM reads. NV: 16-wide tiles of the rank,
 // NK: 32-wide steps of the cache row; EXACT when both equal the shape's own.
-template <int NV, int NK, bool EXACT>
-__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) void latent_attend_mfma_kernel(
+template <int NV, int NK, bool EXACT, int HG>
+__global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))) void latent_attend_mfma_kernel(
     const uint16_t* __restrict__ qa, const uint16_t* __restrict__ q_rot, int64_t q_stride, int64_t q_head,
     const uint16_t* __restrict__ cache, int row, const int32_t* __restrict__ tables, int64_t bt_stride,
     const int32_t* __restrict__ bt_row, const int64_t* __restrict__ positions, int ntok, int heads, int rank, int rot,
@@ -165,9 +166,9 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     float* __restrict__ ws_ml) {
     constexpr int LDR = NV * 16 + 16;  // padded LDS row: sixteen rows' 32-byte pieces fall into distinct banks
     constexpr int LDS_ = 64 + 4, NW = NV / 4, LDQ = NK * 32 + 8;
-    constexpr int kTile = 64 * LDR > 16 * LDQ ? 64 * LDR : 16 * LDQ;
+    constexpr int NT = kNT * HG, kTile = 64 * LDR > 16 * HG * LDQ ? 64 * LDR : 16 * HG * LDQ;
     __shared__ __attribute__((aligned(16))) uint16_t s_c[kTile];  // first the query, then the latent tile
-    __shared__ __attribute__((aligned(16))) float s_s[16 * LDS_];  // scores [head][key of the tile]
+    __shared__ __attribute__((aligned(16))) float s_scores[HG * 16 * LDS_];  // scores [head][key of the tile]
     const int t = blockIdx.z;
     const int pos = (int)positions[t];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
@@ -176,9 +177,11 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     if (part >= sp.parts) return;
     const int nk = EXACT ? NK : row / 32;
     const int nv = EXACT ? NV : (rank + 15) / 16;
-    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6) & 3, hg = __builtin_amdgcn_readfirstlane(tid >> 8);
     const int c = lane & 15, g = lane >> 4;
-    const int h0 = blockIdx.y * 16;
+    const int h0 = blockIdx.y * 16 * HG;  // the workgroup's first head
+    float* s_s = s_scores + hg * 16 * LDS_;
 
     const int first = sp.p0 + part * sp.per;
     const int np = min(sp.per, sp.np - part * sp.per);
@@ -204,7 +207,7 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
 
     // the query rows of this head group, [latent | rotated | 0], through LDS into MFMA operands
     const bool vec = rank % 8 == 0;
-    for (int e = tid; e < 16 * NK * 4; e += kNT) {
+    for (int e = tid; e < HG * 16 * NK * 4; e += NT) {
         const int hh = e / (NK * 4), d = (e - hh * (NK * 4)) * 8, h = h0 + hh;
         s16x8 f = {0, 0, 0, 0, 0, 0, 0, 0};
         if (h < heads && d < row) {
@@ -227,7 +230,7 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     __syncthreads();
     s16x8 qf[NK];
 #pragma unroll
-    for (int s = 0; s < NK; ++s) qf[s] = *reinterpret_cast<const s16x8*>(&s_c[c * LDQ + 32 * s + 8 * g]);
+    for (int s = 0; s < NK; ++s) qf[s] = *reinterpret_cast<const s16x8*>(&s_c[(16 * hg + c) * LDQ + 32 * s + 8 * g]);
 
     f32x4 o[NW];
 #pragma unroll
@@ -253,7 +256,7 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
         __syncthreads();  // the query operands, or the previous tile, are consumed
 #pragma unroll
         for (int s = 0; s < NK; ++s)
-            if ((EXACT || s < nk) && 32 * s < NV * 16)
+            if ((EXACT || s < nk) && 32 * s < NV * 16 && s % HG == hg)  // the groups share the copy
                 *reinterpret_cast<s16x8*>(&s_c[(16 * wave + c) * LDR + 32 * s + 8 * g]) = kf[s];
         f32x4 sv = (sa + sb) * scale_log2;  // token tb + 4 g + i, head c
         if (edge) {
@@ -321,7 +324,7 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     }
     l += __shfl_xor(l, 16, kWave);  // the sum over all keys, the same in every wave
     l += __shfl_xor(l, 32, kWave);
-    const int h = h0 + c;
+    const int h = h0 + 16 * hg + c;
     if (h >= heads) return;
     if (sp.parts == 1) {
         const float inv = 1.f / l;
@@ -663,10 +666,13 @@ extern "C" size_t skyrl_latent_attend_workspace_bytes(int32_t T_, int32_t heads,
     return recs * ((size_t)((rank + 15) / 16) * 16 + 2) * sizeof(float) + 16;
 }
 
-#define LAUNCH_ATTEND(NV, NK, EX)                                                                                     \
-    hipLaunchKernelGGL((latent_attend_mfma_kernel<NV, NK, EX>), dim3(nparts, (heads + 15) / 16, T_), dim3(kNT), 0, s,  \
-                       q_, r_, q_stride, q_head, c_, row, block_tables, bt_stride, bt_row, positions, T_, heads, rank, \
-                       rot_dim, scale * kLog2e, window, part_min, nparts, o_, ws_o, ws_ml)
+#define LAUNCH_ATTEND_(NV, NK, EX, HG)                                                                               \
+    hipLaunchKernelGGL((latent_attend_mfma_kernel<NV, NK, EX, HG>), dim3(nparts, (heads + 16 * HG - 1) / (16 * HG), T_), \
+                       dim3(kNT * HG), 0, s, q_, r_, q_stride, q_head, c_, row, block_tables, bt_stride, bt_row,     \
+                       positions, T_, heads, rank, rot_dim, scale * kLog2e, window, part_min, nparts, o_, ws_o, ws_ml)
+#define LAUNCH_ATTEND(NV, NK, EX)                    \
+    if (heads > 16) LAUNCH_ATTEND_(NV, NK, EX, 2);   \
+    else LAUNCH_ATTEND_(NV, NK, EX, 1)
 
 extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_stride, int64_t q_head,
                                    const void* cache, int32_t row, const int32_t* block_tables, int64_t bt_stride,
@@ -701,11 +707,17 @@ extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_
     float* ws_o = reinterpret_cast<float*>(workspace);
     float* ws_ml = ws_o ? ws_o + (size_t)T_ * heads * nparts * (((rank + 15) / 16) * 16) : nullptr;
     const int nk = row / 32, nv = (rank + 15) / 16;
-    if (nv <= 4 && nk <= 4) LAUNCH_ATTEND(4, 4, false);
-    else if (nv <= 8 && nk <= 6) LAUNCH_ATTEND(8, 6, false);
-    else if (nv <= 16 && nk <= 10) LAUNCH_ATTEND(16, 10, false);
-    else if (rank == 512 && nk == 18) LAUNCH_ATTEND(32, 18, true);
-    else LAUNCH_ATTEND(32, 20, false);
+    if (nv <= 4 && nk <= 4) {
+        LAUNCH_ATTEND(4, 4, false);
+    } else if (nv <= 8 && nk <= 6) {
+        LAUNCH_ATTEND(8, 6, false);
+    } else if (nv <= 16 && nk <= 10) {
+        LAUNCH_ATTEND(16, 10, false);
+    } else if (rank == 512 && nk == 18) {
+        LAUNCH_ATTEND(32, 18, true);
+    } else {
+        LAUNCH_ATTEND(32, 20, false);
+    }
     int rc = check_launch("latent_attend_mfma_kernel");
     if (rc != SKYRL_OK || nparts == 1) return rc;
     hipLaunchKernelGGL(latent_merge_kernel, dim3(heads, T_), dim3(kWave * 2), 0, s, ws_o, ws_ml, positions, T_, heads, rank,

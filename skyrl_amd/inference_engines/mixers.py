@@ -171,7 +171,7 @@ class LatentAttention:
     # ---- decode split
     def nparts(self, tokens: int, max_ctx: int) -> int:
         ctx = min(max_ctx, self.window + BLOCK_SIZE) if self.window else max_ctx
-        return kernels.choose_nparts(tokens, (self.heads + 15) // 16, ctx, target_waves=ATTEND_WORKGROUPS)
+        return kernels.choose_nparts(tokens, (self.heads + 31) // 32, ctx, target_waves=ATTEND_WORKGROUPS)
 
     def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
         from .. import _ffi
