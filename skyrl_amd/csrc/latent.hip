@@ -153,9 +153,11 @@ __device__ __forceinline__ s16x4 lds_read_tr(const uint16_t* p) {
 }
 
 // ---- decode form, MFMA ------------------------------------------------------------------------
-// grid (nparts, ceil(heads / (16 HG)), tokens), four waves per group of 16 heads. A tile is four pages, one
-// per wave of a group for the scores; for the values each wave takes a quarter of the rank over all 64
-// keys. With HG = 2 two head groups share the tile in LDS and its HBM reads. NV: 16-wide tiles of the rank,
+// grid (nparts, ceil(heads / (16 HG)), tokens), four waves per group of 16 heads. A tile is four pages, staged
+// through registers into LDS in whole 1 KB pieces (a page is contiguous; row-by-row operand loads from
+// HBM ran at half the rate), one page per wave, the next tile's loads in flight. Each wave scores one
+// page for its head group; for the values it takes a quarter of the rank over all 64 keys. With HG = 2
+// two head groups share the tile and each stages half of it. NV: 16-wide tiles of the rank,
 // NK: 32-wide steps of the cache row; EXACT when both equal the shape's own.
 template <int NV, int NK, bool EXACT, int HG>
 __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))) void latent_attend_mfma_kernel(
@@ -164,10 +166,10 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
     const int32_t* __restrict__ bt_row, const int64_t* __restrict__ positions, int ntok, int heads, int rank, int rot,
     float scale_log2, int window, int part_min, int nparts, uint16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml) {
-    constexpr int LDR = NV * 16 + 16;  // padded LDS row: sixteen rows' 32-byte pieces fall into distinct banks
-    constexpr int LDS_ = 64 + 4, NW = NV / 4, LDQ = NK * 32 + 8;
-    constexpr int NT = kNT * HG, kTile = 64 * LDR > 16 * HG * LDQ ? 64 * LDR : 16 * HG * LDQ;
-    __shared__ __attribute__((aligned(16))) uint16_t s_c[kTile];  // first the query, then the latent tile
+    constexpr int LDR = NK * 32 + 8;  // padded LDS row
+    constexpr int LDS_ = 64 + 4, NW = NV / 4, NT = kNT * HG;
+    constexpr int NL = (NK + HG - 1) / HG;  // 16-byte pieces of its page per lane
+    __shared__ __attribute__((aligned(16))) uint16_t s_c[64 * LDR];  // first the query, then the tile
     __shared__ __attribute__((aligned(16))) float s_scores[HG * 16 * LDS_];  // scores [head][key of the tile]
     const int t = blockIdx.z;
     const int pos = (int)positions[t];
@@ -186,21 +188,27 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
     const int first = sp.p0 + part * sp.per;
     const int np = min(sp.per, sp.np - part * sp.per);
     const int32_t* bt = tables + (int64_t)bt_row[t] * bt_stride + first;
-    const uint16_t* kbase = cache + (int64_t)c * row + 8 * g;
-    s16x8 kf[NK];  // this wave's page of the current tile, then of the next
     // Pages come in windows of 64, whose block ids a wave holds by lane (no table load ahead of a page's).
     // Loads are unconditional, the last page again past the end: a branch around them would turn every
     // wait into one for all loads in flight.
+    const int rc = EXACT ? NK * 4 : nk * 4;  // pieces per row
+    auto piece = [&](int k) { return min(lane + 64 * (hg + HG * k), 16 * rc - 1); };
+    int lds_at[NL];
+#pragma unroll
+    for (int k = 0; k < NL; ++k) {
+        const int e = piece(k), r = e / rc;
+        lds_at[k] = (16 * wave + r) * LDR + (e - r * rc) * 8;
+    }
+    s16x8 st_[NL];
     int tbl = 0, npw = 0;
     auto window_at = [&](int w0) {
         npw = min(64, np - w0);
         tbl = bt[w0 + min(lane, npw - 1)];
     };
     auto load_page = [&](int j) {
-        const uint16_t* p = kbase + (int64_t)__builtin_amdgcn_readlane(tbl, min(j, npw - 1)) * kBS * row;
+        const uint16_t* p = cache + (int64_t)__builtin_amdgcn_readlane(tbl, min(j, npw - 1)) * kBS * row;
 #pragma unroll
-        for (int s = 0; s < NK; ++s)
-            if (EXACT || s < nk) kf[s] = *reinterpret_cast<const s16x8*>(p + 32 * s);
+        for (int k = 0; k < NL; ++k) st_[k] = *reinterpret_cast<const s16x8*>(p + piece(k) * 8);
     };
     window_at(0);
     load_page(wave);
@@ -225,12 +233,12 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
                 }
             }
         }
-        *reinterpret_cast<s16x8*>(&s_c[hh * LDQ + d]) = f;
+        *reinterpret_cast<s16x8*>(&s_c[hh * LDR + d]) = f;
     }
     __syncthreads();
     s16x8 qf[NK];
 #pragma unroll
-    for (int s = 0; s < NK; ++s) qf[s] = *reinterpret_cast<const s16x8*>(&s_c[(16 * hg + c) * LDQ + 32 * s + 8 * g]);
+    for (int s = 0; s < NK; ++s) qf[s] = *reinterpret_cast<const s16x8*>(&s_c[(16 * hg + c) * LDR + 32 * s + 8 * g]);
 
     f32x4 o[NW];
 #pragma unroll
@@ -240,24 +248,26 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
         const int tb = (first + w0 + j0 + wave) * kBS;  // this wave's page
         const bool edge = j0 + wave >= npw || tb < lo || tb + kBS - 1 > pos;
         if (edge) {  // a masked slot may hold anything: 0 * NaN must not reach the sums
-            const bool ok = j0 + wave < npw && tb + c >= lo && tb + c <= pos;
 #pragma unroll
-            for (int s = 0; s < NK; ++s)
-                if (!ok) kf[s] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
-        }
-        f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = sa;
-#pragma unroll
-        for (int s = 0; s < NK; ++s) {
-            if (EXACT || s < nk) {
-                if (s & 1) sb = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sb, 0, 0, 0);
-                else sa = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sa, 0, 0, 0);
+            for (int k = 0; k < NL; ++k) {
+                const int tok = tb + piece(k) / rc;
+                if (!(j0 + wave < npw && tok >= lo && tok <= pos)) st_[k] = s16x8{0, 0, 0, 0, 0, 0, 0, 0};
             }
         }
         __syncthreads();  // the query operands, or the previous tile, are consumed
 #pragma unroll
-        for (int s = 0; s < NK; ++s)
-            if ((EXACT || s < nk) && 32 * s < NV * 16 && s % HG == hg)  // the groups share the copy
-                *reinterpret_cast<s16x8*>(&s_c[(16 * wave + c) * LDR + 32 * s + 8 * g]) = kf[s];
+        for (int k = 0; k < NL; ++k) *reinterpret_cast<s16x8*>(&s_c[lds_at[k]]) = st_[k];
+        load_page(j0 + 4 + wave);
+        __syncthreads();
+        f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = sa;
+#pragma unroll
+        for (int s = 0; s < NK; ++s) {
+            if (EXACT || s < nk) {
+                const s16x8 kf = *reinterpret_cast<const s16x8*>(&s_c[(16 * wave + c) * LDR + 32 * s + 8 * g]);
+                if (s & 1) sb = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], sb, 0, 0, 0);
+                else sa = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], sa, 0, 0, 0);
+            }
+        }
         f32x4 sv = (sa + sb) * scale_log2;  // token tb + 4 g + i, head c
         if (edge) {
 #pragma unroll
@@ -267,7 +277,6 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
             }
         }
         *reinterpret_cast<f32x4*>(&s_s[c * LDS_ + 16 * wave + 4 * g]) = sv;
-        load_page(j0 + 4 + wave);
         __syncthreads();
         // every wave: weights of all 64 keys, the lane's own 16 in the order of the MFMA operand
         f32x4 x[4];
