@@ -130,8 +130,7 @@ __global__ __launch_bounds__(kNT) void latent_attend_plain_kernel(
     }
 }
 
-// Pages [p0, p0 + np) of a token's context cut into shares of `per` pages, a multiple of the workgroup's
-// four; parts = number of shares.
+// Pages [p0, p0 + np) of a token's context cut into shares of `per` pages; parts = number of shares.
 struct PageSplit {
     int p0, per, parts, np;
 };
@@ -139,8 +138,7 @@ __device__ __forceinline__ PageSplit page_split(int lo, int pos, int part_min, i
     PageSplit s;
     s.p0 = lo / kBS;
     s.np = pos / kBS - s.p0 + 1;
-    const int per = max((s.np + nparts - 1) / nparts, part_min / kBS);
-    s.per = (per + 3) / 4 * 4;
+    s.per = max((s.np + nparts - 1) / nparts, part_min / kBS);
     s.parts = (s.np + s.per - 1) / s.per;
     return s;
 }
