@@ -24,7 +24,7 @@ def hybrid_config(z):
            "mixer": {"heads": z["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
                      "mask": {"size": z["window"]},
                      "rot": {"base": 10000.0, "dims": 64,
-                             "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+                             "scaling": {"factor": 16.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
     dlt = {"type": "delta", "mlp": {"kind": "dense", "ff": z["ff"]},
            "mixer": {"heads": z["delta_heads"], "kv_heads": z["delta_kv"], "dim": 128, "vdim": 128, "conv": 4}}
     return {"architecture": "Dovidra", "layers": [lat, dlt, lat, dlt], "loop": {"start": 1, "stop": 3, "times": 2},

@@ -943,7 +943,7 @@ __global__ __launch_bounds__(NT, W) void policy_train_split_kernel(
     const float inv_t = HAS_T ? 1.f / temp : 1.f;
     // dL/dz = glp (onehot - p) - gent p (logp + H) with logp = z - L and p = 2^((z - L) log2e):
     //   gg = p (ca z + cb), ca = -gent, cb = -glp - gent (H - L); the label's element adds glp.
-    // Two packed fma, one exp2 and one multiply per element (the per-element label compare and the
+    // Two fma, one exp2 and one multiply per element (the per-element label compare and the
     // separate subtract / scale are gone): the sweep is less VALU per byte, which matters when the
     // chip's clock drops under sustained HBM load (policy_train)
     const float cy = -L * kLog2e;
@@ -958,7 +958,7 @@ __global__ __launch_bounds__(NT, W) void policy_train_split_kernel(
             typedef float f2 __attribute__((ext_vector_type(2)));
             const f2 l2 = {kLog2e, kLog2e}, c2 = {cy, cy}, a2 = {ca, ca}, b2 = {cb, cb};
 #pragma unroll
-            for (int j = 0; j < 8; j += 2) {  // packed fma pairs (v_pk_fma_f32)
+            for (int j = 0; j < 8; j += 2) {  // in pairs
                 const f2 z = {tval(x[j]), tval(x[j + 1])};
                 const f2 y = __builtin_elementwise_fma(z, l2, c2);
                 const f2 t = __builtin_elementwise_fma(a2, z, b2);

@@ -92,7 +92,7 @@ def paged_latents(g, lens, rank, rot, dtype, spare=3):
 
 
 ATTEND = [  # heads, rank, rot, window
-    (3, 40, 12, 37), (16, 64, 16, 96), (5, 33, 6, 1), (17, 128, 32, None), (4, 256, 64, 65), (16, 512, 64, 130),
+    (3, 40, 12, 37), (16, 80, 24, 72), (5, 33, 6, 1), (17, 128, 32, None), (4, 256, 64, 65), (16, 512, 64, 130),
     (20, 512, 128, None), (2, 24, 2, 16), (2, 700, 20, 33)]
 
 
@@ -158,7 +158,7 @@ def test_latent_write(heads, dim, rot, rank, dtype):
 
 PREFILL = [  # heads, dim, rot, vdim, rank, window, [(start, tokens)]
     (3, 20, 12, 28, 40, 37, [(0, 70), (5, 33)]),
-    (4, 32, 16, 80, 64, 96, [(0, 130), (300, 64), (95, 40)]),
+    (6, 40, 24, 72, 48, 80, [(0, 130), (300, 64), (79, 40)]),
     (2, 128, 64, 128, 512, 100, [(0, 300), (1000, 129)]),
     (2, 64, 64, 64, 96, None, [(17, 200)]),
     (1, 130, 62, 140, 50, 1, [(3, 35)]),
@@ -210,7 +210,7 @@ def test_latent_prefill(heads, dim, rot, vdim, rank, window, segs):
 
 # ---------------------------------------------------------------- gated delta rule
 DELTA = [  # heads, kv_heads, dim, vdim, taps
-    (4, 2, 24, 36, 3), (2, 1, 64, 32, 4), (2, 2, 128, 128, 4), (3, 3, 18, 10, 1), (2, 1, 200, 130, 9), (1, 1, 16, 200, 2),
+    (4, 2, 24, 36, 3), (3, 1, 64, 48, 3), (2, 2, 128, 128, 4), (3, 3, 18, 10, 1), (2, 1, 200, 130, 9), (1, 1, 16, 200, 2),
     (2, 2, 5, 3, 8)]
 
 
@@ -429,6 +429,25 @@ def test_graph_replays_match_eager_steps():
             rows.append(s.step([{"id": "x", "tokens": toks[i:i + 1], "want": [0]}]))
         outs.append(torch.cat(rows[1:]))
     model_close(outs[0], outs[1].double(), torch.bfloat16)
+
+
+@pytest.mark.parametrize("rows", [3, 40])
+def test_graph_replays_at_larger_layers(rows):
+    """The same with library products of a real model's size in the captured step: every replay against
+    the eager step on its own cache and state."""
+    cfg = config([latent(heads=8, dim=128, rot_dim=64, vdim=128, kv_rank=512, window=40),
+                  delta(heads=8, kv_heads=4, dim=128, vdim=128, conv=4)], width=1024, ff=2048, vocab=4096)
+    m, _ = build(cfg, torch.bfloat16)
+    prompts = [tokens_of(cfg, 10 + i % 7, i) for i in range(rows)]
+    ids = [f"r{i}" for i in range(rows)]
+    sessions = [TraceSession(m, 64 * rows, max_live=rows, use_graphs=g) for g in (True, False)]
+    for s in sessions:
+        s.step([{"id": k, "tokens": p, "want": []} for k, p in zip(ids, prompts)])
+    for t in range(6):
+        step = [{"id": k, "tokens": [(31 * t + 7 * i) % cfg["vocab"]], "want": [0]} for i, k in enumerate(ids)]
+        a, b = (s.step(step) for s in sessions)
+        model_close(a, b.double(), torch.bfloat16)
+        torch.cuda.synchronize()
 
 
 def test_steps_without_wanted_logits_keep_their_inputs():
