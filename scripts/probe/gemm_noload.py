@@ -47,7 +47,7 @@ def run():
     print(json.dumps({"lib": "product"}), flush=True)
     lsb.gemm_sweep(shapes)
     for name in VARIANTS:
-        _ffi._lib = None
+        _ffi._libs.clear()
         _ffi.LIB_PATH = os.path.join(HERE, f"libgemm_{name}.so")
         print(json.dumps({"lib": name}), flush=True)
         lsb.gemm_sweep(shapes)
