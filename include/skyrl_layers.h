@@ -17,21 +17,35 @@
 extern "C" {
 #endif
 
-/* ---- norms, activations, logits -------------------------------------------------------------
+/* ---- embedding, norms, activations, convolution state, logits ---------------------------------
+ *   skyrl_embed     out f32 [n, H] = scale * table T [vocab, H] at tokens i64 [n].
  *   skyrl_add_norm  hidden f32 [n, H] += delta T [n, H] (may be NULL) and += step T [H] (may be
- *                   NULL: one vector for every row); out T [n, H] = norm(hidden) * weight T [H].
+ *                   NULL: one vector for every row); out T [n, H] = norm(hidden) * (w_base + weight T [H]):
+ *                   w_base 0 for a weight stored as it is, 1 for one stored as its distance from 1.
  *                   kind 0: layer norm without bias (mean taken off, variance = mean squared
  *                   deviation), 1: RMS norm; eps inside the root. H <= 8192.
- *   skyrl_gate_mul  out T [n, I] = act(gate) * up of gate_up T [n, 2I] (gate | up);
- *                   act 0: silu, 1: gelu in its tanh form. The product is f32, rounded once.
+ *   skyrl_gate_mul  out T [n, I] (row stride out_stride) from gate | up of gate_up T [n, 2I] (row stride
+ *                   gu_stride): act 0: silu(gate) * up, 1: gelu(gate) * up in gelu's tanh form, 2: with
+ *                   g = min(gate, limit) and u = up clamped to +-limit, g * sigmoid(alpha g) * (u + 1).
+ *                   f32 throughout, rounded once. alpha and limit are of act 2.
+ *   skyrl_conv_save stores the last `taps` rows of every sequence's columns [0, channels) of x T [T, stride]
+ *                   in ring T [rows, taps, channels], the row of position p at p % taps. Sequences: tokens
+ *                   [cu[s], cu[s+1]) of row rows[s] (< 0: skipped), positions consecutive from positions[cu[s]].
  *   skyrl_softcap   out f32 = cap * tanh(x / cap) over count elements of x T (cap <= 0: a copy). */
 #define SKYRL_NORM_LAYER 0
 #define SKYRL_NORM_RMS 1
 #define SKYRL_ACT_SILU 0
 #define SKYRL_ACT_GELU_TANH 1
-int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, int32_t n, int32_t H,
-                   float eps, int32_t kind, void* out, int32_t dtype, void* stream);
-int skyrl_gate_mul(const void* gate_up, int64_t n, int32_t I, int32_t act, void* out, int32_t dtype, void* stream);
+#define SKYRL_ACT_CLAMPED 2
+int skyrl_embed(const int64_t* tokens, const void* table, int64_t n, int32_t H, float scale, float* out, int32_t dtype,
+                void* stream);
+int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, float w_base, int32_t n,
+                   int32_t H, float eps, int32_t kind, void* out, int32_t dtype, void* stream);
+int skyrl_gate_mul(const void* gate_up, int64_t gu_stride, int64_t n, int32_t I, int32_t act, float alpha, float limit,
+                   void* out, int64_t out_stride, int32_t dtype, void* stream);
+int skyrl_conv_save(const void* x, int64_t stride, int32_t channels, int32_t taps, const int32_t* cu,
+                    const int32_t* rows, const int64_t* positions, int32_t nseq, void* ring, int32_t dtype,
+                    void* stream);
 int skyrl_softcap(const void* x, float* out, int64_t count, float cap, int32_t dtype, void* stream);
 
 /* ---- latent attention over a paged latent cache ----------------------------------------------
@@ -96,8 +110,7 @@ int skyrl_latent_prefill(const void* q, int64_t q_stride, const void* k_nope, in
  * consecutive from positions[cu[s]].
  *   skyrl_delta_scan       token by token, the state in registers: decode steps and short portions.
  *                          save_conv 1 also stores the convolution inputs and needs every sequence to
- *                          have one token; otherwise skyrl_delta_save follows.
- *   skyrl_delta_save       stores the last inputs of every sequence.
+ *                          have one token; otherwise skyrl_conv_save of the channels follows.
  *   Prompt form, for portions of many tokens, in chunks of 64: chunk i32 [nchunks, 4] (first token,
  *   tokens <= 64, sequence, 0), chunks of one sequence consecutive and in order, cut from its first
  *   token on; d16, v16 = dim, vdim up to a multiple of 16. dim <= 256.
@@ -109,7 +122,7 @@ int skyrl_latent_prefill(const void* q, int64_t q_stride, const void* k_nope, in
  *                          blocks below and on the diagonal), G f32
  *                          [nchunks, heads, 64] (summed log decays).
  *   skyrl_delta_chain      3: sequential over the chunks seq_chunks[i] .. seq_chunks[i + 1] - 1 of sequence
- *                          seq0 + i: reads and writes S, o f32 [T, heads, vdim]. skyrl_delta_save stores
+ *                          seq0 + i: reads and writes S, o f32 [T, heads, vdim]. skyrl_conv_save stores
  *                          the convolution inputs.
  *   skyrl_delta_out        4: out T of tokens [first, T) from o. */
 typedef struct skyrl_delta_shape {
@@ -120,9 +133,6 @@ int skyrl_delta_scan(const skyrl_delta_shape* shape, const void* proj, int64_t p
                      const float* a_log, const float* dt_bias, const void* norm_w, const int32_t* cu,
                      const int32_t* rows, const int64_t* positions, int32_t nseq, float* state, void* conv_state,
                      int32_t save_conv, void* out, int64_t out_stride, int32_t dtype, void* stream);
-int skyrl_delta_save(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride, const int32_t* cu,
-                     const int32_t* rows, const int64_t* positions, int32_t nseq, void* conv_state, int32_t dtype,
-                     void* stream);
 int skyrl_delta_conv(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride, const void* conv_w,
                      const float* a_log, const float* dt_bias, const int32_t* chunk, int32_t nchunks,
                      const int32_t* cu, const int32_t* rows, const int64_t* positions, const void* conv_state,
@@ -137,6 +147,59 @@ int skyrl_delta_chain(const skyrl_delta_shape* shape, const int32_t* chunk, cons
 int skyrl_delta_out(const skyrl_delta_shape* shape, const float* o, const void* proj, int64_t proj_stride,
                     const void* norm_w, int32_t first, int32_t T, void* out, int64_t out_stride, int32_t dtype,
                     void* stream);
+
+/* ---- differential attention over a paged key / value cache -------------------------------------
+ * A query head has two maps, each an attention of its own over the same values: a_m = softmax(scale
+ * q_m . k_m) v, o = a_1 - lambda a_2, out = o / rms(o) (1 - diff) sigmoid(gate), the root mean square (eps
+ * inside) over the head's vdim values. Query head h reads key / value head h / (heads / kv_heads).
+ * proj T [T, proj_stride]: q (heads x 2 x dim) | k (kv_heads x 2 x dim) | v (kv_heads x vdim), with k and v
+ * only if `kv` (else the keys and values are another layer's, in its cache). Each channel passes a causal
+ * convolution over time (conv_t f32 [taps, channels], last tap on the current token; state as under
+ * skyrl_conv_save), then the first rot_dims of every map of q and k are rotated (interleaved pairs;
+ * cos_sin f32 [max_pos, rot_dims] = cos | sin halves, amplitude included).
+ * Padded sizes: dp = dim up to a multiple of 16, vp = vdim likewise. Queries T [T, heads, 2 dp], map m
+ * from m dp on, zeros between. Cache: keys T [num_blocks, kv_heads, 16, 2 dp], values transposed T
+ * [num_blocks, kv_heads, vp, 16]; padding must hold zeros. slot = block * 16 + offset. Token t of a
+ * step belongs to row bt_row[t] of block_tables, which is also its sequence (cu, rows), and attends to
+ * positions [0, positions[t]].
+ *   skyrl_diff_write      tokens [first, first + count): convolution, rotation, queries out, keys and values
+ *                         into the cache at slots[t] (< 0: no write). save_conv 1 also stores the
+ *                         convolution inputs and needs every sequence to have one token; otherwise
+ *                         skyrl_conv_save follows. Padding is not written.
+ *   skyrl_diff_write_runs the same (bf16, dim and vdim multiples of 8, taps <= 8) by runs i32 [nruns, 2]: first
+ *                         token, count <= 8 of one sequence, whose slots lie in one half of a block.
+ *   skyrl_diff_attend     one query row per token; gate T points at head 0 of token 0 (row stride
+ *                         gate_stride); lambda f32 [1]; out T (row stride out_stride), head h at h * vdim.
+ *                         nparts waves share a token's keys (MFMA form, bf16), each at least part_min >= 16
+ *                         keys, a multiple of 16; nparts > 1 needs skyrl_diff_attend_workspace_bytes. f32, and
+ *                         shapes outside the MFMA form (skyrl_diff_mfma == 0), take a plain kernel and
+ *                         ignore nparts.
+ *   skyrl_diff_prefill    prompt form (bf16, skyrl_diff_mfma != 0): one workgroup per (tile, head); tiles i32
+ *                         [ntiles, 4]: first token, token count (<= 128), position of the first token, row
+ *                         of block_tables. */
+typedef struct skyrl_diff_shape {
+    int32_t heads, kv_heads, dim, vdim, rot_dims, taps, kv;
+    float scale, diff, eps;
+} skyrl_diff_shape;
+int skyrl_diff_write(const skyrl_diff_shape* shape, const void* proj, int64_t proj_stride, const float* conv_t,
+                     const int32_t* cu, const int32_t* rows, const int32_t* bt_row, const int64_t* positions,
+                     const int64_t* slots, const float* cos_sin, void* ring, int32_t save_conv, int32_t first,
+                     int32_t count, void* q, void* k_cache, void* v_cache, int32_t dtype, void* stream);
+int skyrl_diff_write_runs(const skyrl_diff_shape* shape, const void* proj, int64_t proj_stride, const float* conv_t,
+                          const int32_t* cu, const int32_t* rows, const int32_t* bt_row, const int64_t* positions,
+                          const int64_t* slots, const float* cos_sin, const void* ring, const int32_t* runs,
+                          int32_t nruns, void* q, void* k_cache, void* v_cache, void* stream);
+int skyrl_diff_mfma(const skyrl_diff_shape* shape, int32_t dtype);
+size_t skyrl_diff_attend_workspace_bytes(const skyrl_diff_shape* shape, int32_t T, int32_t nparts);
+int skyrl_diff_attend(const skyrl_diff_shape* shape, const void* q, const void* gate, int64_t gate_stride,
+                      const void* k_cache, const void* v_cache, const int32_t* block_tables, int64_t bt_stride,
+                      const int32_t* bt_row, const int64_t* positions, int32_t T, const float* lambda,
+                      int32_t part_min, int32_t nparts, void* out, int64_t out_stride, void* workspace, int32_t dtype,
+                      void* stream);
+int skyrl_diff_prefill(const skyrl_diff_shape* shape, const void* q, const void* gate, int64_t gate_stride,
+                       const void* k_cache, const void* v_cache, const int32_t* block_tables, int64_t bt_stride,
+                       const int32_t* tiles, int32_t ntiles, const float* lambda, void* out, int64_t out_stride,
+                       void* stream);
 
 #ifdef __cplusplus
 }

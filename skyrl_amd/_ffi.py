@@ -230,11 +230,21 @@ class DeltaShape(ctypes.Structure):
     ]
 
 
+class DiffShape(ctypes.Structure):
+    """Mirror of ``skyrl_diff_shape`` (include/skyrl_layers.h)."""
+
+    _fields_ = [(n, ctypes.c_int32) for n in ("heads", "kv_heads", "dim", "vdim", "rot_dims", "taps", "kv")] + [
+        (n, ctypes.c_float) for n in ("scale", "diff", "eps")]
+
+
 # the exported surface of include/skyrl_layers.h, in a library of its own (libskyrl_layers.so)
 _DS = ctypes.POINTER(DeltaShape)
+_FS = ctypes.POINTER(DiffShape)
 LAYERS_SIGNATURES = {
-    "skyrl_add_norm": (_INT, [_P, _P, _P, _P, _I32, _I32, _F, _I32, _P, _I32, _P]),
-    "skyrl_gate_mul": (_INT, [_P, _I64, _I32, _I32, _P, _I32, _P]),
+    "skyrl_embed": (_INT, [_P, _P, _I64, _I32, _F, _P, _I32, _P]),
+    "skyrl_add_norm": (_INT, [_P, _P, _P, _P, _F, _I32, _I32, _F, _I32, _P, _I32, _P]),
+    "skyrl_gate_mul": (_INT, [_P, _I64, _I64, _I32, _I32, _F, _F, _P, _I64, _I32, _P]),
+    "skyrl_conv_save": (_INT, [_P, _I64, _I32, _I32, _P, _P, _P, _I32, _P, _I32, _P]),
     "skyrl_softcap": (_INT, [_P, _P, _I64, _F, _I32, _P]),
     "skyrl_latent_write": (_INT, [_P, _I64, _I32, _I32, _I32, _I32, _I32, _P, _F, _P, _P, _P, _P, _I32, _I32, _P]),
     "skyrl_latent_attend_mfma": (_INT, [_I32, _I32, _I32, _I32]),
@@ -245,11 +255,17 @@ LAYERS_SIGNATURES = {
     "skyrl_latent_prefill": (_INT, [_P, _I64, _P, _I64, _P, _P, _I64, _P, _I32, _I32, _I32, _I32, _I32, _F, _I32, _P,
                                     _I64, _P]),
     "skyrl_delta_scan": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I32, _P, _I64, _I32, _P]),
-    "skyrl_delta_save": (_INT, [_DS, _P, _I64, _P, _P, _P, _I32, _P, _I32, _P]),
     "skyrl_delta_conv": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P]),
     "skyrl_delta_chunk": (_INT, [_DS, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P]),
     "skyrl_delta_chain": (_INT, [_DS, _P, _P, _I32, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P]),
     "skyrl_delta_out": (_INT, [_DS, _P, _P, _I64, _P, _I32, _I32, _P, _I64, _I32, _P]),
+    "skyrl_diff_write": (_INT, [_FS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _P, _P, _P, _I32, _P]),
+    "skyrl_diff_write_runs": (_INT, [_FS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _P]),
+    "skyrl_diff_mfma": (_INT, [_FS, _I32]),
+    "skyrl_diff_attend_workspace_bytes": (_SZ, [_FS, _I32, _I32]),
+    "skyrl_diff_attend": (_INT, [_FS, _P, _P, _I64, _P, _P, _P, _I64, _P, _P, _I32, _P, _I32, _I32, _P, _I64, _P, _I32,
+                                 _P]),
+    "skyrl_diff_prefill": (_INT, [_FS, _P, _P, _I64, _P, _P, _P, _I64, _P, _I32, _P, _P, _I64, _P]),
 }
 
 # entry points with a per-call variant form (name + "_ex": the same arguments, then the variant)

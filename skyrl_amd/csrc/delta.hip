@@ -17,7 +17,7 @@
 //   U = U0 - W S,   O = diag(e^G) Q S + P U,   S <- e^{G_n} S + K^T diag(e^{G_n - G}) U.
 // Everything is f32, the products on the f32 matrix instructions (v_mfma_f32_16x16x4_f32): a lane's
 // four consecutive k values of a 16-step feed four instructions, the same permutation of k on both sides.
-#include "elem.h"
+#include "conv.h"
 
 namespace skyrl {
 namespace {
@@ -25,7 +25,6 @@ namespace {
 constexpr int kNT = 256;
 constexpr int kMaxTaps = 64;
 constexpr int kC = 64;       // tokens per chunk
-constexpr int kWindow = 8;   // convolution taps held in registers by the prompt form
 
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
@@ -38,34 +37,11 @@ struct Dims {
     __host__ __device__ int channels() const { return 2 * K * D + H * V; }
 };
 
-// silu(causal convolution) of channel ch at token t of a sequence whose first token is t0 at position p0;
-// inputs before t0 come from the stored ones (the input of position p at p % taps; r = pos % taps). Up to
-// kWindow taps every load is in flight at once.
 template <typename T>
 __device__ __forceinline__ float conv_silu(const T* __restrict__ proj, int64_t stride, const T* __restrict__ w,
                                            const T* __restrict__ ring, int channels, int taps, int ch, int t, int t0,
                                            int pos, int r) {
-    float y = 0.f;
-    auto input = [&](int back) -> float {
-        if (t - back >= t0) return ld(proj + (int64_t)(t - back) * stride + ch);
-        const int slot = r - back < 0 ? r - back + taps : r - back;
-        return ld(ring + (int64_t)slot * channels + ch);
-    };
-    if (taps <= kWindow) {
-        float x[kWindow], f[kWindow];
-#pragma unroll
-        for (int back = 0; back < kWindow; ++back) {
-            const bool on = back < taps && back <= pos;
-            x[back] = on ? input(back) : 0.f;
-            f[back] = on ? ld(w + (int64_t)ch * taps + taps - 1 - back) : 0.f;
-        }
-#pragma unroll
-        for (int back = 0; back < kWindow; ++back) y += x[back] * f[back];
-    } else {
-        for (int back = 0; back < taps && back <= pos; ++back)
-            y += input(back) * ld(w + (int64_t)ch * taps + taps - 1 - back);
-    }
-    return siluf_(y);
+    return siluf_(short_conv(proj, stride, w, ring, channels, taps, ch, t, t0, pos, r));
 }
 
 // NT threads, RPT state rows per thread: thread (cg, rg) holds columns 4 cg .. 4 cg + 3 of rows rg, rg + RG, ...
@@ -222,22 +198,6 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void de
     }
 }
 
-template <typename T>
-__global__ __launch_bounds__(kNT) void delta_save_kernel(Dims d, const T* __restrict__ proj, int64_t stride,
-                                                         const int32_t* __restrict__ cu,
-                                                         const int32_t* __restrict__ rows,
-                                                         const int64_t* __restrict__ positions,
-                                                         T* __restrict__ conv_state) {
-    const int s = blockIdx.y, row = rows[s];
-    if (row < 0) return;
-    const int t0 = cu[s], t1 = cu[s + 1];
-    const int ch = blockIdx.x * kNT + threadIdx.x, n = d.channels();
-    if (ch >= n || t0 >= t1) return;
-    const int64_t pos0 = positions[t0];
-    for (int t = max(t0, t1 - d.taps); t < t1; ++t)
-        conv_state[((int64_t)row * d.taps + (pos0 + t - t0) % d.taps) * n + ch] = proj[(int64_t)t * stride + ch];
-}
-
 // ---- prompt form ------------------------------------------------------------------------------
 struct SeqRef {
     const int32_t* chunk;  // [nchunks, 4]: first token, tokens, sequence, 0
@@ -280,36 +240,36 @@ __global__ __launch_bounds__(kNT) void delta_conv_kernel(Dims d, SeqRef sq, cons
         return ld(ring + (int64_t)((pos0 + i) % d.taps) * ch_all + ch);
     };
     const int nch = keys ? 2 * D : min(kNT, d.H * d.V - ((int)blockIdx.y - d.K) * kNT);
-    const bool held = d.taps <= kWindow, carry = nch <= kNT;  // carry: one channel per thread, inputs stay in registers
-    constexpr int kSub = 16, kBack = kWindow - 1;
+    const bool held = d.taps <= kConvWindow, carry = nch <= kNT;  // carry: one channel per thread, inputs stay in registers
+    constexpr int kSub = 16, kBack = kConvWindow - 1;
     float x[kBack + kSub];
     for (int i0 = 0; i0 < n; i0 += kSub) {
         const int m = min(kSub, n - i0);
         for (int e = tid; e < nch; e += kNT) {
             const int ch = !keys ? 2 * d.K * D + ((int)blockIdx.y - d.K) * kNT + e
                                  : e < D ? kh * D + e : (d.K + kh) * D + (e - D);
-            float w[kWindow];
+            float w[kConvWindow];
             if (held) {
                 if (carry && i0 > 0) {
 #pragma unroll
                     for (int j = 0; j < kBack; ++j) x[j] = x[j + kSub];
                 } else {
 #pragma unroll
-                    for (int j = 0; j < kBack; ++j) x[j] = j >= kWindow - d.taps ? input(ch, i0 - kBack + j) : 0.f;
+                    for (int j = 0; j < kBack; ++j) x[j] = j >= kConvWindow - d.taps ? input(ch, i0 - kBack + j) : 0.f;
                 }
 #pragma unroll
                 for (int j = 0; j < kSub; ++j)
                     x[kBack + j] = ld(proj + (int64_t)(t0 + min(i0 + j, n - 1)) * stride + ch);
 #pragma unroll
-                for (int j = 0; j < kWindow; ++j)
-                    w[j] = j >= kWindow - d.taps ? ld(conv_w + (int64_t)ch * d.taps + j - (kWindow - d.taps)) : 0.f;
+                for (int j = 0; j < kConvWindow; ++j)
+                    w[j] = j >= kConvWindow - d.taps ? ld(conv_w + (int64_t)ch * d.taps + j - (kConvWindow - d.taps)) : 0.f;
             }
 #pragma unroll
             for (int i = 0; i < kSub; ++i) {
                 float y = 0.f;
                 if (held) {
 #pragma unroll
-                    for (int j = 0; j < kWindow; ++j) y += x[i + j] * w[j];
+                    for (int j = 0; j < kConvWindow; ++j) y += x[i + j] * w[j];
                 } else if (i < m) {
                     for (int j = 0; j < d.taps; ++j)
                         y += input(ch, i0 + i - (d.taps - 1) + j) * ld(conv_w + (int64_t)ch * d.taps + j);
@@ -751,24 +711,6 @@ extern "C" int skyrl_delta_scan(const skyrl_delta_shape* shape, const void* proj
         else LAUNCH_SCAN(1024, 16);
     })
     return check_launch("delta_scan_kernel");
-}
-
-extern "C" int skyrl_delta_save(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride,
-                                const int32_t* cu, const int32_t* rows, const int64_t* positions, int32_t nseq,
-                                void* conv_state, int32_t dtype, void* stream) {
-    SKYRL_REQUIRE_T(dtype, "delta_save");
-    const char* bad = bad_shape(shape);
-    SKYRL_REQUIRE(!bad, bad);
-    const Dims d = dims_of(shape);
-    SKYRL_REQUIRE(nseq >= 0 && nseq <= 65535 && proj_stride >= proj_width(d), "delta_save: bad sizes");
-    if (nseq == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(proj && cu && rows && positions && conv_state, "delta_save: null pointer");
-    SKYRL_DISPATCH_T(dtype, {
-        hipLaunchKernelGGL((delta_save_kernel<T>), dim3((d.channels() + kNT - 1) / kNT, nseq), dim3(kNT), 0,
-                           as_stream(stream), d, reinterpret_cast<const T*>(proj), proj_stride, cu, rows, positions,
-                           reinterpret_cast<T*>(conv_state));
-    })
-    return check_launch("delta_save_kernel");
 }
 
 extern "C" int skyrl_delta_conv(const skyrl_delta_shape* shape, const void* proj, int64_t proj_stride,

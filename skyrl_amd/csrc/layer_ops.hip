@@ -1,7 +1,7 @@
-// Norms, gated activations and the logit cap of the hybrid decoders (include/skyrl_layers.h). The
-// residual stream stays f32 in HBM: the add, the norm and the optional per-pass step vector of a
-// looped layer stack are one pass over a row.
-#include "elem.h"
+// Embedding, norms, gated activations, convolution state and the logit cap of the hybrid decoders
+// (include/skyrl_layers.h). The residual stream stays f32 in HBM: the add, the norm and the optional
+// per-pass step vector of a looped layer stack are one pass over a row.
+#include "conv.h"
 
 namespace skyrl {
 namespace {
@@ -11,8 +11,9 @@ constexpr int kNT = 256;
 // One block per row, the row in registers: kMaxV groups of VEC elements per thread.
 template <typename T, int VEC, int kMaxV>
 __global__ __launch_bounds__(kNT) void add_norm_kernel(const T* __restrict__ delta, float* __restrict__ h,
-                                                       const T* __restrict__ step, const T* __restrict__ w, int H,
-                                                       float eps, int kind, T* __restrict__ out) {
+                                                       const T* __restrict__ step, const T* __restrict__ w,
+                                                       float w_base, int H, float eps, int kind,
+                                                       T* __restrict__ out) {
     __shared__ float s_red[kNT / kWave];
     const int64_t base = (int64_t)blockIdx.x * H;
     const int nv = H / VEC;
@@ -64,37 +65,83 @@ __global__ __launch_bounds__(kNT) void add_norm_kernel(const T* __restrict__ del
         if (v < nv) {
             if constexpr (VEC == 4) {
                 const float4 a = ld4(w + 4 * v);
-                st4(out + base + 4 * v,
-                    make_float4(x[k][0] * r * a.x, x[k][1] * r * a.y, x[k][2] * r * a.z, x[k][3] * r * a.w));
+                st4(out + base + 4 * v, make_float4(x[k][0] * r * (w_base + a.x), x[k][1] * r * (w_base + a.y),
+                                                    x[k][2] * r * (w_base + a.z), x[k][3] * r * (w_base + a.w)));
             } else {
-                st(out + base + v, x[k][0] * r * ld(w + v));
+                st(out + base + v, x[k][0] * r * (w_base + ld(w + v)));
             }
         }
     }
 }
 
-__device__ __forceinline__ float activate(float x, int act) {
-    if (act == SKYRL_ACT_SILU) return siluf_(x);
-    return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+struct Gate {
+    int act;
+    float alpha, limit;  // of the clamped form
+};
+
+// The gated product of one pair.
+__device__ __forceinline__ float gated(float g, float u, const Gate& f) {
+    if (f.act == SKYRL_ACT_SILU) return siluf_(g) * u;
+    if (f.act == SKYRL_ACT_CLAMPED) {
+        g = fminf(g, f.limit);
+        u = fminf(fmaxf(u, -f.limit), f.limit);
+        return g / (1.f + expf(-f.alpha * g)) * (u + 1.f);
+    }
+    return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
 }
 
 template <typename T, int VEC>
-__global__ __launch_bounds__(kNT) void gate_mul_kernel(const T* __restrict__ gu, int64_t n, int I, int act,
-                                                       T* __restrict__ out) {
+__global__ __launch_bounds__(kNT) void gate_mul_kernel(const T* __restrict__ gu, int64_t gu_stride, int64_t n, int I,
+                                                       Gate f, T* __restrict__ out, int64_t out_stride) {
     const int iv = I / VEC;
     const int64_t total = n * iv;
     for (int64_t e = (int64_t)blockIdx.x * kNT + threadIdx.x; e < total; e += (int64_t)gridDim.x * kNT) {
         const int64_t row = e / iv;
         const int c = (int)(e - row * iv) * VEC;
-        const T* g = gu + row * 2 * I + c;
+        const T* g = gu + row * gu_stride + c;
         if constexpr (VEC == 4) {
             const float4 a = ld4(g), b = ld4(g + I);
-            st4(out + row * I + c, make_float4(activate(a.x, act) * b.x, activate(a.y, act) * b.y,
-                                               activate(a.z, act) * b.z, activate(a.w, act) * b.w));
+            st4(out + row * out_stride + c,
+                make_float4(gated(a.x, b.x, f), gated(a.y, b.y, f), gated(a.z, b.z, f), gated(a.w, b.w, f)));
         } else {
-            st(out + row * I + c, activate(ld(g), act) * ld(g + I));
+            st(out + row * out_stride + c, gated(ld(g), ld(g + I), f));
         }
     }
+}
+
+// out[row] = scale * table[tokens[row]], f32.
+template <typename T, int VEC>
+__global__ __launch_bounds__(kNT) void embed_kernel(const int64_t* __restrict__ tokens, const T* __restrict__ table,
+                                                    int64_t n, int H, float scale, float* __restrict__ out) {
+    const int hv = H / VEC;
+    const int64_t total = n * hv;
+    for (int64_t e = (int64_t)blockIdx.x * kNT + threadIdx.x; e < total; e += (int64_t)gridDim.x * kNT) {
+        const int64_t row = e / hv;
+        const int c = (int)(e - row * hv) * VEC;
+        const T* src = table + tokens[row] * H + c;
+        if constexpr (VEC == 4) {
+            const float4 a = ld4(src);
+            st4(out + row * H + c, make_float4(a.x * scale, a.y * scale, a.z * scale, a.w * scale));
+        } else {
+            out[row * H + c] = ld(src) * scale;
+        }
+    }
+}
+
+// The last inputs of every sequence's convolutions into its ring. grid (channels / kNT, sequences).
+template <typename T>
+__global__ __launch_bounds__(kNT) void conv_save_kernel(const T* __restrict__ x, int64_t stride, int channels, int taps,
+                                                        const int32_t* __restrict__ cu,
+                                                        const int32_t* __restrict__ rows,
+                                                        const int64_t* __restrict__ positions, T* __restrict__ ring) {
+    const int s = blockIdx.y, row = rows[s];
+    if (row < 0) return;
+    const int t0 = cu[s], t1 = cu[s + 1];
+    const int ch = blockIdx.x * kNT + threadIdx.x;
+    if (ch >= channels || t0 >= t1) return;
+    const int64_t pos0 = positions[t0];
+    for (int t = max(t0, t1 - taps); t < t1; ++t)
+        ring[((int64_t)row * taps + (pos0 + t - t0) % taps) * channels + ch] = x[(int64_t)t * stride + ch];
 }
 
 template <typename T>
@@ -117,10 +164,11 @@ unsigned grid_for(int64_t items) {
 using namespace skyrl;
 
 #define LAUNCH_NORM(V, K) \
-    hipLaunchKernelGGL((add_norm_kernel<T, V, K>), dim3(n), dim3(kNT), 0, s, d, hidden, st_, w, H, eps, kind, o)
+    hipLaunchKernelGGL((add_norm_kernel<T, V, K>), dim3(n), dim3(kNT), 0, s, d, hidden, st_, w, w_base, H, eps, \
+                       kind, o)
 
-extern "C" int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, int32_t n,
-                              int32_t H, float eps, int32_t kind, void* out, int32_t dtype, void* stream) {
+extern "C" int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, float w_base,
+                              int32_t n, int32_t H, float eps, int32_t kind, void* out, int32_t dtype, void* stream) {
     SKYRL_REQUIRE_T(dtype, "add_norm");
     SKYRL_REQUIRE(n >= 0 && H > 0 && H <= 8192, "add_norm: H must be in [1, 8192]");
     SKYRL_REQUIRE(kind == SKYRL_NORM_LAYER || kind == SKYRL_NORM_RMS, "add_norm: unknown norm kind");
@@ -145,24 +193,60 @@ extern "C" int skyrl_add_norm(const void* delta, float* hidden, const void* step
     return check_launch("add_norm_kernel");
 }
 
-extern "C" int skyrl_gate_mul(const void* gate_up, int64_t n, int32_t I, int32_t act, void* out, int32_t dtype,
-                              void* stream) {
+extern "C" int skyrl_gate_mul(const void* gate_up, int64_t gu_stride, int64_t n, int32_t I, int32_t act, float alpha,
+                              float limit, void* out, int64_t out_stride, int32_t dtype, void* stream) {
     SKYRL_REQUIRE_T(dtype, "gate_mul");
-    SKYRL_REQUIRE(n >= 0 && I > 0, "gate_mul: bad sizes");
-    SKYRL_REQUIRE(act == SKYRL_ACT_SILU || act == SKYRL_ACT_GELU_TANH, "gate_mul: unknown activation");
+    SKYRL_REQUIRE(n >= 0 && I > 0 && gu_stride >= 2 * (int64_t)I && out_stride >= I, "gate_mul: bad sizes");
+    SKYRL_REQUIRE(act == SKYRL_ACT_SILU || act == SKYRL_ACT_GELU_TANH || act == SKYRL_ACT_CLAMPED,
+                  "gate_mul: unknown activation");
     if (n == 0) return SKYRL_OK;
     SKYRL_REQUIRE(gate_up && out, "gate_mul: null pointer");
+    const Gate f{act, alpha, limit};
     SKYRL_DISPATCH_T(dtype, {
         const T* g = reinterpret_cast<const T*>(gate_up);
         T* o = reinterpret_cast<T*>(out);
-        if (I % 4 == 0)
+        const uintptr_t mis = (reinterpret_cast<uintptr_t>(g) | reinterpret_cast<uintptr_t>(o)) & (4 * sizeof(T) - 1);
+        if (I % 4 == 0 && gu_stride % 4 == 0 && out_stride % 4 == 0 && mis == 0)
             hipLaunchKernelGGL((gate_mul_kernel<T, 4>), dim3(grid_for(n * (I / 4))), dim3(kNT), 0, as_stream(stream),
-                               g, n, I, act, o);
+                               g, gu_stride, n, I, f, o, out_stride);
         else
-            hipLaunchKernelGGL((gate_mul_kernel<T, 1>), dim3(grid_for(n * I)), dim3(kNT), 0, as_stream(stream), g, n,
-                               I, act, o);
+            hipLaunchKernelGGL((gate_mul_kernel<T, 1>), dim3(grid_for(n * I)), dim3(kNT), 0, as_stream(stream), g,
+                               gu_stride, n, I, f, o, out_stride);
     })
     return check_launch("gate_mul_kernel");
+}
+
+extern "C" int skyrl_embed(const int64_t* tokens, const void* table, int64_t n, int32_t H, float scale, float* out,
+                           int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "embed");
+    SKYRL_REQUIRE(n >= 0 && H > 0, "embed: bad sizes");
+    if (n == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(tokens && table && out, "embed: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        const T* w = reinterpret_cast<const T*>(table);
+        if (H % 4 == 0)
+            hipLaunchKernelGGL((embed_kernel<T, 4>), dim3(grid_for(n * (H / 4))), dim3(kNT), 0, as_stream(stream),
+                               tokens, w, n, H, scale, out);
+        else
+            hipLaunchKernelGGL((embed_kernel<T, 1>), dim3(grid_for(n * H)), dim3(kNT), 0, as_stream(stream), tokens, w,
+                               n, H, scale, out);
+    })
+    return check_launch("embed_kernel");
+}
+
+extern "C" int skyrl_conv_save(const void* x, int64_t stride, int32_t channels, int32_t taps, const int32_t* cu,
+                               const int32_t* rows, const int64_t* positions, int32_t nseq, void* ring, int32_t dtype,
+                               void* stream) {
+    SKYRL_REQUIRE_T(dtype, "conv_save");
+    SKYRL_REQUIRE(channels > 0 && taps > 0 && stride >= channels && nseq >= 0 && nseq <= 65535, "conv_save: bad sizes");
+    if (nseq == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(x && cu && rows && positions && ring, "conv_save: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        hipLaunchKernelGGL((conv_save_kernel<T>), dim3((channels + kNT - 1) / kNT, nseq), dim3(kNT), 0,
+                           as_stream(stream), reinterpret_cast<const T*>(x), stride, channels, taps, cu, rows,
+                           positions, reinterpret_cast<T*>(ring));
+    })
+    return check_launch("conv_save_kernel");
 }
 
 extern "C" int skyrl_softcap(const void* x, float* out, int64_t count, float cap, int32_t dtype, void* stream) {

@@ -3,10 +3,12 @@ state) and feed-forward, part of which may run several times with the same weigh
 
 Dovidra is such a design: latent attention under a sliding window beside gated delta rule layers,
 bias-free layer norms before each half, tanh-form GELU gates, a looped range of layers that adds one
-learned vector per pass, and a tanh cap on the logits. The model is what config.json lists; the
-mechanisms are mixers.py.
+learned vector per pass, and a tanh cap on the logits. Lipedra is another: differential attention, some
+layers over an earlier layer's keys and values, beside clamped gates with biases in parallel layers (one
+RMS norm, mixer and feed-forward in the same two matrix products), and a scaled embedding. The model is
+what config.json lists; the mechanisms are mixers.py; `DESIGNS` holds what a design fixes.
 
-The residual stream is f32. One pass of the HIP norm kernel adds the previous half-layer's output and
+The residual stream is f32. One pass of the HIP norm kernel adds the previous sublayer's output and
 (at the start of a loop pass) its vector, stores the stream and writes the next product's input.
 
 HybridDecoder has PagedDecoder's interface (model.py), so the engine's scheduler, runner, sampler and
@@ -16,7 +18,7 @@ and decode others at the same time (`forward_portions`).
 
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Any, Dict, Iterable, Iterator, List, Optional, Tuple
 
 import torch
@@ -24,10 +26,26 @@ import torch.nn.functional as F
 
 from . import kernels
 from . import layer_kernels as lk
-from .mixers import FEEDFORWARDS, MIXERS, PROMPT_MIN, Weights, chunk_plan, prompt_plan
+from .mixers import FEEDFORWARDS, MIXERS, PROMPT_MIN, Products, Weights
 from .model import StepInputs
 
 DEFAULT_MAX_MODEL_LEN = 32768
+
+
+@dataclass(frozen=True)
+class Design:
+    """What a design fixes for every model of it."""
+
+    norm: str                # of layer_kernels.NORMS
+    norm_base: float = 0.0   # added to the stored norm weights
+    parallel: bool = False   # mixer and feed-forward read one norm and are added together
+    mlp: Dict[str, Any] = field(default_factory=dict)  # feed-forward constants
+
+
+DESIGNS = {
+    "Dovidra": Design(norm="layer", mlp={"act": "gelu_tanh"}),
+    "Lipedra": Design(norm="rms", norm_base=1.0, parallel=True, mlp={"act": "clamped", "alpha": 1.702, "bias": True}),
+}
 
 
 @dataclass
@@ -40,8 +58,10 @@ class LayerRun:
 class HybridSpec:
     """What the engine reads of a model, and the layer order."""
 
+    design: Design
     vocab_size: int
     hidden_size: int
+    embed_scale: float
     norm_eps: float
     logit_softcap: Optional[float]
     layers: List[Dict[str, Any]]
@@ -64,6 +84,14 @@ class HybridSpec:
                 raise ValueError(f"unknown layer type {e['type']!r} (known: {sorted(MIXERS)})")
             if e.get("mlp") and e["mlp"]["kind"] not in FEEDFORWARDS:
                 raise ValueError(f"unknown feed-forward {e['mlp']['kind']!r} (known: {sorted(FEEDFORWARDS)})")
+        for i, e in enumerate(layers):
+            j = e["mixer"].get("kv_from")
+            if j is None:
+                continue
+            m = layers[j]["mixer"] if 0 <= j < i else None
+            if m is None or layers[j]["type"] != e["type"] or m.get("kv_from") is not None \
+                    or any(m.get(k) != e["mixer"].get(k) for k in ("kv_heads", "dim", "vdim")):
+                raise ValueError(f"layer {i}: kv_from {j} is no earlier layer with such keys and values of its own")
         n, loop = len(layers), cfg.get("loop")
         runs, times = [], 0
         if loop:
@@ -77,7 +105,8 @@ class HybridSpec:
         else:
             runs = [LayerRun(i) for i in range(n)]
         eos = cfg.get("eos_token_id")
-        return cls(vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]), norm_eps=float(cfg["norm"]["eps"]),
+        return cls(design=DESIGNS[cfg["architecture"]], vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+                   embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), norm_eps=float(cfg["norm"]["eps"]),
                    logit_softcap=float(cfg["logit_softcap"]) if cfg.get("logit_softcap") else None, layers=layers,
                    runs=runs, loop_times=times,
                    max_position_embeddings=int(cfg.get("max_position_embeddings") or DEFAULT_MAX_MODEL_LEN),
@@ -86,20 +115,23 @@ class HybridSpec:
 
 class HybridCache:
     """Cache or state of every layer run: a looped layer has one per pass. Paged runs share the
-    sequences' block tables; recurrent runs are indexed by the request's persistent batch row."""
+    sequences' block tables; recurrent state is indexed by the request's persistent batch row. A run that
+    reads another layer's keys and values holds that layer's last run's."""
 
     def __init__(self, model: "HybridDecoder", num_blocks: int, num_rows: int):
         self.num_blocks, self.num_rows = num_blocks, num_rows
-        self.runs = [model.layers[r.layer]["mixer"].make_state(num_blocks, num_rows, model.device)
-                     for r in model.spec.runs]
+        self.runs, last = [], {}
+        for r in model.spec.runs:
+            mixer = model.layers[r.layer]["mixer"]
+            source = () if mixer.kv_from is None else (last[mixer.kv_from],)
+            last[r.layer] = mixer.make_state(num_blocks, num_rows, model.device, *source)
+            self.runs.append(last[r.layer])
 
 
 class HybridDecoder:
     """Weights + forward of a hybrid decoder over a HybridCache."""
 
     portions = True         # serves steps that mix prompt portions with decoded tokens
-    plain_lm_head = False   # logits are more than hidden . head^T (cap, f32)
-
     def __init__(self, config: Dict[str, Any], device, dtype: torch.dtype = torch.bfloat16,
                  seed: Optional[int] = 0, max_model_len: Optional[int] = None):
         if dtype not in (torch.bfloat16, torch.float32):
@@ -115,25 +147,38 @@ class HybridDecoder:
     # recurrent state cannot be shared by prefix
     @property
     def prefix_cacheable(self) -> bool:
-        return all(MIXERS[self.spec.layers[r.layer]["type"]].paged for r in self.spec.runs)
+        return all(MIXERS[e["type"]].prefix_cacheable(e["mixer"]) for e in self.spec.layers)
+
+    # logits = hidden . lm_head^T: the sampler may run in that product's epilogue
+    @property
+    def plain_lm_head(self) -> bool:
+        return self.spec.logit_softcap is None
 
     # ---------------------------------------------------------------- weights
     def _alloc(self, seed: Optional[int]):
         s = self.spec
         w = Weights(self.device, self.dtype, seed, s.initializer_range)
         H = s.hidden_size
+        norm = (lambda: w.zeros(H)) if s.design.norm_base else (lambda: w.ones(H))
         self.embed = w.matrix(s.vocab_size, H)
         self.layers: List[Dict[str, Any]] = []
         for e in s.layers:
-            mlp = e.get("mlp")
-            self.layers.append({
-                "norm1": w.ones(H),
-                "mixer": MIXERS[e["type"]](e["mixer"], H, s.norm_eps, self.max_model_len, w),
-                "norm2": w.ones(H) if mlp else None,
-                "mlp": FEEDFORWARDS[mlp["kind"]](mlp, H, w) if mlp else None,
-            })
+            mixer = MIXERS[e["type"]](e["mixer"], H, s.norm_eps, self.max_model_len, w)
+            mlp = FEEDFORWARDS[e["mlp"]["kind"]](e["mlp"], H, w, **s.design.mlp) if e.get("mlp") else None
+            joined = hasattr(mixer, "inner")  # its products are Products'
+            L = {"mixer": mixer, "mlp": mlp, "norm1": norm(), "norm2": None}
+            if s.design.parallel and mlp is not None:
+                if not joined:
+                    raise ValueError(f"{e['type']!r} layers cannot be parallel to a feed-forward")
+                L["subs"] = [(L["norm1"], Products([mixer, mlp], H, w))]
+            else:
+                L["subs"] = [(L["norm1"], Products([mixer], H, w) if joined else mixer)]
+                if mlp is not None:
+                    L["norm2"] = norm()
+                    L["subs"].append((L["norm2"], Products([mlp], H, w)))
+            self.layers.append(L)
         self.loop_step = w.matrix(s.loop_times, H) if s.loop_times else None
-        self.norm = w.ones(H)
+        self.norm = norm()
         self.lm_head = w.matrix(s.vocab_size, H)
 
     def _param_views(self) -> Dict[str, torch.Tensor]:
@@ -146,8 +191,9 @@ class HybridDecoder:
             out[p + "norm1"] = L["norm1"]
             for name, t in L["mixer"].params():
                 out[p + "mix." + name] = t
-            if L["mlp"] is not None:
+            if L["norm2"] is not None:
                 out[p + "norm2"] = L["norm2"]
+            if L["mlp"] is not None:
                 for name, t in L["mlp"].params():
                     out[p + "mlp." + name] = t
         return out
@@ -208,38 +254,36 @@ class HybridDecoder:
         return tokens < PROMPT_MIN
 
     def plan(self, seq_lens: List[int], starts: List[int], n_short: int):
-        """Host plan of the prompt forms, numpy arrays: {window: (seg, tiles, rows, longest)} of the paged
-        mixers' windows and {"chunks": (chunk, seq_chunks)} of the recurrent ones."""
+        """Host plan of the prompt forms, tuples of numpy arrays and sizes by the mixers' keys (host_plans)."""
         if n_short == len(seq_lens):
             return None
-        first = sum(seq_lens[:n_short])
-        plan = {"chunks": chunk_plan(seq_lens, n_short, first)}
-        for w in {L["mixer"].window for L in self.layers if L["mixer"].paged}:
-            plan[w] = prompt_plan(seq_lens, starts, n_short, first, w)
+        plan, first = {}, sum(seq_lens[:n_short])
+        for L in self.layers:
+            for key, make in L["mixer"].host_plans(seq_lens, starts, n_short, first):
+                if key not in plan:
+                    plan[key] = make()
         return plan
 
     # ---------------------------------------------------------------- forward
     def _run_layers(self, inp: StepInputs, cache: HybridCache, want: Optional[torch.Tensor], trail=None):
         """Final-norm output of the wanted tokens (None: all). `trail` collects the residual after every
         layer run (inspection)."""
-        eps = self.spec.norm_eps
-        h = F.embedding(inp.tokens, self.embed).float()
+        s = self.spec
+        norm = dict(eps=s.norm_eps, kind=s.design.norm, base=s.design.norm_base)
+        h = lk.embed(inp.tokens, self.embed, s.embed_scale)
         x = torch.empty(h.shape, dtype=self.dtype, device=self.device)
         delta = None
         ws = self.workspace if inp.one_token else self.portion_workspace
-        for r, state in zip(self.spec.runs, cache.runs):
-            L = self.layers[r.layer]
+        for r, state in zip(s.runs, cache.runs):
             step = None if r.step is None else self.loop_step[r.step]
-            lk.add_norm(delta, h, L["norm1"], eps, step=step, out=x)
-            delta = L["mixer"].forward(x, inp, state, ws)
-            if L["mlp"] is not None:
-                lk.add_norm(delta, h, L["norm2"], eps, out=x)
-                delta = L["mlp"].forward(x)
+            for weight, sub in self.layers[r.layer]["subs"]:
+                lk.add_norm(delta, h, weight, step=step, out=x, **norm)
+                delta, step = sub.forward(x, inp, state, ws), None
             if trail is not None:
                 trail.append(h + delta.float())
         if want is None:
-            return lk.add_norm(delta, h, self.norm, eps, out=x)
-        return lk.add_norm(None if delta is None else delta[want], h[want], self.norm, eps)
+            return lk.add_norm(delta, h, self.norm, out=x, **norm)
+        return lk.add_norm(None if delta is None else delta[want], h[want], self.norm, **norm)
 
     def forward_decode(self, inp: StepInputs, cache: HybridCache) -> torch.Tensor:
         """One token per row: final hidden states [n, H]."""

@@ -14,7 +14,7 @@ from .. import _ffi
 from ..ops import _ptr, _require_gpu, _stream
 
 NORMS = {"layer": 0, "rms": 1}
-ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
 _DTYPES = {torch.bfloat16: _ffi.BF16, torch.float32: _ffi.F32}
 
 
@@ -36,10 +36,28 @@ def _check(t: Optional[torch.Tensor], name: str, dtype, shape=None, contiguous: 
         raise ValueError(f"{name} must be contiguous")
 
 
+def _check_view(t: torch.Tensor, name: str, dtype, shape):
+    """Any row stride, unit column stride."""
+    if t.dtype != dtype or tuple(t.shape) != tuple(shape) or (t.shape[1] > 1 and t.stride(1) != 1):
+        raise ValueError(f"{name} must be {dtype} {tuple(shape)} with unit column stride")
+
+
+def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float) -> torch.Tensor:
+    """f32 rows of the embedding table times scale."""
+    dev = _require_gpu(tokens, table)
+    n, H = tokens.shape[0], table.shape[1]
+    _check(tokens, "tokens", torch.int64, (n,))
+    _check(table, "table", table.dtype)
+    out = torch.empty((n, H), dtype=torch.float32, device=dev)
+    _ffi.call("skyrl_embed", _ptr(tokens), _ptr(table), n, H, float(scale), _ptr(out), _code(table), _stream(dev))
+    return out
+
+
 def add_norm(delta: Optional[torch.Tensor], hidden: torch.Tensor, weight: torch.Tensor, eps: float,
              kind: str = "layer", step: Optional[torch.Tensor] = None,
-             out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """hidden (f32, in place) += delta and += step (one vector for every row), then the norm."""
+             out: Optional[torch.Tensor] = None, base: float = 0.0) -> torch.Tensor:
+    """hidden (f32, in place) += delta and += step (one vector for every row), then the norm, times
+    base + weight (base 1: the weight is stored as its distance from 1)."""
     dev = _require_gpu(hidden, weight, delta, step, out)
     n, H = hidden.shape
     _check(hidden, "hidden", torch.float32)
@@ -49,19 +67,39 @@ def add_norm(delta: Optional[torch.Tensor], hidden: torch.Tensor, weight: torch.
     if out is None:
         out = torch.empty((n, H), dtype=weight.dtype, device=dev)
     _check(out, "out", weight.dtype, (n, H))
-    _ffi.call("skyrl_add_norm", _ptr(delta), _ptr(hidden), _ptr(step), _ptr(weight), n, H, float(eps), NORMS[kind],
-              _ptr(out), _code(weight), _stream(dev))
+    _ffi.call("skyrl_add_norm", _ptr(delta), _ptr(hidden), _ptr(step), _ptr(weight), float(base), n, H, float(eps),
+              NORMS[kind], _ptr(out), _code(weight), _stream(dev))
     return out
 
 
-def gate_mul(gate_up: torch.Tensor, act: str) -> torch.Tensor:
-    """act(gate) * up of the fused [n, 2I] projection."""
-    dev = _require_gpu(gate_up)
+def gate_mul(gate_up: torch.Tensor, act: str, alpha: float = 1.0, limit: float = 0.0,
+             out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The gated product of the fused [n, 2I] projection (skyrl_gate_mul); both may be column ranges."""
+    dev = _require_gpu(gate_up, out)
     n, I2 = gate_up.shape
-    _check(gate_up, "gate_up", gate_up.dtype)
-    out = torch.empty((n, I2 // 2), dtype=gate_up.dtype, device=dev)
-    _ffi.call("skyrl_gate_mul", _ptr(gate_up), n, I2 // 2, ACTIVATIONS[act], _ptr(out), _code(gate_up), _stream(dev))
+    _check_view(gate_up, "gate_up", gate_up.dtype, (n, I2))
+    if out is None:
+        out = torch.empty((n, I2 // 2), dtype=gate_up.dtype, device=dev)
+    _check_view(out, "out", gate_up.dtype, (n, I2 // 2))
+    _ffi.call("skyrl_gate_mul", _ptr(gate_up), gate_up.stride(0), n, I2 // 2, ACTIVATIONS[act], float(alpha),
+              float(limit), _ptr(out), out.stride(0), _code(gate_up), _stream(dev))
     return out
+
+
+def conv_save(x: torch.Tensor, channels: int, cu, rows, positions, ring: torch.Tensor) -> None:
+    """Store the last inputs of each sequence's short convolutions, columns [0, channels) of x."""
+    dev = _require_gpu(x, cu, rows, positions, ring)
+    T, n = x.shape[0], rows.shape[0]
+    if x.dim() != 2 or x.shape[1] < channels or x.stride(1) != 1:
+        raise ValueError(f"x must be [T, >= {channels}] with unit column stride")
+    _check(cu, "cu", torch.int32, (n + 1,))
+    _check(rows, "rows", torch.int32, (n,))
+    _check(positions, "positions", torch.int64, (T,))
+    if ring.dim() != 3 or ring.shape[2] != channels:
+        raise ValueError("ring must be [rows, taps, channels]")
+    _check(ring, "ring", x.dtype)
+    _ffi.call("skyrl_conv_save", _ptr(x), x.stride(0), channels, ring.shape[1], _ptr(cu), _ptr(rows), _ptr(positions),
+              n, _ptr(ring), _code(x), _stream(dev))
 
 
 def softcap(x: torch.Tensor, cap: Optional[float]) -> torch.Tensor:
@@ -236,14 +274,6 @@ def delta_scan(sh, proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, st
     return out
 
 
-def delta_save(sh, proj, cu, rows, positions, conv_state) -> None:
-    """Store the last inputs of each sequence's convolutions."""
-    dev = _require_gpu(proj, cu, rows, positions, conv_state)
-    n = _check_delta(sh, proj, cu, rows, positions, conv_state)
-    _ffi.call("skyrl_delta_save", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(cu), _ptr(rows),
-              _ptr(positions), n, _ptr(conv_state), _code(proj), _stream(dev))
-
-
 CHUNK = 64  # tokens per chunk of the prompt form
 
 
@@ -255,7 +285,7 @@ def delta_prompt(sh, proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, 
                  first_seq: int, first_token: int, out) -> torch.Tensor:
     """Chunked form over the sequences from first_seq on, whose tokens are [first_token, T): chunk int32
     [n, 4] and seq_chunks int32 [sequences + 1] (mixers.chunk_plan). `state` is updated in place; the
-    convolution inputs are delta_save's."""
+    convolution inputs are conv_save's."""
     dev = _require_gpu(proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, state, conv_state, chunk,
                        seq_chunks, out)
     n = _check_delta(sh, proj, cu, rows, positions, conv_state, state)
@@ -282,4 +312,129 @@ def delta_prompt(sh, proj, conv_w, a_log, dt_bias, norm_w, cu, rows, positions, 
               _ptr(positions), _ptr(qk), _ptr(kt), _ptr(W), _ptr(U), _ptr(P), _ptr(G), _ptr(state), _ptr(o), st)
     _ffi.call("skyrl_delta_out", ref, _ptr(o), _ptr(proj), proj.stride(0), _ptr(norm_w), first_token, T, _ptr(out),
               out.stride(0), _code(proj), st)
+    return out
+
+
+# ---------------------------------------------------------------- differential attention
+RUN = 8  # tokens per thread of the prompt's write
+
+
+def diff_shape(heads, kv_heads, dim, vdim, rot_dims, taps, kv, scale, diff, eps) -> _ffi.DiffShape:
+    """kv: the projection has keys and values (False: the layer reads another's)."""
+    return _ffi.DiffShape(heads, kv_heads, dim, vdim, rot_dims, taps, int(kv), scale, diff, eps)
+
+
+def diff_channels(sh) -> int:
+    """Channels of the short convolutions: q | k | v."""
+    return 2 * sh.heads * sh.dim + (sh.kv_heads * (2 * sh.dim + sh.vdim) if sh.kv else 0)
+
+
+def diff_pads(sh):
+    """(columns of a cached key or padded query row, rows of a cached value tile)."""
+    return (sh.dim + 15) // 16 * 32, (sh.vdim + 15) // 16 * 16
+
+
+def diff_mfma(sh, dtype) -> bool:
+    """Whether the matrix kernels (split decode, prompt form) take the shape."""
+    return bool(_ffi.query("skyrl_diff_mfma", ctypes.byref(sh), _DTYPES[dtype]))
+
+
+def diff_runs_fit(sh, proj) -> bool:
+    return (proj.dtype == torch.bfloat16 and sh.dim % 8 == 0 and sh.vdim % 8 == 0 and sh.taps <= 8
+            and proj.stride(0) % 8 == 0 and proj.data_ptr() % 16 == 0)
+
+
+def _check_diff_cache(sh, k_cache, v_cache, dtype):
+    kw, vp = diff_pads(sh)
+    _check(k_cache, "k_cache", dtype, (k_cache.shape[0], sh.kv_heads, 16, kw))
+    _check(v_cache, "v_cache", dtype, (k_cache.shape[0], sh.kv_heads, vp, 16))
+
+
+def diff_write(sh, proj, conv_t, cu, rows, bt_row, positions, slots, cos_sin, ring, k_cache, v_cache,
+               save_conv: bool = False, q=None, first: int = 0, count: Optional[int] = None, runs=None) -> torch.Tensor:
+    """Convolution, rotation, queries out [T, heads, padded], keys and values into the cache, for tokens
+    [first, first + count) or, with `runs` int32 [n, 2] (mixers.run_plan), for those. conv_t f32 [taps,
+    channels]; a given `q` is filled in place."""
+    dev = _require_gpu(proj, conv_t, cu, rows, bt_row, positions, slots, cos_sin, ring, k_cache, v_cache, runs, q)
+    T, n, ch = proj.shape[0], rows.shape[0], diff_channels(sh)
+    if proj.dim() != 2 or proj.shape[1] < ch or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, >= {ch}] with unit column stride")
+    _check(conv_t, "conv_t", torch.float32, (sh.taps, ch))
+    _check(cu, "cu", torch.int32, (n + 1,))
+    _check(rows, "rows", torch.int32, (n,))
+    _check(bt_row, "bt_row", torch.int32, (T,))
+    _check(positions, "positions", torch.int64, (T,))
+    _check(slots, "slots", torch.int64, (T,))
+    if cos_sin.dim() != 2 or cos_sin.shape[1] != sh.rot_dims:
+        raise ValueError("cos_sin must be [max_pos, rot_dims]")
+    _check(cos_sin, "cos_sin", torch.float32)
+    _check(ring, "ring", proj.dtype, (ring.shape[0], sh.taps, ch))
+    _check_diff_cache(sh, k_cache, v_cache, proj.dtype)
+    kw = diff_pads(sh)[0]
+    if q is None:
+        make = torch.empty if kw == 2 * sh.dim else torch.zeros  # the padding must be zero
+        q = make((T, sh.heads, kw), dtype=proj.dtype, device=dev)
+    _check(q, "q", proj.dtype, (T, sh.heads, kw))
+    ref, st = ctypes.byref(sh), _stream(dev)
+    args = (ref, _ptr(proj), proj.stride(0), _ptr(conv_t), _ptr(cu), _ptr(rows), _ptr(bt_row), _ptr(positions),
+            _ptr(slots), _ptr(cos_sin), _ptr(ring))
+    if runs is not None:
+        _check(runs, "runs", torch.int32, (runs.shape[0], 2))
+        for a in range(0, runs.shape[0], 65535):  # the grid's limit
+            part = runs[a:a + 65535]
+            _ffi.call("skyrl_diff_write_runs", *args, _ptr(part), part.shape[0], _ptr(q), _ptr(k_cache), _ptr(v_cache),
+                      st)
+        return q
+    count = T - first if count is None else count
+    if not 0 <= first <= first + count <= T:
+        raise ValueError("diff_write: token range outside the step")
+    _ffi.call("skyrl_diff_write", *args, int(save_conv), first, count, _ptr(q), _ptr(k_cache), _ptr(v_cache),
+              _code(proj), st)
+    return q
+
+
+def diff_workspace_bytes(sh, tokens: int, nparts: int) -> int:
+    return int(_ffi.query("skyrl_diff_attend_workspace_bytes", ctypes.byref(sh), tokens, nparts))
+
+
+def _check_diff_io(sh, q, gate, lam, out):
+    T = q.shape[0]
+    _check(q, "q", q.dtype, (T, sh.heads, diff_pads(sh)[0]))
+    _check_view(gate, "gate", q.dtype, (T, sh.heads))
+    _check(lam, "lambda", torch.float32, (1,))
+    _check_view(out, "out", q.dtype, (T, sh.heads * sh.vdim))
+
+
+def diff_attend(sh, q, gate, k_cache, v_cache, block_tables, bt_row, positions, lam, out, nparts: int = 1,
+                part_min: int = 64, workspace=None) -> torch.Tensor:
+    """One query row per token over its sequence's pages; gate [T, heads] before its sigmoid."""
+    dev = _require_gpu(q, gate, k_cache, v_cache, block_tables, bt_row, positions, lam, out)
+    T = q.shape[0]
+    _check_diff_io(sh, q, gate, lam, out)
+    _check_diff_cache(sh, k_cache, v_cache, q.dtype)
+    _check_table(block_tables, bt_row, positions, T)
+    ws = None
+    if nparts > 1 and diff_mfma(sh, q.dtype):
+        need = diff_workspace_bytes(sh, T, nparts)
+        ws = workspace.get(need) if workspace is not None else torch.empty(need, dtype=torch.uint8, device=dev)
+    else:
+        nparts = 1
+    _ffi.call("skyrl_diff_attend", ctypes.byref(sh), _ptr(q), _ptr(gate), gate.stride(0), _ptr(k_cache), _ptr(v_cache),
+              _ptr(block_tables), block_tables.stride(0), _ptr(bt_row), _ptr(positions), T, _ptr(lam), part_min, nparts,
+              _ptr(out), out.stride(0), _ptr(ws), _code(q), _stream(dev))
+    return out
+
+
+def diff_prefill(sh, q, gate, k_cache, v_cache, block_tables, tiles, lam, out) -> torch.Tensor:
+    """Prompt tiles int32 [n, 4] (mixers.tile_plan) over their sequences' pages, which already hold the
+    portion's own keys and values."""
+    dev = _require_gpu(q, gate, k_cache, v_cache, block_tables, tiles, lam, out)
+    _check_diff_io(sh, q, gate, lam, out)
+    _check_diff_cache(sh, k_cache, v_cache, torch.bfloat16)
+    if block_tables.dtype != torch.int32 or block_tables.dim() != 2 or block_tables.stride(1) != 1:
+        raise ValueError("block_tables must be int32 [n, blocks] with unit column stride")
+    _check(tiles, "tiles", torch.int32, (tiles.shape[0], 4))
+    _ffi.call("skyrl_diff_prefill", ctypes.byref(sh), _ptr(q), _ptr(gate), gate.stride(0), _ptr(k_cache),
+              _ptr(v_cache), _ptr(block_tables), block_tables.stride(0), _ptr(tiles), tiles.shape[0], _ptr(lam),
+              _ptr(out), out.stride(0), _stream(dev))
     return out

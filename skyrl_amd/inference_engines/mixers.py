@@ -1,10 +1,15 @@
-"""Layer mechanisms of the hybrid decoders: latent attention, gated delta rule, gated MLP.
+"""Layer mechanisms of the hybrid decoders: latent attention, gated delta rule, differential
+attention, gated MLP.
 
 A mechanism owns its weights (fused where one product serves several tensors), names them for
 loading and saving, sizes and allocates its cache or state, and runs a step over it with the HIP
 kernels of layer_kernels.py; matrix products are hipBLASLt through torch. Every size and constant is
 a parameter; nothing here knows a particular model. `MIXERS` and `FEEDFORWARDS` map the type names of
 a config.json to these classes.
+
+A sublayer is `forward(x, inp, state, workspace)`. Differential attention and the MLP leave their input
+and output products to `Products`, which runs one sublayer, or a mixer and a feed-forward that read the
+same input side by side in the same two products.
 
 A step is a StepInputs (model.py): tokens of several sequences, each with its own first position. In
 a portion step the first `n_short` sequences (single decoded tokens and short portions) come first;
@@ -40,6 +45,15 @@ class Weights:
         if seed is not None:
             self.gen = torch.Generator(device=self.device)
             self.gen.manual_seed(seed)
+
+        self.tables: Dict[Tuple, torch.Tensor] = {}
+
+    def rotary(self, rot: Dict[str, Any], max_pos: int) -> torch.Tensor:
+        """rotary_table on the device, one for all layers of equal rotation."""
+        key = (repr(sorted(rot.items(), key=lambda kv: kv[0])), max_pos)
+        if key not in self.tables:
+            self.tables[key] = rotary_table(rot, max_pos).to(self.device)
+        return self.tables[key]
 
     def matrix(self, *shape) -> torch.Tensor:
         t = torch.empty(shape, dtype=self.dtype, device=self.device)
@@ -118,12 +132,73 @@ def chunk_plan(seq_lens: List[int], first_seq: int, first_token: int):
     return np.asarray(chunk, dtype=np.int32).reshape(-1, 4), np.asarray(ends, dtype=np.int32)
 
 
+def tile_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token: int) -> np.ndarray:
+    """Query tiles int32 [m, 4] of full causal attention of sequences first_seq..: first token, tokens,
+    position of the first, sequence; the tiles with the most keys first."""
+    tiles, tok = [], first_token
+    for i in range(first_seq, len(seq_lens)):
+        L, s = seq_lens[i], starts[i]
+        tiles += [(tok + a, min(PREFILL_TILE, L - a), s + a, i) for a in range(0, L, PREFILL_TILE)]
+        tok += L
+    tiles.sort(key=lambda t: -(t[1] + t[2]))
+    return np.asarray(tiles, dtype=np.int32).reshape(-1, 4)
+
+
+def run_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token: int) -> np.ndarray:
+    """Runs int32 [n, 2] (first token, tokens) of sequences first_seq.., cut where a position is a
+    multiple of lk.RUN, so that a run's cache slots are consecutive."""
+    runs, tok = [], first_token
+    for i in range(first_seq, len(seq_lens)):
+        L, s = seq_lens[i], starts[i]
+        cuts = np.unique(np.concatenate([[0, L], np.arange(-s % lk.RUN, L, lk.RUN)]))
+        runs.append(np.stack([tok + cuts[:-1], np.diff(cuts)], 1))
+        tok += L
+    return np.concatenate(runs).astype(np.int32)
+
+
+class Products:
+    """The input and the output product of sublayers that read the same input and whose outputs are
+    summed: the parts' input rows stacked and their output columns side by side, one product each. Parts
+    start at multiples of 8 elements (16 bytes). A part has `in_rows`, `out_cols`, `in_bias`, `out_bias`,
+    takes its views of the weights in `bind` and computes `inner(proj, out, ...)` between the products."""
+
+    def __init__(self, parts: List[Any], width: int, w: Weights):
+        self.parts, self.ranges = parts, []
+        a = c = 0
+        for p in parts:
+            self.ranges.append((a, c))
+            a, c = a + (p.in_rows + 7) // 8 * 8, c + (p.out_cols + 7) // 8 * 8
+        if sum(p.out_bias for p in parts) > 1:
+            raise ValueError("one part at most may have an output bias")
+        self.w_in, self.w_out = w.matrix(a, width), w.matrix(width, c)
+        self.b_in = w.zeros(a) if any(p.in_bias for p in parts) else None
+        self.b_out = w.zeros(width) if any(p.out_bias for p in parts) else None
+        self.padded = any(p.out_cols % 8 for p in parts)
+        for p, (a, c) in zip(parts, self.ranges):
+            p.bind(self.w_in[a:a + p.in_rows], self.b_in[a:a + p.in_rows] if p.in_bias else None,
+                   self.w_out[:, c:c + p.out_cols], self.b_out if p.out_bias else None)
+
+    def forward(self, x: torch.Tensor, inp, state, workspace) -> torch.Tensor:
+        proj = F.linear(x, self.w_in, self.b_in)
+        make = torch.zeros if self.padded else torch.empty  # padding columns meet weights: they must be finite
+        cat = make((x.shape[0], self.w_out.shape[1]), dtype=x.dtype, device=x.device)
+        for p, (a, c) in zip(self.parts, self.ranges):
+            p.inner(proj[:, a:a + p.in_rows], cat[:, c:c + p.out_cols], inp, state, workspace)
+        return F.linear(cat, self.w_out, self.b_out)
+
+
 class LatentAttention:
     """Attention over low-rank latents shared by all heads, with a rotated key part beside them and
     an optional sliding window. Caches [blocks, 16, row]: per token the normed latent | the rotated key
     part."""
 
     paged = True
+    kv_from = None
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        """Whether a page's content depends on the tokens before it alone, with no state beside the pages."""
+        return True
 
     def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
         self.heads, self.dim, self.rot_dim = int(m["heads"]), int(m["dim"]), int(m["rot_dim"])
@@ -135,7 +210,7 @@ class LatentAttention:
         if self.rot_dim % 2:
             raise ValueError("rot_dim must be even")
         self.eps, self.width, self.dtype = eps, width, w.dtype
-        self.cos_sin = rotary_table(m["rot"], max_pos).to(w.device)
+        self.cos_sin = w.rotary(m["rot"], max_pos)
         H, qd = self.heads, self.dim + self.rot_dim
         self.wproj = w.matrix(H * qd + self.rank + self.rot_dim, width)
         self.dkv_norm = w.ones(self.rank)
@@ -167,6 +242,10 @@ class LatentAttention:
     def make_state(self, num_blocks: int, num_rows: int, device) -> torch.Tensor:
         return torch.zeros((num_blocks, BLOCK_SIZE, lk.latent_row(self.rank, self.rot_dim)), dtype=self.dtype,
                            device=device)
+
+    # ---- plans
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        yield self.window, lambda: prompt_plan(seq_lens, starts, first_seq, first_token, self.window)
 
     # ---- decode split
     def nparts(self, tokens: int, max_ctx: int) -> int:
@@ -218,7 +297,11 @@ class GatedDelta:
     request): the f32 matrix of every head and the convolutions' last inputs."""
 
     paged = False
-    window = None
+    kv_from = None
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        return False
 
     def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
         self.heads, self.kv_heads = int(m["heads"]), int(m["kv_heads"])
@@ -263,6 +346,9 @@ class GatedDelta:
     def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
         return 0
 
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        yield "chunks", lambda: chunk_plan(seq_lens, first_seq, first_token)
+
     # ---- step
     def forward(self, x: torch.Tensor, inp, state, workspace) -> torch.Tensor:
         S, ring = state
@@ -279,25 +365,143 @@ class GatedDelta:
             lk.delta_prompt(self.shape, proj, *args, inp.cu, inp.rows, inp.positions, S, ring, chunk, seq_chunks, k,
                             inp.short_tokens, out)
         if not inp.one_token:
-            lk.delta_save(self.shape, proj, inp.cu, inp.rows, inp.positions, ring)
+            lk.conv_save(proj, lk.delta_channels(self.shape), inp.cu, inp.rows, inp.positions, ring)
         return F.linear(out, self.wo)
 
 
-class GatedMLP:
-    """down(act(gate x) * up x), gate and up fused."""
+class DifferentialAttention:
+    """Full causal attention in two softmax maps per head over the same values, their weighted difference
+    normed per head and gated; short causal convolutions and partial interleaved rotation on its
+    projections. Caches, per layer with keys of its own, K [blocks, kv_heads, 16, both maps] and V
+    transposed [blocks, kv_heads, vdim, 16]; state per row: the convolutions' last inputs. A layer with
+    `kv_from` reads the cache of that layer and has queries only."""
 
-    def __init__(self, m: Dict[str, Any], width: int, w: Weights, act: str = "gelu_tanh"):
-        self.ff, self.act = int(m["ff"]), act
-        self.wgu = w.matrix(2 * self.ff, width)
-        self.wd = w.matrix(width, self.ff)
+    paged = True
+    in_bias, out_bias = True, False
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        return int(m["conv"]) == 1
+
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+        self.heads, self.kv_heads = int(m["heads"]), int(m["kv_heads"])
+        self.dim, self.vdim, self.taps, self.diff = int(m["dim"]), int(m["vdim"]), int(m["conv"]), float(m["diff"])
+        self.kv_from = None if m.get("kv_from") is None else int(m["kv_from"])
+        rot = m["rot"]
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if int(rot["dims"]) % 2 or int(rot["dims"]) > self.dim:
+            raise ValueError("rot.dims must be even and at most dim")
+        self.shape = lk.diff_shape(self.heads, self.kv_heads, self.dim, self.vdim, int(rot["dims"]), self.taps,
+                                   self.kv_from is None, float(m["scale"]), self.diff, eps)
+        self.dtype = w.dtype
+        self.cos_sin = w.rotary(rot, max_pos)
+        self.channels = lk.diff_channels(self.shape)
+        self.in_rows, self.out_cols = self.channels + self.heads, self.heads * self.vdim
+        self.conv = w.matrix(self.channels, self.taps)
+        self.lq1, self.lk1, self.lq2, self.lk2 = (w.matrix(self.dim) for _ in range(4))
+        self.conv_t = w.zeros(self.taps, self.channels, dtype=torch.float32)  # the kernels' form of conv
+        self.lam = w.zeros(1, dtype=torch.float32)
+        self.refresh()
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.w_in, self.b_in, self.wo = w_in, b_in, w_out
+
+    def _rows(self):
+        qk, v = 2 * self.heads * self.dim, self.kv_heads * self.vdim
+        own = self.kv_from is None
+        return (("q", qk),) + ((("k", 2 * self.kv_heads * self.dim), ("v", v)) if own else ())
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        yield from split_rows(self.w_in, self._rows() + (("g", self.heads),))
+        yield from split_rows(self.b_in, [(n + ".b", r) for n, r in self._rows()])
+        yield from split_rows(self.conv, [(n + ".conv", r) for n, r in self._rows()])
+        yield from (("lq1", self.lq1), ("lk1", self.lk1), ("lq2", self.lq2), ("lk2", self.lk2), ("o", self.wo))
+
+    def refresh(self) -> None:
+        """Recompute derived tensors, in place, after the weights changed."""
+        self.conv_t.copy_(self.conv.t())
+        a, b = ((q.float() * k.float()).sum() for q, k in ((self.lq1, self.lk1), (self.lq2, self.lk2)))
+        self.lam.copy_(torch.exp(a) - torch.exp(b) + self.diff)
+
+    # ---- cache
+    def block_bytes(self) -> int:
+        if self.kv_from is not None:
+            return 0
+        return self.kv_heads * BLOCK_SIZE * sum(lk.diff_pads(self.shape)) * self.dtype.itemsize
+
+    def row_bytes(self) -> int:
+        return self.taps * self.channels * self.dtype.itemsize
+
+    def make_state(self, num_blocks: int, num_rows: int, device, source=None):
+        """source: the state of the layer whose keys and values this one reads."""
+        ring = torch.zeros((num_rows, self.taps, self.channels), dtype=self.dtype, device=device)
+        if source is not None:
+            return source[0], source[1], ring
+        kw, vp = lk.diff_pads(self.shape)
+        zeros = lambda *tail: torch.zeros((num_blocks, self.kv_heads) + tail, dtype=self.dtype, device=device)  # noqa: E731
+        return zeros(BLOCK_SIZE, kw), zeros(vp, BLOCK_SIZE), ring
+
+    # ---- plans
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        yield "tiles", lambda: (tile_plan(seq_lens, starts, first_seq, first_token),
+                                run_plan(seq_lens, starts, first_seq, first_token))
+
+    def nparts(self, tokens: int, max_ctx: int) -> int:
+        groups = -(-(self.heads // self.kv_heads) // 8)  # a wave takes eight query heads of a key head
+        return kernels.choose_nparts(tokens, self.kv_heads * groups, max_ctx)
+
+    def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
+        return lk.diff_workspace_bytes(self.shape, tokens, self.nparts(tokens, max_ctx))
+
+    # ---- step
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
+        k_cache, v_cache, ring = state
+        T = proj.shape[0]
+        seqs = (inp.cu, inp.rows, inp.bt_row, inp.positions, inp.slots, self.cos_sin, ring, k_cache, v_cache)
+        prompt = inp.plan is not None and lk.diff_mfma(self.shape, self.dtype)
+        ts = inp.short_tokens if prompt else T
+        runs = inp.plan["tiles"][1] if prompt and lk.diff_runs_fit(self.shape, proj) else None
+        q = lk.diff_write(self.shape, proj, self.conv_t, *seqs, save_conv=inp.one_token,
+                          count=T if runs is None else ts)
+        if runs is not None:
+            lk.diff_write(self.shape, proj, self.conv_t, *seqs, q=q, runs=runs)
+        if not inp.one_token and self.taps > 1:
+            lk.conv_save(proj, self.channels, inp.cu, inp.rows, inp.positions, ring)
+        gate = proj[:, self.channels:]
+        for a in range(0, ts, 32768):  # the decode form's grid limit
+            b = min(ts, a + 32768)
+            lk.diff_attend(self.shape, q[a:b], gate[a:b], k_cache, v_cache, inp.block_tables, inp.bt_row[a:b],
+                           inp.positions[a:b], self.lam, out[a:b], nparts=self.nparts(b - a, inp.max_ctx),
+                           part_min=kernels.MIN_PARTITION, workspace=workspace)
+        if ts < T:
+            lk.diff_prefill(self.shape, q, gate, k_cache, v_cache, inp.block_tables, inp.plan["tiles"][0], self.lam, out)
+
+
+class GatedMLP:
+    """down(gated product of gate x and up x), gate and up fused: `act` of layer_kernels.ACTIVATIONS, with
+    m["limit"] for the clamped one; `bias`: on every projection."""
+
+    def __init__(self, m: Dict[str, Any], width: int, w: Weights, act: str = "gelu_tanh", alpha: float = 1.0,
+                 bias: bool = False):
+        self.ff, self.act, self.alpha = int(m["ff"]), act, alpha
+        self.limit = float(m["limit"]) if act == "clamped" else 0.0
+        self.in_rows, self.out_cols = 2 * self.ff, self.ff
+        self.in_bias = self.out_bias = bias
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.wgu, self.bgu, self.wd, self.bd = w_in, b_in, w_out, b_out
 
     def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
         yield from split_rows(self.wgu, (("gate", self.ff), ("up", self.ff)))
         yield "down", self.wd
+        if self.in_bias:
+            yield from split_rows(self.bgu, (("gate.b", self.ff), ("up.b", self.ff)))
+            yield "down.b", self.bd
 
-    def forward(self, x: torch.Tensor) -> torch.Tensor:
-        return F.linear(lk.gate_mul(F.linear(x, self.wgu), self.act), self.wd)
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
+        lk.gate_mul(proj, self.act, self.alpha, self.limit, out=out)
 
 
-MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta}
+MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "attention": DifferentialAttention}
 FEEDFORWARDS = {"dense": GatedMLP}

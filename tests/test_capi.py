@@ -43,10 +43,16 @@ def test_layers_library_matches_its_header():
 
 def test_layers_entries_validate_on_host():
     p, sh = ctypes.c_void_p(16), _ffi.DeltaShape(3, 2, 8, 8, 4, 1e-5)
+    diff = lambda *a: ctypes.byref(_ffi.DiffShape(*a, 0.5, 0.3, 1e-5))  # noqa: E731
+    good = diff(4, 2, 12, 8, 4, 3, 1)
+    rows = (p, p, p, p, p, p)
     for name, args, msg in (
-            ("skyrl_add_norm", (None, p, None, p, 1, 9000, 1e-5, 0, p, _ffi.BF16, None), "H must be"),
-            ("skyrl_add_norm", (None, p, None, p, 1, 64, 1e-5, 0, p, _ffi.I64, None), "dtype"),
-            ("skyrl_gate_mul", (p, 1, 8, 7, p, _ffi.F32, None), "activation"),
+            ("skyrl_add_norm", (None, p, None, p, 0.0, 1, 9000, 1e-5, 0, p, _ffi.BF16, None), "H must be"),
+            ("skyrl_add_norm", (None, p, None, p, 0.0, 1, 64, 1e-5, 0, p, _ffi.I64, None), "dtype"),
+            ("skyrl_gate_mul", (p, 16, 1, 8, 7, 1.0, 0.0, p, 8, _ffi.F32, None), "activation"),
+            ("skyrl_gate_mul", (p, 15, 1, 8, 2, 1.0, 0.0, p, 8, _ffi.F32, None), "sizes"),
+            ("skyrl_embed", (p, p, 1, 0, 1.0, p, _ffi.F32, None), "sizes"),
+            ("skyrl_conv_save", (p, 7, 8, 3, p, p, p, 1, p, _ffi.F32, None), "sizes"),
             ("skyrl_latent_write", (p, 10, 1, 1, 4, 4, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "proj_stride"),
             ("skyrl_latent_write", (p, 100, 1, 1, 4, 4, 40, p, 1e-5, p, p, p, p, 40, _ffi.F32, None), "multiple of 32"),
             ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 8, 1, p, p, _ffi.BF16, None),
@@ -56,7 +62,19 @@ def test_layers_entries_validate_on_host():
             ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 65, p, 1, 1, 16, 16, 16, 1.0, 0, p, 16, None), "vt_stride"),
             ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 64, p, 1, 1, 250, 16, 16, 1.0, 0, p, 16, None), "256"),
             ("skyrl_delta_scan", (ctypes.byref(sh), p, 100, p, p, p, p, p, p, p, 1, p, p, 1, p, 24, _ffi.F32, None),
-             "multiple of kv_heads")):
+             "multiple of kv_heads"),
+            ("skyrl_diff_write", (diff(3, 2, 8, 8, 4, 3, 1), p, 100, p, *rows, p, 0, 0, 1, p, p, p, _ffi.F32, None),
+             "multiple of kv_heads"),
+            ("skyrl_diff_write", (diff(4, 2, 8, 8, 10, 3, 1), p, 100, p, *rows, p, 0, 0, 1, p, p, p, _ffi.F32, None),
+             "rot_dims"),
+            ("skyrl_diff_write", (good, p, 100, p, *rows, p, 0, 0, 1, p, p, p, _ffi.F32, None), "sizes"),
+            ("skyrl_diff_write_runs", (good, p, 160, p, *rows, p, p, 1, p, p, p, None), "multiples of 8"),
+            ("skyrl_diff_attend", (good, p, p, 4, p, p, p, 8, p, p, 1, p, 8, 1, p, 32, p, _ffi.BF16, None), "part_min"),
+            ("skyrl_diff_attend", (good, p, p, 4, p, p, p, 8, p, p, 1, p, 64, 2, p, 32, None, _ffi.BF16, None),
+             "workspace"),
+            ("skyrl_diff_attend", (good, p, p, 4, p, p, p, 8, p, p, 1, p, 64, 1, p, 31, None, _ffi.F32, None), "sizes"),
+            ("skyrl_diff_prefill", (diff(4, 2, 130, 8, 4, 3, 1), p, p, 4, p, p, p, 8, p, 1, p, p, 32, None), "dim <= 128"),
+            ("skyrl_diff_prefill", (good, p, p, 3, p, p, p, 8, p, 1, p, p, 32, None), "sizes")):
         with pytest.raises(_ffi.SkyrlHipError, match=msg):
             _ffi.call(name, *args)
 

@@ -264,7 +264,7 @@ class DeltaCase:
             chunk, ends = (torch.from_numpy(a).to(DEV) for a in mixers.chunk_plan(lens, k, first))
             lk.delta_prompt(self.sh, proj, *self.dev, cu, rows, pos, self.S, self.ring, chunk, ends, k, first, out)
         if not one:
-            lk.delta_save(self.sh, proj, cu, rows, pos, self.ring)
+            lk.conv_save(proj, lk.delta_channels(self.sh), cu, rows, pos, self.ring)
         return out.split(lens)
 
 
