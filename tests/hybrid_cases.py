@@ -93,3 +93,81 @@ def make_weights(cfg, seed=0):
     vec("final.norm", W)
     mat("head", cfg["vocab"], W, 3.0)
     return {k: v.to(torch.bfloat16) for k, v in w.items()}
+
+
+# ---------------------------------------------------------------- parallel layers of differential attention
+def diff_attention(heads=4, kv_heads=2, dim=20, vdim=28, conv=3, rot_dims=8, diff=0.35, scale=None, base=700.0,
+                   scaling=True, kv_from=None):
+    rot = {"base": base, "dims": rot_dims}
+    if scaling:
+        rot["scaling"] = {"factor": 5.0, "original": 48, "fast": 6.0, "slow": 0.4}
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv, "diff": diff, "rot": rot,
+         "scale": scale or 1.4 / math.sqrt(dim)}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m}
+
+
+def parallel_config(layers, width=72, vocab=203, ff=(100, 1.3), scale=2.7, eps=4e-5, no_mlp=()):
+    layers = [dict(e, mlp=None if i in no_mlp else {"kind": "dense", "ff": ff[0] + 4 * i, "limit": ff[1] + 0.2 * i})
+              for i, e in enumerate(layers)]
+    return {"architecture": "Lipedra", "layers": layers, "norm": {"eps": eps}, "embedding": {"scale": scale},
+            "vocab": vocab, "width": width}
+
+
+PARALLEL = {
+    # sizes no vector width divides, two layers on one cache with other constants than its owner, no feed-forward
+    "odd": parallel_config([diff_attention(), diff_attention(heads=6, kv_heads=3, dim=22, vdim=11, conv=5, rot_dims=22),
+                            diff_attention(heads=6, kv_heads=3, dim=22, vdim=11, conv=2, rot_dims=22, kv_from=1, diff=0.7,
+                                           scale=0.5),
+                            diff_attention(heads=4, kv_heads=2, kv_from=0, conv=4)], no_mlp=(2,)),
+    # exact matrix-kernel shapes, many query heads per key head (more than one group), no scaling
+    "wide": parallel_config([diff_attention(heads=20, kv_heads=1, dim=32, vdim=64, rot_dims=16, scaling=False, conv=4),
+                             diff_attention(heads=2, kv_heads=2, dim=64, vdim=128, rot_dims=64, conv=1),
+                             diff_attention(heads=20, kv_heads=1, dim=32, vdim=64, rot_dims=16, scaling=False, kv_from=0,
+                                            conv=4)], width=128, ff=(96, 0.7)),
+    # padded shapes of the matrix kernels: both maps in one step, values beyond one tile count, many taps
+    "padded": parallel_config([diff_attention(heads=3, kv_heads=1, dim=48, vdim=24, rot_dims=2, conv=8),
+                               diff_attention(heads=8, kv_heads=4, dim=16, vdim=136, rot_dims=6, conv=11),
+                               diff_attention(heads=2, kv_heads=1, dim=104, vdim=200, rot_dims=40, conv=6)], width=56,
+                              ff=(68, 2.5), scale=0.6),
+}
+
+
+def make_parallel_weights(cfg, seed=0):
+    """bf16 tensors by checkpoint name: biases, norm offsets and gates far from trivial, feed-forward
+    projections that reach the clamp."""
+    g = torch.Generator().manual_seed(seed)
+    W, w = cfg["width"], {}
+
+    def rand(name, *shape, gain=1.0):
+        w[name] = torch.randn(*shape, generator=g) * gain
+
+    def proj(name, rows, cols, gain=1.0, bias=True):
+        rand(name, rows, cols, gain=gain / math.sqrt(cols))
+        if bias:
+            rand(name + ".b", rows, gain=0.3)
+
+    rand("embed", cfg["vocab"], W)
+    for i, e in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        q = p + "mix."
+        rand(p + "norm1", W, gain=0.3)
+        rows = [("q", 2 * m["heads"] * m["dim"])]
+        if m.get("kv_from") is None:
+            rows += [("k", 2 * m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])]
+        for n, r in rows:
+            proj(q + n, r, W, 1.3)
+            rand(q + n + ".conv", r, m["conv"], gain=1 / math.sqrt(m["conv"]))
+        for n in ("lq1", "lk1", "lq2", "lk2"):
+            rand(q + n, m["dim"], gain=0.25)
+        proj(q + "g", m["heads"], W, 1.5, bias=False)
+        proj(q + "o", W, m["heads"] * m["vdim"], 1.5, bias=False)
+        if e.get("mlp"):
+            ff = e["mlp"]["ff"]
+            proj(p + "mlp.gate", ff, W, 1.5)
+            proj(p + "mlp.up", ff, W, 1.5)
+            proj(p + "mlp.down", W, ff)
+    rand("final.norm", W, gain=0.3)
+    proj("head", cfg["vocab"], W, 3.0, bias=False)
+    return {k: v.to(torch.bfloat16) for k, v in w.items()}
