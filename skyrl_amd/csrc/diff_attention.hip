@@ -14,6 +14,8 @@
 //
 // Prompt form (diff_prefill): flash style, eight waves of 16 queries of one head share a tile of 64 keys and
 // values in LDS, read straight from the pages; each wave keeps both maps' sums and combines them in registers.
+// A map's running maximum is only raised when the scores outgrow it by kSlack, so that the sums are rescaled
+// at the first tile and seldom after.
 #include "conv.h"
 
 namespace skyrl {
@@ -597,6 +599,7 @@ __global__ __launch_bounds__(2 * kWave) void diff_merge_kernel(Dims d, const flo
 
 // ---- prompt form ----------------------------------------------------------------------------------
 constexpr int kKT = 64;        // keys per LDS tile
+constexpr float kSlack = 8.f;  // a running maximum may lag by this (base 2): weights stay below 2^8
 constexpr int kPNT = 512;
 
 // KM: 32-wide steps of one map's key columns (with dp % 32 == 16 the middle step belongs to both maps, the
@@ -697,13 +700,13 @@ __global__ __launch_bounds__(kPNT) __attribute__((amdgpu_waves_per_eu(2))) void 
         if (kp0 > wq1 || wq0 > last) continue;  // no key of this tile for this wave
         const bool edge = kp1 > wq0;
         s16x8 pf[2][2];  // [map][32-key step]
-        float alpha[2];
+        f32x4 sc[2][4];
+        float top[2];
         bool grown = false;
 #pragma unroll
         for (int mp = 0; mp < 2; ++mp) {
-            f32x4 sc[4];
 #pragma unroll
-            for (int tt = 0; tt < 4; ++tt) sc[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+            for (int tt = 0; tt < 4; ++tt) sc[mp][tt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int s = 0; s < KM; ++s) {
                 if (EXACT || s < km) {
@@ -711,7 +714,7 @@ __global__ __launch_bounds__(kPNT) __attribute__((amdgpu_waves_per_eu(2))) void 
 #pragma unroll
                     for (int tt = 0; tt < 4; ++tt) {
                         const s16x8 kf = *reinterpret_cast<const s16x8*>(&s_k[(16 * tt + c) * LDK + col]);
-                        sc[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[mp][s], sc[tt], 0, 0, 0);
+                        sc[mp][tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[mp][s], sc[mp][tt], 0, 0, 0);
                     }
                 }
             }
@@ -721,18 +724,29 @@ __global__ __launch_bounds__(kPNT) __attribute__((amdgpu_waves_per_eu(2))) void 
                 for (int tt = 0; tt < 4; ++tt)
 #pragma unroll
                     for (int i = 0; i < 4; ++i)
-                        if (16 * tt + i > seen) sc[tt][i] = -INFINITY;
+                        if (16 * tt + i > seen) sc[mp][tt][i] = -INFINITY;
             }
             float bm = -INFINITY;
 #pragma unroll
             for (int tt = 0; tt < 4; ++tt)
-                bm = fmaxf(bm, fmaxf(fmaxf(sc[tt][0], sc[tt][1]), fmaxf(sc[tt][2], sc[tt][3])));
+                bm = fmaxf(bm, fmaxf(fmaxf(sc[mp][tt][0], sc[mp][tt][1]), fmaxf(sc[mp][tt][2], sc[mp][tt][3])));
             bm = fmaxf(bm, __shfl_xor(bm, 16, kWave));
             bm = fmaxf(bm, __shfl_xor(bm, 32, kWave));
-            const float mn = fmaxf(m[mp], bm * scale_log2);  // scale > 0; finite from the first tile on
-            alpha[mp] = fast_exp2(m[mp] - mn);
-            grown |= mn > m[mp];
-            float sum = 0.f;
+            top[mp] = bm * scale_log2;  // scale > 0
+            grown |= top[mp] > m[mp] + kSlack;
+        }
+        if (__any(grown)) {  // at the first tile; later seldom
+#pragma unroll
+            for (int mp = 0; mp < 2; ++mp) {
+                const float mn = fmaxf(m[mp], top[mp]), alpha = fast_exp2(m[mp] - mn);
+                m[mp] = mn;
+                l[mp] = l[mp] * alpha;
+#pragma unroll
+                for (int n = 0; n < NV; ++n) o[mp][n] = o[mp][n] * alpha;
+            }
+        }
+#pragma unroll
+        for (int mp = 0; mp < 2; ++mp) {
 #pragma unroll
             for (int kk = 0; kk < 2; ++kk) {
                 uint32_t pk[4];
@@ -741,22 +755,13 @@ __global__ __launch_bounds__(kPNT) __attribute__((amdgpu_waves_per_eu(2))) void 
                     float p[4];
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
-                        p[i] = fast_exp2(fmaf(sc[2 * kk + bb][i], scale_log2, -mn));
-                        sum += p[i];
+                        p[i] = fast_exp2(fmaf(sc[mp][2 * kk + bb][i], scale_log2, -m[mp]));
+                        l[mp] += p[i];
                     }
                     pk[2 * bb] = pack_bf16x2(p[0], p[1]);
                     pk[2 * bb + 1] = pack_bf16x2(p[2], p[3]);
                 }
                 pf[mp][kk] = __builtin_bit_cast(s16x8, make_uint4(pk[0], pk[1], pk[2], pk[3]));
-            }
-            l[mp] = l[mp] * alpha[mp] + sum;
-            m[mp] = mn;
-        }
-        if (__any(grown)) {
-#pragma unroll
-            for (int n = 0; n < NV; ++n) {
-                o[0][n] = o[0][n] * alpha[0];
-                o[1][n] = o[1][n] * alpha[1];
             }
         }
 #pragma unroll
@@ -822,7 +827,6 @@ Dims dims_of(const skyrl_diff_shape* s) {
 }
 bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
-template <typename T>
 bool wide(const Dims& d, const void* proj, int64_t stride) {  // every piece of eight channels is one head's and aligned
     return d.D % 8 == 0 && d.V % 8 == 0 && stride % 8 == 0 && aligned16(proj);
 }
@@ -854,7 +858,7 @@ extern "C" int skyrl_diff_write(const skyrl_diff_shape* shape, const void* proj,
                        positions, slots, cos_sin, reinterpret_cast<T*>(ring), save_conv, first,                       \
                        reinterpret_cast<T*>(q), reinterpret_cast<T*>(k_cache), reinterpret_cast<T*>(v_cache))
     SKYRL_DISPATCH_T(dtype, {
-        if (wide<T>(d, proj, proj_stride)) LAUNCH_WRITE(8);
+        if (wide(d, proj, proj_stride)) LAUNCH_WRITE(8);
         else LAUNCH_WRITE(1);
     })
     return check_launch("diff_write_kernel");
@@ -869,7 +873,7 @@ extern "C" int skyrl_diff_write_runs(const skyrl_diff_shape* shape, const void* 
     SKYRL_REQUIRE(!bad, bad);
     const Dims d = dims_of(shape);
     SKYRL_REQUIRE(nruns >= 0 && nruns <= 65535 && proj_stride >= d.channels(), "diff_write_runs: bad sizes");
-    SKYRL_REQUIRE(wide<uint16_t>(d, proj, proj_stride) && d.taps <= kConvWindow,
+    SKYRL_REQUIRE(wide(d, proj, proj_stride) && d.taps <= kConvWindow,
                   "diff_write_runs: dim, vdim and proj_stride must be multiples of 8, proj aligned, taps <= 8");
     if (nruns == 0) return SKYRL_OK;
     SKYRL_REQUIRE(proj && conv_t && cu && rows && bt_row && positions && slots && ring && runs && q &&

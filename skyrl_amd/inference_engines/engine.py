@@ -615,7 +615,7 @@ class ModelRunner:
         self.max_num_seqs = max_num_seqs
         self.max_blocks = _blocks_needed(model.max_model_len)
         self.use_graphs = use_graphs
-        self.buckets = [b for b in self.BUCKETS if b < max_num_seqs] + [max_num_seqs]
+        self.buckets = [b for b in self.BUCKETS if model.min_bucket <= b < max_num_seqs] + [max_num_seqs]
         self.cache = None
         R = max_num_seqs
         pin = torch.cuda.is_available()

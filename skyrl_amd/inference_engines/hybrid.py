@@ -154,6 +154,11 @@ class HybridDecoder:
     def plain_lm_head(self) -> bool:
         return self.spec.logit_softcap is None
 
+    # a biased product of one row copies the bias first instead of adding it in the library's kernel
+    @property
+    def min_bucket(self) -> int:
+        return 2 if self.spec.design.mlp.get("bias") else 1
+
     # ---------------------------------------------------------------- weights
     def _alloc(self, seed: Optional[int]):
         s = self.spec

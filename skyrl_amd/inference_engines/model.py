@@ -128,6 +128,7 @@ class PagedDecoder:
     portions = False         # a step is a prefill or a decode
     plain_lm_head = True     # logits = hidden . lm_head^T (the sampler may run in that product's epilogue)
     prefix_cacheable = True  # a block's K/V depend on the token prefix alone
+    min_bucket = 1           # rows of the smallest decode step
 
     def __init__(self, hf_config, device, dtype: torch.dtype = torch.bfloat16, seed: Optional[int] = 0,
                  max_model_len: Optional[int] = None):
