@@ -28,6 +28,7 @@ from __future__ import annotations
 import asyncio
 import collections
 import dataclasses
+import gc
 import heapq
 import itertools
 import time
@@ -701,8 +702,18 @@ class ModelRunner:
         if self._pool is None:
             self._pool = torch.cuda.graph_pool_handle()
         graph = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(graph, pool=self._pool):
-            hidden = self._forward_hidden(inp)
+        # A cyclic collection inside the capture would destroy what a discarded engine left (its graphs,
+        # events, pinned buffers) with runtime calls that a capture forbids: an error in a destructor ends
+        # the process. So collect now, and not until the capture is over.
+        gc.collect()
+        collecting = gc.isenabled()
+        gc.disable()
+        try:
+            with torch.cuda.graph(graph, pool=self._pool):
+                hidden = self._forward_hidden(inp)
+        finally:
+            if collecting:
+                gc.enable()
         self._graphs[nb] = (graph, hidden)
         return self._graphs[nb]
 

@@ -403,6 +403,30 @@ def test_graph_replays_at_larger_layers(rows):
         torch.cuda.synchronize()
 
 
+def test_no_garbage_collection_inside_a_capture():
+    """A discarded engine's graphs must not be destroyed while another engine captures: with a collection
+    due at every allocation, none runs inside a capture."""
+    import gc
+
+    cfg = CONFIGS["plain"]
+    m, _ = build(cfg, torch.bfloat16)
+    prompts = [tokens_of(cfg, 5, 1)]
+    old = generate(m, prompts, 40, temperature=0.0, max_tokens=3, ignore_eos=True)[1]
+    old.cycle = old  # only the collector frees it
+    del old
+    phases, threshold = [], gc.get_threshold()
+    note = lambda phase, info: phases.append(torch.cuda.is_current_stream_capturing())  # noqa: E731
+    gc.callbacks.append(note)
+    gc.set_threshold(1, 1, 1)
+    try:
+        out, eng = generate(m, prompts, 40, temperature=0.0, max_tokens=3, ignore_eos=True)
+    finally:
+        gc.set_threshold(*threshold)
+        gc.callbacks.remove(note)
+    assert len(eng.runner._graphs) > 0 and len(out["response_ids"][0]) == 3
+    assert phases and not any(phases) and gc.isenabled()
+
+
 def test_steps_without_wanted_logits_keep_their_inputs():
     """Decode steps that fetch nothing run ahead of the host: their staged inputs must not be overwritten."""
     cfg = CONFIGS["plain"]
