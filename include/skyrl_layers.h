@@ -18,12 +18,20 @@ extern "C" {
 #endif
 
 /* ---- embedding, norms, activations, convolution state, logits ---------------------------------
- *   skyrl_embed     out f32 [n, H] = scale * table T [vocab, H] at tokens i64 [n].
+ *   skyrl_embed     out f32 [n, H] = scale * table T [vocab, H] at tokens i64 [n]. With turns f64 [(H + 1) / 2] the
+ *                   position's vector is added: sine (even columns) and cosine (odd) of positions[row] *
+ *                   turns[column / 2] revolutions. x T [n, H] (may be NULL): the same rounded.
  *   skyrl_add_norm  hidden f32 [n, H] += delta T [n, H] (may be NULL) and += step T [H] (may be
  *                   NULL: one vector for every row); out T [n, H] = norm(hidden) * (w_base + weight T [H]):
  *                   w_base 0 for a weight stored as it is, 1 for one stored as its distance from 1.
  *                   kind 0: layer norm without bias (mean taken off, variance = mean squared
  *                   deviation), 1: RMS norm; eps inside the root. H <= 8192.
+ *   skyrl_norm_add  for sublayers whose output is normed: with rms(v) = v / sqrt(mean(v^2) + eps) over a row of H,
+ *                   m = a T [n, H], or, with two outputs, share (rms(a) wa + rms(b) wb) (wa, wb T [H]); hidden f32 +=
+ *                   rms(m) * weight; out T = hidden, or rms(hidden) * final_weight if that is given. weight and
+ *                   final_weight T hold one number for all columns or H (weight_n, final_n). H <= 8192.
+ *   skyrl_xielu     out T [n, I] = ap x^2 + x / 2 for x > 0, an (exp(x) - 1 - x) + x / 2 otherwise, ap = softplus(p),
+ *                   an = 1/2 + softplus(q) from pq T [2].
  *   skyrl_gate_mul  out T [n, I] (row stride out_stride) from gate | up of gate_up T [n, 2I] (row stride
  *                   gu_stride): act 0: silu(gate) * up, 1: gelu(gate) * up in gelu's tanh form, 2: with
  *                   g = min(gate, limit) and u = up clamped to +-limit, g * sigmoid(alpha g) * (u + 1).
@@ -37,8 +45,13 @@ extern "C" {
 #define SKYRL_ACT_SILU 0
 #define SKYRL_ACT_GELU_TANH 1
 #define SKYRL_ACT_CLAMPED 2
-int skyrl_embed(const int64_t* tokens, const void* table, int64_t n, int32_t H, float scale, float* out, int32_t dtype,
-                void* stream);
+int skyrl_embed(const int64_t* tokens, const void* table, int64_t n, int32_t H, float scale, const int64_t* positions,
+                const double* turns, float* out, void* x, int32_t dtype, void* stream);
+int skyrl_norm_add(const void* a, const void* wa, const void* b, const void* wb, float share, float* hidden,
+                   const void* weight, int32_t weight_n, const void* final_weight, int32_t final_n, int32_t n,
+                   int32_t H, float eps, void* out, int32_t dtype, void* stream);
+int skyrl_xielu(const void* x, int64_t stride, int64_t n, int32_t I, const void* pq, void* out, int64_t out_stride,
+                int32_t dtype, void* stream);
 int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, float w_base, int32_t n,
                    int32_t H, float eps, int32_t kind, void* out, int32_t dtype, void* stream);
 int skyrl_gate_mul(const void* gate_up, int64_t gu_stride, int64_t n, int32_t I, int32_t act, float alpha, float limit,
@@ -200,6 +213,110 @@ int skyrl_diff_prefill(const skyrl_diff_shape* shape, const void* q, const void*
                        const void* k_cache, const void* v_cache, const int32_t* block_tables, int64_t bt_stride,
                        const int32_t* tiles, int32_t ntiles, const float* lambda, void* out, int64_t out_stride,
                        void* stream);
+
+/* ---- short convolutions of a prompt's tokens ---------------------------------------------------
+ * Causal convolution of columns [0, channels) of x T [T, stride] (conv_t f32 [taps, channels], last tap on the
+ * current token; inputs before the step from the ring as under skyrl_conv_save, zero before position 0), plus
+ * bias f32 [channels] (may be NULL), then the activation, at the tokens of chunks i32 [nchunks, 4] (first token,
+ * tokens <= 64, sequence, 0). Consecutive sections of the channels, each units x size, go to rows T [T, units,
+ * padded] and / or transposed to cols T [nchunks, units, padded, 64], zero past a chunk's end (either may be NULL;
+ * padding is not written). */
+#define SKYRL_CONV_NONE 0
+#define SKYRL_CONV_SILU 1
+typedef struct skyrl_conv_section {
+    int32_t units, size, padded;
+    void *rows, *cols;
+} skyrl_conv_section;
+int skyrl_conv_chunk(const void* x, int64_t stride, int32_t channels, int32_t taps, const float* conv_t,
+                     const float* bias, int32_t act, const int32_t* chunk, int32_t nchunks, const int32_t* cu,
+                     const int32_t* rows, const int64_t* positions, const void* ring,
+                     const skyrl_conv_section* sections, int32_t nsections, int32_t dtype, void* stream);
+
+/* ---- gated linear recurrence (RG-LRU) ----------------------------------------------------------
+ * proj T [T, proj_stride]: output gate y (width) | recurrence input (width). u = the input's short convolution
+ * plus bias. With u cut into `blocks` equal parts, r and i = sigmoid(W u + b) per part; log a = rate r; S <- a S +
+ * sqrt(1 - a^2) i u per channel; out = S gelu(y) (tanh form). gate_w T [blocks, 2 (r, i), np, kp] zero-padded (np, kp:
+ * a part's size up to a multiple of 16, of 32), gate_b f32 [2, width], rate f32 [width].
+ * State per row: S f32 [rows, width] and the convolution's ring T [rows, taps, width]. A sequence that starts at
+ * position 0 starts from zero, whatever the row holds.
+ *   skyrl_rglru_step    decode: token s is the one token of sequence s, row rows[s] (< 0: skipped).
+ *   skyrl_rglru_prompt  u T [T, width] from skyrl_conv_chunk; chunks as there, seq_chunks[i] .. seq_chunks[i + 1] - 1
+ *                       those of sequence seq0 + i. Scratch: hbuf, abuf f32 [T, width], s_in f32 [nchunks, width].
+ *                       skyrl_conv_save stores the ring. */
+int skyrl_rglru_step(const void* proj, int64_t proj_stride, int32_t width, int32_t blocks, int32_t taps,
+                     const float* conv_t, const float* conv_b, const void* gate_w, const float* gate_b,
+                     const float* rate, const int32_t* rows, const int64_t* positions, int32_t n, float* state,
+                     void* ring, void* out, int64_t out_stride, int32_t dtype, void* stream);
+int skyrl_rglru_prompt(const void* proj, int64_t proj_stride, int32_t width, int32_t blocks, const void* u,
+                       const void* gate_w, const float* gate_b, const float* rate, const int32_t* chunk,
+                       int32_t nchunks, const int32_t* seq_chunks, int32_t seq0, int32_t nseq, const int32_t* cu,
+                       const int32_t* rows, const int64_t* positions, float* state, float* hbuf, float* abuf,
+                       float* s_in, void* out, int64_t out_stride, int32_t dtype, void* stream);
+
+/* ---- grouped attention with normed queries and keys, a window and an output gate ---------------
+ * proj T [T, proj_stride]: q (heads x dim) | k (kv_heads x dim) | v (kv_heads x vdim). q and k are RMS-normed per
+ * head (weights T [dim]); out = softmax(scale q . k) v over the positions [max(0, pos - window + 1), pos] (window
+ * <= 0: all) times sigmoid(gate), gate T of the output's layout. Query head h reads key / value head h / (heads /
+ * kv_heads). dp = dim up to a multiple of 32, vp = vdim to one of 16: queries T [T, heads, dp], keys T [num_blocks,
+ * kv_heads, 16, dp], values transposed T [num_blocks, kv_heads, vp, 16]; padding must hold zeros and is not
+ * written. slot = block * 16 + offset; token t belongs to row bt_row[t] of block_tables.
+ *   skyrl_attn_write    tokens [first, first + count), or, with runs i32 [count, 2] (first token, tokens <= 8 of one
+ *                       sequence whose slots lie in one half of a block; bf16, dim and vdim multiples of 8), those.
+ *                       Keys and values go to slots[t] (< 0: no write).
+ *   skyrl_attn_attend   one query row per token. nparts waves share a token's keys (MFMA form, bf16), each at least
+ *                       part_min >= 16 keys, a multiple of 16; nparts > 1 needs skyrl_attn_attend_workspace_bytes. f32,
+ *                       and shapes outside the MFMA form (skyrl_attn_mfma == 0), take a plain kernel and ignore nparts.
+ *   skyrl_attn_prefill  prompt form (bf16, skyrl_attn_mfma != 0): one workgroup per (tile, head); tiles i32 [ntiles, 4]:
+ *                       first token, token count (<= 128), position of the first token, row of block_tables. */
+typedef struct skyrl_attn_shape {
+    int32_t heads, kv_heads, dim, vdim, window;
+    float scale, eps;
+} skyrl_attn_shape;
+int skyrl_attn_write(const skyrl_attn_shape* shape, const void* proj, int64_t proj_stride, const void* q_norm,
+                     const void* k_norm, const int64_t* slots, const int32_t* runs, int32_t first, int32_t count,
+                     void* q, void* k_cache, void* v_cache, int32_t dtype, void* stream);
+int skyrl_attn_mfma(const skyrl_attn_shape* shape, int32_t dtype);
+size_t skyrl_attn_attend_workspace_bytes(const skyrl_attn_shape* shape, int32_t T, int32_t nparts);
+int skyrl_attn_attend(const skyrl_attn_shape* shape, const void* q, const void* gate, int64_t gate_stride,
+                      const void* k_cache, const void* v_cache, const int32_t* block_tables, int64_t bt_stride,
+                      const int32_t* bt_row, const int64_t* positions, int32_t T, int32_t part_min, int32_t nparts,
+                      void* out, int64_t out_stride, void* workspace, int32_t dtype, void* stream);
+int skyrl_attn_prefill(const skyrl_attn_shape* shape, const void* q, const void* gate, int64_t gate_stride,
+                       const void* k_cache, const void* v_cache, const int32_t* block_tables, int64_t bt_stride,
+                       const int32_t* tiles, int32_t ntiles, void* out, int64_t out_stride, void* stream);
+
+/* ---- state space mixer (Mamba-2) ----------------------------------------------------------------
+ * proj T [T, proj_stride]: z (heads x vdim) | x (heads x vdim) | B (groups x state) | C (groups x state) | dt
+ * (heads). x, B and C pass a short convolution with bias and silu. Head h with group h / (heads / groups): dt =
+ * softplus(dt + dt_bias); S <- exp(-exp(A_log) dt) S + dt B x^T; y = S^T C + skip x.
+ * State per row: S f32 [rows, heads, state, ppad], ppad = vdim up to a multiple of 4, and the convolution's ring T
+ * [rows, taps, heads vdim + 2 groups state]. A sequence that starts at position 0 starts from zero.
+ *   skyrl_ssd_scan    token by token over each sequence's tokens [cu[s], cu[s+1]) (row rows[s] < 0: skipped); y T.
+ *                     save_conv 1 also stores the convolution inputs and needs every sequence to have one token;
+ *                     otherwise skyrl_conv_save follows.
+ *   skyrl_ssd_prompt  bf16, state <= 256, from skyrl_conv_chunk's outputs: xt [nchunks, heads, vp, 64], bt [nchunks,
+ *                     groups, np, 64], brow and crow [T, groups, np] (vp, np: vdim, state up to a multiple of 16, of
+ *                     32; padding zero). super i32 [nsuper, 4]: first chunk, chunks, sequence, 1 if the sequence has
+ *                     several such runs + 2 if its last; pick i32 [npick]: the runs that are followed by another of
+ *                     their sequence; chain i32 [nchain, 2]: first run and number of runs of the sequences with
+ *                     several. Scratch: runs f32 [nsuper, heads, np, vp], gtot f32 [nsuper, heads].
+ *   skyrl_gated_norm  out T [n, width] = rms over each of `groups` equal parts of y silu(z), times weight T [width]. */
+typedef struct skyrl_ssd_shape {
+    int32_t heads, vdim, state, groups, taps;
+} skyrl_ssd_shape;
+int skyrl_ssd_scan(const skyrl_ssd_shape* shape, const void* proj, int64_t proj_stride, const float* conv_t,
+                   const float* conv_b, const float* a_log, const float* dt_bias, const float* skip, const int32_t* cu,
+                   const int32_t* rows, const int64_t* positions, int32_t nseq, float* state, void* ring,
+                   int32_t save_conv, void* y, int64_t y_stride, int32_t dtype, void* stream);
+int skyrl_ssd_prompt(const skyrl_ssd_shape* shape, const void* xt, const void* bt, const void* brow, const void* crow,
+                     const void* dt_raw, int64_t dt_stride, const float* a_log, const float* dt_bias,
+                     const float* skip, const int32_t* chunk, const int32_t* super, int32_t nsuper,
+                     const int32_t* pick, int32_t npick, const int32_t* chain, int32_t nchain, const int32_t* cu,
+                     const int32_t* rows, const int64_t* positions, float* state, float* runs, float* gtot, void* y,
+                     int64_t y_stride, void* stream);
+int skyrl_gated_norm(const void* y, int64_t y_stride, const void* z, int64_t z_stride, const void* weight, int64_t n,
+                     int32_t width, int32_t groups, float eps, void* out, int64_t out_stride, int32_t dtype,
+                     void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,6 +1,7 @@
 """Plain CPU restatement of the hybrid decoders (Dovidra: latent attention + gated delta rule layers;
-Lipedra: differential attention in parallel layers), one function per mechanism, whole sequences at a
-time, in the dtype of its weights (float64 in the tests).
+Lipedra: differential attention in parallel layers; Foduzen: gated linear recurrences, and windowed
+attention beside a state space mixer, behind norms of the sublayers' outputs), one function per mechanism,
+whole sequences at a time, in the dtype of its weights (float64 in the tests).
 Test infrastructure only: nothing under skyrl_amd/ imports it and it shares no code with it.
 
 `w` maps tensor names to CPU tensors; `cfg` is the parsed config.json.
@@ -208,6 +209,127 @@ def clamped_ff(h, w, p, limit):
     return (g * torch.sigmoid(1.702 * g) * (u + 1)) @ w[p + "down"].T + w[p + "down.b"]
 
 
+def softplus(z):
+    return torch.where(z > 0, z, torch.zeros_like(z)) + torch.log1p(torch.exp(-z.abs()))
+
+
+def rms(x, eps):
+    """x over its root mean square (last dimension)."""
+    return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+
+def sinusoid(positions, width, base=10000.0):
+    """Position vectors [T, width]: sines on the even entries, cosines of the same angle after them."""
+    out = torch.zeros(len(positions), width, dtype=torch.float64)
+    for e in range(width):
+        a = positions.double() * base ** (-(e - e % 2) / width)
+        out[:, e] = torch.cos(a) if e % 2 else torch.sin(a)
+    return out
+
+
+def block_gates(u, w, name):
+    """Sigmoid of a block-diagonal affine map: block b of u times the matrix w[name][b] [out, in]."""
+    blocks, size = w[name].shape[0], w[name].shape[1]
+    out = torch.zeros_like(u)
+    for b in range(blocks):
+        cols = slice(b * size, (b + 1) * size)
+        out[:, cols] = torch.sigmoid(u[:, cols] @ w[name][b].T + w[name + ".b"][b])
+    return out
+
+
+def gated_linear_recurrence(u, r, i, lam, state=None):
+    """S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t per channel, log a = -8 r softplus(lam); all states [T, C]."""
+    log_a = -8.0 * r * softplus(lam)
+    a, into = torch.exp(log_a), torch.sqrt(-torch.expm1(2 * log_a)) * i * u
+    S = torch.zeros(u.shape[1], dtype=u.dtype) if state is None else state.clone()
+    out = torch.zeros_like(u)
+    for t in range(u.shape[0]):
+        S = a[t] * S + into[t]
+        out[t] = S
+    return out
+
+
+def rglru_mixer(h, w, p):
+    y = gelu_tanh(h @ w[p + "y"].T + w[p + "y.b"])
+    u = short_conv(h @ w[p + "x"].T + w[p + "x.b"], w[p + "conv"]) + w[p + "conv.b"]
+    S = gated_linear_recurrence(u, block_gates(u, w, p + "ra"), block_gates(u, w, p + "ri"), w[p + "lam"])
+    return (S * y) @ w[p + "o"].T
+
+
+def gated_window_attention(h, w, p, m, eps):
+    """Normed queries and keys, no rotation, a sliding window, an elementwise output gate."""
+    T, H, G, D, V = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    proj = lambda n: h @ w[p + n].T + w[p + n + ".b"]  # noqa: E731
+    q = rms_norm(proj("q").view(T, H, D), w[p + "q.norm"], eps)
+    k = rms_norm(proj("k").view(T, G, D), w[p + "k.norm"], eps)
+    group = torch.tensor([hh // (H // G) for hh in range(H)])
+    size = m["mask"]["size"] if m.get("mask") else None
+    o = window_attention(q, k[:, group], proj("v").view(T, G, V)[:, group], m["scale"], size).reshape(T, H * V)
+    return (o * torch.sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T + w[p + "o.b"]
+
+
+def state_space_recurrence(x, B, C, dt, A_log, D, state=None):
+    """x [T, H, P], B and C [T, H, N], dt [T, H] -> y [T, H, P] and the final state [H, N, P]."""
+    T, H, P = x.shape
+    S = torch.zeros(H, B.shape[-1], P, dtype=x.dtype) if state is None else state.clone()
+    y = torch.zeros_like(x)
+    for t in range(T):
+        for h in range(H):
+            decay = torch.exp(-torch.exp(A_log[h]) * dt[t, h])
+            S[h] = decay * S[h] + dt[t, h] * torch.outer(B[t, h], x[t, h])
+            y[t, h] = S[h].T @ C[t, h] + D[h] * x[t, h]
+    return y, S
+
+
+def grouped_gated_norm(y, z, weight, groups, eps):
+    """rms over each of `groups` equal parts of y silu(z), times the weight."""
+    T, n = y.shape
+    return rms((y * silu(z)).view(T, groups, n // groups), eps).view(T, n) * weight
+
+
+def state_space_mixer(h, w, p, m, eps):
+    T, H, P, N, G = h.shape[0], m["heads"], m["vdim"], m["state"], m["groups"]
+    inner = H * P
+    u = h @ w[p + "in"].T
+    z, xbc, dt = u[:, :inner], u[:, inner:2 * inner + 2 * G * N], u[:, 2 * inner + 2 * G * N:]
+    xbc = silu(short_conv(xbc, w[p + "conv"]) + w[p + "conv.b"])
+    group = torch.tensor([hh // (H // G) for hh in range(H)])
+    x = xbc[:, :inner].view(T, H, P)
+    B = xbc[:, inner:inner + G * N].view(T, G, N)[:, group]
+    C = xbc[:, inner + G * N:].view(T, G, N)[:, group]
+    y, _ = state_space_recurrence(x, B, C, softplus(dt + w[p + "dt_bias"]), w[p + "A_log"], w[p + "D"])
+    y = grouped_gated_norm(y.reshape(T, inner), z, w[p + "norm"], m["norm_groups"], eps)
+    return y @ w[p + "o"].T
+
+
+def side_by_side(left, right, w, p, eps):
+    """Half the sum of two mixers' outputs, each normed over the model width."""
+    return (rms_norm(left, w[p + "left.out"], eps) + rms_norm(right, w[p + "right.out"], eps)) / 2
+
+
+def xielu(z, p, q):
+    neg = torch.where(z > 0, torch.zeros_like(z), z)
+    return torch.where(z > 0, softplus(p) * z * z, (0.5 + softplus(q)) * (torch.expm1(neg) - neg)) + z / 2
+
+
+def xielu_ff(h, w, p):
+    return xielu(h @ w[p + "up"].T, *w[p + "act"]) @ w[p + "down"].T
+
+
+def output_norm_layer(x, w, i, entry, eps):
+    """Foduzen: each sublayer reads the residual and its output is normed (one number as the weight)."""
+    p, m = f"l{i}.", entry["mixer"]
+    if entry["type"] == "rglru":
+        y = rglru_mixer(x, w, p + "mix.")
+    else:
+        y = side_by_side(gated_window_attention(x, w, p + "mix.left.", m["left"], eps),
+                         state_space_mixer(x, w, p + "mix.right.", m["right"], eps), w, p + "mix.", eps)
+    x = x + rms_norm(y, w[p + "norm1"], eps)
+    if entry.get("mlp"):
+        x = x + rms_norm(xielu_ff(x, w, p + "mlp."), w[p + "norm2"], eps)
+    return x
+
+
 def layer(x, w, i, entry, eps):
     """Dovidra: two halves, each behind a norm of its own."""
     p = f"l{i}."
@@ -245,19 +367,24 @@ def layer_runs(cfg):
 
 def forward(tokens, w, cfg):
     """Logits [T, vocab] and the residual after every layer run [runs, T, width]."""
-    eps = cfg["norm"]["eps"]
-    parallel = cfg["architecture"] == "Lipedra"
+    eps, design = cfg["norm"]["eps"], cfg["architecture"]
     x = w["embed"][torch.as_tensor(tokens)]
-    if parallel:
+    if design != "Dovidra":
         x = x * cfg["embedding"]["scale"]
+    if design == "Foduzen":
+        x = x + sinusoid(torch.arange(len(tokens)), cfg["width"]).to(x.dtype)
     trail, kvs = [], {}
     for i, t in layer_runs(cfg):
         if t is not None:
             x = x + w["loop.step"][t]
         e = cfg["layers"][i]
-        x = parallel_layer(x, w, i, e, eps, kvs) if parallel else layer(x, w, i, e, eps)
+        if design == "Lipedra":
+            x = parallel_layer(x, w, i, e, eps, kvs)
+        else:
+            x = (output_norm_layer if design == "Foduzen" else layer)(x, w, i, e, eps)
         trail.append(x)
-    logits = (rms_norm_about_one if parallel else layer_norm)(x, w["final.norm"], eps) @ w["head"].T
+    norm = {"Dovidra": layer_norm, "Lipedra": rms_norm_about_one, "Foduzen": rms_norm}[design]
+    logits = norm(x, w["final.norm"], eps) @ w["head"].T
     cap = cfg.get("logit_softcap")
     if cap:
         logits = cap * torch.tanh(logits / cap)

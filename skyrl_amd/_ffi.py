@@ -237,11 +237,35 @@ class DiffShape(ctypes.Structure):
         (n, ctypes.c_float) for n in ("scale", "diff", "eps")]
 
 
+class ConvSection(ctypes.Structure):
+    """Mirror of ``skyrl_conv_section`` (include/skyrl_layers.h)."""
+
+    _fields_ = [(n, ctypes.c_int32) for n in ("units", "size", "padded")] + [
+        (n, ctypes.c_void_p) for n in ("rows", "cols")]
+
+
+class AttnShape(ctypes.Structure):
+    """Mirror of ``skyrl_attn_shape`` (include/skyrl_layers.h)."""
+
+    _fields_ = [(n, ctypes.c_int32) for n in ("heads", "kv_heads", "dim", "vdim", "window")] + [
+        (n, ctypes.c_float) for n in ("scale", "eps")]
+
+
+class SSDShape(ctypes.Structure):
+    """Mirror of ``skyrl_ssd_shape`` (include/skyrl_layers.h)."""
+
+    _fields_ = [(n, ctypes.c_int32) for n in ("heads", "vdim", "state", "groups", "taps")]
+
+
 # the exported surface of include/skyrl_layers.h, in a library of its own (libskyrl_layers.so)
 _DS = ctypes.POINTER(DeltaShape)
 _FS = ctypes.POINTER(DiffShape)
+_AS = ctypes.POINTER(AttnShape)
+_SS = ctypes.POINTER(SSDShape)
 LAYERS_SIGNATURES = {
-    "skyrl_embed": (_INT, [_P, _P, _I64, _I32, _F, _P, _I32, _P]),
+    "skyrl_embed": (_INT, [_P, _P, _I64, _I32, _F, _P, _P, _P, _P, _I32, _P]),
+    "skyrl_norm_add": (_INT, [_P, _P, _P, _P, _F, _P, _P, _I32, _P, _I32, _I32, _I32, _F, _P, _I32, _P]),
+    "skyrl_xielu": (_INT, [_P, _I64, _I64, _I32, _P, _P, _I64, _I32, _P]),
     "skyrl_add_norm": (_INT, [_P, _P, _P, _P, _F, _I32, _I32, _F, _I32, _P, _I32, _P]),
     "skyrl_gate_mul": (_INT, [_P, _I64, _I64, _I32, _I32, _F, _F, _P, _I64, _I32, _P]),
     "skyrl_conv_save": (_INT, [_P, _I64, _I32, _I32, _P, _P, _P, _I32, _P, _I32, _P]),
@@ -266,6 +290,21 @@ LAYERS_SIGNATURES = {
     "skyrl_diff_attend": (_INT, [_FS, _P, _P, _I64, _P, _P, _P, _I64, _P, _P, _I32, _P, _I32, _I32, _P, _I64, _P, _I32,
                                  _P]),
     "skyrl_diff_prefill": (_INT, [_FS, _P, _P, _I64, _P, _P, _P, _I64, _P, _I32, _P, _P, _I64, _P]),
+    "skyrl_conv_chunk": (_INT, [_P, _I64, _I32, _I32, _P, _P, _I32, _P, _I32, _P, _P, _P, _P,
+                                ctypes.POINTER(ConvSection), _I32, _I32, _P]),
+    "skyrl_rglru_step": (_INT, [_P, _I64, _I32, _I32, _I32, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _I64, _I32,
+                                _P]),
+    "skyrl_rglru_prompt": (_INT, [_P, _I64, _I32, _I32, _P, _P, _P, _P, _P, _I32, _P, _I32, _I32, _P, _P, _P, _P, _P,
+                                  _P, _P, _P, _I64, _I32, _P]),
+    "skyrl_attn_write": (_INT, [_AS, _P, _I64, _P, _P, _P, _P, _I32, _I32, _P, _P, _P, _I32, _P]),
+    "skyrl_attn_mfma": (_INT, [_AS, _I32]),
+    "skyrl_attn_attend_workspace_bytes": (_SZ, [_AS, _I32, _I32]),
+    "skyrl_attn_attend": (_INT, [_AS, _P, _P, _I64, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _I64, _P, _I32, _P]),
+    "skyrl_attn_prefill": (_INT, [_AS, _P, _P, _I64, _P, _P, _P, _I64, _P, _I32, _P, _I64, _P]),
+    "skyrl_ssd_scan": (_INT, [_SS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I32, _P, _I64, _I32, _P]),
+    "skyrl_ssd_prompt": (_INT, [_SS, _P, _P, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I32, _P, _I32, _P, _I32, _P, _P, _P,
+                                _P, _P, _P, _P, _I64, _P]),
+    "skyrl_gated_norm": (_INT, [_P, _I64, _P, _I64, _P, _I64, _I32, _I32, _F, _P, _I64, _I32, _P]),
 }
 
 # entry points with a per-call variant form (name + "_ex": the same arguments, then the variant)

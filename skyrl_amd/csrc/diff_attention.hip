@@ -17,19 +17,14 @@
 // A map's running maximum is only raised when the scores outgrow it by kSlack, so that the sums are rescaled
 // at the first tile and seldom after.
 #include "conv.h"
+#include "paged.h"
 
 namespace skyrl {
 namespace {
 
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-typedef short s16x8 __attribute__((ext_vector_type(8)));
-typedef float f32x4 __attribute__((ext_vector_type(4)));
-
-constexpr int kBS = 16;  // tokens per cache block
 constexpr int kNT = 256;
 constexpr int kGroup = 8;  // query heads per decode wave
 constexpr int kRun = 8;    // tokens per thread of the prompt's write
-constexpr float kLog2e = 1.4426950408889634f;
 
 struct Dims {
     int H, G, D, V, rot, taps, kv;
@@ -42,34 +37,6 @@ struct Dims {
     __host__ __device__ int R() const { return H / G; }
     __host__ __device__ int groups() const { return (R() + kGroup - 1) / kGroup; }
 };
-
-template <typename T, int VEC>
-__device__ __forceinline__ void ldv(const T* p, float (&o)[VEC]) {
-    if constexpr (VEC == 1) {
-        o[0] = ld(p);
-    } else {
-        static_assert(VEC == 8);
-        const float4 a = ld4(p), b = ld4(p + 4);
-        o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w;
-        o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
-    }
-}
-__device__ __forceinline__ void st8(float* p, const float (&v)[8]) {
-    st4(p, make_float4(v[0], v[1], v[2], v[3]));
-    st4(p + 4, make_float4(v[4], v[5], v[6], v[7]));
-}
-__device__ __forceinline__ void st8(uint16_t* p, const float (&v)[8]) {
-    *reinterpret_cast<uint4*>(p) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]),
-                                              pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
-}
-__device__ __forceinline__ void unpack8(uint4 x, float (&o)[8]) {
-    const uint32_t w[4] = {x.x, x.y, x.z, x.w};
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        o[2 * i] = __uint_as_float(w[i] << 16);
-        o[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
-    }
-}
 
 // Where a channel goes: 0 query, 1 key, 2 value; head; column d of map `map`.
 struct Place {
@@ -103,53 +70,6 @@ __device__ __forceinline__ void rotate8(float (&y)[8], int d, int rot, const flo
             const float c = cs[(d + i) / 2], s = cs[h2 + (d + i) / 2], u = y[i], v = y[i + 1];
             y[i] = u * c - v * s;
             y[i + 1] = v * c + u * s;
-        }
-    }
-}
-
-// Convolution of VEC channels at one token; x0: the token's own inputs.
-template <typename T, int VEC>
-__device__ __forceinline__ void conv_at(const T* __restrict__ proj, int64_t stride, const float* __restrict__ conv_t,
-                                        const T* __restrict__ ring, int channels, int taps, int ch, int t, int t0,
-                                        int pos, float (&y)[VEC], float (&x0)[VEC]) {
-    constexpr int W = 4;
-    const int r = pos % taps;
-    auto input = [&](int back, float (&x)[VEC]) {
-        if (t - back >= t0) {
-            ldv<T, VEC>(proj + (int64_t)(t - back) * stride + ch, x);
-        } else {
-            const int slot = r - back < 0 ? r - back + taps : r - back;
-            ldv<T, VEC>(ring + (int64_t)slot * channels + ch, x);
-        }
-    };
-#pragma unroll
-    for (int i = 0; i < VEC; ++i) y[i] = 0.f;
-    if (taps <= W) {
-        float x[W][VEC], f[W][VEC];
-#pragma unroll
-        for (int back = 0; back < W; ++back) {
-            if (back < taps && back <= pos) {
-                input(back, x[back]);
-                ldv<float, VEC>(conv_t + (int64_t)(taps - 1 - back) * channels + ch, f[back]);
-            } else {
-#pragma unroll
-                for (int i = 0; i < VEC; ++i) x[back][i] = f[back][i] = 0.f;
-            }
-        }
-#pragma unroll
-        for (int back = 0; back < W; ++back)
-#pragma unroll
-            for (int i = 0; i < VEC; ++i) y[i] += x[back][i] * f[back][i];
-#pragma unroll
-        for (int i = 0; i < VEC; ++i) x0[i] = x[0][i];
-    } else {
-        input(0, x0);
-        for (int back = 0; back < taps && back <= pos; ++back) {
-            float x[VEC], f[VEC];
-            input(back, x);
-            ldv<float, VEC>(conv_t + (int64_t)(taps - 1 - back) * channels + ch, f);
-#pragma unroll
-            for (int i = 0; i < VEC; ++i) y[i] += x[i] * f[i];
         }
     }
 }
@@ -380,27 +300,6 @@ __global__ __launch_bounds__(kNT) void diff_attend_plain_kernel(
         const int e = threadIdx.x + a * kNT;
         if (e < d.V) st(out + (int64_t)t * out_stride + (int64_t)h * d.V + e, acc[0][a] * r);
     }
-}
-
-// Four consecutive outputs of a head from column e on.
-__device__ __forceinline__ void store4(uint16_t* orow, int e, int V, bool vec, const float (&v)[4]) {
-    if (vec && e + 4 <= V) {
-        *reinterpret_cast<uint2*>(orow + e) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
-    } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-            if (e + i < V) orow[e + i] = f32_to_bf16(v[i]);
-    }
-}
-__device__ __forceinline__ bool out_vec(const uint16_t* out, int64_t out_stride, int V) {
-    return V % 4 == 0 && out_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0;
-}
-
-// A context of ctx tokens over at most nparts waves, each share a multiple of 16 and at least part_min tokens.
-__device__ __forceinline__ void ctx_split(int ctx, int part_min, int nparts, int& part, int& np) {
-    const int p = ((ctx + nparts - 1) / nparts + kBS - 1) / kBS * kBS;
-    part = max(p, part_min);
-    np = (ctx + part - 1) / part;
 }
 
 // ---- decode form ----------------------------------------------------------------------------------
@@ -825,7 +724,6 @@ const char* bad_shape(const skyrl_diff_shape* sh) {
 Dims dims_of(const skyrl_diff_shape* s) {
     return Dims{s->heads, s->kv_heads, s->dim, s->vdim, s->rot_dims, s->taps, s->kv, s->scale, s->diff, s->eps};
 }
-bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
 bool wide(const Dims& d, const void* proj, int64_t stride) {  // every piece of eight channels is one head's and aligned
     return d.D % 8 == 0 && d.V % 8 == 0 && stride % 8 == 0 && aligned16(proj);

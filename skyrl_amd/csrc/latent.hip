@@ -26,7 +26,6 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int kBS = 16;  // tokens per cache block
 constexpr int kNT = 256;
-constexpr float kLog2e = 1.4426950408889634f;
 
 template <typename T>
 __global__ __launch_bounds__(kNT) void latent_write_kernel(T* __restrict__ proj, int64_t stride, int heads, int dim,
@@ -636,7 +635,6 @@ __global__ __launch_bounds__(512 / QT) __attribute__((amdgpu_waves_per_eu(2))) v
     }
 }
 
-bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
 }  // namespace
 }  // namespace skyrl

@@ -74,6 +74,126 @@ __global__ __launch_bounds__(kNT) void add_norm_kernel(const T* __restrict__ del
     }
 }
 
+// Norms of sublayer outputs added to the residual. Up to two outputs per row; the row in registers: kMaxV
+// groups of VEC elements per thread.
+template <typename T>
+struct NormAdd {
+    const T *a, *wa, *b, *wb;  // b, wa, wb: only with two outputs
+    float share;
+    float* h;
+    const T* g;
+    int gs;  // 0: g is one number, 1: a vector
+    const T* gf;
+    int fs;
+    T* out;
+    int H;
+    float eps;
+};
+
+template <typename T, int VEC>
+__device__ __forceinline__ void ldw(const T* p, float (&o)[VEC]) {
+    if constexpr (VEC == 4) {
+        const float4 v = ld4(p);
+        o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
+    } else {
+        o[0] = ld(p);
+    }
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void stw(T* p, const float (&v)[VEC]) {
+    if constexpr (VEC == 4) st4(p, make_float4(v[0], v[1], v[2], v[3]));
+    else st(p, v[0]);
+}
+// A weight's VEC values at element e: a vector's, or one number.
+template <typename T, int VEC>
+__device__ __forceinline__ void weights_at(const T* w, int step, int e, float (&o)[VEC]) {
+    if (step) {
+        ldw<T, VEC>(w + e, o);
+    } else {
+        const float x = ld(w);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) o[j] = x;
+    }
+}
+
+template <typename T, int VEC, int kMaxV, bool PAIR>
+__global__ __launch_bounds__(kNT) void norm_add_kernel(NormAdd<T> p) {
+    __shared__ float s_red[kNT / kWave];
+    const int64_t base = (int64_t)blockIdx.x * p.H;
+    const int nv = p.H / VEC;
+    float a[kMaxV][VEC], b[PAIR ? kMaxV : 1][VEC], h[kMaxV][VEC];
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int k = 0; k < kMaxV; ++k) {
+        const int v = threadIdx.x + k * kNT;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            a[k][j] = h[k][j] = 0.f;
+            if constexpr (PAIR) b[k][j] = 0.f;
+        }
+        if (v < nv) {
+            ldw<T, VEC>(p.a + base + VEC * v, a[k]);
+            if constexpr (PAIR) ldw<T, VEC>(p.b + base + VEC * v, b[k]);
+            ldw<float, VEC>(p.h + base + VEC * v, h[k]);
+        }
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            sa += a[k][j] * a[k][j];
+            if constexpr (PAIR) sb += b[k][j] * b[k][j];
+        }
+    }
+    float r = 1.f / sqrtf(block_total<kNT>(sa, s_red) / (float)p.H + p.eps);
+    if constexpr (PAIR) {
+        const float rb = 1.f / sqrtf(block_total<kNT>(sb, s_red) / (float)p.H + p.eps);
+        float ss = 0.f;
+#pragma unroll
+        for (int k = 0; k < kMaxV; ++k) {
+            const int v = threadIdx.x + k * kNT;
+            if (v < nv) {
+                float wa[VEC], wb[VEC];
+                ldw<T, VEC>(p.wa + VEC * v, wa);
+                ldw<T, VEC>(p.wb + VEC * v, wb);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) {
+                    a[k][j] = p.share * (a[k][j] * r * wa[j] + b[k][j] * rb * wb[j]);
+                    ss += a[k][j] * a[k][j];
+                }
+            }
+        }
+        r = 1.f / sqrtf(block_total<kNT>(ss, s_red) / (float)p.H + p.eps);
+    }
+    float sh = 0.f;
+#pragma unroll
+    for (int k = 0; k < kMaxV; ++k) {
+        const int v = threadIdx.x + k * kNT;
+        if (v < nv) {
+            float g[VEC];
+            weights_at<T, VEC>(p.g, p.gs, VEC * v, g);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) {
+                h[k][j] += a[k][j] * r * g[j];
+                sh += h[k][j] * h[k][j];
+            }
+            stw<float, VEC>(p.h + base + VEC * v, h[k]);
+        }
+    }
+    float rf = 1.f;
+    if (p.gf) rf = 1.f / sqrtf(block_total<kNT>(sh, s_red) / (float)p.H + p.eps);
+#pragma unroll
+    for (int k = 0; k < kMaxV; ++k) {
+        const int v = threadIdx.x + k * kNT;
+        if (v < nv) {
+            if (p.gf) {
+                float g[VEC];
+                weights_at<T, VEC>(p.gf, p.fs, VEC * v, g);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) h[k][j] *= rf * g[j];
+            }
+            stw<T, VEC>(p.out + base + VEC * v, h[k]);
+        }
+    }
+}
+
 struct Gate {
     int act;
     float alpha, limit;  // of the clamped form
@@ -109,10 +229,47 @@ __global__ __launch_bounds__(kNT) void gate_mul_kernel(const T* __restrict__ gu,
     }
 }
 
-// out[row] = scale * table[tokens[row]], f32.
+// xIELU with the learned pair (p, q): ap = softplus(p), an = 1/2 + softplus(q).
+template <typename T>
+__device__ __forceinline__ float xielu(float z, float ap, float an) {
+    const float zn = fminf(z, 0.f);
+    float em;
+    if constexpr (sizeof(T) == 2) em = exp_<T>(zn) - 1.f;
+    else em = expm1f(zn);
+    return (z > 0.f ? ap * z * z : an * (em - zn)) + 0.5f * z;
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(kNT) void xielu_kernel(const T* __restrict__ x, int64_t stride, int64_t n, int I,
+                                                    const T* __restrict__ pq, T* __restrict__ out,
+                                                    int64_t out_stride) {
+    const float ap = softplusf_(ld(pq)), an = 0.5f + softplusf_(ld(pq + 1));
+    const int iv = I / VEC;
+    const int64_t total = n * iv;
+    for (int64_t e = (int64_t)blockIdx.x * kNT + threadIdx.x; e < total; e += (int64_t)gridDim.x * kNT) {
+        const int64_t row = e / iv;
+        const int c = (int)(e - row * iv) * VEC;
+        float v[VEC];
+        ldv<T, VEC>(x + row * stride + c, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[j] = xielu<T>(v[j], ap, an);
+        stv(out + row * out_stride + c, v);
+    }
+}
+
+// Sine and cosine of pos * turns revolutions: the revolution's fraction is formed in f64.
+__device__ __forceinline__ void position_pair(int64_t pos, double turns, float& s, float& c) {
+    const double x = (double)pos * turns;
+    sincospif(2.f * (float)(x - rint(x)), &s, &c);
+}
+
+// out[row] = scale * table[tokens[row]] (+ the position's vector), f32; x the same as T.
 template <typename T, int VEC>
 __global__ __launch_bounds__(kNT) void embed_kernel(const int64_t* __restrict__ tokens, const T* __restrict__ table,
-                                                    int64_t n, int H, float scale, float* __restrict__ out) {
+                                                    int64_t n, int H, float scale,
+                                                    const int64_t* __restrict__ positions,
+                                                    const double* __restrict__ turns, float* __restrict__ out,
+                                                    T* __restrict__ x) {
     const int hv = H / VEC;
     const int64_t total = n * hv;
     for (int64_t e = (int64_t)blockIdx.x * kNT + threadIdx.x; e < total; e += (int64_t)gridDim.x * kNT) {
@@ -121,9 +278,28 @@ __global__ __launch_bounds__(kNT) void embed_kernel(const int64_t* __restrict__ 
         const T* src = table + tokens[row] * H + c;
         if constexpr (VEC == 4) {
             const float4 a = ld4(src);
-            st4(out + row * H + c, make_float4(a.x * scale, a.y * scale, a.z * scale, a.w * scale));
+            float4 v = make_float4(a.x * scale, a.y * scale, a.z * scale, a.w * scale);
+            if (turns) {
+                const int64_t pos = positions[row];
+                float s, k;
+                position_pair(pos, turns[c / 2], s, k);
+                v.x += s;
+                v.y += k;
+                position_pair(pos, turns[c / 2 + 1], s, k);
+                v.z += s;
+                v.w += k;
+            }
+            st4(out + row * H + c, v);
+            if (x) st4(x + row * H + c, v);
         } else {
-            out[row * H + c] = ld(src) * scale;
+            float v = ld(src) * scale;
+            if (turns) {
+                float s, k;
+                position_pair(positions[row], turns[c / 2], s, k);
+                v += c & 1 ? k : s;
+            }
+            out[row * H + c] = v;
+            if (x) st(x + row * H + c, v);
         }
     }
 }
@@ -216,22 +392,72 @@ extern "C" int skyrl_gate_mul(const void* gate_up, int64_t gu_stride, int64_t n,
     return check_launch("gate_mul_kernel");
 }
 
-extern "C" int skyrl_embed(const int64_t* tokens, const void* table, int64_t n, int32_t H, float scale, float* out,
-                           int32_t dtype, void* stream) {
+extern "C" int skyrl_embed(const int64_t* tokens, const void* table, int64_t n, int32_t H, float scale,
+                           const int64_t* positions, const double* turns, float* out, void* x, int32_t dtype,
+                           void* stream) {
     SKYRL_REQUIRE_T(dtype, "embed");
     SKYRL_REQUIRE(n >= 0 && H > 0, "embed: bad sizes");
     if (n == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(tokens && table && out, "embed: null pointer");
+    SKYRL_REQUIRE(tokens && table && out && (positions || !turns), "embed: null pointer");
     SKYRL_DISPATCH_T(dtype, {
         const T* w = reinterpret_cast<const T*>(table);
+        T* xo = reinterpret_cast<T*>(x);
         if (H % 4 == 0)
             hipLaunchKernelGGL((embed_kernel<T, 4>), dim3(grid_for(n * (H / 4))), dim3(kNT), 0, as_stream(stream),
-                               tokens, w, n, H, scale, out);
+                               tokens, w, n, H, scale, positions, turns, out, xo);
         else
             hipLaunchKernelGGL((embed_kernel<T, 1>), dim3(grid_for(n * H)), dim3(kNT), 0, as_stream(stream), tokens, w,
-                               n, H, scale, out);
+                               n, H, scale, positions, turns, out, xo);
     })
     return check_launch("embed_kernel");
+}
+
+#define LAUNCH_NORM_ADD(V, K)                                                                                   if (b) hipLaunchKernelGGL((norm_add_kernel<T, V, K, true>), dim3(n), dim3(kNT), 0, as_stream(stream), p);     else hipLaunchKernelGGL((norm_add_kernel<T, V, K, false>), dim3(n), dim3(kNT), 0, as_stream(stream), p)
+
+extern "C" int skyrl_norm_add(const void* a, const void* wa, const void* b, const void* wb, float share, float* hidden,
+                              const void* weight, int32_t weight_n, const void* final_weight, int32_t final_n,
+                              int32_t n, int32_t H, float eps, void* out, int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "norm_add");
+    SKYRL_REQUIRE(n >= 0 && H > 0 && H <= 8192, "norm_add: H must be in [1, 8192]");
+    SKYRL_REQUIRE((weight_n == 1 || weight_n == H) && (!final_weight || final_n == 1 || final_n == H),
+                  "norm_add: a weight has 1 or H values");
+    if (n == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(a && hidden && weight && out && (!b || (wa && wb)), "norm_add: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        auto t = [](const void* q) { return reinterpret_cast<const T*>(q); };
+        const NormAdd<T> p{t(a), t(wa), t(b), t(wb), share, hidden, t(weight), weight_n > 1, t(final_weight),
+                           final_n > 1, reinterpret_cast<T*>(out), H, eps};
+        if (H % 4 == 0) {
+            if (H <= 4 * kNT) { LAUNCH_NORM_ADD(4, 1); }
+            else if (H <= 8 * kNT) { LAUNCH_NORM_ADD(4, 2); }
+            else if (H <= 16 * kNT) { LAUNCH_NORM_ADD(4, 4); }
+            else { LAUNCH_NORM_ADD(4, 8); }
+        } else {
+            if (H <= 4 * kNT) { LAUNCH_NORM_ADD(1, 4); }
+            else { LAUNCH_NORM_ADD(1, 32); }
+        }
+    })
+    return check_launch("norm_add_kernel");
+}
+
+extern "C" int skyrl_xielu(const void* x, int64_t stride, int64_t n, int32_t I, const void* pq, void* out,
+                           int64_t out_stride, int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "xielu");
+    SKYRL_REQUIRE(n >= 0 && I > 0 && stride >= I && out_stride >= I, "xielu: bad sizes");
+    if (n == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(x && pq && out, "xielu: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        const T* in = reinterpret_cast<const T*>(x);
+        T* o = reinterpret_cast<T*>(out);
+        const T* w = reinterpret_cast<const T*>(pq);
+        if (I % 8 == 0 && stride % 8 == 0 && out_stride % 8 == 0 && aligned16(in) && aligned16(o))
+            hipLaunchKernelGGL((xielu_kernel<T, 8>), dim3(grid_for(n * (I / 8))), dim3(kNT), 0, as_stream(stream), in,
+                               stride, n, I, w, o, out_stride);
+        else
+            hipLaunchKernelGGL((xielu_kernel<T, 1>), dim3(grid_for(n * I)), dim3(kNT), 0, as_stream(stream), in,
+                               stride, n, I, w, o, out_stride);
+    })
+    return check_launch("xielu_kernel");
 }
 
 extern "C" int skyrl_conv_save(const void* x, int64_t stride, int32_t channels, int32_t taps, const int32_t* cu,

@@ -5,11 +5,16 @@ Dovidra is such a design: latent attention under a sliding window beside gated d
 bias-free layer norms before each half, tanh-form GELU gates, a looped range of layers that adds one
 learned vector per pass, and a tanh cap on the logits. Lipedra is another: differential attention, some
 layers over an earlier layer's keys and values, beside clamped gates with biases in parallel layers (one
-RMS norm, mixer and feed-forward in the same two matrix products), and a scaled embedding. The model is
-what config.json lists; the mechanisms are mixers.py; `DESIGNS` holds what a design fixes.
+RMS norm, mixer and feed-forward in the same two matrix products), and a scaled embedding. Foduzen is a
+third: gated linear recurrences, and layers of windowed attention beside a state space mixer, which read
+the residual itself and whose outputs are normed (one number as the weight), xIELU feed-forwards, sinusoidal
+position vectors. The model is what config.json lists; the mechanisms are mixers.py; `DESIGNS` holds what a
+design fixes.
 
 The residual stream is f32. One pass of the HIP norm kernel adds the previous sublayer's output and
-(at the start of a loop pass) its vector, stores the stream and writes the next product's input.
+(at the start of a loop pass) its vector, stores the stream and writes the next product's input; where
+outputs are normed, one pass norms the sublayer's output (or joins and norms two), adds it, stores the
+stream and writes the next product's input, at the end the final norm.
 
 HybridDecoder has PagedDecoder's interface (model.py), so the engine's scheduler, runner, sampler and
 weight updates serve it unchanged; besides, it takes portions: a step may continue several prompts
@@ -18,6 +23,7 @@ and decode others at the same time (`forward_portions`).
 
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass, field
 from typing import Any, Dict, Iterable, Iterator, List, Optional, Tuple
 
@@ -26,7 +32,7 @@ import torch.nn.functional as F
 
 from . import kernels
 from . import layer_kernels as lk
-from .mixers import FEEDFORWARDS, MIXERS, PROMPT_MIN, Products, Weights
+from .mixers import FEEDFORWARDS, MIXERS, PLAIN_FEEDFORWARDS, PROMPT_MIN, Products, SideBySide, Weights
 from .model import StepInputs
 
 DEFAULT_MAX_MODEL_LEN = 32768
@@ -40,11 +46,16 @@ class Design:
     norm_base: float = 0.0   # added to the stored norm weights
     parallel: bool = False   # mixer and feed-forward read one norm and are added together
     mlp: Dict[str, Any] = field(default_factory=dict)  # feed-forward constants
+    feedforwards: Dict[str, Any] = field(default_factory=lambda: FEEDFORWARDS)
+    output_norms: bool = False  # sublayers read the residual, their outputs are normed
+    scalar_norms: bool = False  # a norm's weight is one number
+    sinusoid: Optional[float] = None  # base of the position vectors added to the embedding
 
 
 DESIGNS = {
     "Dovidra": Design(norm="layer", mlp={"act": "gelu_tanh"}),
     "Lipedra": Design(norm="rms", norm_base=1.0, parallel=True, mlp={"act": "clamped", "alpha": 1.702, "bias": True}),
+    "Foduzen": Design(norm="rms", output_norms=True, scalar_norms=True, sinusoid=10000.0, feedforwards=PLAIN_FEEDFORWARDS),
 }
 
 
@@ -78,12 +89,14 @@ class HybridSpec:
 
     @classmethod
     def from_config(cls, cfg: Dict[str, Any]) -> "HybridSpec":
-        layers = cfg["layers"]
+        layers, design = cfg["layers"], DESIGNS[cfg["architecture"]]
         for e in layers:
             if e["type"] not in MIXERS:
                 raise ValueError(f"unknown layer type {e['type']!r} (known: {sorted(MIXERS)})")
-            if e.get("mlp") and e["mlp"]["kind"] not in FEEDFORWARDS:
-                raise ValueError(f"unknown feed-forward {e['mlp']['kind']!r} (known: {sorted(FEEDFORWARDS)})")
+            if e.get("mlp") and e["mlp"]["kind"] not in design.feedforwards:
+                raise ValueError(f"unknown feed-forward {e['mlp']['kind']!r} (known: {sorted(design.feedforwards)})")
+            if (e["type"] == "parallel") and not design.output_norms:
+                raise ValueError("mixers side by side need a design that norms outputs")
         for i, e in enumerate(layers):
             j = e["mixer"].get("kv_from")
             if j is None:
@@ -94,6 +107,8 @@ class HybridSpec:
                 raise ValueError(f"layer {i}: kv_from {j} is no earlier layer with such keys and values of its own")
         n, loop = len(layers), cfg.get("loop")
         runs, times = [], 0
+        if loop and design.output_norms:
+            raise ValueError("this design has no looped layers")
         if loop:
             a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
             if not 0 <= a <= b <= n or times < 0:
@@ -105,7 +120,7 @@ class HybridSpec:
         else:
             runs = [LayerRun(i) for i in range(n)]
         eos = cfg.get("eos_token_id")
-        return cls(design=DESIGNS[cfg["architecture"]], vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
+        return cls(design=design, vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]),
                    embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), norm_eps=float(cfg["norm"]["eps"]),
                    logit_softcap=float(cfg["logit_softcap"]) if cfg.get("logit_softcap") else None, layers=layers,
                    runs=runs, loop_times=times,
@@ -157,33 +172,44 @@ class HybridDecoder:
     # a biased product of one row copies the bias first instead of adding it in the library's kernel
     @property
     def min_bucket(self) -> int:
-        return 2 if self.spec.design.mlp.get("bias") else 1
+        subs = [sub for L in self.layers for _, sub in L["subs"]]
+        return 2 if any(isinstance(sub, Products) and sub.biased for sub in subs) else 1
 
     # ---------------------------------------------------------------- weights
     def _alloc(self, seed: Optional[int]):
         s = self.spec
         w = Weights(self.device, self.dtype, seed, s.initializer_range)
         H = s.hidden_size
-        norm = (lambda: w.zeros(H)) if s.design.norm_base else (lambda: w.ones(H))
+        d = s.design
+        size = () if d.scalar_norms else (H,)
+        norm = (lambda: w.zeros(*size)) if d.norm_base else (lambda: w.ones(*size))
         self.embed = w.matrix(s.vocab_size, H)
         self.layers: List[Dict[str, Any]] = []
         for e in s.layers:
             mixer = MIXERS[e["type"]](e["mixer"], H, s.norm_eps, self.max_model_len, w)
-            mlp = FEEDFORWARDS[e["mlp"]["kind"]](e["mlp"], H, w, **s.design.mlp) if e.get("mlp") else None
+            mlp = d.feedforwards[e["mlp"]["kind"]](e["mlp"], H, w, **d.mlp) if e.get("mlp") else None
             joined = hasattr(mixer, "inner")  # its products are Products'
             L = {"mixer": mixer, "mlp": mlp, "norm1": norm(), "norm2": None}
-            if s.design.parallel and mlp is not None:
+            if d.parallel and mlp is not None:
                 if not joined:
                     raise ValueError(f"{e['type']!r} layers cannot be parallel to a feed-forward")
                 L["subs"] = [(L["norm1"], Products([mixer, mlp], H, w))]
             else:
-                L["subs"] = [(L["norm1"], Products([mixer], H, w) if joined else mixer)]
+                if isinstance(mixer, SideBySide):
+                    sub = Products(mixer.parts, H, w, apart=True)
+                else:
+                    sub = Products([mixer], H, w) if joined else mixer
+                L["subs"] = [(L["norm1"], sub)]
                 if mlp is not None:
                     L["norm2"] = norm()
                     L["subs"].append((L["norm2"], Products([mlp], H, w)))
             self.layers.append(L)
         self.loop_step = w.matrix(s.loop_times, H) if s.loop_times else None
         self.norm = norm()
+        self.turns = None  # revolutions per position of each pair of the position vector's columns
+        if d.sinusoid:
+            i = torch.arange((H + 1) // 2, dtype=torch.float64)
+            self.turns = (d.sinusoid ** (-2.0 * i / H) / (2 * math.pi)).to(self.device)
         self.lm_head = w.matrix(s.vocab_size, H)
 
     def _param_views(self) -> Dict[str, torch.Tensor]:
@@ -260,20 +286,22 @@ class HybridDecoder:
 
     def plan(self, seq_lens: List[int], starts: List[int], n_short: int):
         """Host plan of the prompt forms, tuples of numpy arrays and sizes by the mixers' keys (host_plans)."""
-        if n_short == len(seq_lens):
-            return None
         plan, first = {}, sum(seq_lens[:n_short])
         for L in self.layers:
+            if n_short == len(seq_lens) and not getattr(L["mixer"], "plans_short", False):
+                continue  # the per-token forms need none
             for key, make in L["mixer"].host_plans(seq_lens, starts, n_short, first):
                 if key not in plan:
                     plan[key] = make()
-        return plan
+        return plan or None
 
     # ---------------------------------------------------------------- forward
     def _run_layers(self, inp: StepInputs, cache: HybridCache, want: Optional[torch.Tensor], trail=None):
         """Final-norm output of the wanted tokens (None: all). `trail` collects the residual after every
         layer run (inspection)."""
         s = self.spec
+        if s.design.output_norms:
+            return self._run_output_normed(inp, cache, want, trail)
         norm = dict(eps=s.norm_eps, kind=s.design.norm, base=s.design.norm_base)
         h = lk.embed(inp.tokens, self.embed, s.embed_scale)
         x = torch.empty(h.shape, dtype=self.dtype, device=self.device)
@@ -289,6 +317,32 @@ class HybridDecoder:
         if want is None:
             return lk.add_norm(delta, h, self.norm, out=x, **norm)
         return lk.add_norm(None if delta is None else delta[want], h[want], self.norm, **norm)
+
+    def _run_output_normed(self, inp: StepInputs, cache: HybridCache, want: Optional[torch.Tensor], trail=None):
+        s = self.spec
+        x = torch.empty((inp.tokens.shape[0], s.hidden_size), dtype=self.dtype, device=self.device)
+        h = lk.embed(inp.tokens, self.embed, s.embed_scale, None if self.turns is None else inp.positions, self.turns, x)
+        ws = self.workspace if inp.one_token else self.portion_workspace
+        last = len(s.runs) - 1
+        for i, (r, state) in enumerate(zip(s.runs, cache.runs)):
+            L = self.layers[r.layer]
+            for k, (weight, sub) in enumerate(L["subs"]):
+                delta = sub.forward(x, inp, state, ws)
+                join = {}
+                if isinstance(delta, tuple):
+                    join = {"pair": L["mixer"].out_norms, "share": L["mixer"].SHARE}
+                if i == last and k == len(L["subs"]) - 1:
+                    if trail is not None:
+                        lk.norm_add(delta, (full := h.clone()), weight, s.norm_eps, **join)
+                        trail.append(full)
+                    if want is not None:
+                        delta = tuple(t[want] for t in delta) if join else delta[want]
+                        h, x = h[want], None
+                    return lk.norm_add(delta, h, weight, s.norm_eps, final=self.norm, out=x, **join)
+                lk.norm_add(delta, h, weight, s.norm_eps, out=x, **join)
+            if trail is not None:
+                trail.append(h.clone())
+        raise ValueError("a model needs a layer")
 
     def forward_decode(self, inp: StepInputs, cache: HybridCache) -> torch.Tensor:
         """One token per row: final hidden states [n, H]."""

@@ -42,14 +42,22 @@ def _check_view(t: torch.Tensor, name: str, dtype, shape):
         raise ValueError(f"{name} must be {dtype} {tuple(shape)} with unit column stride")
 
 
-def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float) -> torch.Tensor:
-    """f32 rows of the embedding table times scale."""
-    dev = _require_gpu(tokens, table)
+def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float, positions: Optional[torch.Tensor] = None,
+          turns: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """f32 rows of the embedding table times scale, plus, with `turns` f64 [(H + 1) // 2], each position's sine
+    and cosine vector; `x`: filled with the same in the table's type."""
+    dev = _require_gpu(tokens, table, positions, turns, x)
     n, H = tokens.shape[0], table.shape[1]
     _check(tokens, "tokens", torch.int64, (n,))
     _check(table, "table", table.dtype)
+    if (positions is None) != (turns is None):
+        raise ValueError("positions and turns go together")
+    _check(positions, "positions", torch.int64, (n,))
+    _check(turns, "turns", torch.float64, ((H + 1) // 2,))
+    _check(x, "x", table.dtype, (n, H))
     out = torch.empty((n, H), dtype=torch.float32, device=dev)
-    _ffi.call("skyrl_embed", _ptr(tokens), _ptr(table), n, H, float(scale), _ptr(out), _code(table), _stream(dev))
+    _ffi.call("skyrl_embed", _ptr(tokens), _ptr(table), n, H, float(scale), _ptr(positions), _ptr(turns), _ptr(out),
+              _ptr(x), _code(table), _stream(dev))
     return out
 
 
@@ -69,6 +77,46 @@ def add_norm(delta: Optional[torch.Tensor], hidden: torch.Tensor, weight: torch.
     _check(out, "out", weight.dtype, (n, H))
     _ffi.call("skyrl_add_norm", _ptr(delta), _ptr(hidden), _ptr(step), _ptr(weight), float(base), n, H, float(eps),
               NORMS[kind], _ptr(out), _code(weight), _stream(dev))
+    return out
+
+
+def norm_add(delta, hidden: torch.Tensor, weight: torch.Tensor, eps: float, pair=None, share: float = 0.5,
+             final: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """hidden (f32, in place) += rms(delta) * weight. With `pair` = (wa, wb) `delta` is two outputs (a, b), joined
+    to share (rms(a) wa + rms(b) wb) first. Returns hidden in the weight's type, or rms(hidden) * final. A weight
+    is one number (a 0-d tensor) or a vector."""
+    a, b = delta if pair is not None else (delta, None)
+    wa, wb = pair if pair is not None else (None, None)
+    dev = _require_gpu(a, b, wa, wb, hidden, weight, final, out)
+    n, H = hidden.shape
+    _check(hidden, "hidden", torch.float32)
+    for t, name in ((a, "delta"), (b, "second delta")):
+        _check(t, name, weight.dtype, (n, H))
+    for t, name in ((wa, "first pair weight"), (wb, "second pair weight")):
+        _check(t, name, weight.dtype, (H,))
+    for t, name in ((weight, "weight"), (final, "final weight")):
+        if t is not None and tuple(t.shape) not in ((), (H,)):
+            raise ValueError(f"{name} must be one number or [{H}]")
+        _check(t, name, weight.dtype)
+    if out is None:
+        out = torch.empty((n, H), dtype=weight.dtype, device=dev)
+    _check(out, "out", weight.dtype, (n, H))
+    _ffi.call("skyrl_norm_add", _ptr(a), _ptr(wa), _ptr(b), _ptr(wb), float(share), _ptr(hidden), _ptr(weight),
+              weight.numel(), _ptr(final), 0 if final is None else final.numel(), n, H, float(eps), _ptr(out),
+              _code(weight), _stream(dev))
+    return out
+
+
+def xielu(x: torch.Tensor, pq: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """xIELU of x [n, I] with the learned pair pq; both may be column ranges."""
+    dev = _require_gpu(x, pq, out)
+    n, I = x.shape
+    _check_view(x, "x", x.dtype, (n, I))
+    _check(pq, "pq", x.dtype, (2,))
+    if out is None:
+        out = torch.empty((n, I), dtype=x.dtype, device=dev)
+    _check_view(out, "out", x.dtype, (n, I))
+    _ffi.call("skyrl_xielu", _ptr(x), x.stride(0), n, I, _ptr(pq), _ptr(out), out.stride(0), _code(x), _stream(dev))
     return out
 
 
@@ -437,4 +485,293 @@ def diff_prefill(sh, q, gate, k_cache, v_cache, block_tables, tiles, lam, out) -
     _ffi.call("skyrl_diff_prefill", ctypes.byref(sh), _ptr(q), _ptr(gate), gate.stride(0), _ptr(k_cache),
               _ptr(v_cache), _ptr(block_tables), block_tables.stride(0), _ptr(tiles), tiles.shape[0], _ptr(lam),
               _ptr(out), out.stride(0), _stream(dev))
+    return out
+
+
+# ---------------------------------------------------------------- short convolutions of prompts
+def _check_steps(cu, rows, positions, T: Optional[int] = None):
+    n = rows.shape[0]
+    _check(rows, "rows", torch.int32, (n,))
+    _check(cu, "cu", torch.int32, (n + 1,))
+    _check(positions, "positions", torch.int64, (positions.shape[0] if T is None else T,))
+    return n
+
+
+def conv_chunk(x: torch.Tensor, conv_t: torch.Tensor, bias: Optional[torch.Tensor], silu: bool, chunk, cu, rows,
+               positions, ring, sections) -> None:
+    """Convolution, bias and activation of x's first columns at the tokens of `chunk` int32 [n, 4]
+    (mixers.chunk_plan). sections: (units, size, padded, rows or None, cols or None) over consecutive channels,
+    rows [T, units, padded], cols [chunks, units, padded, CHUNK] in x's type."""
+    dev = _require_gpu(x, conv_t, bias, chunk, cu, rows, positions, ring)
+    taps, ch = conv_t.shape
+    T, nc = x.shape[0], chunk.shape[0]
+    if x.dim() != 2 or x.shape[1] < ch or (ch > 1 and x.stride(1) != 1):
+        raise ValueError(f"x must be [T, >= {ch}] with unit column stride")
+    _check(conv_t, "conv_t", torch.float32)
+    _check(bias, "bias", torch.float32, (ch,))
+    _check(chunk, "chunk", torch.int32, (nc, 4))
+    _check_steps(cu, rows, positions, T)
+    _check(ring, "ring", x.dtype, (ring.shape[0], taps, ch))
+    sec = (_ffi.ConvSection * len(sections))()
+    for i, (units, size, padded, by_row, by_col) in enumerate(sections):
+        _check(by_row, "rows of a section", x.dtype, (T, units, padded))
+        _check(by_col, "cols of a section", x.dtype, (nc, units, padded, CHUNK))
+        sec[i] = _ffi.ConvSection(units, size, padded, *(None if t is None else t.data_ptr() for t in (by_row, by_col)))
+    for a in range(0, nc, 65535):  # the grid's limit
+        n = min(65535, nc - a)
+        part = (_ffi.ConvSection * len(sections))()
+        for i, s in enumerate(sec):
+            cols = sections[i][4]
+            part[i] = _ffi.ConvSection(s.units, s.size, s.padded, s.rows, None if cols is None else cols[a:].data_ptr())
+        _ffi.call("skyrl_conv_chunk", _ptr(x), x.stride(0), ch, taps, _ptr(conv_t), _ptr(bias), int(silu),
+                  _ptr(chunk[a:a + n]), n, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(ring), part, len(sections),
+                  _code(x), _stream(dev))
+
+
+# ---------------------------------------------------------------- gated linear recurrence
+def rglru_pads(width: int, blocks: int):
+    """(padded outputs, padded inputs) of a block's gate matrices."""
+    size = width // blocks
+    return (size + 15) // 16 * 16, (size + 31) // 32 * 32
+
+
+def _check_rglru(proj, width, blocks, gate_w, gate_b, rate, state, out):
+    T = proj.shape[0]
+    if proj.dim() != 2 or proj.shape[1] < 2 * width or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, >= {2 * width}] with unit column stride")
+    _check(gate_w, "gate_w", proj.dtype, (blocks, 2) + rglru_pads(width, blocks))
+    _check(gate_b, "gate_b", torch.float32, (2, width))
+    _check(rate, "rate", torch.float32, (width,))
+    _check(state, "state", torch.float32, (state.shape[0], width))
+    _check_view(out, "out", proj.dtype, (T, width))
+
+
+def rglru_step(proj, width: int, blocks: int, conv_t, conv_b, gate_w, gate_b, rate, rows, positions, state, ring,
+               out) -> None:
+    """One token per sequence: state and ring updated in place."""
+    dev = _require_gpu(proj, conv_t, conv_b, gate_w, gate_b, rate, rows, positions, state, ring, out)
+    n, taps = proj.shape[0], conv_t.shape[0]
+    _check_rglru(proj, width, blocks, gate_w, gate_b, rate, state, out)
+    _check(conv_t, "conv_t", torch.float32, (taps, width))
+    _check(conv_b, "conv_b", torch.float32, (width,))
+    _check(rows, "rows", torch.int32, (n,))
+    _check(positions, "positions", torch.int64, (n,))
+    _check(ring, "ring", proj.dtype, (state.shape[0], taps, width))
+    _ffi.call("skyrl_rglru_step", _ptr(proj), proj.stride(0), width, blocks, taps, _ptr(conv_t), _ptr(conv_b),
+              _ptr(gate_w), _ptr(gate_b), _ptr(rate), _ptr(rows), _ptr(positions), n, _ptr(state), _ptr(ring), _ptr(out),
+              out.stride(0), _code(proj), _stream(dev))
+
+
+def rglru_prompt(proj, width: int, blocks: int, u, gate_w, gate_b, rate, chunk, seq_chunks, seq0: int, cu, rows,
+                 positions, state, out) -> None:
+    """Tokens of the chunks, of the sequences from seq0 on; u [T, width] is conv_chunk's."""
+    dev = _require_gpu(proj, u, gate_w, gate_b, rate, chunk, seq_chunks, cu, rows, positions, state, out)
+    T, nc = proj.shape[0], chunk.shape[0]
+    _check_rglru(proj, width, blocks, gate_w, gate_b, rate, state, out)
+    n = _check_steps(cu, rows, positions, T) - seq0
+    _check(u, "u", proj.dtype, (T, width))
+    _check(chunk, "chunk", torch.int32, (nc, 4))
+    _check(seq_chunks, "seq_chunks", torch.int32, (n + 1,))
+    h, a = (torch.empty((T, width), dtype=torch.float32, device=dev) for _ in range(2))
+    s_in = torch.empty((nc, width), dtype=torch.float32, device=dev)
+    _ffi.call("skyrl_rglru_prompt", _ptr(proj), proj.stride(0), width, blocks, _ptr(u), _ptr(gate_w), _ptr(gate_b),
+              _ptr(rate), _ptr(chunk), nc, _ptr(seq_chunks), seq0, n, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(state),
+              _ptr(h), _ptr(a), _ptr(s_in), _ptr(out), out.stride(0), _code(proj), _stream(dev))
+
+
+# ---------------------------------------------------------------- windowed attention with an output gate
+def attn_shape(heads, kv_heads, dim, vdim, window, scale, eps) -> _ffi.AttnShape:
+    return _ffi.AttnShape(heads, kv_heads, dim, vdim, int(window or 0), scale, eps)
+
+
+def attn_channels(sh) -> int:
+    """Columns of the projection: q | k | v."""
+    return (sh.heads + sh.kv_heads) * sh.dim + sh.kv_heads * sh.vdim
+
+
+def attn_pads(sh):
+    """(columns of a cached key or padded query row, rows of a cached value tile)."""
+    return (sh.dim + 31) // 32 * 32, (sh.vdim + 15) // 16 * 16
+
+
+def attn_mfma(sh, dtype) -> bool:
+    """Whether the matrix kernels (split decode, prompt form) take the shape."""
+    return bool(_ffi.query("skyrl_attn_mfma", ctypes.byref(sh), _DTYPES[dtype]))
+
+
+def attn_runs_fit(sh, proj) -> bool:
+    return (proj.dtype == torch.bfloat16 and sh.dim % 8 == 0 and sh.dim <= 512 and sh.vdim % 8 == 0
+            and proj.stride(0) % 8 == 0 and proj.data_ptr() % 16 == 0)
+
+
+def _check_attn_cache(sh, k_cache, v_cache, dtype):
+    dp, vp = attn_pads(sh)
+    _check(k_cache, "k_cache", dtype, (k_cache.shape[0], sh.kv_heads, 16, dp))
+    _check(v_cache, "v_cache", dtype, (k_cache.shape[0], sh.kv_heads, vp, 16))
+
+
+def attn_write(sh, proj, q_norm, k_norm, slots, k_cache, v_cache, q=None, count: Optional[int] = None,
+               runs=None) -> torch.Tensor:
+    """Normed queries out [T, heads, padded], normed keys and values into the cache, for the first `count` tokens
+    or, with `runs` int32 [n, 2] (mixers.run_plan), for those. A given `q` is filled in place."""
+    dev = _require_gpu(proj, q_norm, k_norm, slots, k_cache, v_cache, q, runs)
+    T, dp = proj.shape[0], attn_pads(sh)[0]
+    if proj.dim() != 2 or proj.shape[1] < attn_channels(sh) or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, >= {attn_channels(sh)}] with unit column stride")
+    _check(q_norm, "q_norm", proj.dtype, (sh.dim,))
+    _check(k_norm, "k_norm", proj.dtype, (sh.dim,))
+    _check(slots, "slots", torch.int64, (T,))
+    _check_attn_cache(sh, k_cache, v_cache, proj.dtype)
+    if q is None:
+        make = torch.empty if dp == sh.dim else torch.zeros  # the padding must be zero
+        q = make((T, sh.heads, dp), dtype=proj.dtype, device=dev)
+    _check(q, "q", proj.dtype, (T, sh.heads, dp))
+    if runs is not None:
+        _check(runs, "runs", torch.int32, (runs.shape[0], 2))
+        n = runs.shape[0]
+    else:
+        n = T if count is None else count
+        if not 0 <= n <= T:
+            raise ValueError("attn_write: token range outside the step")
+    _ffi.call("skyrl_attn_write", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(q_norm), _ptr(k_norm), _ptr(slots),
+              _ptr(runs), 0, n, _ptr(q), _ptr(k_cache), _ptr(v_cache), _code(proj), _stream(dev))
+    return q
+
+
+def attn_workspace_bytes(sh, tokens: int, nparts: int) -> int:
+    return int(_ffi.query("skyrl_attn_attend_workspace_bytes", ctypes.byref(sh), tokens, nparts))
+
+
+def _check_attn_io(sh, q, gate, out):
+    T = q.shape[0]
+    _check(q, "q", q.dtype, (T, sh.heads, attn_pads(sh)[0]))
+    _check_view(gate, "gate", q.dtype, (T, sh.heads * sh.vdim))
+    _check_view(out, "out", q.dtype, (T, sh.heads * sh.vdim))
+
+
+def attn_attend(sh, q, gate, k_cache, v_cache, block_tables, bt_row, positions, out, nparts: int = 1,
+                part_min: int = 64, workspace=None) -> torch.Tensor:
+    """One query row per token over its window's pages; gate [T, heads * vdim] before its sigmoid."""
+    dev = _require_gpu(q, gate, k_cache, v_cache, block_tables, bt_row, positions, out)
+    T = q.shape[0]
+    _check_attn_io(sh, q, gate, out)
+    _check_attn_cache(sh, k_cache, v_cache, q.dtype)
+    _check_table(block_tables, bt_row, positions, T)
+    ws = None
+    if nparts > 1 and attn_mfma(sh, q.dtype):
+        need = attn_workspace_bytes(sh, T, nparts)
+        ws = workspace.get(need) if workspace is not None else torch.empty(need, dtype=torch.uint8, device=dev)
+    else:
+        nparts = 1
+    _ffi.call("skyrl_attn_attend", ctypes.byref(sh), _ptr(q), _ptr(gate), gate.stride(0), _ptr(k_cache), _ptr(v_cache),
+              _ptr(block_tables), block_tables.stride(0), _ptr(bt_row), _ptr(positions), T, part_min, nparts, _ptr(out),
+              out.stride(0), _ptr(ws), _code(q), _stream(dev))
+    return out
+
+
+def attn_prefill(sh, q, gate, k_cache, v_cache, block_tables, tiles, out) -> torch.Tensor:
+    """Prompt tiles int32 [n, 4] (mixers.tile_plan) over their sequences' pages, which already hold the
+    portion's own keys and values."""
+    dev = _require_gpu(q, gate, k_cache, v_cache, block_tables, tiles, out)
+    _check_attn_io(sh, q, gate, out)
+    _check_attn_cache(sh, k_cache, v_cache, torch.bfloat16)
+    if block_tables.dtype != torch.int32 or block_tables.dim() != 2 or block_tables.stride(1) != 1:
+        raise ValueError("block_tables must be int32 [n, blocks] with unit column stride")
+    _check(tiles, "tiles", torch.int32, (tiles.shape[0], 4))
+    _ffi.call("skyrl_attn_prefill", ctypes.byref(sh), _ptr(q), _ptr(gate), gate.stride(0), _ptr(k_cache),
+              _ptr(v_cache), _ptr(block_tables), block_tables.stride(0), _ptr(tiles), tiles.shape[0], _ptr(out),
+              out.stride(0), _stream(dev))
+    return out
+
+
+# ---------------------------------------------------------------- state space mixer
+def ssd_shape(heads, vdim, state, groups, taps) -> _ffi.SSDShape:
+    return _ffi.SSDShape(heads, vdim, state, groups, taps)
+
+
+def ssd_channels(sh) -> int:
+    """Channels of the short convolution: x | B | C."""
+    return sh.heads * sh.vdim + 2 * sh.groups * sh.state
+
+
+def ssd_width(sh) -> int:
+    """Columns of the projection: z | x | B | C | dt."""
+    return sh.heads * sh.vdim + ssd_channels(sh) + sh.heads
+
+
+def ssd_ppad(sh) -> int:
+    return (sh.vdim + 3) // 4 * 4
+
+
+def ssd_prompt_fits(sh, dtype) -> bool:
+    return dtype == torch.bfloat16 and sh.state <= 256
+
+
+def ssd_slices(sh) -> int:
+    """Workgroups per head of the prompt form: 64 value columns each."""
+    return (sh.vdim + 63) // 64
+
+
+def _check_ssd(sh, proj, conv_t, conv_b, a_log, dt_bias, skip, state, ring, y):
+    T, ch = proj.shape[0], ssd_channels(sh)
+    if proj.dim() != 2 or proj.shape[1] < ssd_width(sh) or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, >= {ssd_width(sh)}] with unit column stride")
+    _check(conv_t, "conv_t", torch.float32, (sh.taps, ch))
+    _check(conv_b, "conv_b", torch.float32, (ch,))
+    for t, name in ((a_log, "a_log"), (dt_bias, "dt_bias"), (skip, "skip")):
+        _check(t, name, torch.float32, (sh.heads,))
+    _check(state, "state", torch.float32, (state.shape[0], sh.heads, sh.state, ssd_ppad(sh)))
+    _check(ring, "ring", proj.dtype, (state.shape[0], sh.taps, ch))
+    _check_view(y, "y", proj.dtype, (T, sh.heads * sh.vdim))
+
+
+def ssd_scan(sh, proj, conv_t, conv_b, a_log, dt_bias, skip, cu, rows, positions, state, ring, save_conv, y) -> None:
+    """Token by token over each sequence's tokens [cu[s], cu[s + 1]) into y [T, heads * vdim], before the gated
+    norm; state and (save_conv: one token per sequence) convolution inputs updated in place."""
+    dev = _require_gpu(proj, conv_t, conv_b, a_log, dt_bias, skip, cu, rows, positions, state, ring, y)
+    _check_ssd(sh, proj, conv_t, conv_b, a_log, dt_bias, skip, state, ring, y)
+    n = _check_steps(cu, rows, positions, proj.shape[0])
+    _ffi.call("skyrl_ssd_scan", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(conv_t), _ptr(conv_b), _ptr(a_log),
+              _ptr(dt_bias), _ptr(skip), _ptr(cu), _ptr(rows), _ptr(positions), n, _ptr(state), _ptr(ring),
+              int(save_conv), _ptr(y), y.stride(0), _code(proj), _stream(dev))
+
+
+def ssd_prompt(sh, proj, conv_t, conv_b, a_log, dt_bias, skip, cu, rows, positions, state, ring, chunk, super_, pick,
+               chain, y) -> None:
+    """Chunked form over the chunks int32 [n, 4] and runs of chunks (mixers.walk_plan); `state` is updated in
+    place, the convolution inputs are conv_save's."""
+    dev = _require_gpu(proj, conv_t, conv_b, a_log, dt_bias, skip, cu, rows, positions, state, ring, chunk, super_, pick,
+                       chain, y)
+    _check_ssd(sh, proj, conv_t, conv_b, a_log, dt_bias, skip, state, ring, y)
+    T, nc, ns = proj.shape[0], chunk.shape[0], super_.shape[0]
+    _check(super_, "super", torch.int32, (ns, 4))
+    _check(pick, "pick", torch.int32, (pick.shape[0],))
+    _check(chain, "chain", torch.int32, (chain.shape[0], 2))
+    H, P, N, G = sh.heads, sh.vdim, sh.state, sh.groups
+    vp, np_, inner = (P + 15) // 16 * 16, (N + 31) // 32 * 32, H * P
+    make = torch.empty if (vp, np_) == (P, N) else torch.zeros  # padding meets the other operand: zero
+    xt, bt = (make(s, dtype=proj.dtype, device=dev) for s in ((nc, H, vp, CHUNK), (nc, G, np_, CHUNK)))
+    brow, crow = (make((T, G, np_), dtype=proj.dtype, device=dev) for _ in range(2))
+    conv_chunk(proj[:, inner:], conv_t, conv_b, True, chunk, cu, rows, positions, ring,
+               ((H, P, vp, None, xt), (G, N, np_, brow, bt), (G, N, np_, crow, None)))
+    multi = pick.shape[0] > 0
+    runs = torch.empty((ns if multi else 1, H, np_, vp), dtype=torch.float32, device=dev)
+    gtot = torch.empty((ns if multi else 1, H), dtype=torch.float32, device=dev)
+    dt = proj[:, inner + ssd_channels(sh):]
+    _ffi.call("skyrl_ssd_prompt", ctypes.byref(sh), _ptr(xt), _ptr(bt), _ptr(brow), _ptr(crow), _ptr(dt), dt.stride(0),
+              _ptr(a_log), _ptr(dt_bias), _ptr(skip), _ptr(chunk), _ptr(super_), ns, _ptr(pick), pick.shape[0],
+              _ptr(chain), chain.shape[0], _ptr(cu), _ptr(rows), _ptr(positions), _ptr(state), _ptr(runs), _ptr(gtot),
+              _ptr(y), y.stride(0), _stream(dev))
+
+
+def gated_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float,
+               out: torch.Tensor) -> torch.Tensor:
+    """rms over each of `groups` equal parts of y silu(z), times weight; y, z and out may be column ranges."""
+    dev = _require_gpu(y, z, weight, out)
+    n, W = y.shape
+    for t, name in ((y, "y"), (z, "z"), (out, "out")):
+        _check_view(t, name, weight.dtype, (n, W))
+    _check(weight, "weight", weight.dtype, (W,))
+    _ffi.call("skyrl_gated_norm", _ptr(y), y.stride(0), _ptr(z), z.stride(0), _ptr(weight), n, W, groups, float(eps),
+              _ptr(out), out.stride(0), _code(weight), _stream(dev))
     return out

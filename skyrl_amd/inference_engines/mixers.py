@@ -1,5 +1,5 @@
 """Layer mechanisms of the hybrid decoders: latent attention, gated delta rule, differential
-attention, gated MLP.
+attention, gated linear recurrence, windowed attention beside a state space mixer, gated and plain MLPs.
 
 A mechanism owns its weights (fused where one product serves several tensors), names them for
 loading and saving, sizes and allocates its cache or state, and runs a step over it with the HIP
@@ -7,9 +7,9 @@ kernels of layer_kernels.py; matrix products are hipBLASLt through torch. Every 
 a parameter; nothing here knows a particular model. `MIXERS` and `FEEDFORWARDS` map the type names of
 a config.json to these classes.
 
-A sublayer is `forward(x, inp, state, workspace)`. Differential attention and the MLP leave their input
-and output products to `Products`, which runs one sublayer, or a mixer and a feed-forward that read the
-same input side by side in the same two products.
+A sublayer is `forward(x, inp, state, workspace)`. Most leave their input and output products to
+`Products`, which runs one sublayer, a mixer and a feed-forward that read the same input side by side in
+the same two products, or two mixers whose outputs are normed apart and joined (`SideBySide`).
 
 A step is a StepInputs (model.py): tokens of several sequences, each with its own first position. In
 a portion step the first `n_short` sequences (single decoded tokens and short portions) come first;
@@ -132,15 +132,16 @@ def chunk_plan(seq_lens: List[int], first_seq: int, first_token: int):
     return np.asarray(chunk, dtype=np.int32).reshape(-1, 4), np.asarray(ends, dtype=np.int32)
 
 
-def tile_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token: int) -> np.ndarray:
-    """Query tiles int32 [m, 4] of full causal attention of sequences first_seq..: first token, tokens,
-    position of the first, sequence; the tiles with the most keys first."""
+def tile_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token: int,
+              window: Optional[int] = None) -> np.ndarray:
+    """Query tiles int32 [m, 4] of causal attention of sequences first_seq..: first token, tokens, position
+    of the first, sequence; the tiles with the most keys (in `window`) first."""
     tiles, tok = [], first_token
     for i in range(first_seq, len(seq_lens)):
         L, s = seq_lens[i], starts[i]
         tiles += [(tok + a, min(PREFILL_TILE, L - a), s + a, i) for a in range(0, L, PREFILL_TILE)]
         tok += L
-    tiles.sort(key=lambda t: -(t[1] + t[2]))
+    tiles.sort(key=lambda t: -(t[1] + min(t[2], window or t[2])))
     return np.asarray(tiles, dtype=np.int32).reshape(-1, 4)
 
 
@@ -156,30 +157,71 @@ def run_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token
     return np.concatenate(runs).astype(np.int32)
 
 
+WALK_WORKGROUPS = 1024  # of the state space prompt walk: four per CU
+WALK_CHUNKS = 4         # chunks per run at least: a run's state is written and read once more
+
+
+def walk_plan(seq_lens: List[int], first_seq: int, first_token: int, per_run: int):
+    """Host plan of the state space prompt form of sequences first_seq..: (chunk int32 [n, 4], super int32 [m, 4],
+    pick int32 [k], chain int32 [j, 2]). Sequences are cut into runs of chunks so that about WALK_WORKGROUPS
+    workgroups walk them, per_run of them per run (skyrl_ssd_prompt)."""
+    chunk, ends = chunk_plan(seq_lens, first_seq, first_token)
+    size = max(WALK_CHUNKS, -(-len(chunk) * per_run // WALK_WORKGROUPS))
+    runs, pick, chain = [], [], []
+    for i in range(len(ends) - 1):
+        n = int(ends[i + 1] - ends[i])
+        k = max(1, round(n / size))
+        cuts = [ends[i] + n * j // k for j in range(k + 1)]
+        if k > 1:
+            chain.append((len(runs), k))
+            pick += range(len(runs), len(runs) + k - 1)
+        runs += [(a, b - a, first_seq + i, (k > 1) + 2 * (b == ends[i + 1])) for a, b in zip(cuts, cuts[1:])]
+    i32 = lambda x, *tail: np.asarray(x, dtype=np.int32).reshape(-1, *tail)  # noqa: E731
+    return chunk, i32(runs, 4), i32(pick), i32(chain, 2)
+
+
 class Products:
     """The input and the output product of sublayers that read the same input and whose outputs are
     summed: the parts' input rows stacked and their output columns side by side, one product each. Parts
     start at multiples of 8 elements (16 bytes). A part has `in_rows`, `out_cols`, `in_bias`, `out_bias`,
-    takes its views of the weights in `bind` and computes `inner(proj, out, ...)` between the products."""
+    takes its views of the weights in `bind` and computes `inner(proj, out, ...)` between the products.
+    With `apart` every part has an output product and a state of its own, and the outputs are a tuple."""
 
-    def __init__(self, parts: List[Any], width: int, w: Weights):
-        self.parts, self.ranges = parts, []
+    def __init__(self, parts: List[Any], width: int, w: Weights, apart: bool = False):
+        self.parts, self.ranges, self.apart = parts, [], apart
         a = c = 0
         for p in parts:
             self.ranges.append((a, c))
             a, c = a + (p.in_rows + 7) // 8 * 8, c + (p.out_cols + 7) // 8 * 8
+        self.w_in = w.matrix(a, width)
+        self.b_in = w.zeros(a) if any(p.in_bias for p in parts) else None
+        if apart:
+            self.outs = [(w.matrix(width, p.out_cols), w.zeros(width) if p.out_bias else None) for p in parts]
+            for p, (a, _), (wo, bo) in zip(parts, self.ranges, self.outs):
+                p.bind(self.w_in[a:a + p.in_rows], self.b_in[a:a + p.in_rows] if p.in_bias else None, wo, bo)
+            return
         if sum(p.out_bias for p in parts) > 1:
             raise ValueError("one part at most may have an output bias")
-        self.w_in, self.w_out = w.matrix(a, width), w.matrix(width, c)
-        self.b_in = w.zeros(a) if any(p.in_bias for p in parts) else None
+        self.w_out = w.matrix(width, c)
         self.b_out = w.zeros(width) if any(p.out_bias for p in parts) else None
         self.padded = any(p.out_cols % 8 for p in parts)
         for p, (a, c) in zip(parts, self.ranges):
             p.bind(self.w_in[a:a + p.in_rows], self.b_in[a:a + p.in_rows] if p.in_bias else None,
                    self.w_out[:, c:c + p.out_cols], self.b_out if p.out_bias else None)
 
-    def forward(self, x: torch.Tensor, inp, state, workspace) -> torch.Tensor:
+    @property
+    def biased(self) -> bool:
+        return self.b_in is not None or any(p.out_bias for p in self.parts)
+
+    def forward(self, x: torch.Tensor, inp, state, workspace):
         proj = F.linear(x, self.w_in, self.b_in)
+        if self.apart:
+            outs = []
+            for p, (a, _), (wo, bo), st in zip(self.parts, self.ranges, self.outs, state):
+                o = torch.empty((x.shape[0], p.out_cols), dtype=x.dtype, device=x.device)
+                p.inner(proj[:, a:a + p.in_rows], o, inp, st, workspace)
+                outs.append(F.linear(o, wo, bo))
+            return tuple(outs)
         make = torch.zeros if self.padded else torch.empty  # padding columns meet weights: they must be finite
         cat = make((x.shape[0], self.w_out.shape[1]), dtype=x.dtype, device=x.device)
         for p, (a, c) in zip(self.parts, self.ranges):
@@ -277,7 +319,7 @@ class LatentAttention:
                         self.cos_sin, cache)
         qw = H * (self.dim + self.rot_dim)
         out = torch.empty((T, H * self.vdim), dtype=self.dtype, device=x.device)
-        prompt = inp.plan is not None and lk.prefill_fits(self.dim, self.rot_dim, self.vdim, self.dtype)
+        prompt = inp.plan is not None and self.window in inp.plan and lk.prefill_fits(self.dim, self.rot_dim, self.vdim, self.dtype)
         ts = inp.short_tokens if prompt else T
         q = proj[:, :qw]
         for a in range(0, ts, 32768):  # the decode form's grid limit
@@ -356,7 +398,8 @@ class GatedDelta:
         out = torch.empty((x.shape[0], self.heads * self.vdim), dtype=self.dtype, device=x.device)
         args = (self.conv, self.a_log, self.dt_bias, self.norm)
         n = inp.rows.shape[0]
-        k = inp.n_short if inp.plan is not None and lk.delta_prompt_fits(self.shape) else n
+        prompt = inp.plan is not None and "chunks" in inp.plan and lk.delta_prompt_fits(self.shape)
+        k = inp.n_short if prompt else n
         if k:
             lk.delta_scan(self.shape, proj, *args, inp.cu[:k + 1], inp.rows[:k], inp.positions, S, ring,
                           inp.one_token, out)
@@ -459,7 +502,7 @@ class DifferentialAttention:
         k_cache, v_cache, ring = state
         T = proj.shape[0]
         seqs = (inp.cu, inp.rows, inp.bt_row, inp.positions, inp.slots, self.cos_sin, ring, k_cache, v_cache)
-        prompt = inp.plan is not None and lk.diff_mfma(self.shape, self.dtype)
+        prompt = inp.plan is not None and "tiles" in inp.plan and lk.diff_mfma(self.shape, self.dtype)
         ts = inp.short_tokens if prompt else T
         runs = inp.plan["tiles"][1] if prompt and lk.diff_runs_fit(self.shape, proj) else None
         q = lk.diff_write(self.shape, proj, self.conv_t, *seqs, save_conv=inp.one_token,
@@ -476,6 +519,313 @@ class DifferentialAttention:
                            part_min=kernels.MIN_PARTITION, workspace=workspace)
         if ts < T:
             lk.diff_prefill(self.shape, q, gate, k_cache, v_cache, inp.block_tables, inp.plan["tiles"][0], self.lam, out)
+
+
+class ShortConv:
+    """Weights of a biased causal convolution per channel, `conv` [channels, taps] and `conv.b`, and the
+    transposed f32 filters that the kernels read."""
+
+    def __init__(self, channels: int, taps: int, w: Weights):
+        self.conv, self.bias = w.matrix(channels, taps), w.zeros(channels, dtype=torch.float32)
+        self.conv_t = w.zeros(taps, channels, dtype=torch.float32)
+        self.refresh()
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        yield from (("conv", self.conv), ("conv.b", self.bias))
+
+    def refresh(self) -> None:
+        self.conv_t.copy_(self.conv.t())
+
+
+class GatedLinearRecurrence:
+    """Recurrent block of a real gated linear recurrence (RG-LRU): a gelu branch gates a branch of short
+    convolution and recurrence, whose two gates are block-diagonal. State per row: the f32 channels and the
+    convolution's last inputs."""
+
+    paged = False
+    kv_from = None
+    plans_short = True
+    in_bias, out_bias = True, False
+    RATE = 8.0  # log decay = -RATE r softplus(lam)
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        return False
+
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+        self.channels, self.blocks, self.taps = int(m["width"]), int(m["blocks"]), int(m["conv"])
+        if self.channels % self.blocks:
+            raise ValueError("the recurrence's width must be a multiple of blocks")
+        C, n = self.channels, self.channels // self.blocks
+        self.dtype = w.dtype
+        self.in_rows, self.out_cols = 2 * C, C
+        self.conv = ShortConv(C, self.taps, w)
+        self.ra, self.ri = w.matrix(self.blocks, n, n), w.matrix(self.blocks, n, n)
+        self.gate_b = w.zeros(2, C, dtype=torch.float32)
+        self.lam = w.zeros(C, dtype=torch.float32)
+        self.gate_w = w.zeros(self.blocks, 2, *lk.rglru_pads(C, self.blocks))  # the kernels' form of ra, ri
+        self.rate = w.zeros(C, dtype=torch.float32)
+        self.refresh()
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.w_in, self.b_in, self.wo = w_in, b_in, w_out
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        C = self.channels
+        yield from split_rows(self.w_in, (("y", C), ("x", C)))
+        yield from split_rows(self.b_in, (("y.b", C), ("x.b", C)))
+        yield from self.conv.params()
+        for i, (name, t) in enumerate((("ra", self.ra), ("ri", self.ri))):
+            yield name, t
+            yield name + ".b", self.gate_b[i].view(self.blocks, -1)
+        yield from (("lam", self.lam), ("o", self.wo))
+
+    def refresh(self) -> None:
+        """Recompute derived tensors, in place, after the weights changed."""
+        self.conv.refresh()
+        n = self.ra.shape[1]
+        self.gate_w[:, 0, :n, :n].copy_(self.ra)
+        self.gate_w[:, 1, :n, :n].copy_(self.ri)
+        self.rate.copy_(-self.RATE * F.softplus(self.lam.double(), threshold=50.0))
+
+    # ---- state
+    def block_bytes(self) -> int:
+        return 0
+
+    def row_bytes(self) -> int:
+        return self.channels * (4 + self.taps * self.dtype.itemsize)
+
+    def make_state(self, num_blocks: int, num_rows: int, device):
+        return (torch.zeros((num_rows, self.channels), dtype=torch.float32, device=device),
+                torch.zeros((num_rows, self.taps, self.channels), dtype=self.dtype, device=device))
+
+    def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
+        return 0
+
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        yield "all_chunks", lambda: chunk_plan(seq_lens, 0, 0)
+
+    # ---- step
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
+        S, ring = state
+        C = self.channels
+        gates = (self.gate_w, self.gate_b, self.rate)
+        if inp.one_token:
+            lk.rglru_step(proj, C, self.blocks, self.conv.conv_t, self.conv.bias, *gates, inp.rows, inp.positions, S,
+                          ring, out)
+            return
+        chunk, seq_chunks = inp.plan["all_chunks"]
+        u = torch.empty((proj.shape[0], C), dtype=self.dtype, device=proj.device)
+        x, seqs = proj[:, C:], (inp.cu, inp.rows, inp.positions)
+        lk.conv_chunk(x, self.conv.conv_t, self.conv.bias, False, chunk, *seqs, ring, ((1, C, C, u.unsqueeze(1), None),))
+        lk.rglru_prompt(proj, C, self.blocks, u, *gates, chunk, seq_chunks, 0, *seqs, S, out)
+        lk.conv_save(x, C, *seqs, ring)
+
+
+class WindowAttention:
+    """Grouped attention with RMS-normed queries and keys, no rotation, an optional sliding window and an
+    elementwise output gate; biases on its projections but the gate's. Caches K [blocks, kv_heads, 16, dim] and V
+    transposed [blocks, kv_heads, vdim, 16], sizes padded."""
+
+    paged = True
+    kv_from = None
+    in_bias, out_bias = True, True
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        return True
+
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+        self.heads, self.kv_heads = int(m["heads"]), int(m["kv_heads"])
+        self.dim, self.vdim = int(m["dim"]), int(m["vdim"])
+        mask = m.get("mask")
+        self.window = int(mask["size"]) if mask and mask.get("size") else None
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.shape = lk.attn_shape(self.heads, self.kv_heads, self.dim, self.vdim, self.window, float(m["scale"]), eps)
+        self.dtype = w.dtype
+        self.qkv = lk.attn_channels(self.shape)
+        self.out_cols = self.heads * self.vdim
+        self.in_rows = self.qkv + self.out_cols
+        self.q_norm, self.k_norm = w.ones(self.dim), w.ones(self.dim)
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.w_in, self.b_in, self.wo, self.bo = w_in, b_in, w_out, b_out
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        rows = (("q", self.heads * self.dim), ("k", self.kv_heads * self.dim), ("v", self.kv_heads * self.vdim))
+        yield from split_rows(self.w_in, rows + (("g", self.out_cols),))
+        yield from split_rows(self.b_in, [(n + ".b", r) for n, r in rows])
+        yield from (("q.norm", self.q_norm), ("k.norm", self.k_norm), ("o", self.wo), ("o.b", self.bo))
+
+    def refresh(self) -> None:
+        pass
+
+    # ---- cache
+    def block_bytes(self) -> int:
+        return self.kv_heads * BLOCK_SIZE * sum(lk.attn_pads(self.shape)) * self.dtype.itemsize
+
+    def row_bytes(self) -> int:
+        return 0
+
+    def make_state(self, num_blocks: int, num_rows: int, device):
+        dp, vp = lk.attn_pads(self.shape)
+        zeros = lambda *tail: torch.zeros((num_blocks, self.kv_heads) + tail, dtype=self.dtype, device=device)  # noqa: E731
+        return zeros(BLOCK_SIZE, dp), zeros(vp, BLOCK_SIZE)
+
+    # ---- plans
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        args = (seq_lens, starts, first_seq, first_token)
+        yield ("tiles", self.window), lambda: (tile_plan(*args, self.window),)
+        yield "runs", lambda: (run_plan(*args),)
+
+    def nparts(self, tokens: int, max_ctx: int) -> int:
+        ctx = min(max_ctx, self.window + BLOCK_SIZE) if self.window else max_ctx
+        groups = -(-(self.heads // self.kv_heads) // 16)  # a wave takes 16 query heads of a key head
+        return kernels.choose_nparts(tokens, self.kv_heads * groups, ctx)
+
+    def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
+        return lk.attn_workspace_bytes(self.shape, tokens, self.nparts(tokens, max_ctx))
+
+    # ---- step
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
+        k_cache, v_cache = state
+        T = proj.shape[0]
+        key = ("tiles", self.window)
+        prompt = inp.plan is not None and key in inp.plan and lk.attn_mfma(self.shape, self.dtype)
+        ts = inp.short_tokens if prompt else T
+        runs = inp.plan["runs"][0] if prompt and lk.attn_runs_fit(self.shape, proj) else None
+        args = (self.q_norm, self.k_norm, inp.slots, k_cache, v_cache)
+        q = lk.attn_write(self.shape, proj, *args, count=T if runs is None else ts)
+        if runs is not None:
+            lk.attn_write(self.shape, proj, *args, q=q, runs=runs)
+        gate = proj[:, self.qkv:]
+        for a in range(0, ts, 32768):  # the decode form's grid limit
+            b = min(ts, a + 32768)
+            lk.attn_attend(self.shape, q[a:b], gate[a:b], k_cache, v_cache, inp.block_tables, inp.bt_row[a:b],
+                           inp.positions[a:b], out[a:b], nparts=self.nparts(b - a, inp.max_ctx),
+                           part_min=kernels.MIN_PARTITION, workspace=workspace)
+        if ts < T:
+            lk.attn_prefill(self.shape, q, gate, k_cache, v_cache, inp.block_tables, inp.plan[key][0], out)
+
+
+class StateSpace:
+    """State space mixer with a scalar decay per head (Mamba-2): biased short convolutions, a gate before a
+    norm in equal parts. State per row: the f32 matrix of every head and the convolutions' last inputs."""
+
+    paged = False
+    kv_from = None
+    in_bias, out_bias = False, False
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        return False
+
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+        self.heads, self.vdim, self.state = int(m["heads"]), int(m["vdim"]), int(m["state"])
+        self.groups, self.taps, self.norm_groups = int(m["groups"]), int(m["conv"]), int(m["norm_groups"])
+        self.width = self.heads * self.vdim
+        if self.heads % self.groups or self.width % self.norm_groups:
+            raise ValueError("heads must be a multiple of groups, heads * vdim of norm_groups")
+        self.shape = lk.ssd_shape(self.heads, self.vdim, self.state, self.groups, self.taps)
+        self.eps, self.dtype = eps, w.dtype
+        self.channels = lk.ssd_channels(self.shape)
+        self.in_rows, self.out_cols = lk.ssd_width(self.shape), self.width
+        self.conv = ShortConv(self.channels, self.taps, w)
+        self.a_log, self.dt_bias, self.skip = (w.zeros(self.heads, dtype=torch.float32) for _ in range(3))
+        self.norm = w.ones(self.width)
+        self.plan_key = ("walk", self.heads * lk.ssd_slices(self.shape))
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.w_in, self.wo = w_in, w_out
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        yield "in", self.w_in
+        yield from self.conv.params()
+        yield from (("dt_bias", self.dt_bias), ("A_log", self.a_log), ("D", self.skip), ("norm", self.norm),
+                    ("o", self.wo))
+
+    def refresh(self) -> None:
+        self.conv.refresh()
+
+    # ---- state
+    def block_bytes(self) -> int:
+        return 0
+
+    def row_bytes(self) -> int:
+        return (4 * self.heads * self.state * lk.ssd_ppad(self.shape)
+                + self.taps * self.channels * self.dtype.itemsize)
+
+    def make_state(self, num_blocks: int, num_rows: int, device):
+        return (torch.zeros((num_rows, self.heads, self.state, lk.ssd_ppad(self.shape)), dtype=torch.float32,
+                            device=device),
+                torch.zeros((num_rows, self.taps, self.channels), dtype=self.dtype, device=device))
+
+    def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
+        return 0
+
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        yield self.plan_key, lambda: walk_plan(seq_lens, first_seq, first_token, self.plan_key[1])
+
+    # ---- step
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
+        S, ring = state
+        y = torch.empty((proj.shape[0], self.width), dtype=self.dtype, device=proj.device)
+        args = (self.conv.conv_t, self.conv.bias, self.a_log, self.dt_bias, self.skip)
+        n = inp.rows.shape[0]
+        prompt = inp.plan is not None and self.plan_key in inp.plan and lk.ssd_prompt_fits(self.shape, self.dtype)
+        k = inp.n_short if prompt else n
+        if k:
+            lk.ssd_scan(self.shape, proj, *args, inp.cu[:k + 1], inp.rows[:k], inp.positions, S, ring, inp.one_token, y)
+        if k < n:
+            lk.ssd_prompt(self.shape, proj, *args, inp.cu, inp.rows, inp.positions, S, ring, *inp.plan[self.plan_key], y)
+        if not inp.one_token:
+            lk.conv_save(proj[:, self.width:], self.channels, inp.cu, inp.rows, inp.positions, ring)
+        lk.gated_norm(y, proj[:, :self.width], self.norm, self.norm_groups, self.eps, out)
+
+
+class SideBySide:
+    """Two mixers over the same input, one input product, each output normed over the model's width: the
+    layer's output norm joins them, half the sum of both (layer_kernels.norm_add)."""
+
+    LEFT, RIGHT, SHARE = WindowAttention, StateSpace, 0.5
+    kv_from = None
+
+    @classmethod
+    def prefix_cacheable(cls, m: Dict[str, Any]) -> bool:
+        return cls.LEFT.prefix_cacheable(m["left"]) and cls.RIGHT.prefix_cacheable(m["right"])
+
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+        self.parts = [c(m[side], width, eps, max_pos, w) for c, side in ((self.LEFT, "left"), (self.RIGHT, "right"))]
+        self.out_norms = (w.ones(width), w.ones(width))
+        self.paged = any(p.paged for p in self.parts)
+        self.plans_short = any(getattr(p, "plans_short", False) for p in self.parts)
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        for side, part, norm in zip(("left.", "right."), self.parts, self.out_norms):
+            for name, t in part.params():
+                yield side + name, t
+            yield side + "out", norm
+
+    def refresh(self) -> None:
+        for p in self.parts:
+            p.refresh()
+
+    def block_bytes(self) -> int:
+        return sum(p.block_bytes() for p in self.parts)
+
+    def row_bytes(self) -> int:
+        return sum(p.row_bytes() for p in self.parts)
+
+    def make_state(self, num_blocks: int, num_rows: int, device):
+        return tuple(p.make_state(num_blocks, num_rows, device) for p in self.parts)
+
+    def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
+        return max(p.workspace_bytes(tokens, max_ctx) for p in self.parts)
+
+    def host_plans(self, *args):
+        for p in self.parts:
+            yield from p.host_plans(*args)
 
 
 class GatedMLP:
@@ -503,5 +853,26 @@ class GatedMLP:
         lk.gate_mul(proj, self.act, self.alpha, self.limit, out=out)
 
 
-MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "attention": DifferentialAttention}
+class PlainMLP:
+    """down(xIELU(up x)); the activation's two learned numbers are `act`."""
+
+    in_bias = out_bias = False
+
+    def __init__(self, m: Dict[str, Any], width: int, w: Weights):
+        self.in_rows = self.out_cols = int(m["ff"])
+        self.act = w.zeros(2)
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.wu, self.wd = w_in, w_out
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        yield from (("up", self.wu), ("down", self.wd), ("act", self.act))
+
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
+        lk.xielu(proj, self.act, out=out)
+
+
+MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "attention": DifferentialAttention,
+          "rglru": GatedLinearRecurrence, "parallel": SideBySide}
 FEEDFORWARDS = {"dense": GatedMLP}
+PLAIN_FEEDFORWARDS = {"dense": PlainMLP}

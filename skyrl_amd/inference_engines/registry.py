@@ -30,7 +30,7 @@ def _hf_paged(config: Dict[str, Any], folder: str, device, dtype, max_model_len,
                         max_model_len=max_model_len)
 
 
-ARCHITECTURES: Dict[str, Callable] = {"Dovidra": _hybrid, "Lipedra": _hybrid}
+ARCHITECTURES: Dict[str, Callable] = {"Dovidra": _hybrid, "Lipedra": _hybrid, "Foduzen": _hybrid}
 HF_MODEL_TYPES: Dict[str, Callable] = {t: _hf_paged for t in ("qwen2", "llama", "mistral", "qwen3")}
 
 
