@@ -1,8 +1,8 @@
 """Throughput of the hybrid decoders beside the closest dense decoder (Qwen2 layers) of equal size,
 through the engine's own runner (scheduled batches, HIP sampler included): `python bench.py --hybrid`.
 
-All models have random weights, the same width, heads, feed-forward, vocabulary and number of layer
-runs. Prints one JSON line: tokens/s of prompts (one long, eight short) and of decode steps at several
+All models have random weights, the same width, heads, feed-forward weights, vocabulary and number of
+layer runs. Prints one JSON line: tokens/s of prompts (one long, eight short) and of decode steps at several
 batch sizes. `--hybrid-model` and `--hybrid-phase` restrict it, e.g. under a profiler."""
 
 from __future__ import annotations
@@ -14,7 +14,7 @@ SIZES = {  # layers that resemble a 2B and an 8B model's
     "2k": dict(width=2048, ff=6144, heads=16, window=1024, delta_heads=32, delta_kv=16, vocab=32768),
     "4k": dict(width=4096, ff=12288, heads=32, window=1024, delta_heads=64, delta_kv=32, vocab=32768),
 }
-MODELS = ("dovidra", "lipedra", "qwen2")
+MODELS = ("dovidra", "lipedra", "foduzen", "qwen2")
 RUNS = 6  # layer runs: latent, (delta, latent, delta) ... as below
 PROMPTS = ((1, 8192), (8, 1024))
 DECODES = ((1, 2048), (64, 2048), (256, 2048))
@@ -44,6 +44,19 @@ def parallel_config(z):
             "vocab": z["vocab"], "width": z["width"]}
 
 
+def normed_config(z):
+    """Four layers of gated linear recurrence (as wide as the model, blocks of 128) and two of windowed attention with
+    the dense model's heads beside a state space mixer (twice the width, heads of 64, state 128)."""
+    rec = {"width": z["width"], "blocks": z["width"] // 128, "conv": 4}
+    left = {"heads": z["heads"], "kv_heads": max(2, z["heads"] // 8), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+            "mask": {"size": z["window"]}}
+    right = {"heads": z["width"] // 32, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+    layers = [{"type": "parallel", "mixer": {"left": left, "right": right}} if i % 3 == 2 else {"type": "rglru", "mixer": rec}
+              for i in range(RUNS)]
+    return {"architecture": "Foduzen", "layers": [dict(e, mlp={"kind": "dense", "ff": z["ff"] * 3 // 2}) for e in layers],
+            "norm": {"eps": 1e-6}, "embedding": {"scale": z["width"] ** 0.5}, "vocab": z["vocab"], "width": z["width"]}
+
+
 def dense_config(z):
     from transformers import Qwen2Config
 
@@ -59,7 +72,7 @@ def build(kind, z, max_len):
     from skyrl_amd.inference_engines.model import PagedDecoder
 
     if kind != "qwen2":
-        config = {"dovidra": hybrid_config, "lipedra": parallel_config}[kind](z)
+        config = {"dovidra": hybrid_config, "lipedra": parallel_config, "foduzen": normed_config}[kind](z)
         return HybridDecoder(config, "cuda:0", dtype=torch.bfloat16, seed=0, max_model_len=max_len)
     return PagedDecoder(dense_config(z), "cuda:0", seed=0, max_model_len=max_len)
 

@@ -171,3 +171,112 @@ def make_parallel_weights(cfg, seed=0):
     rand("final.norm", W, gain=0.3)
     proj("head", cfg["vocab"], W, 3.0, bias=False)
     return {k: v.to(torch.bfloat16) for k, v in w.items()}
+
+
+# ---------------------------------------------------------------- output-normed recurrent and side-by-side layers
+def rglru(width=60, blocks=3, conv=3):
+    return {"type": "rglru", "mixer": {"width": width, "blocks": blocks, "conv": conv}}
+
+
+def attend(heads=4, kv_heads=2, dim=20, vdim=28, window=37, scale=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale or 1.6 / math.sqrt(dim)}
+    if window:
+        m["mask"] = {"size": window}
+    return m
+
+
+def ssd(heads=3, vdim=20, state=18, groups=1, conv=5, norm_groups=2):
+    return {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "conv": conv, "norm_groups": norm_groups}
+
+
+def side(left=None, right=None):
+    return {"type": "parallel", "mixer": {"left": left or attend(), "right": right or ssd()}}
+
+
+def normed_config(layers, width=72, vocab=199, ff=100, scale=3.3, eps=2e-5, no_mlp=()):
+    layers = [dict(e, mlp=None if i in no_mlp else {"kind": "dense", "ff": ff + 4 * i}) for i, e in enumerate(layers)]
+    return {"architecture": "Foduzen", "layers": layers, "norm": {"eps": eps}, "embedding": {"scale": scale},
+            "vocab": vocab, "width": width}
+
+
+NORMED = {
+    # sizes no vector width divides, an odd state, one tap, no feed-forward in two layers
+    "odd": normed_config([rglru(), side(), rglru(width=50, blocks=2, conv=1), side(attend(heads=3, kv_heads=3, dim=17, vdim=9, window=16),
+                          ssd(heads=4, vdim=14, state=11, groups=2, conv=2, norm_groups=2))], width=70, no_mlp=(1, 2)),
+    # shapes the matrix kernels take exactly, one key head, window 1 tile and a half, groups shared by heads
+    "wide": normed_config([side(attend(heads=16, kv_heads=1, dim=64, vdim=128, window=96),
+                                ssd(heads=4, vdim=64, state=128, groups=2, conv=4, norm_groups=1)),
+                           rglru(width=256, blocks=2, conv=4), rglru(width=128, blocks=8, conv=4)], width=128, ff=96),
+    # padded shapes: many query heads, values of more than one slice, nine taps, no window
+    "padded": normed_config([rglru(width=96, blocks=6, conv=9),
+                             side(attend(heads=20, kv_heads=1, dim=40, vdim=24, window=None),
+                                  ssd(heads=6, vdim=72, state=40, groups=3, conv=7, norm_groups=2)),
+                             side(attend(heads=2, kv_heads=2, dim=136, vdim=152, window=3),
+                                  ssd(heads=2, vdim=24, state=160, groups=1, conv=1, norm_groups=2))], width=88, ff=60,
+                            scale=0.8, no_mlp=(0,)),
+}
+
+
+def make_normed_weights(cfg, seed=0):
+    """bf16 tensors by checkpoint name: decays from short to long memory, norms, gates and biases far from trivial."""
+    g = torch.Generator().manual_seed(seed)
+    W, w = cfg["width"], {}
+
+    def rand(name, *shape, gain=1.0, mean=0.0):
+        w[name] = mean + torch.randn(*shape, generator=g) * gain
+
+    def mat(name, rows, cols, gain=1.0, bias=False):
+        rand(name, rows, cols, gain=gain / math.sqrt(cols))
+        if bias:
+            rand(name + ".b", rows, gain=0.4)
+
+    def conv(q, channels, taps):
+        rand(q + "conv", channels, taps, gain=1 / math.sqrt(taps))
+        rand(q + "conv.b", channels, gain=0.3)
+
+    def number(name):
+        w[name] = (1 + 0.4 * torch.randn((), generator=g))
+
+    rand("embed", cfg["vocab"], W)
+    for i, e in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        q = p + "mix."
+        number(p + "norm1")
+        if e["type"] == "rglru":
+            C, b = m["width"], m["blocks"]
+            mat(q + "y", C, W, 1.3 / cfg["embedding"]["scale"] ** 0.5, bias=True)
+            mat(q + "x", C, W, 1.3 / cfg["embedding"]["scale"] ** 0.5, bias=True)
+            conv(q, C, m["conv"])
+            for n in ("ra", "ri"):
+                rand(q + n, b, C // b, C // b, gain=1.5 / math.sqrt(C // b))
+                rand(q + n + ".b", b, C // b, gain=0.7)
+            rand(q + "lam", C, gain=3.0, mean=-4.0)
+            mat(q + "o", W, C)
+        else:
+            a, s, l, r = m["left"], m["right"], q + "left.", q + "right."
+            mat(l + "q", a["heads"] * a["dim"], W, bias=True)
+            mat(l + "k", a["kv_heads"] * a["dim"], W, bias=True)
+            mat(l + "v", a["kv_heads"] * a["vdim"], W, bias=True)
+            rand(l + "q.norm", a["dim"], gain=0.3, mean=1.0)
+            rand(l + "k.norm", a["dim"], gain=0.3, mean=1.0)
+            mat(l + "g", a["heads"] * a["vdim"], W)
+            mat(l + "o", W, a["heads"] * a["vdim"], bias=True)
+            inner, ch = s["heads"] * s["vdim"], s["heads"] * s["vdim"] + 2 * s["groups"] * s["state"]
+            mat(r + "in", inner + ch + s["heads"], W, 0.8)
+            conv(r, ch, s["conv"])
+            rand(r + "dt_bias", s["heads"], gain=1.0, mean=-1.5)
+            rand(r + "A_log", s["heads"], gain=1.5, mean=-1.0)
+            rand(r + "D", s["heads"])
+            rand(r + "norm", inner, gain=0.3, mean=1.0)
+            mat(r + "o", W, inner)
+            rand(q + "left.out", W, gain=0.3, mean=1.0)
+            rand(q + "right.out", W, gain=0.3, mean=1.0)
+        if e.get("mlp"):
+            ff = e["mlp"]["ff"]
+            number(p + "norm2")
+            mat(p + "mlp.up", ff, W, 0.8)
+            mat(p + "mlp.down", W, ff)
+            rand(p + "mlp.act", 2, gain=0.8)
+    number("final.norm")
+    mat("head", cfg["vocab"], W, 3.0)
+    return {k: v.to(torch.bfloat16) for k, v in w.items()}

@@ -4,7 +4,7 @@ import asyncio
 
 import torch
 
-from hybrid_cases import make_parallel_weights, make_weights
+from hybrid_cases import make_normed_weights, make_parallel_weights, make_weights
 from oracle import hybrid_ref as ref
 from skyrl_amd.inference_engines.engine import AMDInferenceEngine
 from skyrl_amd.inference_engines.hybrid import HybridDecoder
@@ -14,7 +14,7 @@ DTYPES = [torch.float32, torch.bfloat16]
 
 
 def weights_of(cfg, seed=0):
-    return (make_parallel_weights if cfg["architecture"] == "Lipedra" else make_weights)(cfg, seed)
+    return {"Lipedra": make_parallel_weights, "Foduzen": make_normed_weights, "Dovidra": make_weights}[cfg["architecture"]](cfg, seed)
 
 
 def rms(x):
@@ -30,7 +30,7 @@ def close(got, want, dtype, f32=1e-4, bf16=2e-2):
 
 
 def rnd(g, *shape, dtype=torch.float32, scale=1.0):
-    return (torch.randn(*shape, generator=g) * scale).to(dtype)
+    return (torch.randn(shape, generator=g) * scale).to(dtype)
 
 
 LIMIT = {torch.float32: 2e-5, torch.bfloat16: 4e-2}

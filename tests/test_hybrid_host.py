@@ -7,8 +7,8 @@ import numpy as np
 import pytest
 import torch
 
-from hybrid_cases import (CONFIGS, PARALLEL, config, delta, diff_attention, latent, make_parallel_weights, make_weights,
-                          parallel_config)
+from hybrid_cases import (CONFIGS, NORMED, PARALLEL, attend, config, delta, diff_attention, latent, make_normed_weights,
+                          make_parallel_weights, make_weights, normed_config, parallel_config, rglru, side, ssd)
 from oracle import hybrid_ref as ref
 from skyrl_amd.inference_engines import mixers
 from skyrl_amd.inference_engines.engine import BLOCK_SIZE, EngineCore, ModelRunner, RequestParams
@@ -360,3 +360,120 @@ def test_parallel_plan_and_smallest_decode_step():
     assert set(plan) == {"tiles"} and [len(p) for p in plan["tiles"]] == [1, 5] and m.plan([1, 2], [3, 0], 2) is None
     assert ModelRunner(m, 4, 6).buckets == [2, 4, 6] and ModelRunner(m, 4, 1).buckets == [1]
     assert ModelRunner(HybridDecoder(CONFIGS["once"], "cpu", seed=None, max_model_len=64), 4, 3).buckets == [1, 2, 3]
+
+
+# ---------------------------------------------------------------- output norms, recurrences, mixers side by side
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
+@pytest.mark.parametrize("name", sorted(NORMED))
+def test_normed_weight_names_round_trip(name, dtype):
+    cfg = NORMED[name]
+    m = HybridDecoder(cfg, "cpu", dtype=dtype, seed=None, max_model_len=64)
+    w = make_normed_weights(cfg, 2)
+    assert m.load_weights(w.items()) == len(w)
+    ours = dict(m.hf_named_tensors())
+    assert sorted(ours) == sorted(w) and m.num_params() == sum(t.numel() for t in w.values())
+    for k in w:
+        assert ours[k].shape == w[k].shape and torch.equal(ours[k].float(), w[k].float()), k
+    for i, L in enumerate(m.layers):  # derived tensors follow the weights
+        p, x = f"l{i}.mix.", L["mixer"]
+        if isinstance(x, mixers.GatedLinearRecurrence):
+            n = x.channels // x.blocks
+            assert torch.equal(x.conv.conv_t, w[p + "conv"].float().t())
+            for k, g in enumerate(("ra", "ri")):
+                assert torch.equal(x.gate_w[:, k, :n, :n].float(), w[p + g].float())
+                assert torch.equal(x.gate_b[k], w[p + g + ".b"].float().view(-1))
+            assert not bool(x.gate_w[:, :, n:].any()) and not bool(x.gate_w[..., n:].any())
+            torch.testing.assert_close(x.rate.double(), -8 * ref.softplus(w[p + "lam"].double()), rtol=1e-6, atol=0)
+        else:
+            left, right = x.parts
+            sub = L["subs"][0][1]
+            assert sub.apart and all(a % 8 == 0 for a, _ in sub.ranges) and sub.biased
+            bias = torch.cat([w[p + f"left.{n}.b"] for n in "qkv"])
+            assert torch.equal(left.b_in[:len(bias)].float(), bias.float()) and not bool(left.b_in[len(bias):].any())
+            assert torch.equal(right.conv.conv_t, w[p + "right.conv"].float().t())
+    with pytest.raises(KeyError):
+        m.load_weights([("l0.mix.none", w["final.norm"])])
+    with pytest.raises(ValueError):
+        m.load_weights([("final.norm", torch.ones(cfg["width"]))])
+
+
+def test_normed_checkpoint_registry(tmp_path):
+    from safetensors.torch import save_file
+
+    cfg, w = NORMED["odd"], make_normed_weights(NORMED["odd"], 3)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file(w, str(tmp_path / "model.safetensors"))
+    m = load_decoder(str(tmp_path), "cpu", max_model_len=64)
+    assert isinstance(m, HybridDecoder) and m.plain_lm_head and not m.prefix_cacheable and m.min_bucket == 2
+    assert m.norm.shape == () and m.spec.embed_scale == cfg["embedding"]["scale"]
+    del w["l1.mix.right.D"]
+    save_file(w, str(tmp_path / "model.safetensors"))
+    with pytest.raises(ValueError, match="l1.mix.right.D"):
+        load_decoder(str(tmp_path), "cpu", max_model_len=64)
+
+
+def test_position_turns():
+    m = HybridDecoder(NORMED["odd"], "cpu", seed=None, max_model_len=64)
+    W, pos = NORMED["odd"]["width"], torch.tensor([0, 1, 5, 4000])
+    a = pos[:, None].double() * m.turns[None] * 2 * torch.pi
+    torch.testing.assert_close(torch.stack([a.sin(), a.cos()], -1).view(4, -1)[:, :W], ref.sinusoid(pos, W), rtol=0, atol=1e-9)
+
+
+def test_normed_caches_and_sizes():
+    cfg = NORMED["padded"]
+    m = HybridDecoder(cfg, "cpu", seed=None, max_model_len=64)
+    runs = HybridCache(m, 5, 3).runs
+    S, ring = runs[0]
+    assert S.shape == (3, 96) and S.dtype == torch.float32 and ring.shape == (3, 9, 96)
+    (k, v), (S, ring) = runs[1]
+    assert k.shape == (5, 1, BLOCK_SIZE, 64) and v.shape == (5, 1, 32, BLOCK_SIZE)
+    assert S.shape == (3, 6, 40, 72) and S.dtype == torch.float32 and ring.shape == (3, 7, 6 * 72 + 2 * 3 * 40)
+    flat = [t for r in (runs[0], *runs[1], *runs[2]) for t in r]
+    assert m.row_bytes() == sum(t.numel() * t.itemsize for t in flat if t.shape[0] == 3) // 3
+    assert m.block_bytes() == sum(t.numel() * t.itemsize for t in flat if t.shape[0] == 5) // 5
+
+
+def test_normed_sizes_outside_the_design_are_refused():
+    build = lambda *layers, **kw: HybridDecoder(dict(normed_config(list(layers)), **kw), "cpu", seed=None, max_model_len=8)  # noqa: E731
+    for bad in (rglru(width=60, blocks=7), side(attend(heads=3, kv_heads=2)), side(right=ssd(heads=3, groups=2)),
+                side(right=ssd(norm_groups=7))):
+        with pytest.raises(ValueError):
+            build(bad)
+    with pytest.raises(ValueError, match="looped"):
+        build(rglru(), loop={"start": 0, "stop": 1, "times": 2})
+    with pytest.raises(ValueError, match="side by side"):
+        build(side(), architecture="Lipedra")
+
+
+@pytest.mark.parametrize("lens,per_run", [([1, 3, 40, 200, 129], 6), ([64] * 3, 64), ([8192], 64), ([5, 1000] + [700] * 5, 32), ([100], 4096)])
+def test_walk_plan_covers_every_chunk_once(lens, per_run):
+    first = sum(1 for n in lens if n < 32)
+    tok = sum(lens[:first])
+    chunk, runs, pick, chain = mixers.walk_plan(lens, first, tok, per_run)
+    ref_chunk, ends = mixers.chunk_plan(lens, first, tok)
+    assert (chunk == ref_chunk).all()
+    covered, by_seq = [], {}
+    for r, (a, n, seq, kind) in enumerate(runs.tolist()):
+        assert n > 0 and {int(c) for c in chunk[a:a + n, 2]} == {seq}
+        covered += range(a, a + n)
+        by_seq.setdefault(seq, []).append((r, kind))
+    assert covered == list(range(len(chunk)))
+    many = {s: rs for s, rs in by_seq.items() if len(rs) > 1}
+    assert chain.tolist() == [[rs[0][0], len(rs)] for rs in many.values()]
+    assert pick.tolist() == [r for rs in many.values() for r, _ in rs[:-1]]
+    for rs in by_seq.values():
+        assert [k for _, k in rs] == [(len(rs) > 1) + 2 * (i == len(rs) - 1) for i in range(len(rs))]
+
+
+def test_normed_plans_and_window_tiles():
+    m = HybridDecoder(NORMED["odd"], "cpu", seed=None, max_model_len=64)
+    plan = m.plan([1, 2, 40], [3, 0, 7], 2)
+    assert set(plan) == {"all_chunks", ("tiles", 37), ("tiles", 16), "runs", ("walk", 3), ("walk", 4)}
+    assert plan["all_chunks"][0].tolist() == [[0, 1, 0, 0], [1, 2, 1, 0], [3, 40, 2, 0]] and plan["all_chunks"][1].tolist() == [0, 1, 2, 3]
+    assert plan[("tiles", 16)][0].tolist() == [[3, 40, 7, 2]] and plan[("walk", 3)][1].tolist() == [[0, 1, 2, 2]]
+    assert set(m.plan([1, 2], [3, 0], 2)) == {"all_chunks"}
+    tiles = mixers.tile_plan([300, 200], [0, 1000], 0, 0, 128)
+    assert sorted(tiles[:, 0].tolist()) == [0, 128, 256, 300, 428]
+    keys = [t[1] + min(t[2], 128) for t in tiles.tolist()]
+    assert keys == sorted(keys, reverse=True)
+    assert ModelRunner(m, 4, 6).buckets == [2, 4, 6]
