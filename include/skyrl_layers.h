@@ -1,8 +1,9 @@
 /*
- * skyrl_layers.h — C ABI of libskyrl_layers.so: the decoder-layer mechanisms of the hybrid decoders
- * (inference_engines/hybrid.py) on MI355X (gfx950). A library of its own, so that serving such a
- * model compiles these kernels only. Conventions (status codes, dtype codes, stream order, no
- * allocation, skyrl_last_error()) are those of skyrl_hip.h.
+ * skyrl_layers.h — C ABI of the hybrid decoders' layer libraries (inference_engines/hybrid.py) on MI355X
+ * (gfx950): libskyrl_layers.so (embedding, norms, activations, convolutions) and libskyrl_layer_<name>.so for the
+ * entry points skyrl_<name>_* of one mechanism, so that serving a model compiles its own kernels only.
+ * Conventions (status codes, dtype codes, stream order, no allocation, skyrl_last_error(), one per library) are
+ * those of skyrl_hip.h.
  *
  * `dtype` is the element type T of activations and weights: SKYRL_BF16, or SKYRL_F32 for a model run
  * wholly in 32-bit. The residual stream, norms, rotary angles, attention scores and weights, gates
@@ -30,6 +31,7 @@ extern "C" {
  *                   m = a T [n, H], or, with two outputs, share (rms(a) wa + rms(b) wb) (wa, wb T [H]); hidden f32 +=
  *                   rms(m) * weight; out T = hidden, or rms(hidden) * final_weight if that is given. weight and
  *                   final_weight T hold one number for all columns or H (weight_n, final_n). H <= 8192.
+ *   skyrl_gated_norm  out T [n, width] = rms over each of `groups` equal parts of y silu(z), times weight T [width].
  *   skyrl_xielu     out T [n, I] = ap x^2 + x / 2 for x > 0, an (exp(x) - 1 - x) + x / 2 otherwise, ap = softplus(p),
  *                   an = 1/2 + softplus(q) from pq T [2].
  *   skyrl_gate_mul  out T [n, I] (row stride out_stride) from gate | up of gate_up T [n, 2I] (row stride
@@ -54,6 +56,9 @@ int skyrl_xielu(const void* x, int64_t stride, int64_t n, int32_t I, const void*
                 int32_t dtype, void* stream);
 int skyrl_add_norm(const void* delta, float* hidden, const void* step, const void* weight, float w_base, int32_t n,
                    int32_t H, float eps, int32_t kind, void* out, int32_t dtype, void* stream);
+int skyrl_gated_norm(const void* y, int64_t y_stride, const void* z, int64_t z_stride, const void* weight, int64_t n,
+                     int32_t width, int32_t groups, float eps, void* out, int64_t out_stride, int32_t dtype,
+                     void* stream);
 int skyrl_gate_mul(const void* gate_up, int64_t gu_stride, int64_t n, int32_t I, int32_t act, float alpha, float limit,
                    void* out, int64_t out_stride, int32_t dtype, void* stream);
 int skyrl_conv_save(const void* x, int64_t stride, int32_t channels, int32_t taps, const int32_t* cu,
@@ -240,8 +245,9 @@ int skyrl_conv_chunk(const void* x, int64_t stride, int32_t channels, int32_t ta
  * State per row: S f32 [rows, width] and the convolution's ring T [rows, taps, width]. A sequence that starts at
  * position 0 starts from zero, whatever the row holds.
  *   skyrl_rglru_step    decode: token s is the one token of sequence s, row rows[s] (< 0: skipped).
- *   skyrl_rglru_prompt  u T [T, width] from skyrl_conv_chunk; chunks as there, seq_chunks[i] .. seq_chunks[i + 1] - 1
- *                       those of sequence seq0 + i. Scratch: hbuf, abuf f32 [T, width], s_in f32 [nchunks, width].
+ *   skyrl_rglru_prompt  u T [T, width] from skyrl_conv_chunk; chunks as there, their fourth number the run they belong
+ *                       to; runs i32 [nruns, 4]: first chunk, chunks, sequence, unused; seq_runs[i] .. seq_runs[i + 1]
+ *                       - 1 those of sequence seq0 + i. Scratch: hbuf, abuf f32 [T, width], s_in f32 [nruns, width].
  *                       skyrl_conv_save stores the ring. */
 int skyrl_rglru_step(const void* proj, int64_t proj_stride, int32_t width, int32_t blocks, int32_t taps,
                      const float* conv_t, const float* conv_b, const void* gate_w, const float* gate_b,
@@ -249,8 +255,8 @@ int skyrl_rglru_step(const void* proj, int64_t proj_stride, int32_t width, int32
                      void* ring, void* out, int64_t out_stride, int32_t dtype, void* stream);
 int skyrl_rglru_prompt(const void* proj, int64_t proj_stride, int32_t width, int32_t blocks, const void* u,
                        const void* gate_w, const float* gate_b, const float* rate, const int32_t* chunk,
-                       int32_t nchunks, const int32_t* seq_chunks, int32_t seq0, int32_t nseq, const int32_t* cu,
-                       const int32_t* rows, const int64_t* positions, float* state, float* hbuf, float* abuf,
+                       int32_t nchunks, const int32_t* runs, int32_t nruns, const int32_t* seq_runs, int32_t seq0,
+                       int32_t nseq, const int32_t* cu, const int32_t* rows, const int64_t* positions, float* state, float* hbuf, float* abuf,
                        float* s_in, void* out, int64_t out_stride, int32_t dtype, void* stream);
 
 /* ---- grouped attention with normed queries and keys, a window and an output gate ---------------
@@ -299,8 +305,7 @@ int skyrl_attn_prefill(const skyrl_attn_shape* shape, const void* q, const void*
  *                     32; padding zero). super i32 [nsuper, 4]: first chunk, chunks, sequence, 1 if the sequence has
  *                     several such runs + 2 if its last; pick i32 [npick]: the runs that are followed by another of
  *                     their sequence; chain i32 [nchain, 2]: first run and number of runs of the sequences with
- *                     several. Scratch: runs f32 [nsuper, heads, np, vp], gtot f32 [nsuper, heads].
- *   skyrl_gated_norm  out T [n, width] = rms over each of `groups` equal parts of y silu(z), times weight T [width]. */
+ *                     several. Scratch: scores f32 [nchunks, groups, 10, 256], runs f32 [nsuper, heads, np, vp], gtot f32 [nsuper, heads]. */
 typedef struct skyrl_ssd_shape {
     int32_t heads, vdim, state, groups, taps;
 } skyrl_ssd_shape;
@@ -310,13 +315,10 @@ int skyrl_ssd_scan(const skyrl_ssd_shape* shape, const void* proj, int64_t proj_
                    int32_t save_conv, void* y, int64_t y_stride, int32_t dtype, void* stream);
 int skyrl_ssd_prompt(const skyrl_ssd_shape* shape, const void* xt, const void* bt, const void* brow, const void* crow,
                      const void* dt_raw, int64_t dt_stride, const float* a_log, const float* dt_bias,
-                     const float* skip, const int32_t* chunk, const int32_t* super, int32_t nsuper,
-                     const int32_t* pick, int32_t npick, const int32_t* chain, int32_t nchain, const int32_t* cu,
-                     const int32_t* rows, const int64_t* positions, float* state, float* runs, float* gtot, void* y,
-                     int64_t y_stride, void* stream);
-int skyrl_gated_norm(const void* y, int64_t y_stride, const void* z, int64_t z_stride, const void* weight, int64_t n,
-                     int32_t width, int32_t groups, float eps, void* out, int64_t out_stride, int32_t dtype,
-                     void* stream);
+                     const float* skip, const int32_t* chunk, int32_t nchunks, const int32_t* super,
+                     int32_t nsuper, const int32_t* pick, int32_t npick, const int32_t* chain, int32_t nchain,
+                     const int32_t* cu, const int32_t* rows, const int64_t* positions, float* state, float* scores,
+                     float* runs, float* gtot, void* y, int64_t y_stride, void* stream);
 
 #ifdef __cplusplus
 }

@@ -20,5 +20,6 @@ def require_native():
     """Load the HIP libraries (raises ImportError if one was not built)."""
     from . import _ffi
 
-    _ffi.load_layers()
+    for lib in _ffi.LAYER_LIBS:
+        _ffi.load_layers(lib)
     return _ffi.load()

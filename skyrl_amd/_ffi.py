@@ -21,7 +21,9 @@ import torch  # noqa: F401  (must precede the CDLL load, see module docstring)
 
 LIB_DIR = os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libskyrl_hip.so")
-LAYERS_PATH = os.path.join(LIB_DIR, "libskyrl_layers.so")
+# the hybrid decoders' layer libraries: what every such model needs, and one per mechanism, whose entry points
+# start with skyrl_<name>_
+LAYER_LIBS = ("layers", "latent", "delta", "diff", "rglru", "attn", "ssd")
 
 F32, BF16, I64, I32, U8 = 0, 1, 2, 3, 4
 M_FINAL_LOSS, M_POLICY_LOSS, M_ENTROPY, M_KL, M_CLIP_RATIO, M_MASK_SUM = 0, 1, 2, 3, 4, 5
@@ -257,7 +259,7 @@ class SSDShape(ctypes.Structure):
     _fields_ = [(n, ctypes.c_int32) for n in ("heads", "vdim", "state", "groups", "taps")]
 
 
-# the exported surface of include/skyrl_layers.h, in a library of its own (libskyrl_layers.so)
+# the exported surface of include/skyrl_layers.h, in libraries of its own (LAYER_LIBS)
 _DS = ctypes.POINTER(DeltaShape)
 _FS = ctypes.POINTER(DiffShape)
 _AS = ctypes.POINTER(AttnShape)
@@ -294,16 +296,16 @@ LAYERS_SIGNATURES = {
                                 ctypes.POINTER(ConvSection), _I32, _I32, _P]),
     "skyrl_rglru_step": (_INT, [_P, _I64, _I32, _I32, _I32, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _I64, _I32,
                                 _P]),
-    "skyrl_rglru_prompt": (_INT, [_P, _I64, _I32, _I32, _P, _P, _P, _P, _P, _I32, _P, _I32, _I32, _P, _P, _P, _P, _P,
-                                  _P, _P, _P, _I64, _I32, _P]),
+    "skyrl_rglru_prompt": (_INT, [_P, _I64, _I32, _I32, _P, _P, _P, _P, _P, _I32, _P, _I32, _P, _I32, _I32, _P, _P, _P,
+                                  _P, _P, _P, _P, _P, _I64, _I32, _P]),
     "skyrl_attn_write": (_INT, [_AS, _P, _I64, _P, _P, _P, _P, _I32, _I32, _P, _P, _P, _I32, _P]),
     "skyrl_attn_mfma": (_INT, [_AS, _I32]),
     "skyrl_attn_attend_workspace_bytes": (_SZ, [_AS, _I32, _I32]),
     "skyrl_attn_attend": (_INT, [_AS, _P, _P, _I64, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _I64, _P, _I32, _P]),
     "skyrl_attn_prefill": (_INT, [_AS, _P, _P, _I64, _P, _P, _P, _I64, _P, _I32, _P, _I64, _P]),
     "skyrl_ssd_scan": (_INT, [_SS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I32, _P, _I64, _I32, _P]),
-    "skyrl_ssd_prompt": (_INT, [_SS, _P, _P, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I32, _P, _I32, _P, _I32, _P, _P, _P,
-                                _P, _P, _P, _P, _I64, _P]),
+    "skyrl_ssd_prompt": (_INT, [_SS, _P, _P, _P, _P, _P, _I64, _P, _P, _P, _P, _I32, _P, _I32, _P, _I32, _P, _I32, _P, _P,
+                                _P, _P, _P, _P, _P, _P, _I64, _P]),
     "skyrl_gated_norm": (_INT, [_P, _I64, _P, _I64, _P, _I64, _I32, _I32, _F, _P, _I64, _I32, _P]),
 }
 
@@ -386,15 +388,25 @@ def load() -> ctypes.CDLL:
     return _open(LIB_PATH, SIGNATURES)
 
 
-def load_layers() -> ctypes.CDLL:
-    """libskyrl_layers.so, likewise."""
-    lib = _open(LAYERS_PATH, LAYERS_SIGNATURES)
-    lib.skyrl_last_error.restype = ctypes.c_char_p
-    return lib
+def layer_lib_path(lib: str) -> str:
+    return os.path.join(LIB_DIR, "libskyrl_layers.so" if lib == "layers" else f"libskyrl_layer_{lib}.so")
+
+
+def layer_lib_of(name: str) -> str:
+    """The layer library that exports an entry point of include/skyrl_layers.h."""
+    word = name.split("_")[1]
+    return word if word in LAYER_LIBS else "layers"
+
+
+def load_layers(lib: str = "layers") -> ctypes.CDLL:
+    """One of LAYER_LIBS, likewise."""
+    out = _open(layer_lib_path(lib), {n: s for n, s in LAYERS_SIGNATURES.items() if layer_lib_of(n) == lib})
+    out.skyrl_last_error.restype = ctypes.c_char_p
+    return out
 
 
 def _lib_of(name: str) -> ctypes.CDLL:
-    return load_layers() if name in LAYERS_SIGNATURES else load()
+    return load_layers(layer_lib_of(name)) if name in LAYERS_SIGNATURES else load()
 
 
 def call(name: str, *args) -> int:

@@ -54,21 +54,36 @@ __global__ __launch_bounds__(kNT) void conv_chunk_kernel(ConvArgs<T> p) {
             ldv<T, VEC>(ring + (int64_t)((pos0 + i) % p.taps) * p.channels, o);
         }
     };
+    // all inputs are the step's own: no case to tell apart
+    const bool inner = n == kC && t0 - (p.taps - 1) >= sfirst;
     float y[kRun][VEC];
     float b[VEC];
 #pragma unroll
     for (int v = 0; v < VEC; ++v) b[v] = 0.f;
+    if (r0 >= n) {
+#pragma unroll
+        for (int j = 0; j < kRun; ++j)
+#pragma unroll
+            for (int v = 0; v < VEC; ++v) y[j][v] = 0.f;
+    }
     if (p.bias) ldv<float, VEC>(p.bias + ch, b);
     if (r0 < n) {
         if constexpr (TW > 0) {
             float x[TW - 1 + kRun][VEC];
+            if (inner) {
+                const T* src = p.x + (int64_t)(t0 + r0 - (TW - 1)) * p.stride + ch;
 #pragma unroll
-            for (int k = 0; k < TW - 1 + kRun; ++k) {
-                if (k >= TW - p.taps) {
-                    input(r0 + k - (TW - 1), x[k]);
-                } else {
+                for (int k = 0; k < TW - 1 + kRun; ++k)
+                    ldv<T, VEC>(src + max(k, TW - p.taps) * p.stride, x[k]);  // rows before the filter are not used
+            } else {
 #pragma unroll
-                    for (int v = 0; v < VEC; ++v) x[k][v] = 0.f;
+                for (int k = 0; k < TW - 1 + kRun; ++k) {
+                    if (k >= TW - p.taps) {
+                        input(r0 + k - (TW - 1), x[k]);
+                    } else {
+#pragma unroll
+                        for (int v = 0; v < VEC; ++v) x[k][v] = 0.f;
+                    }
                 }
             }
 #pragma unroll
@@ -106,8 +121,8 @@ __global__ __launch_bounds__(kNT) void conv_chunk_kernel(ConvArgs<T> p) {
     for (int j = 0; j < kRun; ++j)
 #pragma unroll
         for (int v = 0; v < VEC; ++v) {
+            if (p.act == SKYRL_CONV_SILU) y[j][v] = y[j][v] * sigmoid_<T>(y[j][v]);
             if (r0 + j >= n) y[j][v] = 0.f;
-            else if (p.act == SKYRL_CONV_SILU) y[j][v] = y[j][v] * sigmoid_<T>(y[j][v]);
         }
     int k = 0;
     while (k + 1 < p.nsec && ch >= p.sec[k + 1].first) ++k;

@@ -1,4 +1,4 @@
-// Embedding, norms, gated activations, convolution state and the logit cap of the hybrid decoders
+// Embedding, norms, activations, convolution state and the logit cap of the hybrid decoders
 // (include/skyrl_layers.h). The residual stream stays f32 in HBM: the add, the norm and the optional
 // per-pass step vector of a looped layer stack are one pass over a row.
 #include "conv.h"
@@ -329,6 +329,66 @@ __global__ __launch_bounds__(kNT) void softcap_kernel(const T* __restrict__ x, f
     }
 }
 
+// ---- out = rms over each of `groups` equal parts of y silu(z), times w; one workgroup per (token, part) ----
+// Up to kMax groups of VEC values per thread in registers; HOLD false: any length, formed twice.
+template <typename T, int NT, int VEC, int kMax, bool HOLD>
+__global__ __launch_bounds__(NT) void gated_norm_kernel(const T* __restrict__ y, int64_t y_stride,
+                                                        const T* __restrict__ z, int64_t z_stride,
+                                                        const T* __restrict__ w, int groups, int len, float eps,
+                                                        T* __restrict__ out, int64_t out_stride) {
+    __shared__ float s_red[NT / kWave];
+    const int64_t t = blockIdx.x / groups;
+    const int c0 = (int)(blockIdx.x % groups) * len, nv = len / VEC;
+    const T* yp = y + t * y_stride + c0;
+    const T* zp = z + t * z_stride + c0;
+    float a[HOLD ? kMax : 1][VEC];
+    auto form = [&](int v, float (&o)[VEC]) {
+        float zz[VEC];
+        ldv<T, VEC>(yp + VEC * v, o);
+        ldv<T, VEC>(zp + VEC * v, zz);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) o[j] *= zz[j] * sigmoid_<T>(zz[j]);
+    };
+    float ss = 0.f;
+    if constexpr (HOLD) {
+#pragma unroll
+        for (int k = 0; k < kMax; ++k) {
+            const int v = threadIdx.x + k * NT;
+            if (v < nv) {
+                form(v, a[k]);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) ss += a[k][j] * a[k][j];
+            }
+        }
+    } else {
+        for (int v = threadIdx.x; v < nv; v += NT) {
+            form(v, a[0]);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) ss += a[0][j] * a[0][j];
+        }
+    }
+    const float r = 1.f / sqrtf(block_total<NT>(ss, s_red) / (float)len + eps);
+    auto put = [&](int v, float (&o)[VEC]) {
+        float ww[VEC];
+        ldv<T, VEC>(w + c0 + VEC * v, ww);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) o[j] *= r * ww[j];
+        stv(out + t * out_stride + c0 + VEC * v, o);
+    };
+    if constexpr (HOLD) {
+#pragma unroll
+        for (int k = 0; k < kMax; ++k) {
+            const int v = threadIdx.x + k * NT;
+            if (v < nv) put(v, a[k]);
+        }
+    } else {
+        for (int v = threadIdx.x; v < nv; v += NT) {
+            form(v, a[0]);
+            put(v, a[0]);
+        }
+    }
+}
+
 unsigned grid_for(int64_t items) {
     const int64_t b = (items + kNT - 1) / kNT;
     return (unsigned)(b > 8192 ? 8192 : b);
@@ -485,4 +545,34 @@ extern "C" int skyrl_softcap(const void* x, float* out, int64_t count, float cap
                            reinterpret_cast<const T*>(x), out, count, cap);
     })
     return check_launch("softcap_kernel");
+}
+
+#define LAUNCH_GNORM(NT, VEC, K, HOLD)                                                                               \
+    hipLaunchKernelGGL((gated_norm_kernel<T, NT, VEC, K, HOLD>), dim3((unsigned)(n * groups)), dim3(NT), 0,          \
+                       as_stream(stream), y_, y_stride, z_, z_stride, w_, groups, len, eps, o_, out_stride)
+
+extern "C" int skyrl_gated_norm(const void* y, int64_t y_stride, const void* z, int64_t z_stride, const void* weight,
+                                int64_t n, int32_t width, int32_t groups, float eps, void* out, int64_t out_stride,
+                                int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "gated_norm");
+    SKYRL_REQUIRE(n >= 0 && width > 0 && groups > 0 && width % groups == 0 && n * groups < (1ll << 31) &&
+                      y_stride >= width && z_stride >= width && out_stride >= width,
+                  "gated_norm: bad sizes");
+    if (n == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(y && z && weight && out, "gated_norm: null pointer");
+    const int len = width / groups;
+    SKYRL_DISPATCH_T(dtype, {
+        const T* y_ = reinterpret_cast<const T*>(y);
+        const T* z_ = reinterpret_cast<const T*>(z);
+        const T* w_ = reinterpret_cast<const T*>(weight);
+        T* o_ = reinterpret_cast<T*>(out);
+        const bool wide = len % 8 == 0 && y_stride % 8 == 0 && z_stride % 8 == 0 && out_stride % 8 == 0 &&
+                          aligned16(y) && aligned16(z) && aligned16(weight) && aligned16(out);
+        if (wide && len <= 512) LAUNCH_GNORM(64, 8, 1, true);
+        else if (wide && len <= 2048) LAUNCH_GNORM(256, 8, 1, true);
+        else if (wide && len <= 8192) LAUNCH_GNORM(256, 8, 4, true);
+        else if (wide) LAUNCH_GNORM(256, 8, 1, false);
+        else LAUNCH_GNORM(256, 1, 1, false);
+    })
+    return check_launch("gated_norm_kernel");
 }

@@ -7,10 +7,11 @@
 // Decode (rglru_step): the rows are 16 sequences' tokens. Convolution, gates, state update and output gate in
 // one launch.
 //
-// Prompts (rglru_gates, rglru_chain, rglru_out): the rows are consecutive tokens of a chunk of 64. A state from
-// a chunk's own tokens and the product of the decays up to each token give S_t = h_t + A_t S_in, so chunks are
-// independent but for one multiply-add per chunk and channel (rglru_chain). Within a chunk the pairs (A, h)
-// compose along the accumulators: four tokens in a lane, four lane groups by shuffles, four tiles in order.
+// Prompts (rglru_gates, rglru_chain, rglru_out): the rows are consecutive tokens of a chunk of 64, a workgroup
+// walks a run of chunks. A state from the run's own tokens and the product of the decays up to each token give
+// S_t = h_t + A_t S_in, so runs are independent but for one multiply-add per run and channel (rglru_chain).
+// Within a chunk the pairs (A, h) compose along the accumulators: four tokens in a lane, four lane groups by
+// shuffles, four tiles in order.
 #include "conv.h"
 
 namespace skyrl {
@@ -18,9 +19,8 @@ namespace {
 
 constexpr int kNT = 256;
 constexpr int kC = 64;     // tokens per chunk
-// input channels of a block in LDS at a time (prompts)
-template <typename T>
-constexpr int kSlab = sizeof(T) == 2 ? 256 : 128;
+constexpr int kSlab = 128; // input channels of a block in LDS at a time (prompts)
+constexpr int kHeld = 4;   // 32-wide steps of the gate matrices held in registers
 
 typedef short s16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
@@ -39,22 +39,61 @@ struct Gates {
     const float* rate;  // [W]: log a = rate r
 };
 
-// acc += A (16 rows from LDS) B^T (16 rows of w), 32 inputs.
-__device__ __forceinline__ f32x4 product32(const uint16_t* a, const uint16_t* b, int g, f32x4 acc) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const s16x8*>(a + 8 * g),
-                                                   *reinterpret_cast<const s16x8*>(b + 8 * g), acc, 0, 0, 0);
+// A lane's part of 16 rows of a 32-wide operand, and acc += A B^T over it.
+template <typename T>
+struct Frag;
+template <>
+struct Frag<uint16_t> {
+    s16x8 x;
+    __device__ __forceinline__ void load(const uint16_t* row, int g) { x = *reinterpret_cast<const s16x8*>(row + 8 * g); }
+};
+template <>
+struct Frag<float> {
+    float4 x[2];
+    __device__ __forceinline__ void load(const float* row, int g) {
+        x[0] = ld4(row + 4 * g);
+        x[1] = ld4(row + 16 + 4 * g);
+    }
+};
+__device__ __forceinline__ f32x4 product32(const Frag<uint16_t>& a, const Frag<uint16_t>& b, f32x4 acc) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.x, b.x, acc, 0, 0, 0);
 }
-__device__ __forceinline__ f32x4 product32(const float* a, const float* b, int g, f32x4 acc) {
+__device__ __forceinline__ f32x4 product32(const Frag<float>& a, const Frag<float>& b, f32x4 acc) {
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
-        const float4 x = ld4(a + 16 * s + 4 * g), y = ld4(b + 16 * s + 4 * g);
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, acc, 0, 0, 0);
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x[s].x, b.x[s].x, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x[s].y, b.x[s].y, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x[s].z, b.x[s].z, acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x[s].w, b.x[s].w, acc, 0, 0, 0);
     }
     return acc;
 }
+
+// VEC consecutive elements on their way to LDS.
+template <typename T, int VEC>
+struct Piece {
+    static constexpr int kWords = VEC * sizeof(T) / 16;
+    uint4 w[kWords];
+    __device__ __forceinline__ void clear() {
+#pragma unroll
+        for (int i = 0; i < kWords; ++i) w[i] = make_uint4(0, 0, 0, 0);
+    }
+    __device__ __forceinline__ void load(const T* p) {
+#pragma unroll
+        for (int i = 0; i < kWords; ++i) w[i] = reinterpret_cast<const uint4*>(p)[i];
+    }
+    __device__ __forceinline__ void store(T* p) const {
+#pragma unroll
+        for (int i = 0; i < kWords; ++i) reinterpret_cast<uint4*>(p)[i] = w[i];
+    }
+};
+template <typename T>
+struct Piece<T, 1> {
+    T w;
+    __device__ __forceinline__ void clear() { w = 0; }
+    __device__ __forceinline__ void load(const T* p) { w = *p; }
+    __device__ __forceinline__ void store(T* p) const { *p = w; }
+};
 
 // Decay a and input b of S <- a S + b from the gates' sums: b = sqrt(1 - a^2) i u.
 template <typename T>
@@ -87,6 +126,27 @@ __global__ __launch_bounds__(kNT) void rglru_step_kernel(Dims d, const T* __rest
     const int blk = blockIdx.x / ns, split = blockIdx.x - blk * ns, q0 = 16 * blockIdx.y;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c = lane & 15, g = lane >> 4;
+    const int o0 = 64 * split + 16 * wave, ks = d.kp() / 32;
+    const bool on = o0 < d.np();
+    const T* wr = gt.w + ((int64_t)blk * 2 * d.np() + (on ? o0 : 0) + c) * d.kp();
+    const T* wi = wr + (int64_t)d.np() * d.kp();
+    // what does not wait for the convolution: matrices, states, output gates
+    Frag<T> fr[kHeld], fi[kHeld];
+#pragma unroll
+    for (int k = 0; k < kHeld; ++k) {
+        if (k < ks) {
+            fr[k].load(wr + 32 * k, g);
+            fi[k].load(wi + 32 * k, g);
+        }
+    }
+    const int ch_own = blk * d.bs + min(o0 + c, d.bs - 1);
+    float old[4], yg[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int s = min(q0 + 4 * g + i, n - 1), row = rows[s];
+        old[i] = row >= 0 && positions[s] > 0 ? state[(int64_t)row * d.W + ch_own] : 0.f;
+        yg[i] = ld(proj + (int64_t)s * stride + ch_own);
+    }
     const int pieces = d.kp() / VEC;
     for (int e = tid; e < 16 * pieces; e += kNT) {
         const int i = e / pieces, k = (e - i * pieces) * VEC, s = q0 + i;
@@ -106,17 +166,26 @@ __global__ __launch_bounds__(kNT) void rglru_step_kernel(Dims d, const T* __rest
         stv(s_u + i * LD + k, y);
     }
     __syncthreads();
-    const int o0 = 64 * split + 16 * wave;
-    if (o0 >= d.np()) return;
+    if (!on) return;
     f32x4 ar = {0.f, 0.f, 0.f, 0.f}, ai = ar;
-    const T* wr = gt.w + ((int64_t)blk * 2 * d.np() + o0 + c) * d.kp();
-    const T* wi = wr + (int64_t)d.np() * d.kp();
-    for (int k = 0; k < d.kp(); k += 32) {
-        ar = product32(s_u + c * LD + k, wr + k, g, ar);
-        ai = product32(s_u + c * LD + k, wi + k, g, ai);
+    Frag<T> fu;
+#pragma unroll
+    for (int k = 0; k < kHeld; ++k) {
+        if (k < ks) {
+            fu.load(s_u + c * LD + 32 * k, g);
+            ar = product32(fu, fr[k], ar);
+            ai = product32(fu, fi[k], ai);
+        }
+    }
+    for (int k = kHeld; k < ks; ++k) {
+        fu.load(s_u + c * LD + 32 * k, g);
+        fr[0].load(wr + 32 * k, g);
+        fi[0].load(wi + 32 * k, g);
+        ar = product32(fu, fr[0], ar);
+        ai = product32(fu, fi[0], ai);
     }
     if (o0 + c >= d.bs) return;
-    const int ch = blk * d.bs + o0 + c;
+    const int ch = ch_own;
     const float br = gt.bias[ch], bi = gt.bias[d.W + ch], rate = gt.rate[ch];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -124,140 +193,200 @@ __global__ __launch_bounds__(kNT) void rglru_step_kernel(Dims d, const T* __rest
         if (s >= n) break;
         const int row = rows[s];
         if (row < 0) continue;
-        float* st_ = state + (int64_t)row * d.W + ch;
         float a, b;
         recurrence_of<T>(ar[i] + br, ai[i] + bi, ld(s_u + (4 * g + i) * LD + o0 + c), rate, a, b);
-        const float S = positions[s] > 0 ? a * *st_ + b : b;
-        *st_ = S;
-        st(out + (int64_t)s * out_stride + ch, S * gelu_tanh_<T>(ld(proj + (int64_t)s * stride + ch)));
+        const float S = fmaf(a, old[i], b);
+        state[(int64_t)row * d.W + ch] = S;
+        st(out + (int64_t)s * out_stride + ch, S * gelu_tanh_<T>(yg[i]));
     }
 }
 
-// ---- prompts, step 1: gates and each chunk's own states; grid (nb splits, nchunks) ------------------
-template <typename T, int VEC>
-__global__ __launch_bounds__(kNT) void rglru_gates_kernel(Dims d, const T* __restrict__ u, Gates<T> gt,
-                                                          const int32_t* __restrict__ chunk, float* __restrict__ hbuf,
+// ---- prompts, step 1: gates and each run's own states; grid (nb splits, nruns) ----------------------
+// FIT: a block's inputs are one slab, so that its matrices stay in registers and the next chunk's inputs are
+// on their way while a chunk is finished.
+template <typename T, int VEC, bool FIT>
+__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(sizeof(T) == 2 ? 4 : 2))) void rglru_gates_kernel(Dims d, const T* __restrict__ u, Gates<T> gt,
+                                                          const int32_t* __restrict__ chunk,
+                                                          const int32_t* __restrict__ runs, float* __restrict__ hbuf,
                                                           float* __restrict__ abuf) {
-    extern __shared__ __attribute__((aligned(16))) char smem[];
-    T* s_u = reinterpret_cast<T*>(smem);
-    const int kw = min(d.kp(), kSlab<T>), LD = kw + 16 / (int)sizeof(T), ns = d.splits();
+    constexpr int LD = kSlab + 16 / (int)sizeof(T);
+    constexpr int kPieces = FIT && VEC > 1 ? kC * kSlab / VEC / kNT : 1;  // of a thread, per chunk
+    __shared__ __attribute__((aligned(16))) T s_u[kC * LD];
+    const int ns = d.splits(), kp = d.kp();
     const int blk = blockIdx.x / ns, split = blockIdx.x - blk * ns;
-    const int32_t* ck = chunk + 4 * blockIdx.y;
-    const int t0 = ck[0], n = ck[1];
+    const int c0 = runs[4 * blockIdx.y], c1 = c0 + runs[4 * blockIdx.y + 1];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c = lane & 15, g = lane >> 4;
     const int o0 = 64 * split + 16 * wave;
-    const bool on = o0 < d.np();
-    const int tiles = (n + 15) / 16;
-    f32x4 ar[4], ai[4];
+    const bool on = o0 < d.np(), real = on && o0 + c < d.bs;
+    const T* wr = gt.w + ((int64_t)blk * 2 * d.np() + (on ? o0 : 0) + c) * kp;
+    const T* wi = wr + (int64_t)d.np() * kp;
+    const T* ub = u + blk * d.bs;
+    Frag<T> fr[kHeld], fi[kHeld];
+    if constexpr (FIT) {
 #pragma unroll
-    for (int t = 0; t < 4; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const T* wr = gt.w + ((int64_t)blk * 2 * d.np() + (on ? o0 : 0) + c) * d.kp();
-    const T* wi = wr + (int64_t)d.np() * d.kp();
-    for (int k0 = 0; k0 < d.kp(); k0 += kSlab<T>) {
-        const int w = min(kSlab<T>, d.kp() - k0), pieces = w / VEC;
-        __syncthreads();
-        for (int e = tid; e < 16 * tiles * pieces; e += kNT) {
-            const int i = e / pieces, k = (e - i * pieces) * VEC;
-            float y[VEC];
-#pragma unroll
-            for (int v = 0; v < VEC; ++v) y[v] = 0.f;
-            if (i < n && k0 + k < d.bs) ldv<T, VEC>(u + (int64_t)(t0 + i) * d.W + blk * d.bs + k0 + k, y);
-            stv(s_u + i * LD + k, y);
+        for (int k = 0; k < kHeld; ++k) {
+            if (32 * k < kp) {
+                fr[k].load(wr + 32 * k, g);
+                fi[k].load(wi + 32 * k, g);
+            }
         }
-        __syncthreads();
-        if (!on) continue;
-        for (int k = 0; k < w; k += 32) {
+    }
+    const int och = real ? o0 + c : 0, ch = blk * d.bs + och;
+    const float br = gt.bias[ch], bi = gt.bias[d.W + ch], rate = gt.rate[ch];
+    float CA = 1.f, CB = 0.f;  // decay and state over the run so far
+
+    // token e / pieces of a chunk, inputs k0 + VEC (e % pieces) .. of the block, zero past their ends
+    auto fetch = [&](int t0, int n, int k0, int e, int pieces, Piece<T, VEC>& y) {
+        const int i = e / pieces, k = (e - i * pieces) * VEC;
+        y.clear();
+        if (i < n && k0 + k < d.bs) y.load(ub + (int64_t)(t0 + i) * d.W + k0 + k);
+    };
+    auto place = [&](int e, int pieces, const Piece<T, VEC>& y) {
+        const int i = e / pieces, k = (e - i * pieces) * VEC;
+        y.store(s_u + i * LD + k);
+    };
+    Piece<T, VEC> held[kPieces];
+    const int fitp = kp / VEC;
+    if constexpr (kPieces > 1) {
 #pragma unroll
-            for (int t = 0; t < 4; ++t) {
-                if (t < tiles) {
-                    ar[t] = product32(s_u + (16 * t + c) * LD + k, wr + k0 + k, g, ar[t]);
-                    ai[t] = product32(s_u + (16 * t + c) * LD + k, wi + k0 + k, g, ai[t]);
+        for (int j = 0; j < kPieces; ++j)
+            if (tid + j * kNT < kC * fitp) fetch(chunk[4 * c0], chunk[4 * c0 + 1], 0, tid + j * kNT, fitp, held[j]);
+    }
+    for (int ci = c0; ci < c1; ++ci) {
+        const int t0 = chunk[4 * ci], n = chunk[4 * ci + 1];
+        f32x4 ar[4], ai[4];
+#pragma unroll
+        for (int t = 0; t < 4; ++t) ar[t] = ai[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int k0 = 0; k0 < kp; k0 += kSlab) {
+            const int w = min(kSlab, kp - k0), pieces = w / VEC;
+            __syncthreads();
+            if constexpr (kPieces > 1) {
+#pragma unroll
+                for (int j = 0; j < kPieces; ++j)
+                    if (tid + j * kNT < kC * fitp) place(tid + j * kNT, fitp, held[j]);
+            } else {
+                for (int e = tid; e < kC * pieces; e += kNT) {
+                    Piece<T, VEC> y;
+                    fetch(t0, n, k0, e, pieces, y);
+                    place(e, pieces, y);
+                }
+            }
+            __syncthreads();
+            if constexpr (kPieces > 1) {
+                if (ci + 1 < c1) {
+#pragma unroll
+                    for (int j = 0; j < kPieces; ++j)
+                        if (tid + j * kNT < kC * fitp)
+                            fetch(chunk[4 * ci + 4], chunk[4 * ci + 5], 0, tid + j * kNT, fitp, held[j]);
+                }
+            }
+            if (!on) continue;
+#pragma unroll
+            for (int k = 0; k < kSlab / 32; ++k) {
+                if (32 * k >= w) break;
+                if constexpr (!FIT) {
+                    fr[0].load(wr + k0 + 32 * k, g);
+                    fi[0].load(wi + k0 + 32 * k, g);
+                }
+#pragma unroll
+                for (int t = 0; t < 4; ++t) {
+                    Frag<T> fu;
+                    fu.load(s_u + (16 * t + c) * LD + 32 * k, g);
+                    ar[t] = product32(fu, fr[FIT ? k : 0], ar[t]);
+                    ai[t] = product32(fu, fi[FIT ? k : 0], ai[t]);
                 }
             }
         }
-    }
-    if (!on) return;
-    const bool real = o0 + c < d.bs;
-    const int ch = blk * d.bs + (real ? o0 + c : 0);
-    const float br = gt.bias[ch], bi = gt.bias[d.W + ch], rate = gt.rate[ch];
-    float CA = 1.f, CB = 0.f;  // decay and state over the tiles so far
+        if (!on) continue;
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
-        if (t >= tiles) break;
-        float A[4], B[4];  // prefixes of this lane's four tokens
+        for (int t = 0; t < 4; ++t) {
+            if (16 * t >= n) break;
+            float A[4], B[4];  // prefixes of this lane's four tokens
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int j = 16 * t + 4 * g + i;
-            float a = 1.f, b = 0.f;
-            if (j < n)
-                recurrence_of<T>(ar[t][i] + br, ai[t][i] + bi, ld(u + (int64_t)(t0 + j) * d.W + ch), rate, a, b);
-            A[i] = i ? a * A[i - 1] : a;
-            B[i] = i ? fmaf(a, B[i - 1], b) : b;
-        }
-        float TA = A[3], TB = B[3];
-#pragma unroll
-        for (int o = 16; o <= 32; o <<= 1) {
-            const float pa = __shfl_up(TA, o, kWave), pb = __shfl_up(TB, o, kWave);
-            if (lane >= o) {
-                TB = fmaf(TA, pb, TB);
-                TA *= pa;
+            for (int i = 0; i < 4; ++i) {
+                const int j = 16 * t + 4 * g + i;
+                float x, a, b;
+                if constexpr (FIT) x = ld(s_u + j * LD + och);
+                else x = ld(ub + (int64_t)(t0 + min(j, n - 1)) * d.W + och);
+                recurrence_of<T>(ar[t][i] + br, ai[t][i] + bi, x, rate, a, b);
+                if (j >= n) {
+                    a = 1.f;
+                    b = 0.f;
+                }
+                A[i] = i ? a * A[i - 1] : a;
+                B[i] = i ? fmaf(a, B[i - 1], b) : b;
             }
-        }
-        float ea = __shfl_up(TA, 16, kWave), eb = __shfl_up(TB, 16, kWave);
-        if (g == 0) {
-            ea = 1.f;
-            eb = 0.f;
-        }
-        const float PA = ea * CA, PB = fmaf(ea, CB, eb);
+            float TA = A[3], TB = B[3];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int j = 16 * t + 4 * g + i;
-            if (j < n && real) {
-                const int64_t e = (int64_t)(t0 + j) * d.W + ch;
-                hbuf[e] = fmaf(A[i], PB, B[i]);
-                abuf[e] = A[i] * PA;
+            for (int o = 16; o <= 32; o <<= 1) {
+                const float pa = __shfl_up(TA, o, kWave), pb = __shfl_up(TB, o, kWave);
+                if (lane >= o) {
+                    TB = fmaf(TA, pb, TB);
+                    TA *= pa;
+                }
             }
+            float ea = __shfl_up(TA, 16, kWave), eb = __shfl_up(TB, 16, kWave);
+            if (g == 0) {
+                ea = 1.f;
+                eb = 0.f;
+            }
+            const float PA = ea * CA, PB = fmaf(ea, CB, eb);
+            const int64_t e = (int64_t)(t0 + 16 * t + 4 * g) * d.W + ch;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if (16 * t + 4 * g + i < n && real) {
+                    hbuf[e + i * d.W] = fmaf(A[i], PB, B[i]);
+                    abuf[e + i * d.W] = A[i] * PA;
+                }
+            }
+            const float la = __shfl(TA, 48 + c, kWave), lb = __shfl(TB, 48 + c, kWave);
+            CB = fmaf(la, CB, lb);
+            CA *= la;
         }
-        const float la = __shfl(TA, 48 + c, kWave), lb = __shfl(TB, 48 + c, kWave);
-        CB = fmaf(la, CB, lb);
-        CA *= la;
     }
 }
 
-// ---- step 2: the state before every chunk, and the sequence's last; grid (ceil(W / 64), nseq) -------
+// ---- step 2: the state before every run, and the sequence's last; grid (ceil(W / 64), nseq) ---------
 __global__ __launch_bounds__(kWave) void rglru_chain_kernel(int W, const int32_t* __restrict__ chunk,
-                                                            const int32_t* __restrict__ seq_chunks,
+                                                            const int32_t* __restrict__ runs,
+                                                            const int32_t* __restrict__ seq_runs,
                                                             const int32_t* __restrict__ cu,
                                                             const int32_t* __restrict__ rows,
                                                             const int64_t* __restrict__ positions, int seq0,
                                                             const float* __restrict__ hbuf,
                                                             const float* __restrict__ abuf, float* __restrict__ state,
                                                             float* __restrict__ s_in) {
-    constexpr int kAhead = 16;
-    const int ch = blockIdx.x * kWave + threadIdx.x, si = blockIdx.y, seq = seq0 + si, row = rows[seq];
-    const int c0 = seq_chunks[si], c1 = seq_chunks[si + 1];
-    if (ch >= W || row < 0 || c0 >= c1) return;
-    float* st_ = state + (int64_t)row * W + ch;
+    constexpr int kAhead = 32;
+    const int lane = threadIdx.x, ch = blockIdx.x * kWave + lane, si = blockIdx.y, seq = seq0 + si, row = rows[seq];
+    const int r0 = seq_runs[si], r1 = seq_runs[si + 1];
+    if (row < 0 || r0 >= r1) return;
+    const bool on = ch < W;
+    const int col = on ? ch : 0;
+    float* st_ = state + (int64_t)row * W + col;
     float S = positions[cu[seq]] > 0 ? *st_ : 0.f;
-    for (int b0 = c0; b0 < c1; b0 += kAhead) {
+    for (int b0 = r0; b0 < r1; b0 += kAhead) {
+        int last = 0;  // the last token of run b0 + lane
+        if (lane < kAhead && b0 + lane < r1) {
+            const int ci = runs[4 * (b0 + lane)] + runs[4 * (b0 + lane) + 1] - 1;
+            last = chunk[4 * ci] + chunk[4 * ci + 1] - 1;
+        }
         float a[kAhead], h[kAhead];
 #pragma unroll
         for (int i = 0; i < kAhead; ++i) {
-            const int ci = min(b0 + i, c1 - 1);
-            const int64_t e = (int64_t)(chunk[4 * ci] + chunk[4 * ci + 1] - 1) * W + ch;
+            const int64_t e = (int64_t)__builtin_amdgcn_readlane(last, i) * W + col;
             a[i] = abuf[e];
             h[i] = hbuf[e];
         }
 #pragma unroll
         for (int i = 0; i < kAhead; ++i) {
-            if (b0 + i < c1) {
-                s_in[(int64_t)(b0 + i) * W + ch] = S;
+            if (b0 + i < r1) {
+                if (on) s_in[(int64_t)(b0 + i) * W + col] = S;
                 S = fmaf(a[i], S, h[i]);
             }
         }
     }
-    *st_ = S;
+    if (on) *st_ = S;
 }
 
 // ---- step 3: out = (h + A S_in) gelu(y); grid (ceil(W / (256 VEC)), nchunks, 4): 16 tokens each -----
@@ -268,10 +397,10 @@ __global__ __launch_bounds__(kNT) void rglru_out_kernel(int W, const int32_t* __
                                                         const float* __restrict__ s_in, const T* __restrict__ proj,
                                                         int64_t stride, T* __restrict__ out, int64_t out_stride) {
     const int ch = (blockIdx.x * kNT + threadIdx.x) * VEC;
-    const int t0 = chunk[4 * blockIdx.y], n = chunk[4 * blockIdx.y + 1];
+    const int t0 = chunk[4 * blockIdx.y], n = chunk[4 * blockIdx.y + 1], run = chunk[4 * blockIdx.y + 3];
     if (ch >= W) return;
     float S[VEC];
-    ldv<float, VEC>(s_in + (int64_t)blockIdx.y * W + ch, S);
+    ldv<float, VEC>(s_in + (int64_t)run * W + ch, S);
     const int j1 = min(n, 16 * (int)blockIdx.z + 16);
 #pragma unroll 2
     for (int j = 16 * blockIdx.z; j < j1; ++j) {
@@ -331,21 +460,24 @@ extern "C" int skyrl_rglru_step(const void* proj, int64_t proj_stride, int32_t w
     return check_launch("rglru_step_kernel");
 }
 
+#define LAUNCH_GATES(VEC, FIT)                                                                                    \
+    hipLaunchKernelGGL((rglru_gates_kernel<T, VEC, FIT>), grid, dim3(kNT), 0, s, d, u_, gt, chunk, runs, hbuf, abuf)
+
 extern "C" int skyrl_rglru_prompt(const void* proj, int64_t proj_stride, int32_t width, int32_t blocks,
                                   const void* u, const void* gate_w, const float* gate_b, const float* rate,
-                                  const int32_t* chunk, int32_t nchunks, const int32_t* seq_chunks, int32_t seq0,
-                                  int32_t nseq, const int32_t* cu, const int32_t* rows, const int64_t* positions,
+                                  const int32_t* chunk, int32_t nchunks, const int32_t* runs, int32_t nruns,
+                                  const int32_t* seq_runs, int32_t seq0, int32_t nseq, const int32_t* cu, const int32_t* rows, const int64_t* positions,
                                   float* state, float* hbuf, float* abuf, float* s_in, void* out, int64_t out_stride,
                                   int32_t dtype, void* stream) {
     SKYRL_REQUIRE_T(dtype, "rglru_prompt");
     const Dims d{width, blocks, blocks > 0 ? width / blocks : 0, 1};
     const char* bad = bad_dims(d);
     SKYRL_REQUIRE(!bad, bad);
-    SKYRL_REQUIRE(nchunks >= 0 && nchunks <= 65535 && nseq >= 0 && nseq <= 65535 && seq0 >= 0 &&
+    SKYRL_REQUIRE(nchunks >= 0 && nchunks <= 65535 && nruns >= 0 && nruns <= nchunks && nseq >= 0 && nseq <= 65535 && seq0 >= 0 &&
                       proj_stride >= width && out_stride >= width,
                   "rglru_prompt: bad sizes");
     if (nchunks == 0 || nseq == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(proj && u && gate_w && gate_b && rate && chunk && seq_chunks && cu && rows && positions && state &&
+    SKYRL_REQUIRE(proj && u && gate_w && gate_b && rate && chunk && runs && seq_runs && cu && rows && positions && state &&
                       hbuf && abuf && s_in && out,
                   "rglru_prompt: null pointer");
     SKYRL_REQUIRE(aligned16(u) && aligned16(gate_w) && aligned16(hbuf) && aligned16(abuf) && aligned16(s_in),
@@ -356,12 +488,14 @@ extern "C" int skyrl_rglru_prompt(const void* proj, int64_t proj_stride, int32_t
         const T* u_ = reinterpret_cast<const T*>(u);
         const T* p_ = reinterpret_cast<const T*>(proj);
         T* o_ = reinterpret_cast<T*>(out);
-        const size_t lds = tile_bytes<T>(kC, d.kp() < kSlab<T> ? d.kp() : kSlab<T>);
-        const dim3 grid(d.nb * d.splits(), nchunks);
-        if (d.bs % 8 == 0) hipLaunchKernelGGL((rglru_gates_kernel<T, 8>), grid, dim3(kNT), lds, s, d, u_, gt, chunk, hbuf, abuf);
-        else hipLaunchKernelGGL((rglru_gates_kernel<T, 1>), grid, dim3(kNT), lds, s, d, u_, gt, chunk, hbuf, abuf);
+        const dim3 grid(d.nb * d.splits(), nruns);
+        const bool fit = d.kp() <= kSlab;
+        if (d.bs % 8 == 0 && fit) LAUNCH_GATES(8, true);
+        else if (d.bs % 8 == 0) LAUNCH_GATES(8, false);
+        else if (fit) LAUNCH_GATES(1, true);
+        else LAUNCH_GATES(1, false);
         hipLaunchKernelGGL(rglru_chain_kernel, dim3((d.W + kWave - 1) / kWave, nseq), dim3(kWave), 0, s, d.W, chunk,
-                           seq_chunks, cu, rows, positions, seq0, hbuf, abuf, state, s_in);
+                           runs, seq_runs, cu, rows, positions, seq0, hbuf, abuf, state, s_in);
         if (d.W % 8 == 0 && proj_stride % 8 == 0 && out_stride % 8 == 0 && aligned16(p_) && aligned16(o_))
             hipLaunchKernelGGL((rglru_out_kernel<T, 8>), dim3((d.W + 8 * kNT - 1) / (8 * kNT), nchunks, 4), dim3(kNT),
                                0, s, d.W, chunk, hbuf, abuf, s_in, p_, proj_stride, o_, out_stride);

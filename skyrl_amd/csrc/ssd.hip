@@ -4,8 +4,8 @@
 // Token form (ssd_scan): one workgroup per (sequence, head), the state in registers over the sequence's tokens:
 // convolution, step size, decay, update and read-out in one launch. A decode step reads and writes the state once.
 //
-// Prompt form: the convolutions run once for all heads (skyrl_conv_chunk: x and B also transposed), then
-// ssd_walk takes one (run of chunks, head, 64 value columns) per workgroup and walks the chunks of 64 tokens with
+// Prompt form: the convolutions run once for all heads (skyrl_conv_chunk: x and B also transposed), so do the
+// products C B^T of every chunk and group (ssd_scores). ssd_walk takes one (run of chunks, head, 64 value columns) per workgroup and walks the chunks of 64 tokens with
 // the state in registers:
 //   Y = (L o C B^T) X + diag(e^G) C S,   S <- e^{G_n} S + B^T diag(e^{G_n - G} dt) X,
 // G the summed log decays, L_ij = e^{G_i - G_j} dt_j (j <= i), the skip D on L's diagonal. Long sequences are cut
@@ -180,25 +180,61 @@ __device__ __forceinline__ f32x4 mma3(const Split& a, const s16x8& b, f32x4 acc)
 __device__ __forceinline__ f32x4 mma3(const s16x8& a, const Split& b, f32x4 acc) {
     return mma(a, b.hi, mma(a, b.mid, mma(a, b.lo, acc)));
 }
+__device__ __forceinline__ void put16(uint16_t* p, uint4 v) {  // 16 bytes to an address on 8
+    *reinterpret_cast<uint2*>(p) = make_uint2(v.x, v.y);
+    *reinterpret_cast<uint2*>(p + 4) = make_uint2(v.z, v.w);
+}
 // Elements 4 g .. 4 g + 3 of both 16-wide halves of a 32-wide step: the accumulators' order of rows.
 __device__ __forceinline__ s16x8 halves(const uint16_t* p) {
     const s16x4 a = *reinterpret_cast<const s16x4*>(p), b = *reinterpret_cast<const s16x4*>(p + 16);
     return s16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
 }
 
+// C B^T of a chunk and group, transposed (keys in the rows): 16 x 16 tiles at and below the diagonal as the walk's
+// accumulators, query tile w's first at w (w + 1) / 2. grid nchunks G.
+constexpr int kTiles = 10;
+constexpr int kLTerm = 6 * kWave * 8;  // L^T in LDS: 32-key steps 0 .. qt / 2 of each query tile qt
+__device__ __forceinline__ int l_step(int qt, int kk) { return (qt < 2 ? qt : 2 * qt - 2 + kk) * kWave * 8; }
+__global__ __launch_bounds__(kNT) void ssd_scores_kernel(int G, int np, const int32_t* __restrict__ chunk,
+                                                         const uint16_t* __restrict__ brow,
+                                                         const uint16_t* __restrict__ crow, float* __restrict__ scores) {
+    const int ci = blockIdx.x / G, gi = blockIdx.x - ci * G;
+    const int t0 = chunk[4 * ci], n = chunk[4 * ci + 1];
+    const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int64_t bw = (int64_t)G * np;
+    const uint16_t* cr = crow + (t0 + min(16 * wave + c, n - 1)) * bw + gi * np + 8 * g;
+    f32x4 acc[4];
+#pragma unroll
+    for (int tt = 0; tt < 4; ++tt) acc[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < np; k += 32) {
+        const s16x8 q = *reinterpret_cast<const s16x8*>(cr + k);
+#pragma unroll
+        for (int tt = 0; tt < 4; ++tt)
+            if (tt <= wave)
+                acc[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                    *reinterpret_cast<const s16x8*>(brow + (t0 + min(16 * tt + c, n - 1)) * bw + gi * np + 8 * g + k), q,
+                    acc[tt], 0, 0, 0);
+    }
+    float* dst = scores + ((int64_t)blockIdx.x * kTiles + wave * (wave + 1) / 2) * 256 + 4 * lane;
+#pragma unroll
+    for (int tt = 0; tt < 4; ++tt)
+        if (tt <= wave) *reinterpret_cast<f32x4*>(dst + tt * 256) = acc[tt];
+}
+
 // NS: 32-wide steps of the padded state dimension at least. OUT: the second walk; otherwise the first, over the
 // runs that `pick` lists.
 template <int NS, bool OUT>
-__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 4 ? 2 : 1))) void ssd_walk_kernel(
+__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 4 ? 3 : 1))) void ssd_walk_kernel(
     Dims d, SeqRef sq, const int32_t* __restrict__ pick, int slices, const uint16_t* __restrict__ xt,
-    const uint16_t* __restrict__ bt, const uint16_t* __restrict__ brow, const uint16_t* __restrict__ crow,
+    const uint16_t* __restrict__ bt, const float* __restrict__ scores, const uint16_t* __restrict__ crow,
     const uint16_t* __restrict__ dt_raw, int64_t dt_stride, const float* __restrict__ a_log,
     const float* __restrict__ dt_bias, const float* __restrict__ skip, float* __restrict__ state,
     float* __restrict__ runs, float* __restrict__ gtot, uint16_t* __restrict__ y, int64_t y_stride) {
-    constexpr int LDC = NS * 32 + 8, LDB = kC + 8;
+    constexpr int LDC = NS * 32 + 4, LDB = kC + 4;  // rows on 8 bytes
     __shared__ __attribute__((aligned(16))) uint16_t s_c[OUT ? kC * LDC : 8];
     __shared__ __attribute__((aligned(16))) uint16_t s_bt[NS * 32 * LDB];
-    __shared__ __attribute__((aligned(16))) uint16_t s_l[OUT ? 3 * 4 * 2 * kWave * 8 : 8];  // L^T: term, query tile, step
+    __shared__ __attribute__((aligned(16))) uint16_t s_l[OUT ? 3 * kLTerm : 8];  // L^T: term, (query tile, step)
     __shared__ __attribute__((aligned(16))) float s_g[kC], s_d[kC], s_w[kC];
     const int slice = blockIdx.x % slices, hs = blockIdx.x / slices, h = hs % d.H;
     const int ri = OUT ? hs / d.H : pick[hs / d.H];
@@ -239,13 +275,20 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 4 ? 2
             const int pieces = np / 8;
             for (int e = tid; e < kC * pieces; e += kNT) {
                 const int i = e / pieces, x = (e - i * pieces) * 8;
-                *reinterpret_cast<uint4*>(&s_c[i * LDC + x]) =
-                    *reinterpret_cast<const uint4*>(crow + (int64_t)(t0 + min(i, n - 1)) * bw + gi * np + x);
+                put16(&s_c[i * LDC + x],
+                      *reinterpret_cast<const uint4*>(crow + (int64_t)(t0 + min(i, n - 1)) * bw + gi * np + x));
             }
         }
         for (int e = tid; e < np * 8; e += kNT)
-            *reinterpret_cast<uint4*>(&s_bt[(e >> 3) * LDB + (e & 7) * 8]) =
-                *reinterpret_cast<const uint4*>(bt + ((int64_t)ci * bw + gi * np) * kC + e * 8);
+            put16(&s_bt[(e >> 3) * LDB + (e & 7) * 8],
+                  *reinterpret_cast<const uint4*>(bt + ((int64_t)ci * bw + gi * np) * kC + e * 8));
+        f32x4 sc[4];
+        if constexpr (OUT) {
+            const float* src = scores + (((int64_t)ci * d.G + gi) * kTiles + wave * (wave + 1) / 2) * 256 + 4 * lane;
+#pragma unroll
+            for (int tt = 0; tt < 4; ++tt)
+                if (tt <= wave) sc[tt] = *reinterpret_cast<const f32x4*>(src + tt * 256);
+        }
         s16x8 xf[2];
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk)
@@ -277,20 +320,12 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 4 ? 2
             for (int tt = 0; tt < 4; ++tt) {
                 float* dst = &w[tt >> 1][4 * (tt & 1)];
                 if (tt <= wave) {
-                    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-                    const uint16_t* br = brow + (int64_t)(t0 + min(16 * tt + c, n - 1)) * bw + gi * np + 8 * g;
-                    const uint16_t* cr = &s_c[q * LDC + 8 * g];
-#pragma unroll
-                    for (int s = 0; s < NS; ++s)
-                        if (s < ns)
-                            acc = mma(*reinterpret_cast<const s16x8*>(br + 32 * s),
-                                      *reinterpret_cast<const s16x8*>(cr + 32 * s), acc);
                     const int j0 = 16 * tt + 4 * g;
                     const float4 gk = ld4(&s_g[j0]), dk = ld4(&s_d[j0]);
                     const float gv[4] = {gk.x, gk.y, gk.z, gk.w}, dv[4] = {dk.x, dk.y, dk.z, dk.w};
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
-                        const float l = j0 + i <= q ? acc[i] * fast_exp2((gq - gv[i]) * kLog2e) * dv[i] : 0.f;
+                        const float l = j0 + i <= q ? sc[tt][i] * fast_exp2((gq - gv[i]) * kLog2e) * dv[i] : 0.f;
                         dst[i] = j0 + i == q ? l + D : l;
                     }
                 } else {
@@ -302,10 +337,10 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 4 ? 2
             for (int kk = 0; kk < 2; ++kk) {
                 if (kk > wave / 2) break;
                 const Split f = split3(w[kk]);
-                uint16_t* p = &s_l[((wave * 2 + kk) * kWave + lane) * 8];
+                uint16_t* p = &s_l[l_step(wave, kk) + lane * 8];
                 *reinterpret_cast<s16x8*>(p) = f.hi;
-                *reinterpret_cast<s16x8*>(p + 4 * 2 * kWave * 8) = f.mid;
-                *reinterpret_cast<s16x8*>(p + 2 * 4 * 2 * kWave * 8) = f.lo;
+                *reinterpret_cast<s16x8*>(p + kLTerm) = f.mid;
+                *reinterpret_cast<s16x8*>(p + 2 * kLTerm) = f.lo;
             }
             // what the state before the chunk gives: (C S)^T
 #pragma unroll
@@ -331,10 +366,9 @@ __global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(NS <= 4 ? 2
                 for (int qt = 0; qt < 4; ++qt) {
 #pragma unroll
                     for (int kk = 0; kk <= qt / 2; ++kk) {
-                        const uint16_t* p = &s_l[((qt * 2 + kk) * kWave + lane) * 8];
-                        const Split f{*reinterpret_cast<const s16x8*>(p),
-                                      *reinterpret_cast<const s16x8*>(p + 4 * 2 * kWave * 8),
-                                      *reinterpret_cast<const s16x8*>(p + 2 * 4 * 2 * kWave * 8)};
+                        const uint16_t* p = &s_l[l_step(qt, kk) + lane * 8];
+                        const Split f{*reinterpret_cast<const s16x8*>(p), *reinterpret_cast<const s16x8*>(p + kLTerm),
+                                      *reinterpret_cast<const s16x8*>(p + 2 * kLTerm)};
                         o[qt] = mma3(xf[kk], f, o[qt]);
                     }
                     const int tq = 16 * qt + c, p0 = 16 * pt + 4 * g;
@@ -431,66 +465,6 @@ __global__ __launch_bounds__(kNT) void ssd_chain_kernel(Dims d, SeqRef sq, const
     }
 }
 
-// ---- out = rms over each of `groups` equal parts of y silu(z), times w; one workgroup per (token, part) ----
-// Up to kMax groups of VEC values per thread in registers; HOLD false: any length, formed twice.
-template <typename T, int NT, int VEC, int kMax, bool HOLD>
-__global__ __launch_bounds__(NT) void gated_norm_kernel(const T* __restrict__ y, int64_t y_stride,
-                                                        const T* __restrict__ z, int64_t z_stride,
-                                                        const T* __restrict__ w, int groups, int len, float eps,
-                                                        T* __restrict__ out, int64_t out_stride) {
-    __shared__ float s_red[NT / kWave];
-    const int64_t t = blockIdx.x / groups;
-    const int c0 = (int)(blockIdx.x % groups) * len, nv = len / VEC;
-    const T* yp = y + t * y_stride + c0;
-    const T* zp = z + t * z_stride + c0;
-    float a[HOLD ? kMax : 1][VEC];
-    auto form = [&](int v, float (&o)[VEC]) {
-        float zz[VEC];
-        ldv<T, VEC>(yp + VEC * v, o);
-        ldv<T, VEC>(zp + VEC * v, zz);
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) o[j] *= zz[j] * sigmoid_<T>(zz[j]);
-    };
-    float ss = 0.f;
-    if constexpr (HOLD) {
-#pragma unroll
-        for (int k = 0; k < kMax; ++k) {
-            const int v = threadIdx.x + k * NT;
-            if (v < nv) {
-                form(v, a[k]);
-#pragma unroll
-                for (int j = 0; j < VEC; ++j) ss += a[k][j] * a[k][j];
-            }
-        }
-    } else {
-        for (int v = threadIdx.x; v < nv; v += NT) {
-            form(v, a[0]);
-#pragma unroll
-            for (int j = 0; j < VEC; ++j) ss += a[0][j] * a[0][j];
-        }
-    }
-    const float r = 1.f / sqrtf(block_total<NT>(ss, s_red) / (float)len + eps);
-    auto put = [&](int v, float (&o)[VEC]) {
-        float ww[VEC];
-        ldv<T, VEC>(w + c0 + VEC * v, ww);
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) o[j] *= r * ww[j];
-        stv(out + t * out_stride + c0 + VEC * v, o);
-    };
-    if constexpr (HOLD) {
-#pragma unroll
-        for (int k = 0; k < kMax; ++k) {
-            const int v = threadIdx.x + k * NT;
-            if (v < nv) put(v, a[k]);
-        }
-    } else {
-        for (int v = threadIdx.x; v < nv; v += NT) {
-            form(v, a[0]);
-            put(v, a[0]);
-        }
-    }
-}
-
 const char* bad_shape(const skyrl_ssd_shape* sh) {
     if (!sh) return "ssd: null shape";
     if (sh->heads <= 0 || sh->groups <= 0 || sh->heads % sh->groups) return "ssd: heads must be a multiple of groups";
@@ -546,7 +520,7 @@ extern "C" int skyrl_ssd_scan(const skyrl_ssd_shape* shape, const void* proj, in
 
 #define LAUNCH_WALK(NS, OUT, grid, pick)                                                                             \
     hipLaunchKernelGGL((ssd_walk_kernel<NS, OUT>), dim3(grid), dim3(kNT), 0, s, d, sq, pick, slices, u16(xt), u16(bt), \
-                       u16(brow), u16(crow), u16(dt_raw), dt_stride, a_log, dt_bias, skip, state, runs, gtot,        \
+                       scores, u16(crow), u16(dt_raw), dt_stride, a_log, dt_bias, skip, state, runs, gtot,        \
                        reinterpret_cast<uint16_t*>(y), y_stride)
 #define LAUNCH_WALKS(OUT, grid, pick)                      \
     if (d.np() <= 64) LAUNCH_WALK(2, OUT, grid, pick);       \
@@ -555,29 +529,33 @@ extern "C" int skyrl_ssd_scan(const skyrl_ssd_shape* shape, const void* proj, in
 
 extern "C" int skyrl_ssd_prompt(const skyrl_ssd_shape* shape, const void* xt, const void* bt, const void* brow,
                                 const void* crow, const void* dt_raw, int64_t dt_stride, const float* a_log,
-                                const float* dt_bias, const float* skip, const int32_t* chunk, const int32_t* super,
-                                int32_t nsuper, const int32_t* pick, int32_t npick, const int32_t* chain,
+                                const float* dt_bias, const float* skip, const int32_t* chunk, int32_t nchunks,
+                                const int32_t* super, int32_t nsuper, const int32_t* pick, int32_t npick, const int32_t* chain,
                                 int32_t nchain, const int32_t* cu, const int32_t* rows, const int64_t* positions,
-                                float* state, float* runs, float* gtot, void* y, int64_t y_stride, void* stream) {
+                                float* state, float* scores, float* runs, float* gtot, void* y,
+                                int64_t y_stride, void* stream) {
     const char* bad = bad_shape(shape);
     SKYRL_REQUIRE(!bad, bad);
     const Dims d = dims_of(shape);
     const int slices = (d.vp() + 63) / 64;
     SKYRL_REQUIRE(d.N <= 256, "ssd_prompt: state must be at most 256");
-    SKYRL_REQUIRE(nsuper >= 0 && npick >= 0 && nchain >= 0 && nchain <= 65535 && dt_stride >= d.H &&
+    SKYRL_REQUIRE(nchunks >= nsuper && nsuper >= 0 && npick >= 0 && nchain >= 0 && nchain <= 65535 && dt_stride >= d.H &&
                       (int64_t)nsuper * d.H * slices < (1 << 30) && (int64_t)npick * d.H * slices < (1 << 30) &&
                       y_stride >= d.inner(),
                   "ssd_prompt: bad sizes");
     if (nsuper == 0) return SKYRL_OK;
     SKYRL_REQUIRE(xt && bt && brow && crow && dt_raw && a_log && dt_bias && skip && chunk && super && cu && rows &&
-                      positions && state && runs && gtot && y && (pick || !npick) && (chain || !nchain),
+                      positions && state && scores && runs && gtot && y && (pick || !npick) && (chain || !nchain),
                   "ssd_prompt: null pointer");
-    SKYRL_REQUIRE(aligned16(xt) && aligned16(bt) && aligned16(brow) && aligned16(crow), "ssd_prompt: 16-byte alignment");
+    SKYRL_REQUIRE(aligned16(xt) && aligned16(bt) && aligned16(brow) && aligned16(crow) && aligned16(scores),
+                  "ssd_prompt: 16-byte alignment");
     SKYRL_REQUIRE(d.P % 4 || (y_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(y) & 7) == 0),
                   "ssd_prompt: y must be aligned to four elements");
     hipStream_t s = as_stream(stream);
     const SeqRef sq{chunk, super, cu, rows, positions};
     auto u16 = [](const void* p) { return reinterpret_cast<const uint16_t*>(p); };
+    hipLaunchKernelGGL(ssd_scores_kernel, dim3((unsigned)nchunks * d.G), dim3(kNT), 0, s, d.G, d.np(), chunk, u16(brow),
+                       u16(crow), scores);
     if (npick) {
         LAUNCH_WALKS(false, (unsigned)(npick * d.H * slices), pick);
         const int64_t size = (int64_t)d.H * d.np() * d.vp();
@@ -586,34 +564,4 @@ extern "C" int skyrl_ssd_prompt(const skyrl_ssd_shape* shape, const void* xt, co
     }
     LAUNCH_WALKS(true, (unsigned)(nsuper * d.H * slices), nullptr);
     return check_launch("ssd_prompt kernels");
-}
-
-#define LAUNCH_GNORM(NT, VEC, K, HOLD)                                                                               \
-    hipLaunchKernelGGL((gated_norm_kernel<T, NT, VEC, K, HOLD>), dim3((unsigned)(n * groups)), dim3(NT), 0,          \
-                       as_stream(stream), y_, y_stride, z_, z_stride, w_, groups, len, eps, o_, out_stride)
-
-extern "C" int skyrl_gated_norm(const void* y, int64_t y_stride, const void* z, int64_t z_stride, const void* weight,
-                                int64_t n, int32_t width, int32_t groups, float eps, void* out, int64_t out_stride,
-                                int32_t dtype, void* stream) {
-    SKYRL_REQUIRE_T(dtype, "gated_norm");
-    SKYRL_REQUIRE(n >= 0 && width > 0 && groups > 0 && width % groups == 0 && n * groups < (1ll << 31) &&
-                      y_stride >= width && z_stride >= width && out_stride >= width,
-                  "gated_norm: bad sizes");
-    if (n == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(y && z && weight && out, "gated_norm: null pointer");
-    const int len = width / groups;
-    SKYRL_DISPATCH_T(dtype, {
-        const T* y_ = reinterpret_cast<const T*>(y);
-        const T* z_ = reinterpret_cast<const T*>(z);
-        const T* w_ = reinterpret_cast<const T*>(weight);
-        T* o_ = reinterpret_cast<T*>(out);
-        const bool wide = len % 8 == 0 && y_stride % 8 == 0 && z_stride % 8 == 0 && out_stride % 8 == 0 &&
-                          aligned16(y) && aligned16(z) && aligned16(weight) && aligned16(out);
-        if (wide && len <= 512) LAUNCH_GNORM(64, 8, 1, true);
-        else if (wide && len <= 2048) LAUNCH_GNORM(256, 8, 1, true);
-        else if (wide && len <= 8192) LAUNCH_GNORM(256, 8, 4, true);
-        else if (wide) LAUNCH_GNORM(256, 8, 1, false);
-        else LAUNCH_GNORM(256, 1, 1, false);
-    })
-    return check_launch("gated_norm_kernel");
 }

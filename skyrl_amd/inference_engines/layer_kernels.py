@@ -562,20 +562,27 @@ def rglru_step(proj, width: int, blocks: int, conv_t, conv_b, gate_w, gate_b, ra
               out.stride(0), _code(proj), _stream(dev))
 
 
-def rglru_prompt(proj, width: int, blocks: int, u, gate_w, gate_b, rate, chunk, seq_chunks, seq0: int, cu, rows,
+def rglru_workgroups(width: int, blocks: int) -> int:
+    """Workgroups per run of chunks of the prompt form: 64 columns of a block each."""
+    return blocks * ((rglru_pads(width, blocks)[0] + 63) // 64)
+
+
+def rglru_prompt(proj, width: int, blocks: int, u, gate_w, gate_b, rate, chunk, runs, seq_runs, seq0: int, cu, rows,
                  positions, state, out) -> None:
-    """Tokens of the chunks, of the sequences from seq0 on; u [T, width] is conv_chunk's."""
-    dev = _require_gpu(proj, u, gate_w, gate_b, rate, chunk, seq_chunks, cu, rows, positions, state, out)
-    T, nc = proj.shape[0], chunk.shape[0]
+    """Tokens of the chunks, of the sequences from seq0 on (mixers.chunk_runs); u [T, width] is
+    conv_chunk's."""
+    dev = _require_gpu(proj, u, gate_w, gate_b, rate, chunk, runs, seq_runs, cu, rows, positions, state, out)
+    T, nc, nr = proj.shape[0], chunk.shape[0], runs.shape[0]
     _check_rglru(proj, width, blocks, gate_w, gate_b, rate, state, out)
     n = _check_steps(cu, rows, positions, T) - seq0
     _check(u, "u", proj.dtype, (T, width))
     _check(chunk, "chunk", torch.int32, (nc, 4))
-    _check(seq_chunks, "seq_chunks", torch.int32, (n + 1,))
+    _check(runs, "runs", torch.int32, (nr, 4))
+    _check(seq_runs, "seq_runs", torch.int32, (n + 1,))
     h, a = (torch.empty((T, width), dtype=torch.float32, device=dev) for _ in range(2))
-    s_in = torch.empty((nc, width), dtype=torch.float32, device=dev)
+    s_in = torch.empty((nr, width), dtype=torch.float32, device=dev)
     _ffi.call("skyrl_rglru_prompt", _ptr(proj), proj.stride(0), width, blocks, _ptr(u), _ptr(gate_w), _ptr(gate_b),
-              _ptr(rate), _ptr(chunk), nc, _ptr(seq_chunks), seq0, n, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(state),
+              _ptr(rate), _ptr(chunk), nc, _ptr(runs), nr, _ptr(seq_runs), seq0, n, _ptr(cu), _ptr(rows), _ptr(positions), _ptr(state),
               _ptr(h), _ptr(a), _ptr(s_in), _ptr(out), out.stride(0), _code(proj), _stream(dev))
 
 
@@ -756,12 +763,13 @@ def ssd_prompt(sh, proj, conv_t, conv_b, a_log, dt_bias, skip, cu, rows, positio
                ((H, P, vp, None, xt), (G, N, np_, brow, bt), (G, N, np_, crow, None)))
     multi = pick.shape[0] > 0
     runs = torch.empty((ns if multi else 1, H, np_, vp), dtype=torch.float32, device=dev)
+    scores = torch.empty((nc, G, 10, 256), dtype=torch.float32, device=dev)
     gtot = torch.empty((ns if multi else 1, H), dtype=torch.float32, device=dev)
     dt = proj[:, inner + ssd_channels(sh):]
     _ffi.call("skyrl_ssd_prompt", ctypes.byref(sh), _ptr(xt), _ptr(bt), _ptr(brow), _ptr(crow), _ptr(dt), dt.stride(0),
-              _ptr(a_log), _ptr(dt_bias), _ptr(skip), _ptr(chunk), _ptr(super_), ns, _ptr(pick), pick.shape[0],
-              _ptr(chain), chain.shape[0], _ptr(cu), _ptr(rows), _ptr(positions), _ptr(state), _ptr(runs), _ptr(gtot),
-              _ptr(y), y.stride(0), _stream(dev))
+              _ptr(a_log), _ptr(dt_bias), _ptr(skip), _ptr(chunk), nc, _ptr(super_), ns, _ptr(pick), pick.shape[0],
+              _ptr(chain), chain.shape[0], _ptr(cu), _ptr(rows), _ptr(positions), _ptr(state), _ptr(scores), _ptr(runs),
+              _ptr(gtot), _ptr(y), y.stride(0), _stream(dev))
 
 
 def gated_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float,

@@ -157,27 +157,36 @@ def run_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token
     return np.concatenate(runs).astype(np.int32)
 
 
-WALK_WORKGROUPS = 1024  # of the state space prompt walk: four per CU
-WALK_CHUNKS = 4         # chunks per run at least: a run's state is written and read once more
+WALK_WORKGROUPS = 1024  # of the recurrences' prompt walks: four per CU
+WALK_CHUNKS = 4         # chunks per run of the state space walk at least: a run's state is written and read once more
 
 
-def walk_plan(seq_lens: List[int], first_seq: int, first_token: int, per_run: int):
-    """Host plan of the state space prompt form of sequences first_seq..: (chunk int32 [n, 4], super int32 [m, 4],
-    pick int32 [k], chain int32 [j, 2]). Sequences are cut into runs of chunks so that about WALK_WORKGROUPS
-    workgroups walk them, per_run of them per run (skyrl_ssd_prompt)."""
+def chunk_runs(seq_lens: List[int], first_seq: int, first_token: int, per_run: int, least: int = 1):
+    """Sequences first_seq.. as chunks, and their chunks in runs, at least `least` chunks long, so that about
+    WALK_WORKGROUPS workgroups walk them, per_run of them per run: (chunk int32 [n, 4], the fourth number the
+    chunk's run, runs int32 [m, 4]: first chunk, chunks, sequence, 1 if the sequence has several runs + 2 if its
+    last, seq_runs int32 [sequences + 1])."""
     chunk, ends = chunk_plan(seq_lens, first_seq, first_token)
-    size = max(WALK_CHUNKS, -(-len(chunk) * per_run // WALK_WORKGROUPS))
-    runs, pick, chain = [], [], []
+    size = max(least, -(-len(chunk) * per_run // WALK_WORKGROUPS))
+    runs, seq_runs = [], [0]
     for i in range(len(ends) - 1):
         n = int(ends[i + 1] - ends[i])
         k = max(1, round(n / size))
-        cuts = [ends[i] + n * j // k for j in range(k + 1)]
-        if k > 1:
-            chain.append((len(runs), k))
-            pick += range(len(runs), len(runs) + k - 1)
-        runs += [(a, b - a, first_seq + i, (k > 1) + 2 * (b == ends[i + 1])) for a, b in zip(cuts, cuts[1:])]
-    i32 = lambda x, *tail: np.asarray(x, dtype=np.int32).reshape(-1, *tail)  # noqa: E731
-    return chunk, i32(runs, 4), i32(pick), i32(chain, 2)
+        cuts = [int(ends[i]) + n * j // k for j in range(k + 1)]
+        for j, (a, b) in enumerate(zip(cuts, cuts[1:])):
+            chunk[a:b, 3] = len(runs)
+            runs.append((a, b - a, first_seq + i, (k > 1) + 2 * (j == k - 1)))
+        seq_runs.append(len(runs))
+    return chunk, np.asarray(runs, dtype=np.int32).reshape(-1, 4), np.asarray(seq_runs, dtype=np.int32)
+
+
+def walk_plan(seq_lens: List[int], first_seq: int, first_token: int, per_run: int):
+    """Host plan of the state space prompt form of sequences first_seq..: (chunk, runs, pick int32 [k], chain int32
+    [j, 2]) as skyrl_ssd_prompt takes them."""
+    chunk, runs, seq_runs = chunk_runs(seq_lens, first_seq, first_token, per_run, WALK_CHUNKS)
+    chain = [(a, b - a) for a, b in zip(seq_runs, seq_runs[1:]) if b - a > 1]
+    pick = [r for r, kind in enumerate(runs[:, 3]) if kind == 1]
+    return chunk, runs, np.asarray(pick, dtype=np.int32), np.asarray(chain, dtype=np.int32).reshape(-1, 2)
 
 
 class Products:
@@ -234,6 +243,7 @@ class LatentAttention:
     an optional sliding window. Caches [blocks, 16, row]: per token the normed latent | the rotated key
     part."""
 
+    libraries = ("latent",)  # of _ffi.LAYER_LIBS, beside the common one
     paged = True
     kv_from = None
 
@@ -338,6 +348,7 @@ class GatedDelta:
     """Gated delta rule with short causal convolutions on q, k and v. State per row (a running
     request): the f32 matrix of every head and the convolutions' last inputs."""
 
+    libraries = ("delta",)
     paged = False
     kv_from = None
 
@@ -419,6 +430,7 @@ class DifferentialAttention:
     transposed [blocks, kv_heads, vdim, 16]; state per row: the convolutions' last inputs. A layer with
     `kv_from` reads the cache of that layer and has queries only."""
 
+    libraries = ("diff",)
     paged = True
     in_bias, out_bias = True, False
 
@@ -542,6 +554,7 @@ class GatedLinearRecurrence:
     convolution and recurrence, whose two gates are block-diagonal. State per row: the f32 channels and the
     convolution's last inputs."""
 
+    libraries = ("rglru",)
     paged = False
     kv_from = None
     plans_short = True
@@ -565,6 +578,7 @@ class GatedLinearRecurrence:
         self.lam = w.zeros(C, dtype=torch.float32)
         self.gate_w = w.zeros(self.blocks, 2, *lk.rglru_pads(C, self.blocks))  # the kernels' form of ra, ri
         self.rate = w.zeros(C, dtype=torch.float32)
+        self.plan_key = ("runs", lk.rglru_workgroups(C, self.blocks))
         self.refresh()
 
     def bind(self, w_in, b_in, w_out, b_out) -> None:
@@ -603,7 +617,7 @@ class GatedLinearRecurrence:
         return 0
 
     def host_plans(self, seq_lens, starts, first_seq, first_token):
-        yield "all_chunks", lambda: chunk_plan(seq_lens, 0, 0)
+        yield self.plan_key, lambda: chunk_runs(seq_lens, 0, 0, self.plan_key[1])
 
     # ---- step
     def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state, workspace) -> None:
@@ -614,11 +628,11 @@ class GatedLinearRecurrence:
             lk.rglru_step(proj, C, self.blocks, self.conv.conv_t, self.conv.bias, *gates, inp.rows, inp.positions, S,
                           ring, out)
             return
-        chunk, seq_chunks = inp.plan["all_chunks"]
+        chunk, runs, seq_runs = inp.plan[self.plan_key]
         u = torch.empty((proj.shape[0], C), dtype=self.dtype, device=proj.device)
         x, seqs = proj[:, C:], (inp.cu, inp.rows, inp.positions)
         lk.conv_chunk(x, self.conv.conv_t, self.conv.bias, False, chunk, *seqs, ring, ((1, C, C, u.unsqueeze(1), None),))
-        lk.rglru_prompt(proj, C, self.blocks, u, *gates, chunk, seq_chunks, 0, *seqs, S, out)
+        lk.rglru_prompt(proj, C, self.blocks, u, *gates, chunk, runs, seq_runs, 0, *seqs, S, out)
         lk.conv_save(x, C, *seqs, ring)
 
 
@@ -627,6 +641,7 @@ class WindowAttention:
     elementwise output gate; biases on its projections but the gate's. Caches K [blocks, kv_heads, 16, dim] and V
     transposed [blocks, kv_heads, vdim, 16], sizes padded."""
 
+    libraries = ("attn",)
     paged = True
     kv_from = None
     in_bias, out_bias = True, True
@@ -713,6 +728,7 @@ class StateSpace:
     """State space mixer with a scalar decay per head (Mamba-2): biased short convolutions, a gate before a
     norm in equal parts. State per row: the f32 matrix of every head and the convolutions' last inputs."""
 
+    libraries = ("ssd",)
     paged = False
     kv_from = None
     in_bias, out_bias = False, False
@@ -789,6 +805,7 @@ class SideBySide:
     layer's output norm joins them, half the sum of both (layer_kernels.norm_add)."""
 
     LEFT, RIGHT, SHARE = WindowAttention, StateSpace, 0.5
+    libraries = LEFT.libraries + RIGHT.libraries
     kv_from = None
 
     @classmethod

@@ -56,6 +56,18 @@ def build_decoder(config: Dict[str, Any], device, dtype: torch.dtype = torch.bfl
     return decoder_factory(config)(config, folder, device, dtype, max_model_len, seed)
 
 
+def kernel_libraries(config: Dict[str, Any]) -> Tuple[str, ...]:
+    """The layer libraries (_ffi.LAYER_LIBS) that serving the checkpoint needs; none for the paged HF decoders."""
+    if decoder_factory(config) is not _hybrid:
+        return ()
+    from .mixers import MIXERS
+
+    unknown = sorted({e["type"] for e in config["layers"]} - set(MIXERS))
+    if unknown:
+        raise ValueError(f"unknown layer types {unknown} (known: {sorted(MIXERS)})")
+    return ("layers",) + tuple(sorted({lib for e in config["layers"] for lib in MIXERS[e["type"]].libraries}))
+
+
 def checkpoint_tensors(folder: str) -> Iterator[Tuple[str, torch.Tensor]]:
     from safetensors import safe_open
 

@@ -14,7 +14,7 @@ import argparse
 import json
 import os
 import sys
-from typing import Dict, Iterable, Optional
+from typing import Callable, Dict, Iterable, Optional
 
 from .engine import BLOCK_SIZE, EngineCore, ModelRunner, Request
 
@@ -47,7 +47,8 @@ class TraceSession:
         return out
 
 
-def main(argv: Optional[list] = None) -> int:
+def main(argv: Optional[list] = None, prepare: Optional[Callable] = None) -> int:
+    """prepare: called with the names of the kernel libraries that the model needs, before the GPU is used."""
     ap = argparse.ArgumentParser(prog="trace_run", description="replay token steps from stdin, write their logits")
     ap.add_argument("--model", required=True, help="folder with config.json and safetensors weights")
     ap.add_argument("--dtype", required=True, choices=("bfloat16", "float32"))
@@ -58,8 +59,10 @@ def main(argv: Optional[list] = None) -> int:
 
     import torch
 
-    from .registry import load_decoder
+    from .registry import kernel_libraries, load_decoder, read_config
 
+    if prepare is not None:
+        prepare(kernel_libraries(read_config(args.model)))
     if not torch.cuda.is_available():
         print("trace_run needs a GPU", file=sys.stderr)
         return 1

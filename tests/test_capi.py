@@ -33,12 +33,48 @@ def test_ffi_signatures_cover_header():
 
 
 def test_layers_library_matches_its_header():
-    """libskyrl_layers.so exports what include/skyrl_layers.h declares, and is bound name by name."""
+    """The layer libraries export what include/skyrl_layers.h declares, and are bound name by name."""
     names = header_functions("skyrl_layers.h")
     assert "skyrl_latent_attend" in names and "skyrl_delta_scan" in names and sorted(_ffi.LAYERS_SIGNATURES) == names
-    lib = _ffi.load_layers()
-    assert not [n for n in names if not hasattr(lib, n)]
+    assert not [n for n in names if not hasattr(_ffi.load_layers(_ffi.layer_lib_of(n)), n)]
+    assert {_ffi.layer_lib_of(n) for n in names} == set(_ffi.LAYER_LIBS)
     assert not set(names) & set(header_functions())
+
+
+def test_recurrent_layers_entries_validate_on_host():
+    p = ctypes.c_void_p(16)
+    q = ctypes.c_void_p(20)  # not aligned to 16 bytes
+    attn = lambda *a: ctypes.byref(_ffi.AttnShape(*a, 0.5, 1e-5))  # noqa: E731
+    ssd = lambda *a: ctypes.byref(_ffi.SSDShape(*a))  # noqa: E731
+    sec = (_ffi.ConvSection * 4)(_ffi.ConvSection(2, 8, 8, 16, None), _ffi.ConvSection(1, 4, 2, 16, None))
+    seqs = (p, 1, p, p, p)
+    for name, args, msg in (
+            ("skyrl_norm_add", (p, None, None, None, 0.5, p, p, 1, None, 0, 1, 9000, 1e-5, p, _ffi.BF16, None), "H must be"),
+            ("skyrl_norm_add", (p, None, None, None, 0.5, p, p, 7, None, 0, 1, 64, 1e-5, p, _ffi.BF16, None), "1 or H"),
+            ("skyrl_norm_add", (p, None, p, None, 0.5, p, p, 1, None, 0, 1, 64, 1e-5, p, _ffi.BF16, None), "null"),
+            ("skyrl_xielu", (p, 7, 1, 8, p, p, 8, _ffi.F32, None), "bad sizes"),
+            ("skyrl_gated_norm", (p, 8, p, 8, p, 1, 8, 3, 1e-5, p, 8, _ffi.F32, None), "bad sizes"),
+            ("skyrl_embed", (p, p, 1, 8, 1.0, None, p, p, None, _ffi.F32, None), "null"),
+            ("skyrl_conv_chunk", (p, 32, 20, 4, p, None, 0, *seqs, p, sec, 2, _ffi.BF16, None), "bad section"),
+            ("skyrl_conv_chunk", (p, 32, 20, 4, p, None, 0, *seqs, p, sec, 1, _ffi.BF16, None), "cover"),
+            ("skyrl_conv_chunk", (p, 32, 20, 4, p, None, 0, *seqs, p, sec, 4, _ffi.BF16, None), "sections"),
+            ("skyrl_conv_chunk", (p, 32, 16, 4, q, None, 0, *seqs, p, sec, 1, _ffi.BF16, None), "alignment"),
+            ("skyrl_rglru_step", (p, 20, 10, 3, 4, p, p, p, p, p, p, p, 1, p, p, p, 10, _ffi.BF16, None), "multiple of blocks"),
+            ("skyrl_rglru_step", (p, 10, 10, 2, 4, p, p, p, p, p, p, p, 1, p, p, p, 10, _ffi.BF16, None), "bad sizes"),
+            ("skyrl_rglru_step", (p, 8192, 4096, 1, 4, p, p, p, p, p, p, p, 1, p, p, p, 4096, _ffi.BF16, None), "too large"),
+            ("skyrl_rglru_prompt", (p, 20, 10, 2, p, p, p, p, p, 1, p, 2, p, 0, 1, p, p, p, p, p, p, p, p, 10, _ffi.F32, None),
+             "bad sizes"),
+            ("skyrl_attn_write", (attn(3, 2, 8, 8, 0), p, 99, p, p, p, None, 0, 1, p, p, p, _ffi.BF16, None), "multiple of kv_heads"),
+            ("skyrl_attn_write", (attn(2, 1, 9, 8, 0), p, 99, p, p, p, p, 0, 1, p, p, p, _ffi.BF16, None), "runs need"),
+            ("skyrl_attn_attend", (attn(2, 1, 8, 8, 4), p, p, 16, p, p, p, 1, p, p, 1, 64, 3, p, 16, None, _ffi.BF16, None), "workspace"),
+            ("skyrl_attn_attend", (attn(2, 1, 8, 8, 4), p, p, 15, p, p, p, 1, p, p, 1, 64, 1, p, 16, None, _ffi.BF16, None), "bad sizes"),
+            ("skyrl_attn_prefill", (attn(2, 1, 300, 8, 4), p, p, 16, p, p, p, 1, p, 1, p, 16, None), "dim, vdim"),
+            ("skyrl_ssd_scan", (ssd(3, 8, 8, 2, 4), p, 99, p, p, p, p, p, p, p, p, 1, p, p, 0, p, 24, _ffi.BF16, None), "multiple of groups"),
+            ("skyrl_ssd_scan", (ssd(2, 1024, 1024, 1, 4), p, 9999, p, p, p, p, p, p, p, p, 1, p, p, 0, p, 2048, _ffi.BF16, None), "too large"),
+            ("skyrl_ssd_prompt", (ssd(2, 8, 300, 1, 4), p, p, p, p, p, 2, p, p, p, p, 1, p, 1, p, 0, p, 0, p, p, p, p, p, p, p, p,
+                                  16, None), "at most 256")):
+        with pytest.raises(_ffi.SkyrlHipError, match=msg):
+            _ffi.call(name, *args)
 
 
 def test_layers_entries_validate_on_host():
@@ -51,7 +87,7 @@ def test_layers_entries_validate_on_host():
             ("skyrl_add_norm", (None, p, None, p, 0.0, 1, 64, 1e-5, 0, p, _ffi.I64, None), "dtype"),
             ("skyrl_gate_mul", (p, 16, 1, 8, 7, 1.0, 0.0, p, 8, _ffi.F32, None), "activation"),
             ("skyrl_gate_mul", (p, 15, 1, 8, 2, 1.0, 0.0, p, 8, _ffi.F32, None), "sizes"),
-            ("skyrl_embed", (p, p, 1, 0, 1.0, p, _ffi.F32, None), "sizes"),
+            ("skyrl_embed", (p, p, 1, 0, 1.0, None, None, p, None, _ffi.F32, None), "sizes"),
             ("skyrl_conv_save", (p, 7, 8, 3, p, p, p, 1, p, _ffi.F32, None), "sizes"),
             ("skyrl_latent_write", (p, 10, 1, 1, 4, 4, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "proj_stride"),
             ("skyrl_latent_write", (p, 100, 1, 1, 4, 4, 40, p, 1e-5, p, p, p, p, 40, _ffi.F32, None), "multiple of 32"),

@@ -165,8 +165,10 @@ def test_conv_chunk(units, taps, silu, cuts, dtype):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("cuts", CUTS)
 @pytest.mark.parametrize("C,blocks,taps", [(256, 2, 4), (60, 3, 3), (96, 1, 1), (320, 1, 4), (136, 17, 9), (7, 7, 2)])
-def test_rglru(C, blocks, taps, cuts, dtype):
-    """Decays from 1 - 1e-6 to almost nothing, so that a lost or stale state shows."""
+@pytest.mark.parametrize("per_run", [1, 1024])
+def test_rglru(C, blocks, taps, per_run, cuts, dtype):
+    """One run of chunks per sequence and one per chunk or two (skyrl_amd's plan lies between).
+    Decays from 1 - 1e-6 to almost nothing, so that a lost or stale state shows."""
     g = torch.Generator().manual_seed(C)
     n = C // blocks
     m = mixers.GatedLinearRecurrence({"width": C, "blocks": blocks, "conv": taps}, 1, 0.0, 8, mixers.Weights(DEV, dtype, None, 0.0))
@@ -188,7 +190,7 @@ def test_rglru(C, blocks, taps, cuts, dtype):
             pass
 
         inp.cu, inp.rows, inp.positions, inp.one_token = cu, rows, pos, all(k == 1 for k in lens)
-        inp.plan = {"all_chunks": plan_of(mixers.chunk_plan, lens, 0, 0)}
+        inp.plan = {m.plan_key: plan_of(mixers.chunk_runs, lens, 0, 0, per_run)}
         out = torch.full((len(x), C + 3), 7.0, dtype=dtype, device=DEV)
         m.inner(x, out[:, :C], inp, (S, ring), None)
         assert bool((out[:, C:] == 7).all())

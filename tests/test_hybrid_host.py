@@ -412,6 +412,17 @@ def test_normed_checkpoint_registry(tmp_path):
         load_decoder(str(tmp_path), "cpu", max_model_len=64)
 
 
+def test_kernel_libraries_of_a_checkpoint():
+    from skyrl_amd.inference_engines.registry import kernel_libraries
+
+    assert kernel_libraries(NORMED["odd"]) == ("layers", "attn", "rglru", "ssd")
+    assert kernel_libraries(normed_config([rglru()])) == ("layers", "rglru")
+    assert kernel_libraries(PARALLEL["odd"]) == ("layers", "diff") and kernel_libraries(CONFIGS["odd"]) == ("layers", "delta", "latent")
+    assert kernel_libraries({"model_type": "qwen2"}) == ()
+    with pytest.raises(ValueError, match="unknown layer"):
+        kernel_libraries(normed_config([{"type": "none", "mixer": {}}]))
+
+
 def test_position_turns():
     m = HybridDecoder(NORMED["odd"], "cpu", seed=None, max_model_len=64)
     W, pos = NORMED["odd"]["width"], torch.tensor([0, 1, 5, 4000])
@@ -451,11 +462,12 @@ def test_walk_plan_covers_every_chunk_once(lens, per_run):
     tok = sum(lens[:first])
     chunk, runs, pick, chain = mixers.walk_plan(lens, first, tok, per_run)
     ref_chunk, ends = mixers.chunk_plan(lens, first, tok)
-    assert (chunk == ref_chunk).all()
+    assert (chunk[:, :3] == ref_chunk[:, :3]).all()
     covered, by_seq = [], {}
     for r, (a, n, seq, kind) in enumerate(runs.tolist()):
         assert n > 0 and {int(c) for c in chunk[a:a + n, 2]} == {seq}
         covered += range(a, a + n)
+        assert set(chunk[a:a + n, 3].tolist()) == {r}
         by_seq.setdefault(seq, []).append((r, kind))
     assert covered == list(range(len(chunk)))
     many = {s: rs for s, rs in by_seq.items() if len(rs) > 1}
@@ -468,10 +480,12 @@ def test_walk_plan_covers_every_chunk_once(lens, per_run):
 def test_normed_plans_and_window_tiles():
     m = HybridDecoder(NORMED["odd"], "cpu", seed=None, max_model_len=64)
     plan = m.plan([1, 2, 40], [3, 0, 7], 2)
-    assert set(plan) == {"all_chunks", ("tiles", 37), ("tiles", 16), "runs", ("walk", 3), ("walk", 4)}
-    assert plan["all_chunks"][0].tolist() == [[0, 1, 0, 0], [1, 2, 1, 0], [3, 40, 2, 0]] and plan["all_chunks"][1].tolist() == [0, 1, 2, 3]
+    assert set(plan) == {("runs", 3), ("runs", 2), ("tiles", 37), ("tiles", 16), "runs", ("walk", 3), ("walk", 4)}
+    chunk, runs, seq_runs = plan[("runs", 3)]  # short portions too
+    assert chunk.tolist() == [[0, 1, 0, 0], [1, 2, 1, 1], [3, 40, 2, 2]] and seq_runs.tolist() == [0, 1, 2, 3]
+    assert runs.tolist() == [[0, 1, 0, 2], [1, 1, 1, 2], [2, 1, 2, 2]]
     assert plan[("tiles", 16)][0].tolist() == [[3, 40, 7, 2]] and plan[("walk", 3)][1].tolist() == [[0, 1, 2, 2]]
-    assert set(m.plan([1, 2], [3, 0], 2)) == {"all_chunks"}
+    assert set(m.plan([1, 2], [3, 0], 2)) == {("runs", 3), ("runs", 2)}
     tiles = mixers.tile_plan([300, 200], [0, 1000], 0, 0, 128)
     assert sorted(tiles[:, 0].tolist()) == [0, 128, 256, 300, 428]
     keys = [t[1] + min(t[2], 128) for t in tiles.tolist()]
