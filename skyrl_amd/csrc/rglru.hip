@@ -113,7 +113,7 @@ __device__ __forceinline__ void recurrence_of(float zr, float zi, float u, float
 
 // ---- decode: one token per sequence; grid (nb splits, ceil(n / 16)) ---------------------------------
 template <typename T, int VEC>
-__global__ __launch_bounds__(kNT) void rglru_step_kernel(Dims d, const T* __restrict__ proj, int64_t stride,
+__global__ __launch_bounds__(kNT) __attribute__((amdgpu_waves_per_eu(sizeof(T) == 2 ? 4 : 2))) void rglru_step_kernel(Dims d, const T* __restrict__ proj, int64_t stride,
                                                          const float* __restrict__ conv_t,
                                                          const float* __restrict__ conv_b, Gates<T> gt,
                                                          const int32_t* __restrict__ rows,

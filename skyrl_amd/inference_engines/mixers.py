@@ -157,17 +157,20 @@ def run_plan(seq_lens: List[int], starts: List[int], first_seq: int, first_token
     return np.concatenate(runs).astype(np.int32)
 
 
-WALK_WORKGROUPS = 1024  # of the recurrences' prompt walks: four per CU
-WALK_CHUNKS = 4         # chunks per run of the state space walk at least: a run's state is written and read once more
+# Workgroups of a prompt walk: what the CUs hold at once (four and three each).
+LINEAR_WALK = 1024
+STATE_WALK = 768
+WALK_CHUNKS = 4  # chunks per run of the state space walk at least: a run's state is written and read once more
 
 
-def chunk_runs(seq_lens: List[int], first_seq: int, first_token: int, per_run: int, least: int = 1):
+def chunk_runs(seq_lens: List[int], first_seq: int, first_token: int, per_run: int, total: int = LINEAR_WALK,
+               least: int = 1):
     """Sequences first_seq.. as chunks, and their chunks in runs, at least `least` chunks long, so that about
-    WALK_WORKGROUPS workgroups walk them, per_run of them per run: (chunk int32 [n, 4], the fourth number the
+    `total` workgroups walk them, per_run of them per run: (chunk int32 [n, 4], the fourth number the
     chunk's run, runs int32 [m, 4]: first chunk, chunks, sequence, 1 if the sequence has several runs + 2 if its
     last, seq_runs int32 [sequences + 1])."""
     chunk, ends = chunk_plan(seq_lens, first_seq, first_token)
-    size = max(least, -(-len(chunk) * per_run // WALK_WORKGROUPS))
+    size = max(least, -(-len(chunk) * per_run // total))
     runs, seq_runs = [], [0]
     for i in range(len(ends) - 1):
         n = int(ends[i + 1] - ends[i])
@@ -183,7 +186,7 @@ def chunk_runs(seq_lens: List[int], first_seq: int, first_token: int, per_run: i
 def walk_plan(seq_lens: List[int], first_seq: int, first_token: int, per_run: int):
     """Host plan of the state space prompt form of sequences first_seq..: (chunk, runs, pick int32 [k], chain int32
     [j, 2]) as skyrl_ssd_prompt takes them."""
-    chunk, runs, seq_runs = chunk_runs(seq_lens, first_seq, first_token, per_run, WALK_CHUNKS)
+    chunk, runs, seq_runs = chunk_runs(seq_lens, first_seq, first_token, per_run, STATE_WALK, WALK_CHUNKS)
     chain = [(a, b - a) for a, b in zip(seq_runs, seq_runs[1:]) if b - a > 1]
     pick = [r for r, kind in enumerate(runs[:, 3]) if kind == 1]
     return chunk, runs, np.asarray(pick, dtype=np.int32), np.asarray(chain, dtype=np.int32).reshape(-1, 2)

@@ -167,8 +167,7 @@ def test_conv_chunk(units, taps, silu, cuts, dtype):
 @pytest.mark.parametrize("C,blocks,taps", [(256, 2, 4), (60, 3, 3), (96, 1, 1), (320, 1, 4), (136, 17, 9), (7, 7, 2)])
 @pytest.mark.parametrize("per_run", [1, 1024])
 def test_rglru(C, blocks, taps, per_run, cuts, dtype):
-    """One run of chunks per sequence and one per chunk or two (skyrl_amd's plan lies between).
-    Decays from 1 - 1e-6 to almost nothing, so that a lost or stale state shows."""
+    """A run of chunks per chunk, and one per sequence. Decays from 1 - 1e-6 to almost nothing, so that a lost or stale state shows."""
     g = torch.Generator().manual_seed(C)
     n = C // blocks
     m = mixers.GatedLinearRecurrence({"width": C, "blocks": blocks, "conv": taps}, 1, 0.0, 8, mixers.Weights(DEV, dtype, None, 0.0))
