@@ -31,6 +31,12 @@ extern "C" {
  *                   m = a T [n, H], or, with two outputs, share (rms(a) wa + rms(b) wb) (wa, wb T [H]); hidden f32 +=
  *                   rms(m) * weight; out T = hidden, or rms(hidden) * final_weight if that is given. weight and
  *                   final_weight T hold one number for all columns or H (weight_n, final_n). H <= 8192.
+ *   skyrl_gate_norm_add  for sublayers between two norms in `groups` equal parts (norm(v): every part over the root of
+ *                   its own mean square + eps): y = the sum of `parts` consecutive rows of H of a, row rows[i] * parts on
+ *                   (rows NULL: i * parts), times sigmoid(gate T [n, gate_stride] + gate_bias f32 [H]) if gate is
+ *                   given; hidden f32 [n, H] += mult * norm(y) * weight T [H] (fresh: from 0); out T = norm(hidden) *
+ *                   next T [H]. H <= 8192.
+ *   skyrl_tanh      out T [n, I] = tanh of x T [n, I] (row stride `stride`).
  *   skyrl_gated_norm  out T [n, width] = rms over each of `groups` equal parts of y silu(z), times weight T [width].
  *   skyrl_xielu     out T [n, I] = ap x^2 + x / 2 for x > 0, an (exp(x) - 1 - x) + x / 2 otherwise, ap = softplus(p),
  *                   an = 1/2 + softplus(q) from pq T [2].
@@ -61,6 +67,10 @@ int skyrl_gated_norm(const void* y, int64_t y_stride, const void* z, int64_t z_s
                      void* stream);
 int skyrl_gate_mul(const void* gate_up, int64_t gu_stride, int64_t n, int32_t I, int32_t act, float alpha, float limit,
                    void* out, int64_t out_stride, int32_t dtype, void* stream);
+int skyrl_gate_norm_add(const void* a, const int64_t* rows, int32_t parts, const void* gate, int64_t gate_stride,
+                        const float* gate_bias, const void* weight, int32_t groups, float eps, float mult, float* hidden,
+                        int32_t fresh, const void* next, int32_t n, int32_t H, void* out, int32_t dtype, void* stream);
+int skyrl_tanh(const void* x, int64_t stride, int64_t n, int32_t I, void* out, int32_t dtype, void* stream);
 int skyrl_conv_save(const void* x, int64_t stride, int32_t channels, int32_t taps, const int32_t* cu,
                     const int32_t* rows, const int64_t* positions, int32_t nseq, void* ring, int32_t dtype,
                     void* stream);
@@ -71,11 +81,13 @@ int skyrl_softcap(const void* x, float* out, int64_t count, float cap, int32_t d
  * part all heads share (rot_dim), zero padding up to row = a multiple of 32. slot = block * 16 +
  * offset. Token t of a step belongs to row bt_row[t] of block_tables i32 [*, bt_stride] and attends
  * to the cached positions [max(0, positions[t] - window + 1), positions[t]] (window <= 0: all).
- *   skyrl_latent_write   proj T [T, proj_stride]: q (heads x (dim + rot_dim)) | latent (rank) | key
- *                        part (rot_dim). Rotates the q parts in place (interleaved pairs), writes the
- *                        RMS-normed latent (weight T [rank]) and the rotated key part into the cache
- *                        at slots[t] (< 0: no write). cos_sin f32 [max_pos, rot_dim] = cos | sin
- *                        halves, one entry per pair, amplitude included.
+ * Rotations pair neighbouring dimensions, or with `halves` i and i + rot_dim / 2; cos_sin f32 [max_pos, rot_dim] =
+ * cos | sin halves, one entry per pair, amplitude included. sinks f32 [heads] (may be NULL): exp(sink) joins a
+ * head's denominator. gate T [T, gate_stride] (may be NULL): a head's output times sigmoid(gate[t][head]).
+ *   skyrl_latent_write   rows of proj T [T, proj_stride], in place, each part optional: heads > 0: q (heads x (dim +
+ *                        rot_dim)) at the row's start, its rotated parts turned; q_rank > 0: a query latent there,
+ *                        RMS-normed (weight T [q_rank]); rank > 0: at latent_at the key latent (rank) | key part
+ *                        (rot_dim), RMS-normed (weight T [rank]) and turned into the cache at slots[t] (< 0: no write).
  *   skyrl_latent_attend  one query row per token in the latent space: qa T [heads, T, rank] is the
  *                        unrotated query times the key up-projection, q_rot points at the rotated part
  *                        of head 0 of token 0 (token stride q_stride, head stride q_head); out
@@ -96,23 +108,23 @@ int skyrl_softcap(const void* x, float* out, int64_t count, float cap, int32_t d
  *                        of 64 (skyrl_latent_gather zeroes the padding rows). out T [T, out_stride], head h at
  *                        h * vdim. dim + rot_dim <= 256, vdim <= 256, vt_stride % 64 == 0. */
 int skyrl_latent_write(void* proj, int64_t proj_stride, int32_t T, int32_t heads, int32_t dim, int32_t rot_dim,
-                       int32_t rank, const void* norm_weight, float eps, const int64_t* positions,
-                       const int64_t* slots, const float* cos_sin, void* cache, int32_t row, int32_t dtype,
-                       void* stream);
+                       int32_t halves, int32_t q_rank, const void* q_norm, int32_t rank, int32_t latent_at,
+                       const void* norm_weight, float eps, const int64_t* positions, const int64_t* slots,
+                       const float* cos_sin, void* cache, int32_t row, int32_t dtype, void* stream);
 int skyrl_latent_attend_mfma(int32_t rank, int32_t rot_dim, int32_t row, int32_t dtype);
 size_t skyrl_latent_attend_workspace_bytes(int32_t T, int32_t heads, int32_t rank, int32_t nparts);
 int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_stride, int64_t q_head, const void* cache,
                         int32_t row, const int32_t* block_tables, int64_t bt_stride, const int32_t* bt_row,
                         const int64_t* positions, int32_t T, int32_t heads, int32_t rank, int32_t rot_dim,
-                        float scale, int32_t window, int32_t part_min, int32_t nparts, void* out, void* workspace,
-                        int32_t dtype, void* stream);
+                        float scale, int32_t window, int32_t part_min, int32_t nparts, const float* sinks,
+                        const void* gate, int64_t gate_stride, void* out, void* workspace, int32_t dtype, void* stream);
 int skyrl_latent_gather(const void* cache, int32_t row, const int32_t* block_tables, int64_t bt_stride,
                         const int32_t* seg, int32_t nseg, int32_t max_count, int32_t rank, int32_t rot_dim,
                         void* latent, void* k_rot, int32_t dtype, void* stream);
 int skyrl_latent_prefill(const void* q, int64_t q_stride, const void* k_nope, int64_t k_stride, const void* k_rot,
                          const void* v_t, int64_t vt_stride, const int32_t* tiles, int32_t ntiles, int32_t heads,
-                         int32_t dim, int32_t rot_dim, int32_t vdim, float scale, int32_t window, void* out,
-                         int64_t out_stride, void* stream);
+                         int32_t dim, int32_t rot_dim, int32_t vdim, float scale, int32_t window, const float* sinks,
+                         const void* gate, int64_t gate_stride, void* out, int64_t out_stride, void* stream);
 
 /* ---- gated delta rule ------------------------------------------------------------------------
  * proj T [T, proj_stride]: q (kv_heads x dim) | k (kv_heads x dim) | v (heads x vdim) | output gate
@@ -319,6 +331,63 @@ int skyrl_ssd_prompt(const skyrl_ssd_shape* shape, const void* xt, const void* b
                      int32_t nsuper, const int32_t* pick, int32_t npick, const int32_t* chain, int32_t nchain,
                      const int32_t* cu, const int32_t* rows, const int64_t* positions, float* state, float* scores,
                      float* runs, float* gtot, void* y, int64_t y_stride, void* stream);
+
+/* ---- generalized delta rule ------------------------------------------------------------------------
+ * proj T [T, proj_stride]: r | k | v | output gate | removal rate, each heads x dim; wl T [T, wl_stride] the decay
+ * logits (heads x dim); w0, a_bias f32 [heads dim]; norm_w T [heads dim]. Per head, with u = k / sqrt(sum k^2 + 1e-6),
+ * w = exp(-e^(-1/2) sigmoid(wl + w0)) and a = sigmoid(removal rate + a_bias), S the state before the token:
+ *   S' = diag(w) S - (a u) (u^T S) + k v^T;  o = S'^T r;  out = o / sqrt(mean(o^2) + eps) * norm_w * sigmoid(output gate).
+ * State per row: f32 [rows, heads, dim, vpad], vpad = dim up to a multiple of 4. Sequences, rows and chunks as for the
+ * gated delta rule. dim <= 256.
+ *   skyrl_gdelta_scan   token by token, the state in registers: decode steps and short portions.
+ *   Prompt form, chunks of 64, d16 = dim up to a multiple of 16, all f32:
+ *   skyrl_gdelta_chunk  1: what a chunk does to the state, S <- M S + N, and its outputs O + R S: M [nchunks, heads, d16,
+ *                       d16], N [.., d16 values, d16 keys], R and O [.., 64, d16].
+ *   skyrl_gdelta_chain  2: sequences seq0.. of nseq: the states along each sequence's chunks [seq_chunks[i], seq_chunks[i
+ *                       + 1]), updated in `state`, every chunk's first one in first [nchunks, heads, d16 values, d16 keys].
+ *   skyrl_gdelta_out    3: outputs, head norm, weight and gate (gate T [T, gate_stride]: proj's output gate columns). */
+typedef struct {
+    int32_t heads, dim;
+    float eps;
+} skyrl_gdelta_shape;
+int skyrl_gdelta_scan(const skyrl_gdelta_shape* shape, const void* proj, int64_t proj_stride, const void* wl,
+                      int64_t wl_stride, const float* w0, const float* a_bias, const void* norm_w, const int32_t* cu,
+                      const int32_t* rows, const int64_t* positions, int32_t nseq, float* state, void* out,
+                      int64_t out_stride, int32_t dtype, void* stream);
+int skyrl_gdelta_chunk(const skyrl_gdelta_shape* shape, const void* proj, int64_t proj_stride, const void* wl,
+                       int64_t wl_stride, const float* w0, const float* a_bias, const int32_t* chunk, int32_t nchunks,
+                       float* M, float* N, float* R, float* O, int32_t dtype, void* stream);
+int skyrl_gdelta_chain(const skyrl_gdelta_shape* shape, const int32_t* chunk, const int32_t* seq_chunks, int32_t seq0,
+                       int32_t nseq, const int32_t* cu, const int32_t* rows, const int64_t* positions, const float* M,
+                       const float* N, float* state, float* first, void* stream);
+int skyrl_gdelta_out(const skyrl_gdelta_shape* shape, const int32_t* chunk, int32_t nchunks, const float* R,
+                     const float* O, const float* first, const void* gate, int64_t gate_stride, const void* norm_w,
+                     void* out, int64_t out_stride, int32_t dtype, void* stream);
+
+/* ---- routed experts ------------------------------------------------------------------------------------
+ * x T [n, width]. Of `experts` gated feed-forwards (gate_up T [experts, 2, ff, width], down T [experts, width, ff])
+ * each token runs `top`: scores s = sigmoid(router x) (router T [experts, width], f32 sums), choice scores s +
+ * correction f32 [experts]; of `groups` equal groups of neighbours the `keep` with the largest sum of their two largest
+ * choice scores may be chosen from; the `top` largest of those are, ties to the lower index. Pair p = token * top + i.
+ *   skyrl_moe_route    idx i32 [n, top], weight f32 [n, top] (the scores s of the chosen).
+ *   skyrl_moe_tiles    the most tiles of tm rows that npairs pairs can fill.
+ *   skyrl_moe_sort     pairs by expert: order i32 [ntiles, tm] (pair, or -1), tile_expert i32 [ntiles] (-1: unused).
+ *   skyrl_moe_gate_up  act T [ntiles tm, ff], by sorted place = silu(gate x) * up x. tm a multiple of 16; 16, 64 and 128
+ *                      have a matrix form (bf16, width and ff multiples of 8).
+ *   skyrl_moe_down     out T [n top, width], by pair = weight * down act. */
+typedef struct {
+    int32_t width, ff, experts, top, groups, keep;
+} skyrl_moe_shape;
+int skyrl_moe_route(const skyrl_moe_shape* shape, const void* x, int32_t n, const void* router, const float* correction,
+                    int32_t* idx, float* weight, int32_t dtype, void* stream);
+int32_t skyrl_moe_tiles(int32_t experts, int32_t npairs, int32_t tm);
+int skyrl_moe_sort(const int32_t* idx, int32_t npairs, int32_t experts, int32_t tm, int32_t ntiles, int32_t* order,
+                   int32_t* tile_expert, void* stream);
+int skyrl_moe_gate_up(const skyrl_moe_shape* shape, const void* x, const void* w, const int32_t* order,
+                      const int32_t* tile_expert, int32_t tm, int32_t ntiles, void* act, int32_t dtype, void* stream);
+int skyrl_moe_down(const skyrl_moe_shape* shape, const void* act, const void* w, const int32_t* order,
+                   const int32_t* tile_expert, int32_t tm, int32_t ntiles, const float* weight, void* out, int32_t dtype,
+                   void* stream);
 
 #ifdef __cplusplus
 }

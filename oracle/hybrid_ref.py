@@ -1,7 +1,8 @@
 """Plain CPU restatement of the hybrid decoders (Dovidra: latent attention + gated delta rule layers;
 Lipedra: differential attention in parallel layers; Foduzen: gated linear recurrences, and windowed
-attention beside a state space mixer, behind norms of the sublayers' outputs), one function per mechanism,
-whole sequences at a time, in the dtype of its weights (float64 in the tests).
+attention beside a state space mixer, behind norms of the sublayers' outputs; Tativik: latent attention with
+low-rank queries and sinks, a generalized delta rule and routed experts, each gated between two norms), one
+function per mechanism, whole sequences at a time, in the dtype of its weights (float64 in the tests).
 Test infrastructure only: nothing under skyrl_amd/ imports it and it shares no code with it.
 
 `w` maps tensor names to CPU tensors; `cfg` is the parsed config.json.
@@ -330,6 +331,135 @@ def output_norm_layer(x, w, i, entry, eps):
     return x
 
 
+def grouped_rms_norm(x, w, groups, eps):
+    """Every one of `groups` equal consecutive parts over its own root mean square, times the weight."""
+    return rms(x.reshape(x.shape[:-1] + (groups, x.shape[-1] // groups)), eps).reshape(x.shape) * w
+
+
+def rotate_halves(x, positions, rot):
+    """Rotary of the first rot.dims of x [T, ..., D], dimension i paired with i + dims / 2."""
+    f, amp = rotary_frequencies(rot)
+    half = rot["dims"] // 2
+    y = x.clone()
+    for i, fi in enumerate(f):
+        a = positions.to(torch.float64) * fi
+        shape = (-1,) + (1,) * (x.dim() - 2)
+        c, s = ((t * amp).to(x.dtype).view(shape) for t in (torch.cos(a), torch.sin(a)))
+        u, v = x[..., i], x[..., half + i]
+        y[..., i] = u * c - v * s
+        y[..., half + i] = v * c + u * s
+    return y
+
+
+def sink_attention(q, k, v, scale, size, sink):
+    """window_attention whose denominators also hold exp(sink[head])."""
+    T = q.shape[0]
+    s = torch.einsum("ihd,jhd->hij", q, k) * scale
+    d = torch.arange(T)[:, None] - torch.arange(T)[None]
+    see = (d >= 0) & (d < (T if size is None else size))
+    s = s.masked_fill(~see, float("-inf"))
+    top = torch.maximum(s.amax(-1), sink[:, None])[..., None]
+    e = torch.exp(s - top)
+    return torch.einsum("hij,jhv->ihv", e / (e.sum(-1, keepdim=True) + torch.exp(sink[:, None, None] - top)), v)
+
+
+def latent_keys(h, w, p, m, eps):
+    """(normed latents [T, rank], rotated key part [T, rot_dim]): what a layer of its own caches."""
+    down, C = h @ w[p + "dkv"].T, m["kv_rank"]
+    return rms_norm(down[:, :C], w[p + "dkv.norm"], eps), rotate_halves(down[:, C:], torch.arange(h.shape[0]), m["rot"])
+
+
+def sink_latent_attention(h, w, p, m, eps, kv):
+    """kv: (latents, rotated key part), this layer's own or another's."""
+    T = h.shape[0]
+    H, D, R, V = m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+    c_q = rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps)
+    q = (c_q @ w[p + "uq"].T).view(T, H, D + R)
+    q = torch.cat([q[..., :D], rotate_halves(q[..., D:], torch.arange(T), m["rot"])], -1)
+    c, kr = kv
+    k = torch.cat([(c @ w[p + "uk"].T).view(T, H, D), kr[:, None].expand(T, H, R)], -1)
+    v = (c @ w[p + "uv"].T).view(T, H, V)
+    size = m["mask"]["size"] if m.get("mask") else None
+    o = sink_attention(q, k, v, m["scale"], size, w[p + "sink"])
+    o = o * torch.sigmoid(h @ w[p + "g"].T)[:, :, None]
+    return o.reshape(T, H * V) @ w[p + "o"].T
+
+
+def general_delta_recurrence(r, k, v, decay, a, state=None):
+    """All inputs [T, H, D]: S_t = diag(decay) S - (a u) (u^T S) + k v^T with u = unit(k) and S the old state;
+    outputs S_t^T r [T, H, D] and the final state [H, D, D]."""
+    T, H, D = r.shape
+    S = torch.zeros(H, D, D, dtype=r.dtype) if state is None else state.clone()
+    u, out = unit(k), torch.zeros_like(v)
+    for t in range(T):
+        read = torch.einsum("hd,hdv->hv", u[t], S)
+        S = decay[t][..., None] * S - (a[t] * u[t])[..., None] * read[:, None] + k[t][..., None] * v[t][:, None]
+        out[t] = torch.einsum("hd,hdv->hv", r[t], S)
+    return out, S
+
+
+def general_delta_gates(h, w, p):
+    """(decay, removal rate), each [T, heads dim]."""
+    z = torch.tanh(h @ w[p + "w1"].T) @ w[p + "w2"].T + w[p + "w0"].reshape(-1)
+    return torch.exp(-math.exp(-0.5) * torch.sigmoid(z)), torch.sigmoid(h @ w[p + "a"].T + w[p + "a.b"].reshape(-1))
+
+
+def general_delta_mixer(h, w, p, m, eps):
+    T, H, D = h.shape[0], m["heads"], m["dim"]
+    r, k, v = ((h @ w[p + n].T).view(T, H, D) for n in "rkv")
+    decay, a = (t.view(T, H, D) for t in general_delta_gates(h, w, p))
+    o, _ = general_delta_recurrence(r, k, v, decay, a)
+    o = rms(o, eps).reshape(T, H * D) * w[p + "norm"].reshape(-1) * torch.sigmoid(h @ w[p + "g"].T)
+    return o @ w[p + "o"].T
+
+
+def route(scores, correction, top, groups=1, keep=1):
+    """Experts of every token [T, top] and their weights: the largest corrected scores among the `keep` groups whose
+    two largest corrected scores sum highest; the weights are the scores themselves."""
+    T, E = scores.shape
+    choice = scores + correction
+    per = E // groups
+    best = choice.view(T, groups, per).topk(min(2, per), -1).values.sum(-1)
+    kept = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best.topk(keep, -1).indices, True)
+    choice = choice.masked_fill(~kept.repeat_interleave(per, 1), float("-inf"))
+    idx = choice.topk(top, -1).indices
+    return idx, scores.gather(1, idx)
+
+
+def experts_ff(h, w, p, m):
+    """Weighted sum of the chosen experts' gated silu feed-forwards."""
+    ro = m["router"]
+    gr = ro.get("groups") or {"count": 1, "keep": 1}
+    idx, weight = route(torch.sigmoid(h @ w[p + "router"].T), w[p + "correction"], ro["top"], gr["count"], gr["keep"])
+    out = torch.zeros_like(h)
+    for t in range(h.shape[0]):
+        for e, s in zip(idx[t].tolist(), weight[t]):
+            q = f"{p}e{e}."
+            out[t] += s * ((silu(w[q + "gate"] @ h[t]) * (w[q + "up"] @ h[t])) @ w[q + "down"].T)
+    return out
+
+
+def sandwich_layer(x, w, i, entry, cfg, kvs):
+    """Tativik: each sublayer between two norms, its result gated before the second. kvs: latents by layer, extended
+    here."""
+    p, m, eps = f"l{i}.", entry["mixer"], cfg["norm"]["eps"]
+    norm = lambda y, name: grouped_rms_norm(y, w[p + name], cfg["norm"].get("groups", 1), eps)  # noqa: E731
+    gate = lambda h, name: torch.sigmoid(h @ w[p + name].T + w[p + name + ".b"])  # noqa: E731
+    h = norm(x, "norm1")
+    if entry["type"] == "general_delta":
+        y = general_delta_mixer(h, w, p + "mix.", m, eps)
+    else:
+        j = m.get("kv_from")
+        if j is None:
+            kvs[i] = latent_keys(h, w, p + "mix.", m, eps)
+        y = sink_latent_attention(h, w, p + "mix.", m, eps, kvs[i if j is None else j])
+    x = x + cfg["residual_mult"] * norm(y * gate(h, "rg1"), "norm1b")
+    if entry.get("mlp"):
+        h = norm(x, "norm2")
+        x = x + cfg["residual_mult"] * norm(experts_ff(h, w, p + "mlp.", entry["mlp"]) * gate(h, "rg2"), "norm2b")
+    return x
+
+
 def layer(x, w, i, entry, eps):
     """Dovidra: two halves, each behind a norm of its own."""
     p = f"l{i}."
@@ -369,8 +499,10 @@ def forward(tokens, w, cfg):
     """Logits [T, vocab] and the residual after every layer run [runs, T, width]."""
     eps, design = cfg["norm"]["eps"], cfg["architecture"]
     x = w["embed"][torch.as_tensor(tokens)]
-    if design != "Dovidra":
+    if design in ("Lipedra", "Foduzen"):
         x = x * cfg["embedding"]["scale"]
+    if design == "Tativik":
+        x = grouped_rms_norm(x, w["embed.norm"], cfg["norm"].get("groups", 1), eps)
     if design == "Foduzen":
         x = x + sinusoid(torch.arange(len(tokens)), cfg["width"]).to(x.dtype)
     trail, kvs = [], {}
@@ -380,11 +512,16 @@ def forward(tokens, w, cfg):
         e = cfg["layers"][i]
         if design == "Lipedra":
             x = parallel_layer(x, w, i, e, eps, kvs)
+        elif design == "Tativik":
+            x = sandwich_layer(x, w, i, e, cfg, kvs)
         else:
             x = (output_norm_layer if design == "Foduzen" else layer)(x, w, i, e, eps)
         trail.append(x)
-    norm = {"Dovidra": layer_norm, "Lipedra": rms_norm_about_one, "Foduzen": rms_norm}[design]
-    logits = norm(x, w["final.norm"], eps) @ w["head"].T
+    if design == "Tativik":
+        x = grouped_rms_norm(x, w["final.norm"], cfg["norm"].get("groups", 1), eps)
+    else:
+        x = {"Dovidra": layer_norm, "Lipedra": rms_norm_about_one, "Foduzen": rms_norm}[design](x, w["final.norm"], eps)
+    logits = x @ w["head"].T
     cap = cfg.get("logit_softcap")
     if cap:
         logits = cap * torch.tanh(logits / cap)

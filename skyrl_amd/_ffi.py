@@ -23,7 +23,7 @@ LIB_DIR = os.path.join(os.path.dirname(os.path.abspath(__file__)), "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libskyrl_hip.so")
 # the hybrid decoders' layer libraries: what every such model needs, and one per mechanism, whose entry points
 # start with skyrl_<name>_
-LAYER_LIBS = ("layers", "latent", "delta", "diff", "rglru", "attn", "ssd")
+LAYER_LIBS = ("layers", "latent", "delta", "diff", "rglru", "attn", "ssd", "gdelta", "moe")
 
 F32, BF16, I64, I32, U8 = 0, 1, 2, 3, 4
 M_FINAL_LOSS, M_POLICY_LOSS, M_ENTROPY, M_KL, M_CLIP_RATIO, M_MASK_SUM = 0, 1, 2, 3, 4, 5
@@ -259,11 +259,25 @@ class SSDShape(ctypes.Structure):
     _fields_ = [(n, ctypes.c_int32) for n in ("heads", "vdim", "state", "groups", "taps")]
 
 
+class GeneralDeltaShape(ctypes.Structure):
+    """Mirror of ``skyrl_gdelta_shape`` (include/skyrl_layers.h)."""
+
+    _fields_ = [("heads", ctypes.c_int32), ("dim", ctypes.c_int32), ("eps", ctypes.c_float)]
+
+
+class MoeShape(ctypes.Structure):
+    """Mirror of ``skyrl_moe_shape`` (include/skyrl_layers.h)."""
+
+    _fields_ = [(n, ctypes.c_int32) for n in ("width", "ff", "experts", "top", "groups", "keep")]
+
+
 # the exported surface of include/skyrl_layers.h, in libraries of its own (LAYER_LIBS)
 _DS = ctypes.POINTER(DeltaShape)
 _FS = ctypes.POINTER(DiffShape)
 _AS = ctypes.POINTER(AttnShape)
 _SS = ctypes.POINTER(SSDShape)
+_GS = ctypes.POINTER(GeneralDeltaShape)
+_MS = ctypes.POINTER(MoeShape)
 LAYERS_SIGNATURES = {
     "skyrl_embed": (_INT, [_P, _P, _I64, _I32, _F, _P, _P, _P, _P, _I32, _P]),
     "skyrl_norm_add": (_INT, [_P, _P, _P, _P, _F, _P, _P, _I32, _P, _I32, _I32, _I32, _F, _P, _I32, _P]),
@@ -272,14 +286,17 @@ LAYERS_SIGNATURES = {
     "skyrl_gate_mul": (_INT, [_P, _I64, _I64, _I32, _I32, _F, _F, _P, _I64, _I32, _P]),
     "skyrl_conv_save": (_INT, [_P, _I64, _I32, _I32, _P, _P, _P, _I32, _P, _I32, _P]),
     "skyrl_softcap": (_INT, [_P, _P, _I64, _F, _I32, _P]),
-    "skyrl_latent_write": (_INT, [_P, _I64, _I32, _I32, _I32, _I32, _I32, _P, _F, _P, _P, _P, _P, _I32, _I32, _P]),
+    "skyrl_gate_norm_add": (_INT, [_P, _P, _I32, _P, _I64, _P, _P, _I32, _F, _F, _P, _I32, _P, _I32, _I32, _P, _I32, _P]),
+    "skyrl_tanh": (_INT, [_P, _I64, _I64, _I32, _P, _I32, _P]),
+    "skyrl_latent_write": (_INT, [_P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _P, _I32, _I32, _P, _F, _P, _P, _P, _P, _I32,
+                                  _I32, _P]),
     "skyrl_latent_attend_mfma": (_INT, [_I32, _I32, _I32, _I32]),
     "skyrl_latent_attend_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
     "skyrl_latent_attend": (_INT, [_P, _P, _I64, _I64, _P, _I32, _P, _I64, _P, _P, _I32, _I32, _I32, _I32, _F, _I32,
-                                   _I32, _I32, _P, _P, _I32, _P]),
+                                   _I32, _I32, _P, _P, _I64, _P, _P, _I32, _P]),
     "skyrl_latent_gather": (_INT, [_P, _I32, _P, _I64, _P, _I32, _I32, _I32, _I32, _P, _P, _I32, _P]),
     "skyrl_latent_prefill": (_INT, [_P, _I64, _P, _I64, _P, _P, _I64, _P, _I32, _I32, _I32, _I32, _I32, _F, _I32, _P,
-                                    _I64, _P]),
+                                    _P, _I64, _P, _I64, _P]),
     "skyrl_delta_scan": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I32, _P, _I64, _I32, _P]),
     "skyrl_delta_conv": (_INT, [_DS, _P, _I64, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _P]),
     "skyrl_delta_chunk": (_INT, [_DS, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _P]),
@@ -307,6 +324,15 @@ LAYERS_SIGNATURES = {
     "skyrl_ssd_prompt": (_INT, [_SS, _P, _P, _P, _P, _P, _I64, _P, _P, _P, _P, _I32, _P, _I32, _P, _I32, _P, _I32, _P, _P,
                                 _P, _P, _P, _P, _P, _P, _I64, _P]),
     "skyrl_gated_norm": (_INT, [_P, _I64, _P, _I64, _P, _I64, _I32, _I32, _F, _P, _I64, _I32, _P]),
+    "skyrl_gdelta_scan": (_INT, [_GS, _P, _I64, _P, _I64, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I64, _I32, _P]),
+    "skyrl_gdelta_chunk": (_INT, [_GS, _P, _I64, _P, _I64, _P, _P, _P, _I32, _P, _P, _P, _P, _I32, _P]),
+    "skyrl_gdelta_chain": (_INT, [_GS, _P, _P, _I32, _I32, _P, _P, _P, _P, _P, _P, _P, _P]),
+    "skyrl_gdelta_out": (_INT, [_GS, _P, _I32, _P, _P, _P, _P, _I64, _P, _P, _I64, _I32, _P]),
+    "skyrl_moe_route": (_INT, [_MS, _P, _I32, _P, _P, _P, _P, _I32, _P]),
+    "skyrl_moe_tiles": (_I32, [_I32, _I32, _I32]),
+    "skyrl_moe_sort": (_INT, [_P, _I32, _I32, _I32, _I32, _P, _P, _P]),
+    "skyrl_moe_gate_up": (_INT, [_MS, _P, _P, _P, _P, _I32, _I32, _P, _I32, _P]),
+    "skyrl_moe_down": (_INT, [_MS, _P, _P, _P, _P, _I32, _I32, _P, _P, _I32, _P]),
 }
 
 # entry points with a per-call variant form (name + "_ex": the same arguments, then the variant)

@@ -27,42 +27,82 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 constexpr int kBS = 16;  // tokens per cache block
 constexpr int kNT = 256;
 
+// Dimension pairs of the rotation: neighbours, or i with i + rot / 2 (halves).
+struct Pairs {
+    int rot, halves;
+    __device__ __forceinline__ int first(int i) const { return halves ? i : 2 * i; }
+    __device__ __forceinline__ int second(int i) const { return halves ? i + rot / 2 : 2 * i + 1; }
+};
+
+// One workgroup per token. Parts of the row p that are there: the rotated parts of `heads` queries at its start, or
+// (q_rank > 0) a query latent that is normed in place; the key latent and its rotated part at lat_at (rank > 0).
 template <typename T>
 __global__ __launch_bounds__(kNT) void latent_write_kernel(T* __restrict__ proj, int64_t stride, int heads, int dim,
-                                                           int rot, int rank, const T* __restrict__ norm_w, float eps,
-                                                           const int64_t* __restrict__ positions,
+                                                           Pairs pr, int q_rank, const T* __restrict__ q_norm,
+                                                           int rank, int lat_at, const T* __restrict__ norm_w,
+                                                           float eps, const int64_t* __restrict__ positions,
                                                            const int64_t* __restrict__ slots,
                                                            const float* __restrict__ cos_sin, T* __restrict__ cache,
                                                            int row) {
     __shared__ float s_red[kNT / kWave];
     const int t = blockIdx.x;
     T* p = proj + (int64_t)t * stride;
-    const int qd = dim + rot, h2 = rot / 2;
-    const T* lat = p + (int64_t)heads * qd;
+    const int rot = pr.rot, qd = dim + rot, h2 = rot / 2;
     const float* cs = cos_sin + positions[t] * rot;
-    const int64_t slot = slots[t];
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < rank; i += kNT) {
-        const float v = ld(lat + i);
-        ss += v * v;
+    if (q_rank > 0) {
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < q_rank; i += kNT) {
+            const float v = ld(p + i);
+            ss += v * v;
+        }
+        const float r = 1.f / sqrtf(block_total<kNT>(ss, s_red) / (float)q_rank + eps);
+        for (int i = threadIdx.x; i < q_rank; i += kNT) st(p + i, ld(p + i) * r * ld(q_norm + i));
     }
-    const float r = 1.f / sqrtf(block_total<kNT>(ss, s_red) / (float)rank + eps);
-    if (slot >= 0) {
-        T* c = cache + slot * row;
-        for (int i = threadIdx.x; i < rank; i += kNT) st(c + i, ld(lat + i) * r * ld(norm_w + i));
-        for (int i = threadIdx.x; i < h2; i += kNT) {
-            const float u = ld(lat + rank + 2 * i), v = ld(lat + rank + 2 * i + 1);
-            st(c + rank + 2 * i, u * cs[i] - v * cs[h2 + i]);
-            st(c + rank + 2 * i + 1, v * cs[i] + u * cs[h2 + i]);
+    if (rank > 0) {
+        const T* lat = p + lat_at;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < rank; i += kNT) {
+            const float v = ld(lat + i);
+            ss += v * v;
+        }
+        const float r = 1.f / sqrtf(block_total<kNT>(ss, s_red) / (float)rank + eps);
+        const int64_t slot = slots[t];
+        if (slot >= 0) {
+            T* c = cache + slot * row;
+            for (int i = threadIdx.x; i < rank; i += kNT) st(c + i, ld(lat + i) * r * ld(norm_w + i));
+            for (int i = threadIdx.x; i < h2; i += kNT) {
+                const int a = pr.first(i), b = pr.second(i);
+                const float u = ld(lat + rank + a), v = ld(lat + rank + b);
+                st(c + rank + a, u * cs[i] - v * cs[h2 + i]);
+                st(c + rank + b, v * cs[i] + u * cs[h2 + i]);
+            }
         }
     }
     for (int e = threadIdx.x; e < heads * h2; e += kNT) {
         const int h = e / h2, i = e - h * h2;
-        T* q = p + (int64_t)h * qd + dim + 2 * i;
-        const float u = ld(q), v = ld(q + 1);
-        st(q, u * cs[i] - v * cs[h2 + i]);
-        st(q + 1, v * cs[i] + u * cs[h2 + i]);
+        T* q = p + (int64_t)h * qd + dim;
+        const int a = pr.first(i), b = pr.second(i);
+        const float u = ld(q + a), v = ld(q + b);
+        st(q + a, u * cs[i] - v * cs[h2 + i]);
+        st(q + b, v * cs[i] + u * cs[h2 + i]);
     }
+}
+
+// What ends a head's softmax: a learned sink in the denominator and a sigmoid gate on the output, each optional.
+template <typename T>
+struct HeadEnd {
+    const float* sinks;  // [heads]
+    const T* gate;       // logits [token][head]
+    int64_t gate_stride;
+    __device__ __forceinline__ float sink(int h) const { return sinks ? sinks[h] : -INFINITY; }
+    __device__ __forceinline__ float gated(int t, int h) const {
+        return gate ? sigmoidf_(ld(gate + (int64_t)t * gate_stride + h)) : 1.f;
+    }
+};
+// Factor of the value sums with running maximum m and denominator l, all in powers of two; sink in the same units.
+__device__ __forceinline__ float sum_factor(float m, float l, float sink) {
+    const float mm = fmaxf(m, sink), a = fast_exp2(m - mm);
+    return a / (l * a + fast_exp2(sink - mm));
 }
 
 // ---- decode form, plain: one workgroup per (token, head), any rank up to 2048, f32 or bf16 ----
@@ -71,7 +111,7 @@ __global__ __launch_bounds__(kNT) void latent_attend_plain_kernel(
     const T* __restrict__ qa, const T* __restrict__ q_rot, int64_t q_stride, int64_t q_head,
     const T* __restrict__ cache, int row, const int32_t* __restrict__ tables, int64_t bt_stride,
     const int32_t* __restrict__ bt_row, const int64_t* __restrict__ positions, int ntok, int heads, int rank, int rot,
-    float scale, int window, T* __restrict__ out) {
+    float scale, int window, HeadEnd<T> end, T* __restrict__ out) {
     extern __shared__ float s_q[];  // rank + rot
     __shared__ float s_p[kWave];
     constexpr int kAcc = 8;
@@ -122,10 +162,12 @@ __global__ __launch_bounds__(kNT) void latent_attend_plain_kernel(
         }
         __syncthreads();
     }
+    const float sink = end.sink(h), mm = fmaxf(m, sink), a = expf(m - mm);
+    const float f = a / (l * a + expf(sink - mm)) * end.gated(t, h);
 #pragma unroll
     for (int k = 0; k < kAcc; ++k) {
         const int d = threadIdx.x + k * kNT;
-        if (d < rank) st(out + ((int64_t)h * ntok + t) * rank + d, acc[k] / l);
+        if (d < rank) st(out + ((int64_t)h * ntok + t) * rank + d, acc[k] * f);
     }
 }
 
@@ -161,8 +203,8 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
     const uint16_t* __restrict__ qa, const uint16_t* __restrict__ q_rot, int64_t q_stride, int64_t q_head,
     const uint16_t* __restrict__ cache, int row, const int32_t* __restrict__ tables, int64_t bt_stride,
     const int32_t* __restrict__ bt_row, const int64_t* __restrict__ positions, int ntok, int heads, int rank, int rot,
-    float scale_log2, int window, int part_min, int nparts, uint16_t* __restrict__ out, float* __restrict__ ws_o,
-    float* __restrict__ ws_ml) {
+    float scale_log2, int window, int part_min, int nparts, HeadEnd<uint16_t> end, uint16_t* __restrict__ out,
+    float* __restrict__ ws_o, float* __restrict__ ws_ml) {
     constexpr int LDR = NK * 32 + 8;  // padded LDS row
     constexpr int LDS_ = 64 + 4, NW = NV / 4, NT = kNT * HG;
     constexpr int NL = (NK + HG - 1) / HG;  // 16-byte pieces of its page per lane
@@ -333,7 +375,7 @@ __global__ __launch_bounds__(kNT * HG) __attribute__((amdgpu_waves_per_eu(1, 2))
     const int h = h0 + 16 * hg + c;
     if (h >= heads) return;
     if (sp.parts == 1) {
-        const float inv = 1.f / l;
+        const float inv = sum_factor(m, l, end.sink(h) * kLog2e) * end.gated(t, h);
         uint16_t* orow = out + ((int64_t)h * ntok + t) * rank;
 #pragma unroll
         for (int n = 0; n < NW; ++n) {
@@ -365,7 +407,8 @@ __global__ __launch_bounds__(kWave * 2) void latent_merge_kernel(const float* __
                                                                  const float* __restrict__ ws_ml,
                                                                  const int64_t* __restrict__ positions, int ntok,
                                                                  int heads, int rank, int window, int part_min,
-                                                                 int nparts, uint16_t* __restrict__ out) {
+                                                                 int nparts, HeadEnd<uint16_t> end,
+                                                                 uint16_t* __restrict__ out) {
     const int h = blockIdx.x, t = blockIdx.y, lane = threadIdx.x & 63;
     const int pos = (int)positions[t];
     const int lo = window > 0 ? max(0, pos - window + 1) : 0;
@@ -378,7 +421,7 @@ __global__ __launch_bounds__(kWave * 2) void latent_merge_kernel(const float* __
     M = wave_max(M);
     float L = 0.f;
     for (int p = lane; p < sp.parts; p += kWave) L += fast_exp2(ws_ml[(rec + p) * 2] - M) * ws_ml[(rec + p) * 2 + 1];
-    const float inv = 1.f / wave_sum(L);
+    const float inv = sum_factor(M, wave_sum(L), end.sink(h) * kLog2e) * end.gated(t, h);
     uint16_t* orow = out + ((int64_t)h * ntok + t) * rank;
     for (int d = threadIdx.x * 4; d < rp; d += kWave * 8) {
         float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -465,7 +508,7 @@ __global__ __launch_bounds__(512 / QT) __attribute__((amdgpu_waves_per_eu(2))) v
     const uint16_t* __restrict__ q, int64_t q_stride, const uint16_t* __restrict__ k_nope, int64_t k_stride,
     const uint16_t* __restrict__ k_rot, const uint16_t* __restrict__ v_t, int64_t vt_stride,
     const int32_t* __restrict__ tiles, int heads, int dim, int rot, int vdim, float scale_log2, int window,
-    uint16_t* __restrict__ out, int64_t out_stride) {
+    HeadEnd<uint16_t> end, uint16_t* __restrict__ out, int64_t out_stride) {
     constexpr int NT = 512 / QT, QW = 16 * QT;
     constexpr int LDK = NK * 32 + 8, LDV = kKT + 8;
     constexpr int TPK = NT / kKT, KPT = NK * 4 / TPK;     // threads per key row, 16-byte chunks per thread
@@ -617,7 +660,7 @@ __global__ __launch_bounds__(512 / QT) __attribute__((amdgpu_waves_per_eu(2))) v
         s += __shfl_xor(s, 32, kWave);
         const int qi = QW * wave + 16 * qq + c;
         if (qi >= ntok) continue;
-        const float inv = 1.f / s;
+        const float inv = sum_factor(m[qq], s, end.sink(h) * kLog2e) * end.gated(tok0 + qi, h);
         uint16_t* orow = out + (int64_t)(tok0 + qi) * out_stride + (int64_t)h * vdim;
         const bool ovec = vdim % 4 == 0 && out_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0;
 #pragma unroll
@@ -642,21 +685,27 @@ __global__ __launch_bounds__(512 / QT) __attribute__((amdgpu_waves_per_eu(2))) v
 using namespace skyrl;
 
 extern "C" int skyrl_latent_write(void* proj, int64_t proj_stride, int32_t T_, int32_t heads, int32_t dim,
-                                  int32_t rot_dim, int32_t rank, const void* norm_weight, float eps,
-                                  const int64_t* positions, const int64_t* slots, const float* cos_sin, void* cache,
-                                  int32_t row, int32_t dtype, void* stream) {
+                                  int32_t rot_dim, int32_t halves, int32_t q_rank, const void* q_norm, int32_t rank,
+                                  int32_t latent_at, const void* norm_weight, float eps, const int64_t* positions,
+                                  const int64_t* slots, const float* cos_sin, void* cache, int32_t row, int32_t dtype,
+                                  void* stream) {
     SKYRL_REQUIRE_T(dtype, "latent_write");
-    SKYRL_REQUIRE(T_ >= 0 && heads > 0 && dim >= 0 && rot_dim >= 0 && rot_dim % 2 == 0 && rank > 0,
+    SKYRL_REQUIRE(T_ >= 0 && heads >= 0 && dim >= 0 && rot_dim >= 0 && rot_dim % 2 == 0 && rank >= 0 && q_rank >= 0,
                   "latent_write: bad sizes");
-    SKYRL_REQUIRE(row % 32 == 0 && row >= rank + rot_dim, "latent_write: row must be a multiple of 32 >= rank + rot_dim");
-    SKYRL_REQUIRE(proj_stride >= (int64_t)heads * (dim + rot_dim) + rank + rot_dim, "latent_write: proj_stride");
+    SKYRL_REQUIRE(heads == 0 || q_rank == 0, "latent_write: queries or their latent, not both");
+    SKYRL_REQUIRE(rank == 0 || (row % 32 == 0 && row >= rank + rot_dim),
+                  "latent_write: row must be a multiple of 32 >= rank + rot_dim");
+    const int64_t qw = q_rank > 0 ? q_rank : (int64_t)heads * (dim + rot_dim);
+    SKYRL_REQUIRE(proj_stride >= qw && (rank == 0 || (latent_at >= qw && proj_stride >= (int64_t)latent_at + rank + rot_dim)),
+                  "latent_write: proj_stride");
     if (T_ == 0) return SKYRL_OK;
-    SKYRL_REQUIRE(proj && norm_weight && positions && slots && cos_sin && cache, "latent_write: null pointer");
+    SKYRL_REQUIRE(proj && positions && cos_sin && (q_rank == 0 || q_norm) && (rank == 0 || (norm_weight && slots && cache)),
+                  "latent_write: null pointer");
     SKYRL_DISPATCH_T(dtype, {
         hipLaunchKernelGGL((latent_write_kernel<T>), dim3(T_), dim3(kNT), 0, as_stream(stream),
-                           reinterpret_cast<T*>(proj), proj_stride, heads, dim, rot_dim, rank,
-                           reinterpret_cast<const T*>(norm_weight), eps, positions, slots, cos_sin,
-                           reinterpret_cast<T*>(cache), row);
+                           reinterpret_cast<T*>(proj), proj_stride, heads, dim, Pairs{rot_dim, halves}, q_rank,
+                           reinterpret_cast<const T*>(q_norm), rank, latent_at, reinterpret_cast<const T*>(norm_weight),
+                           eps, positions, slots, cos_sin, reinterpret_cast<T*>(cache), row);
     })
     return check_launch("latent_write_kernel");
 }
@@ -674,7 +723,8 @@ extern "C" size_t skyrl_latent_attend_workspace_bytes(int32_t T_, int32_t heads,
 #define LAUNCH_ATTEND_(NV, NK, EX, HG)                                                                               \
     hipLaunchKernelGGL((latent_attend_mfma_kernel<NV, NK, EX, HG>), dim3(nparts, (heads + 16 * HG - 1) / (16 * HG), T_), \
                        dim3(kNT * HG), 0, s, q_, r_, q_stride, q_head, c_, row, block_tables, bt_stride, bt_row,     \
-                       positions, T_, heads, rank, rot_dim, scale * kLog2e, window, part_min, nparts, o_, ws_o, ws_ml)
+                       positions, T_, heads, rank, rot_dim, scale * kLog2e, window, part_min, nparts, end_, o_,  \
+                       ws_o, ws_ml)
 #define LAUNCH_ATTEND(NV, NK, EX)                    \
     if (heads > 16) LAUNCH_ATTEND_(NV, NK, EX, 2);   \
     else LAUNCH_ATTEND_(NV, NK, EX, 1)
@@ -683,8 +733,10 @@ extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_
                                    const void* cache, int32_t row, const int32_t* block_tables, int64_t bt_stride,
                                    const int32_t* bt_row, const int64_t* positions, int32_t T_, int32_t heads,
                                    int32_t rank, int32_t rot_dim, float scale, int32_t window, int32_t part_min,
-                                   int32_t nparts, void* out, void* workspace, int32_t dtype, void* stream) {
+                                   int32_t nparts, const float* sinks, const void* gate, int64_t gate_stride, void* out,
+                                   void* workspace, int32_t dtype, void* stream) {
     SKYRL_REQUIRE_T(dtype, "latent_attend");
+    SKYRL_REQUIRE(!gate || gate_stride >= heads, "latent_attend: gate_stride");
     SKYRL_REQUIRE(T_ >= 0 && T_ <= 65535 && heads > 0 && rank > 0 && rank <= 2048 && rot_dim >= 0,
                   "latent_attend: bad sizes (T <= 65535, rank <= 2048)");
     SKYRL_REQUIRE(row % 32 == 0 && row >= rank + rot_dim, "latent_attend: row must be a multiple of 32 >= rank + rot_dim");
@@ -697,7 +749,8 @@ extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_
                                (rank + rot_dim) * sizeof(float), s, reinterpret_cast<const T*>(qa),
                                reinterpret_cast<const T*>(q_rot), q_stride, q_head, reinterpret_cast<const T*>(cache),
                                row, block_tables, bt_stride, bt_row, positions, T_, heads, rank, rot_dim, scale,
-                               window, reinterpret_cast<T*>(out));
+                               window, HeadEnd<T>{sinks, reinterpret_cast<const T*>(gate), gate_stride},
+                               reinterpret_cast<T*>(out));
         })
         return check_launch("latent_attend_plain_kernel");
     }
@@ -709,6 +762,7 @@ extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_
     const uint16_t* r_ = reinterpret_cast<const uint16_t*>(q_rot);
     const uint16_t* c_ = reinterpret_cast<const uint16_t*>(cache);
     uint16_t* o_ = reinterpret_cast<uint16_t*>(out);
+    const HeadEnd<uint16_t> end_{sinks, reinterpret_cast<const uint16_t*>(gate), gate_stride};
     float* ws_o = reinterpret_cast<float*>(workspace);
     float* ws_ml = ws_o ? ws_o + (size_t)T_ * heads * nparts * (((rank + 15) / 16) * 16) : nullptr;
     const int nk = row / 32, nv = (rank + 15) / 16;
@@ -726,7 +780,7 @@ extern "C" int skyrl_latent_attend(const void* qa, const void* q_rot, int64_t q_
     int rc = check_launch("latent_attend_mfma_kernel");
     if (rc != SKYRL_OK || nparts == 1) return rc;
     hipLaunchKernelGGL(latent_merge_kernel, dim3(heads, T_), dim3(kWave * 2), 0, s, ws_o, ws_ml, positions, T_, heads, rank,
-                       window, part_min, nparts, o_);
+                       window, part_min, nparts, end_, o_);
     return check_launch("latent_merge_kernel");
 }
 
@@ -755,12 +809,13 @@ extern "C" int skyrl_latent_gather(const void* cache, int32_t row, const int32_t
                        as_stream(stream), reinterpret_cast<const uint16_t*>(q), q_stride,                             \
                        reinterpret_cast<const uint16_t*>(k_nope), k_stride, reinterpret_cast<const uint16_t*>(k_rot), \
                        reinterpret_cast<const uint16_t*>(v_t), vt_stride, tiles, heads, dim, rot_dim, vdim,           \
-                       scale * kLog2e, window, reinterpret_cast<uint16_t*>(out), out_stride)
+                       scale * kLog2e, window, end_, reinterpret_cast<uint16_t*>(out), out_stride)
 
 extern "C" int skyrl_latent_prefill(const void* q, int64_t q_stride, const void* k_nope, int64_t k_stride,
                                     const void* k_rot, const void* v_t, int64_t vt_stride, const int32_t* tiles,
                                     int32_t ntiles, int32_t heads, int32_t dim, int32_t rot_dim, int32_t vdim,
-                                    float scale, int32_t window, void* out, int64_t out_stride, void* stream) {
+                                    float scale, int32_t window, const float* sinks, const void* gate,
+                                    int64_t gate_stride, void* out, int64_t out_stride, void* stream) {
     SKYRL_REQUIRE(ntiles >= 0 && heads > 0 && dim >= 0 && rot_dim >= 0 && dim + rot_dim > 0 && dim + rot_dim <= 256 &&
                       vdim > 0 && vdim <= 256,
                   "latent_prefill: dim + rot_dim and vdim must be in [1, 256]");
@@ -769,6 +824,8 @@ extern "C" int skyrl_latent_prefill(const void* q, int64_t q_stride, const void*
     if (ntiles == 0) return SKYRL_OK;
     SKYRL_REQUIRE(q && k_nope && k_rot && v_t && tiles && out, "latent_prefill: null pointer");
     SKYRL_REQUIRE(aligned16(k_nope) && aligned16(k_rot) && aligned16(v_t), "latent_prefill: 16-byte alignment");
+    SKYRL_REQUIRE(!gate || gate_stride >= heads, "latent_prefill: gate_stride");
+    const HeadEnd<uint16_t> end_{sinks, reinterpret_cast<const uint16_t*>(gate), gate_stride};
     const int nk = (dim + rot_dim + 31) / 32, nv = (vdim + 15) / 16;
     const bool vec = dim % 8 == 0 && rot_dim % 8 == 0 && k_stride % 8 == 0 && q_stride % 8 == 0 && aligned16(q);
     if (nk <= 2 && nv <= 8) {

@@ -389,6 +389,136 @@ __global__ __launch_bounds__(NT) void gated_norm_kernel(const T* __restrict__ y,
     }
 }
 
+// ---- a sublayer's result between two norms in equal parts: gated, normed, added to the residual, normed again ----
+template <typename T>
+struct GateNormAdd {
+    const T* a;
+    const int64_t* rows;  // row of a (NULL: the output's own)
+    int parts;            // consecutive rows of a that are summed
+    const T* z;           // gate logits (NULL: no gate) and their bias
+    int64_t z_stride;
+    const float* zb;
+    const T* w;
+    int groups;
+    float eps, mult;
+    float* h;
+    int fresh;  // the residual starts at 0
+    const T* wn;
+    T* out;
+    int H;
+};
+
+// 1 / root mean square of every group of `per` consecutive chunks into s_r, from the chunks' sums of squares s_p: teams
+// of up to 64 lanes. All threads of the block call it; s_p is written by them before.
+__device__ __forceinline__ void group_scales(const float* s_p, float* s_r, int groups, int per, float len, float eps) {
+    __syncthreads();
+    int L = kWave;
+    while (L > 1 && groups * L > kNT) L >>= 1;
+    const int sub = threadIdx.x & (L - 1);
+    for (int g = threadIdx.x / L; g < groups; g += kNT / L) {
+        float s = 0.f;
+        for (int i = sub; i < per; i += L) s += s_p[g * per + i];
+        for (int o = L >> 1; o > 0; o >>= 1) s += __shfl_xor(s, o, kWave);
+        if (sub == 0) s_r[g] = 1.f / sqrtf(s / len + eps);
+    }
+    __syncthreads();
+}
+
+// One block per row, the row in registers. Chunks of VEC elements lie in one group.
+template <typename T, int VEC, int kMaxV>
+__global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p) {
+    extern __shared__ float s_p[];  // a chunk's sum of squares; then the groups' scales
+    __shared__ float s_red[kNT / kWave];
+    const int nv = p.H / VEC, per = nv / p.groups;
+    float* s_r = s_p + nv;
+    const int64_t base = (int64_t)blockIdx.x * p.H;
+    const int64_t row = p.rows ? p.rows[blockIdx.x] : blockIdx.x;
+    const float len = (float)(p.H / p.groups);
+    float y[kMaxV][VEC], h[kMaxV][VEC];
+    float one = 0.f;
+#pragma unroll
+    for (int k = 0; k < kMaxV; ++k) {
+        const int v = threadIdx.x + k * kNT;
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) y[k][j] = h[k][j] = 0.f;
+        if (v < nv) {
+            const T* src = p.a + row * p.parts * p.H + VEC * v;
+            ldw<T, VEC>(src, y[k]);
+            if (!p.fresh) ldw<float, VEC>(p.h + base + VEC * v, h[k]);
+            for (int i = 1; i < p.parts; ++i) {
+                float x[VEC];
+                ldw<T, VEC>(src + (int64_t)i * p.H, x);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) y[k][j] += x[j];
+            }
+            if (p.z) {
+                float z[VEC], b[VEC];
+                ldw<T, VEC>(p.z + blockIdx.x * p.z_stride + VEC * v, z);
+                ldw<float, VEC>(p.zb + VEC * v, b);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) y[k][j] *= sigmoid_<T>(z[j] + b[j]);
+            }
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) ss += y[k][j] * y[k][j];
+            if (p.groups > 1) s_p[v] = ss;
+        }
+        one += ss;
+    }
+    float r1 = 0.f;
+    if (p.groups == 1) r1 = 1.f / sqrtf(block_total<kNT>(one, s_red) / len + p.eps);
+    else group_scales(s_p, s_r, p.groups, per, len, p.eps);
+    one = 0.f;
+#pragma unroll
+    for (int k = 0; k < kMaxV; ++k) {
+        const int v = threadIdx.x + k * kNT;
+        float ss = 0.f;
+        if (v < nv) {
+            const float r = p.groups == 1 ? r1 : s_r[v / per];
+            float w[VEC];
+            ldw<T, VEC>(p.w + VEC * v, w);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) {
+                h[k][j] += p.mult * (y[k][j] * r * w[j]);
+                ss += h[k][j] * h[k][j];
+            }
+            stw<float, VEC>(p.h + base + VEC * v, h[k]);
+            if (p.groups > 1) s_p[v] = ss;  // its own chunks only: the others' scales are not read again before the barrier
+        }
+        one += ss;
+    }
+    if (p.groups == 1) r1 = 1.f / sqrtf(block_total<kNT>(one, s_red) / len + p.eps);
+    else group_scales(s_p, s_r, p.groups, per, len, p.eps);
+#pragma unroll
+    for (int k = 0; k < kMaxV; ++k) {
+        const int v = threadIdx.x + k * kNT;
+        if (v < nv) {
+            const float r = p.groups == 1 ? r1 : s_r[v / per];
+            float w[VEC];
+            ldw<T, VEC>(p.wn + VEC * v, w);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) h[k][j] *= r * w[j];
+            stw<T, VEC>(p.out + base + VEC * v, h[k]);
+        }
+    }
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(kNT) void tanh_kernel(const T* __restrict__ x, int64_t stride, int64_t n, int I,
+                                                   T* __restrict__ out) {
+    const int iv = I / VEC;
+    const int64_t total = n * iv;
+    for (int64_t e = (int64_t)blockIdx.x * kNT + threadIdx.x; e < total; e += (int64_t)gridDim.x * kNT) {
+        const int64_t row = e / iv;
+        const int c = (int)(e - row * iv) * VEC;
+        float v[VEC];
+        ldv<T, VEC>(x + row * stride + c, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[j] = tanhf(v[j]);
+        stv(out + row * I + c, v);
+    }
+}
+
 unsigned grid_for(int64_t items) {
     const int64_t b = (items + kNT - 1) / kNT;
     return (unsigned)(b > 8192 ? 8192 : b);
@@ -518,6 +648,58 @@ extern "C" int skyrl_xielu(const void* x, int64_t stride, int64_t n, int32_t I, 
                                stride, n, I, w, o, out_stride);
     })
     return check_launch("xielu_kernel");
+}
+
+#define LAUNCH_GNA(V, K) \
+    hipLaunchKernelGGL((gate_norm_add_kernel<T, V, K>), dim3(n), dim3(kNT), lds(V), as_stream(stream), p)
+
+extern "C" int skyrl_gate_norm_add(const void* a, const int64_t* rows, int32_t parts, const void* gate,
+                                   int64_t gate_stride, const float* gate_bias, const void* weight, int32_t groups,
+                                   float eps, float mult, float* hidden, int32_t fresh, const void* next, int32_t n,
+                                   int32_t H, void* out, int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "gate_norm_add");
+    SKYRL_REQUIRE(n >= 0 && H > 0 && H <= 8192 && parts > 0, "gate_norm_add: H must be in [1, 8192], parts positive");
+    SKYRL_REQUIRE(groups > 0 && H % groups == 0, "gate_norm_add: H must be a multiple of groups");
+    SKYRL_REQUIRE(!gate || (gate_bias && gate_stride >= H), "gate_norm_add: gate needs a bias and a stride >= H");
+    if (n == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(a && weight && hidden && next && out, "gate_norm_add: null pointer");
+    auto lds = [&](int V) { return groups > 1 ? (size_t)(H / V + groups) * sizeof(float) : (size_t)0; };
+    SKYRL_DISPATCH_T(dtype, {
+        auto t = [](const void* q) { return reinterpret_cast<const T*>(q); };
+        const GateNormAdd<T> p{t(a), rows, parts, t(gate), gate_stride, gate_bias, t(weight), groups, eps, mult, hidden,
+                               fresh, t(next), reinterpret_cast<T*>(out), H};
+        const bool wide = H / groups % 4 == 0 &&
+                          (!gate || (gate_stride % 4 == 0 && reinterpret_cast<uintptr_t>(gate) % (4 * sizeof(T)) == 0));
+        if (wide) {
+            if (H <= 4 * kNT) LAUNCH_GNA(4, 1);
+            else if (H <= 8 * kNT) LAUNCH_GNA(4, 2);
+            else if (H <= 16 * kNT) LAUNCH_GNA(4, 4);
+            else LAUNCH_GNA(4, 8);
+        } else {
+            SKYRL_REQUIRE(lds(1) <= 65536 - 64, "gate_norm_add: too many groups");
+            if (H <= 4 * kNT) LAUNCH_GNA(1, 4);
+            else LAUNCH_GNA(1, 32);
+        }
+    })
+    return check_launch("gate_norm_add_kernel");
+}
+
+extern "C" int skyrl_tanh(const void* x, int64_t stride, int64_t n, int32_t I, void* out, int32_t dtype, void* stream) {
+    SKYRL_REQUIRE_T(dtype, "tanh");
+    SKYRL_REQUIRE(n >= 0 && I > 0 && stride >= I, "tanh: bad sizes");
+    if (n == 0) return SKYRL_OK;
+    SKYRL_REQUIRE(x && out, "tanh: null pointer");
+    SKYRL_DISPATCH_T(dtype, {
+        const T* in = reinterpret_cast<const T*>(x);
+        T* o = reinterpret_cast<T*>(out);
+        if (I % 8 == 0 && stride % 8 == 0 && aligned16(in) && aligned16(o))
+            hipLaunchKernelGGL((tanh_kernel<T, 8>), dim3(grid_for(n * (I / 8))), dim3(kNT), 0, as_stream(stream), in,
+                               stride, n, I, o);
+        else
+            hipLaunchKernelGGL((tanh_kernel<T, 1>), dim3(grid_for(n * I)), dim3(kNT), 0, as_stream(stream), in, stride, n,
+                               I, o);
+    })
+    return check_launch("tanh_kernel");
 }
 
 extern "C" int skyrl_conv_save(const void* x, int64_t stride, int32_t channels, int32_t taps, const int32_t* cu,

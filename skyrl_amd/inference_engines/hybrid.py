@@ -8,13 +8,16 @@ layers over an earlier layer's keys and values, beside clamped gates with biases
 RMS norm, mixer and feed-forward in the same two matrix products), and a scaled embedding. Foduzen is a
 third: gated linear recurrences, and layers of windowed attention beside a state space mixer, which read
 the residual itself and whose outputs are normed (one number as the weight), xIELU feed-forwards, sinusoidal
-position vectors. The model is what config.json lists; the mechanisms are mixers.py; `DESIGNS` holds what a
+position vectors. Tativik is a fourth: latent attention with low-rank queries, sinks and head gates, some layers over an
+earlier layer's latents, and a generalized delta rule; routed experts; every sublayer stands between two norms in equal
+parts and is gated before the second, and the embedding is normed. The model is what config.json lists; the mechanisms are mixers.py; `DESIGNS` holds what a
 design fixes.
 
 The residual stream is f32. One pass of the HIP norm kernel adds the previous sublayer's output and
 (at the start of a loop pass) its vector, stores the stream and writes the next product's input; where
 outputs are normed, one pass norms the sublayer's output (or joins and norms two), adds it, stores the
-stream and writes the next product's input, at the end the final norm.
+stream and writes the next product's input, at the end the final norm. Between two norms likewise: gate, norm, add,
+store, norm.
 
 HybridDecoder has PagedDecoder's interface (model.py), so the engine's scheduler, runner, sampler and
 weight updates serve it unchanged; besides, it takes portions: a step may continue several prompts
@@ -32,7 +35,8 @@ import torch.nn.functional as F
 
 from . import kernels
 from . import layer_kernels as lk
-from .mixers import FEEDFORWARDS, MIXERS, PLAIN_FEEDFORWARDS, PROMPT_MIN, Products, SideBySide, Weights
+from .mixers import (EXPERT_FEEDFORWARDS, FEEDFORWARDS, MIXERS, PLAIN_FEEDFORWARDS, PROMPT_MIN, Gated, Products,
+                     SideBySide, Weights)
 from .model import StepInputs
 
 DEFAULT_MAX_MODEL_LEN = 32768
@@ -50,12 +54,16 @@ class Design:
     output_norms: bool = False  # sublayers read the residual, their outputs are normed
     scalar_norms: bool = False  # a norm's weight is one number
     sinusoid: Optional[float] = None  # base of the position vectors added to the embedding
+    sandwich: bool = False   # sublayers between two norms in equal parts, gated before the second; normed embedding
+    mixers: Dict[str, Dict[str, Any]] = field(default_factory=dict)  # mixer constants by type
 
 
 DESIGNS = {
     "Dovidra": Design(norm="layer", mlp={"act": "gelu_tanh"}),
     "Lipedra": Design(norm="rms", norm_base=1.0, parallel=True, mlp={"act": "clamped", "alpha": 1.702, "bias": True}),
     "Foduzen": Design(norm="rms", output_norms=True, scalar_norms=True, sinusoid=10000.0, feedforwards=PLAIN_FEEDFORWARDS),
+    "Tativik": Design(norm="rms", sandwich=True, feedforwards=EXPERT_FEEDFORWARDS,
+                      mixers={"latent_attention": {"sink": True, "gate": True, "halves": True}}),
 }
 
 
@@ -82,6 +90,8 @@ class HybridSpec:
     eos_token_id: Optional[int] = None
     tie_word_embeddings: bool = False
     initializer_range: float = 0.02
+    norm_groups: int = 1       # equal parts of a row that are normed apart (sandwich)
+    residual_mult: float = 1.0  # of what a sublayer adds (sandwich)
 
     @property
     def num_layers(self) -> int:
@@ -101,13 +111,13 @@ class HybridSpec:
             j = e["mixer"].get("kv_from")
             if j is None:
                 continue
-            m = layers[j]["mixer"] if 0 <= j < i else None
-            if m is None or layers[j]["type"] != e["type"] or m.get("kv_from") is not None \
-                    or any(m.get(k) != e["mixer"].get(k) for k in ("kv_heads", "dim", "vdim")):
+            m, keys = layers[j]["mixer"] if 0 <= j < i else None, getattr(MIXERS[e["type"]], "shared_keys", None)
+            if m is None or keys is None or layers[j]["type"] != e["type"] or m.get("kv_from") is not None \
+                    or any(m.get(k) != e["mixer"].get(k) for k in keys):
                 raise ValueError(f"layer {i}: kv_from {j} is no earlier layer with such keys and values of its own")
         n, loop = len(layers), cfg.get("loop")
         runs, times = [], 0
-        if loop and design.output_norms:
+        if loop and (design.output_norms or design.sandwich):
             raise ValueError("this design has no looped layers")
         if loop:
             a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
@@ -125,7 +135,8 @@ class HybridSpec:
                    logit_softcap=float(cfg["logit_softcap"]) if cfg.get("logit_softcap") else None, layers=layers,
                    runs=runs, loop_times=times,
                    max_position_embeddings=int(cfg.get("max_position_embeddings") or DEFAULT_MAX_MODEL_LEN),
-                   eos_token_id=None if eos is None else int(eos))
+                   eos_token_id=None if eos is None else int(eos), norm_groups=int(cfg["norm"].get("groups") or 1),
+                   residual_mult=float(cfg.get("residual_mult", 1.0)))
 
 
 class HybridCache:
@@ -172,7 +183,7 @@ class HybridDecoder:
     # a biased product of one row copies the bias first instead of adding it in the library's kernel
     @property
     def min_bucket(self) -> int:
-        subs = [sub for L in self.layers for _, sub in L["subs"]]
+        subs = [sub[1] for L in self.layers for sub in L["subs"]]
         return 2 if any(isinstance(sub, Products) and sub.biased for sub in subs) else 1
 
     # ---------------------------------------------------------------- weights
@@ -186,11 +197,16 @@ class HybridDecoder:
         self.embed = w.matrix(s.vocab_size, H)
         self.layers: List[Dict[str, Any]] = []
         for e in s.layers:
-            mixer = MIXERS[e["type"]](e["mixer"], H, s.norm_eps, self.max_model_len, w)
+            mixer = MIXERS[e["type"]](e["mixer"], H, s.norm_eps, self.max_model_len, w, **d.mixers.get(e["type"], {}))
             mlp = d.feedforwards[e["mlp"]["kind"]](e["mlp"], H, w, **d.mlp) if e.get("mlp") else None
             joined = hasattr(mixer, "inner")  # its products are Products'
             L = {"mixer": mixer, "mlp": mlp, "norm1": norm(), "norm2": None}
-            if d.parallel and mlp is not None:
+            if d.sandwich:
+                L["subs"] = [(L["norm1"], Gated(mixer, H, w), norm())]
+                if mlp is not None:
+                    L["norm2"] = norm()
+                    L["subs"].append((L["norm2"], Gated(mlp, H, w), norm()))
+            elif d.parallel and mlp is not None:
                 if not joined:
                     raise ValueError(f"{e['type']!r} layers cannot be parallel to a feed-forward")
                 L["subs"] = [(L["norm1"], Products([mixer, mlp], H, w))]
@@ -206,6 +222,9 @@ class HybridDecoder:
             self.layers.append(L)
         self.loop_step = w.matrix(s.loop_times, H) if s.loop_times else None
         self.norm = norm()
+        self.embed_norm = norm() if d.sandwich else None
+        if d.sandwich and H % s.norm_groups:
+            raise ValueError("the width must be a multiple of norm.groups")
         self.turns = None  # revolutions per position of each pair of the position vector's columns
         if d.sinusoid:
             i = torch.arange((H + 1) // 2, dtype=torch.float64)
@@ -217,6 +236,8 @@ class HybridDecoder:
         out = {"embed": self.embed, "final.norm": self.norm, "head": self.lm_head}
         if self.loop_step is not None:
             out["loop.step"] = self.loop_step
+        if self.embed_norm is not None:
+            out["embed.norm"] = self.embed_norm
         for i, L in enumerate(self.layers):
             p = f"l{i}."
             out[p + "norm1"] = L["norm1"]
@@ -227,6 +248,9 @@ class HybridDecoder:
             if L["mlp"] is not None:
                 for name, t in L["mlp"].params():
                     out[p + "mlp." + name] = t
+            if self.spec.design.sandwich:
+                for k, (_, sub, after) in enumerate(L["subs"], 1):
+                    out.update({f"{p}norm{k}b": after, f"{p}rg{k}": sub.weight, f"{p}rg{k}.b": sub.bias})
         return out
 
     def hf_named_tensors(self) -> Iterator[Tuple[str, torch.Tensor]]:
@@ -253,7 +277,7 @@ class HybridDecoder:
         return sum(int(t.numel()) for t in self._param_views().values())
 
     def release(self):
-        self.embed = self.lm_head = self.norm = self.loop_step = None
+        self.embed = self.lm_head = self.norm = self.loop_step = self.embed_norm = None
         self.layers = []
 
     # ---------------------------------------------------------------- cache and plans
@@ -302,6 +326,8 @@ class HybridDecoder:
         s = self.spec
         if s.design.output_norms:
             return self._run_output_normed(inp, cache, want, trail)
+        if s.design.sandwich:
+            return self._run_sandwich(inp, cache, want, trail)
         norm = dict(eps=s.norm_eps, kind=s.design.norm, base=s.design.norm_base)
         h = lk.embed(inp.tokens, self.embed, s.embed_scale)
         x = torch.empty(h.shape, dtype=self.dtype, device=self.device)
@@ -343,6 +369,30 @@ class HybridDecoder:
             if trail is not None:
                 trail.append(h.clone())
         raise ValueError("a model needs a layer")
+
+    def _run_sandwich(self, inp: StepInputs, cache: HybridCache, want: Optional[torch.Tensor], trail=None):
+        s = self.spec
+        norm = dict(eps=s.norm_eps, groups=s.norm_groups)
+        steps = [(state, *sub) for r, state in zip(s.runs, cache.runs) for sub in self.layers[r.layer]["subs"]]
+        ends = {sum(len(self.layers[q.layer]["subs"]) for q in s.runs[:k + 1]) - 1 for k in range(len(s.runs))}
+        before = [st[1] for st in steps] + [self.norm]  # the norm ahead of every sublayer, then the final one
+        h = torch.empty((inp.tokens.shape[0], s.hidden_size), dtype=torch.float32, device=self.device)
+        x = lk.gate_norm_add(self.embed, h, self.embed_norm, before[0], rows=inp.tokens, fresh=True, **norm)
+        ws = self.workspace if inp.one_token else self.portion_workspace
+        for k, (state, _, sub, after) in enumerate(steps):
+            y, gate = sub.forward(x, inp, state, ws)
+            args = dict(norm, mult=s.residual_mult, parts=sub.rows_per_token, gate_bias=sub.bias)
+            last = k == len(steps) - 1
+            if last and trail is not None:
+                lk.gate_norm_add(y, (full := h.clone()), after, self.norm, gate=gate, **args)
+                trail.append(full)
+            if last and want is not None:
+                y = y.view(-1, sub.rows_per_token, s.hidden_size)[want].view(-1, s.hidden_size)
+                h, gate, x = h[want], gate[want], None
+            x = lk.gate_norm_add(y, h, after, before[k + 1], gate=gate, out=x, **args)
+            if trail is not None and k in ends and not last:
+                trail.append(h.clone())
+        return x
 
     def forward_decode(self, inp: StepInputs, cache: HybridCache) -> torch.Tensor:
         """One token per row: final hidden states [n, H]."""

@@ -107,6 +107,46 @@ def norm_add(delta, hidden: torch.Tensor, weight: torch.Tensor, eps: float, pair
     return out
 
 
+def gate_norm_add(a: torch.Tensor, hidden: torch.Tensor, weight: torch.Tensor, next_weight: torch.Tensor, eps: float,
+                  groups: int = 1, mult: float = 1.0, parts: int = 1, gate: Optional[torch.Tensor] = None,
+                  gate_bias: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None, fresh: bool = False,
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """hidden (f32 [n, H], in place; fresh: from 0) += mult norm(y) weight, y the sum of `parts` consecutive rows of a,
+    times sigmoid(gate + gate_bias) with a gate; returns norm(hidden) next_weight. A norm is an RMS norm in `groups`
+    equal parts of the row. `rows` int64 [n]: which rows of a (parts 1)."""
+    dev = _require_gpu(a, hidden, weight, next_weight, gate, gate_bias, rows, out)
+    n, H = hidden.shape
+    _check(hidden, "hidden", torch.float32)
+    if a.dim() != 2 or a.shape[1] != H or (rows is None and a.shape[0] != n * parts) or (rows is not None and parts != 1):
+        raise ValueError(f"a must be [{n} * parts, {H}], with rows [any, {H}] and one part")
+    _check(a, "a", weight.dtype)
+    _check(weight, "weight", weight.dtype, (H,))
+    _check(next_weight, "next_weight", weight.dtype, (H,))
+    _check(rows, "rows", torch.int64, (n,))
+    if (gate is None) != (gate_bias is None):
+        raise ValueError("gate and gate_bias go together")
+    if gate is not None:
+        _check_view(gate, "gate", weight.dtype, (n, H))
+        _check(gate_bias, "gate_bias", torch.float32, (H,))
+    if out is None:
+        out = torch.empty((n, H), dtype=weight.dtype, device=dev)
+    _check(out, "out", weight.dtype, (n, H))
+    _ffi.call("skyrl_gate_norm_add", _ptr(a), _ptr(rows), parts, _ptr(gate), 0 if gate is None else max(gate.stride(0), H),
+              _ptr(gate_bias), _ptr(weight), groups, float(eps), float(mult), _ptr(hidden), int(fresh), _ptr(next_weight), n, H,
+              _ptr(out), _code(weight), _stream(dev))
+    return out
+
+
+def tanh(x: torch.Tensor) -> torch.Tensor:
+    """tanh of x [n, I] (a column range), contiguous."""
+    dev = _require_gpu(x)
+    n, I = x.shape
+    _check_view(x, "x", x.dtype, (n, I))
+    out = torch.empty((n, I), dtype=x.dtype, device=dev)
+    _ffi.call("skyrl_tanh", _ptr(x), max(x.stride(0), I), n, I, _ptr(out), _code(x), _stream(dev))
+    return out
+
+
 def xielu(x: torch.Tensor, pq: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """xIELU of x [n, I] with the learned pair pq; both may be column ranges."""
     dev = _require_gpu(x, pq, out)
@@ -178,36 +218,56 @@ def _check_table(block_tables, bt_row, positions, T):
     _check(positions, "positions", torch.int64, (T,))
 
 
-def latent_write(proj, heads, dim, rot_dim, rank, norm_weight, eps, positions, slots, cos_sin, cache) -> None:
-    """Rotate the q parts of ``proj`` in place; write the normed latent and the rotated key part."""
-    dev = _require_gpu(proj, norm_weight, positions, slots, cos_sin, cache)
-    T = proj.shape[0]
-    width = heads * (dim + rot_dim) + rank + rot_dim
-    if proj.dim() != 2 or proj.shape[1] != width or proj.stride(1) != 1:
-        raise ValueError(f"proj must be [T, {width}] with unit column stride")
-    _check(norm_weight, "norm_weight", proj.dtype, (rank,))
+def _check_rotation(positions, cos_sin, rot_dim, T):
     _check(positions, "positions", torch.int64, (T,))
-    _check(slots, "slots", torch.int64, (T,))
     if cos_sin.dim() != 2 or cos_sin.shape[1] != rot_dim:
         raise ValueError("cos_sin must be [max_pos, rot_dim]")
     _check(cos_sin, "cos_sin", torch.float32)
-    _check_cache(cache, rank, rot_dim, proj.dtype)
-    _ffi.call("skyrl_latent_write", _ptr(proj), proj.stride(0), T, heads, dim, rot_dim, rank, _ptr(norm_weight),
-              float(eps), _ptr(positions), _ptr(slots), _ptr(cos_sin), _ptr(cache), cache.shape[2], _code(proj),
-              _stream(dev))
+
+
+def latent_write(proj, rot_dim, positions, slots, cos_sin, cache, eps, heads: int = 0, dim: int = 0, q_norm=None,
+                 rank: int = 0, norm_weight=None, halves: bool = False) -> None:
+    """Rows of ``proj`` in place, each part optional: with `heads` the rotated parts of the queries at the row's start
+    are turned, with `q_norm` [q_rank] the query latent there is normed; with `rank` the key latent and its rotated part
+    that follow are normed, turned and written into the cache."""
+    dev = _require_gpu(proj, q_norm, norm_weight, positions, slots, cos_sin, cache)
+    T = proj.shape[0]
+    q_rank = 0 if q_norm is None else q_norm.shape[0]
+    at = q_rank or heads * (dim + rot_dim)
+    width = at + (rank + rot_dim if rank else 0)
+    if (heads and q_rank) or proj.dim() != 2 or proj.shape[1] < width or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, >= {width}] with unit column stride, queries or their latent first")
+    _check_rotation(positions, cos_sin, rot_dim, T)
+    _check(q_norm, "q_norm", proj.dtype, (q_rank,))
+    if rank:
+        _check(norm_weight, "norm_weight", proj.dtype, (rank,))
+        _check(slots, "slots", torch.int64, (T,))
+        _check_cache(cache, rank, rot_dim, proj.dtype)
+    _ffi.call("skyrl_latent_write", _ptr(proj), proj.stride(0), T, heads, dim, rot_dim, int(halves), q_rank, _ptr(q_norm),
+              rank, at, _ptr(norm_weight), float(eps), _ptr(positions), _ptr(slots), _ptr(cos_sin), _ptr(cache),
+              cache.shape[2] if rank else 0, _code(proj), _stream(dev))
+
+
+def _check_end(sinks, gate, heads, T, dtype):
+    _check(sinks, "sinks", torch.float32, (heads,))
+    if gate is not None:
+        _check_view(gate, "gate", dtype, (T, heads))
+    return 0 if gate is None else max(gate.stride(0), heads)
 
 
 def latent_attend(qa, q_rot, cache, rank, rot_dim, block_tables, bt_row, positions, scale, window, nparts=1,
-                  part_min=64, workspace=None) -> torch.Tensor:
+                  part_min=64, workspace=None, sinks=None, gate=None) -> torch.Tensor:
     """Latent-space attention, one query row per token. qa [heads, T, rank]; q_rot [T, heads, rot_dim]
-    (any token and head stride); returns [heads, T, rank]."""
-    dev = _require_gpu(qa, q_rot, cache, block_tables, bt_row, positions)
+    (any token and head stride); returns [heads, T, rank]. sinks f32 [heads]: exp(sink) joins the denominators; gate
+    [T, heads]: outputs times its sigmoid."""
+    dev = _require_gpu(qa, q_rot, cache, block_tables, bt_row, positions, sinks, gate)
     heads, T, R = qa.shape
     _check(qa, "qa", cache.dtype, (heads, T, rank))
     if q_rot.dtype != qa.dtype or tuple(q_rot.shape) != (T, heads, rot_dim) or (rot_dim > 1 and q_rot.stride(2) != 1):
         raise ValueError("q_rot must be [T, heads, rot_dim] with unit last stride")
     _check_cache(cache, rank, rot_dim, qa.dtype)
     _check_table(block_tables, bt_row, positions, T)
+    gate_stride = _check_end(sinks, gate, heads, T, qa.dtype)
     out = torch.empty_like(qa)
     ws = None
     if nparts > 1 and mfma_attend(rank, rot_dim, qa.dtype):
@@ -217,8 +277,8 @@ def latent_attend(qa, q_rot, cache, rank, rot_dim, block_tables, bt_row, positio
         nparts = 1
     _ffi.call("skyrl_latent_attend", _ptr(qa), _ptr(q_rot), q_rot.stride(0), q_rot.stride(1), _ptr(cache),
               cache.shape[2], _ptr(block_tables), block_tables.stride(0), _ptr(bt_row), _ptr(positions), T, heads,
-              rank, rot_dim, float(scale), int(window or 0), part_min, nparts, _ptr(out), _ptr(ws), _code(qa),
-              _stream(dev))
+              rank, rot_dim, float(scale), int(window or 0), part_min, nparts, _ptr(sinks), _ptr(gate), gate_stride,
+              _ptr(out), _ptr(ws), _code(qa), _stream(dev))
     return out
 
 
@@ -240,10 +300,12 @@ def latent_gather(cache, rank, rot_dim, block_tables, seg, nrows: int, max_count
     return latent, k_rot
 
 
-def latent_prefill(q, k_nope, k_rot, v_t, tiles, heads, dim, rot_dim, vdim, scale, window, out) -> torch.Tensor:
+def latent_prefill(q, k_nope, k_rot, v_t, tiles, heads, dim, rot_dim, vdim, scale, window, out, sinks=None,
+                   gate=None) -> torch.Tensor:
     """Windowed attention of prompt tiles over packed keys. q [T, >= heads * (dim + rot_dim)]; k_nope
-    [rows, heads * dim]; k_rot [rows, rot_dim]; v_t [heads * vdim, rows]; out [T, heads * vdim]."""
-    dev = _require_gpu(q, k_nope, k_rot, v_t, tiles, out)
+    [rows, heads * dim]; k_rot [rows, rot_dim]; v_t [heads * vdim, rows]; out [T, heads * vdim]; sinks and gate as in
+    latent_attend."""
+    dev = _require_gpu(q, k_nope, k_rot, v_t, tiles, out, sinks, gate)
     rows = k_nope.shape[0]
     for t, name in ((q, "q"), (k_nope, "k_nope"), (k_rot, "k_rot"), (v_t, "v_t"), (out, "out")):
         if t.dtype != torch.bfloat16 or t.dim() != 2 or t.stride(1) != 1:
@@ -255,9 +317,10 @@ def latent_prefill(q, k_nope, k_rot, v_t, tiles, heads, dim, rot_dim, vdim, scal
     if v_t.shape != (heads * vdim, rows) or rows % 64:
         raise ValueError("v_t must be [heads * vdim, rows] with rows a multiple of 64")
     _check(tiles, "tiles", torch.int32, (tiles.shape[0], 8))
+    gate_stride = _check_end(sinks, gate, heads, q.shape[0], q.dtype)
     _ffi.call("skyrl_latent_prefill", _ptr(q), q.stride(0), _ptr(k_nope), k_nope.stride(0), _ptr(k_rot), _ptr(v_t),
               v_t.stride(0), _ptr(tiles), tiles.shape[0], heads, dim, rot_dim, vdim, float(scale), int(window or 0),
-              _ptr(out), out.stride(0), _stream(dev))
+              _ptr(sinks), _ptr(gate), gate_stride, _ptr(out), out.stride(0), _stream(dev))
     return out
 
 
@@ -782,4 +845,134 @@ def gated_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: i
     _check(weight, "weight", weight.dtype, (W,))
     _ffi.call("skyrl_gated_norm", _ptr(y), y.stride(0), _ptr(z), z.stride(0), _ptr(weight), n, W, groups, float(eps),
               _ptr(out), out.stride(0), _code(weight), _stream(dev))
+    return out
+
+
+# ---------------------------------------------------------------- generalized delta rule
+def gdelta_shape(heads, dim, eps) -> _ffi.GeneralDeltaShape:
+    if not 0 < dim <= 256:
+        raise ValueError("the generalized delta rule takes a dim of at most 256")
+    return _ffi.GeneralDeltaShape(heads, dim, eps)
+
+
+def gdelta_vpad(sh) -> int:
+    return (sh.dim + 3) // 4 * 4
+
+
+def _check_gdelta(sh, proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, out):
+    T, n, HD = proj.shape[0], rows.shape[0], sh.heads * sh.dim
+    if proj.dim() != 2 or proj.shape[1] < 5 * HD or proj.stride(1) != 1:
+        raise ValueError(f"proj must be [T, >= {5 * HD}] with unit column stride")
+    _check_view(wl, "wl", proj.dtype, (T, HD))
+    _check(w0, "w0", torch.float32, (HD,))
+    _check(a_bias, "a_bias", torch.float32, (HD,))
+    _check(norm_w, "norm_w", proj.dtype, (HD,))
+    _check(rows, "rows", torch.int32, (n,))
+    _check(cu, "cu", torch.int32, (n + 1,))
+    _check(positions, "positions", torch.int64, (T,))
+    _check(state, "state", torch.float32, (state.shape[0], sh.heads, sh.dim, gdelta_vpad(sh)))
+    _check_view(out, "out", proj.dtype, (T, HD))
+    return n
+
+
+def gdelta_scan(sh, proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, out) -> torch.Tensor:
+    """Token by token over each sequence's tokens [cu[s], cu[s + 1]); state updated in place. proj [T, >= 5 heads dim]:
+    r | k | v | output gate | removal rate; wl [T, heads dim] the decay logits."""
+    dev = _require_gpu(proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, out)
+    n = rows.shape[0]
+    if cu.shape[0] != n + 1:
+        raise ValueError("cu must be [sequences + 1]")
+    _check_gdelta(sh, proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, out)
+    _ffi.call("skyrl_gdelta_scan", ctypes.byref(sh), _ptr(proj), proj.stride(0), _ptr(wl), wl.stride(0), _ptr(w0),
+              _ptr(a_bias), _ptr(norm_w), _ptr(cu), _ptr(rows), _ptr(positions), n, _ptr(state), _ptr(out), out.stride(0),
+              _code(proj), _stream(dev))
+    return out
+
+
+def gdelta_prompt(sh, proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, chunk, seq_chunks, first_seq: int,
+                  out) -> torch.Tensor:
+    """Chunked form over the sequences from first_seq on: chunk int32 [n, 4] and seq_chunks int32 [sequences + 1]
+    (mixers.chunk_plan). `state` is updated in place."""
+    dev = _require_gpu(proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, chunk, seq_chunks, out)
+    n = _check_gdelta(sh, proj, wl, w0, a_bias, norm_w, cu, rows, positions, state, out)
+    nc, nseq, HD = chunk.shape[0], n - first_seq, sh.heads * sh.dim
+    _check(chunk, "chunk", torch.int32, (nc, 4))
+    _check(seq_chunks, "seq_chunks", torch.int32, (nseq + 1,))
+    d16 = (sh.dim + 15) // 16 * 16
+    f32 = lambda *tail: torch.empty((nc, sh.heads) + tail, dtype=torch.float32, device=dev)  # noqa: E731
+    M, N, S, R, O = f32(d16, d16), f32(d16, d16), f32(d16, d16), f32(CHUNK, d16), f32(CHUNK, d16)
+    st, ref = _stream(dev), ctypes.byref(sh)
+    _ffi.call("skyrl_gdelta_chunk", ref, _ptr(proj), proj.stride(0), _ptr(wl), wl.stride(0), _ptr(w0), _ptr(a_bias),
+              _ptr(chunk), nc, _ptr(M), _ptr(N), _ptr(R), _ptr(O), _code(proj), st)
+    _ffi.call("skyrl_gdelta_chain", ref, _ptr(chunk), _ptr(seq_chunks), first_seq, nseq, _ptr(cu), _ptr(rows),
+              _ptr(positions), _ptr(M), _ptr(N), _ptr(state), _ptr(S), st)
+    gate = proj[:, 3 * HD:4 * HD]
+    _ffi.call("skyrl_gdelta_out", ref, _ptr(chunk), nc, _ptr(R), _ptr(O), _ptr(S), _ptr(gate), proj.stride(0), _ptr(norm_w),
+              _ptr(out), out.stride(0), _code(proj), st)
+    return out
+
+
+# ---------------------------------------------------------------- routed experts
+def moe_shape(width, ff, experts, top, groups=1, keep=1) -> _ffi.MoeShape:
+    if not 0 < experts <= 1024 or groups <= 0 or experts % groups:
+        raise ValueError("experts must be at most 1024 and a multiple of groups")
+    if not 0 < keep <= groups or not 0 < top <= experts // groups * keep:
+        raise ValueError("keep must be in [1, groups] and top at most the experts of the kept groups")
+    return _ffi.MoeShape(width, ff, experts, top, groups, keep)
+
+
+def moe_route(sh, x, router, correction):
+    """(experts int32 [n, top], their scores f32 [n, top]) of every row of x."""
+    dev = _require_gpu(x, router, correction)
+    n = x.shape[0]
+    _check(x, "x", x.dtype, (n, sh.width))
+    _check(router, "router", x.dtype, (sh.experts, sh.width))
+    _check(correction, "correction", torch.float32, (sh.experts,))
+    idx = torch.empty((n, sh.top), dtype=torch.int32, device=dev)
+    weight = torch.empty((n, sh.top), dtype=torch.float32, device=dev)
+    _ffi.call("skyrl_moe_route", ctypes.byref(sh), _ptr(x), n, _ptr(router), _ptr(correction), _ptr(idx), _ptr(weight),
+              _code(x), _stream(dev))
+    return idx, weight
+
+
+def moe_tile(sh, n: int) -> int:
+    """Rows per tile of the experts' products for n tokens."""
+    mean = n * sh.top / sh.experts
+    return 128 if mean >= 96 else 64 if mean >= 16 else 16
+
+
+def moe_sort(sh, idx, tm: int):
+    """(order int32 [tiles, tm], tile_expert int32 [tiles]): the (token, expert) pairs by expert."""
+    dev = _require_gpu(idx)
+    _check(idx, "idx", torch.int32, (idx.shape[0], sh.top))
+    pairs = idx.numel()
+    tiles = int(_ffi.query("skyrl_moe_tiles", sh.experts, pairs, tm))
+    order = torch.empty((tiles, tm), dtype=torch.int32, device=dev)
+    tile_expert = torch.empty((tiles,), dtype=torch.int32, device=dev)
+    _ffi.call("skyrl_moe_sort", _ptr(idx), pairs, sh.experts, tm, tiles, _ptr(order), _ptr(tile_expert), _stream(dev))
+    return order, tile_expert
+
+
+def moe_experts(sh, x, idx, weight, gate_up, down, tm: Optional[int] = None) -> torch.Tensor:
+    """Rows [n * top, width]: every pair's expert output times its weight. gate_up [experts, 2, ff, width], down
+    [experts, width, ff]."""
+    dev = _require_gpu(x, idx, weight, gate_up, down)
+    n = x.shape[0]
+    _check(x, "x", x.dtype, (n, sh.width))
+    _check(idx, "idx", torch.int32, (n, sh.top))
+    _check(weight, "weight", torch.float32, (n, sh.top))
+    _check(gate_up, "gate_up", x.dtype, (sh.experts, 2, sh.ff, sh.width))
+    _check(down, "down", x.dtype, (sh.experts, sh.width, sh.ff))
+    tm = tm or moe_tile(sh, n)
+    out = torch.empty((n * sh.top, sh.width), dtype=x.dtype, device=dev)
+    if n == 0:
+        return out
+    order, tile_expert = moe_sort(sh, idx, tm)
+    tiles = tile_expert.shape[0]
+    act = torch.empty((tiles * tm, sh.ff), dtype=x.dtype, device=dev)
+    ref, st = ctypes.byref(sh), _stream(dev)
+    _ffi.call("skyrl_moe_gate_up", ref, _ptr(x), _ptr(gate_up), _ptr(order), _ptr(tile_expert), tm, tiles, _ptr(act),
+              _code(x), st)
+    _ffi.call("skyrl_moe_down", ref, _ptr(act), _ptr(down), _ptr(order), _ptr(tile_expert), tm, tiles, _ptr(weight),
+              _ptr(out), _code(x), st)
     return out

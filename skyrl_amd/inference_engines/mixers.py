@@ -1,5 +1,6 @@
-"""Layer mechanisms of the hybrid decoders: latent attention, gated delta rule, differential
-attention, gated linear recurrence, windowed attention beside a state space mixer, gated and plain MLPs.
+"""Layer mechanisms of the hybrid decoders: latent attention, gated and generalized delta rules, differential
+attention, gated linear recurrence, windowed attention beside a state space mixer, gated and plain MLPs, routed
+experts.
 
 A mechanism owns its weights (fused where one product serves several tensors), names them for
 loading and saving, sizes and allocates its cache or state, and runs a step over it with the HIP
@@ -9,7 +10,8 @@ a config.json to these classes.
 
 A sublayer is `forward(x, inp, state, workspace)`. Most leave their input and output products to
 `Products`, which runs one sublayer, a mixer and a feed-forward that read the same input side by side in
-the same two products, or two mixers whose outputs are normed apart and joined (`SideBySide`).
+the same two products, or two mixers whose outputs are normed apart and joined (`SideBySide`). `Gated` puts the
+logits of a gate on the sublayer's result beside it.
 
 A step is a StepInputs (model.py): tokens of several sequences, each with its own first position. In
 a portion step the first `n_short` sequences (single decoded tokens and short portions) come first;
@@ -197,15 +199,20 @@ class Products:
     summed: the parts' input rows stacked and their output columns side by side, one product each. Parts
     start at multiples of 8 elements (16 bytes). A part has `in_rows`, `out_cols`, `in_bias`, `out_bias`,
     takes its views of the weights in `bind` and computes `inner(proj, out, ...)` between the products.
-    With `apart` every part has an output product and a state of its own, and the outputs are a tuple."""
+    With `apart` every part has an output product and a state of its own, and the outputs are a tuple. With
+    `beside` that many more input rows, `w_beside`, follow the parts', and forward returns (output, their product)."""
 
-    def __init__(self, parts: List[Any], width: int, w: Weights, apart: bool = False):
-        self.parts, self.ranges, self.apart = parts, [], apart
+    def __init__(self, parts: List[Any], width: int, w: Weights, apart: bool = False, beside: int = 0):
+        self.parts, self.ranges, self.apart, self.beside = parts, [], apart, None
         a = c = 0
         for p in parts:
             self.ranges.append((a, c))
             a, c = a + (p.in_rows + 7) // 8 * 8, c + (p.out_cols + 7) // 8 * 8
+        if beside:
+            self.beside, a = (a, a + beside), a + (beside + 7) // 8 * 8
         self.w_in = w.matrix(a, width)
+        if beside:
+            self.w_beside = self.w_in[self.beside[0]:self.beside[1]]
         self.b_in = w.zeros(a) if any(p.in_bias for p in parts) else None
         if apart:
             self.outs = [(w.matrix(width, p.out_cols), w.zeros(width) if p.out_bias else None) for p in parts]
@@ -238,50 +245,86 @@ class Products:
         cat = make((x.shape[0], self.w_out.shape[1]), dtype=x.dtype, device=x.device)
         for p, (a, c) in zip(self.parts, self.ranges):
             p.inner(proj[:, a:a + p.in_rows], cat[:, c:c + p.out_cols], inp, state, workspace)
-        return F.linear(cat, self.w_out, self.b_out)
+        y = F.linear(cat, self.w_out, self.b_out)
+        return y if self.beside is None else (y, proj[:, self.beside[0]:self.beside[1]])
+
+
+class Gated:
+    """A sublayer and the logits of an elementwise gate on its result, both from the same input: forward returns (rows
+    [n * rows_per_token, width] of which a token's are summed, logits [n, width]); the bias joins where the gate is
+    applied (layer_kernels.gate_norm_add)."""
+
+    def __init__(self, sub, width: int, w: Weights):
+        self.bias = w.zeros(width, dtype=torch.float32)
+        self.rows_per_token = getattr(sub, "rows_per_token", 1)
+        if hasattr(sub, "inner"):
+            self.sub = Products([sub], width, w, beside=width)
+            self.weight = self.sub.w_beside
+        else:
+            self.sub, self.weight = sub, w.matrix(width, width)
+
+    def forward(self, x: torch.Tensor, inp, state, workspace):
+        if isinstance(self.sub, Products):
+            return self.sub.forward(x, inp, state, workspace)
+        return self.sub.forward(x, inp, state, workspace), F.linear(x, self.weight)
 
 
 class LatentAttention:
     """Attention over low-rank latents shared by all heads, with a rotated key part beside them and
     an optional sliding window. Caches [blocks, 16, row]: per token the normed latent | the rotated key
-    part."""
+    part. Queries come from the input or, with `q_rank`, from a normed latent of it. A design may add a learned sink to
+    each head's softmax, a sigmoid gate to each head's output, and pair the rotated dimensions by halves instead of
+    neighbours. A layer with `kv_from` reads the cache of that layer, with up-projections of its own."""
 
     libraries = ("latent",)  # of _ffi.LAYER_LIBS, beside the common one
     paged = True
-    kv_from = None
+    in_bias = out_bias = False
+    shared_keys = ("kv_rank", "rot_dim", "rot")  # equal in a layer and the one whose cache it reads
 
     @staticmethod
     def prefix_cacheable(m: Dict[str, Any]) -> bool:
         """Whether a page's content depends on the tokens before it alone, with no state beside the pages."""
         return True
 
-    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights, sink: bool = False,
+                 gate: bool = False, halves: bool = False):
         self.heads, self.dim, self.rot_dim = int(m["heads"]), int(m["dim"]), int(m["rot_dim"])
         self.vdim, self.rank, self.scale = int(m["vdim"]), int(m["kv_rank"]), float(m["scale"])
+        self.q_rank = int(m["q_rank"]) if m.get("q_rank") else 0
+        self.kv_from = None if m.get("kv_from") is None else int(m["kv_from"])
         mask = m.get("mask")
         self.window = int(mask["size"]) if mask and mask.get("size") else None
         if int(m["rot"]["dims"]) != self.rot_dim:
             raise ValueError("latent attention rotates exactly its rot_dim part: rot.dims must equal rot_dim")
         if self.rot_dim % 2:
             raise ValueError("rot_dim must be even")
-        self.eps, self.width, self.dtype = eps, width, w.dtype
+        self.eps, self.dtype, self.halves = eps, w.dtype, halves
         self.cos_sin = w.rotary(m["rot"], max_pos)
         H, qd = self.heads, self.dim + self.rot_dim
-        self.wproj = w.matrix(H * qd + self.rank + self.rot_dim, width)
-        self.dkv_norm = w.ones(self.rank)
+        own = self.kv_from is None
+        self.q_rows = self.q_rank or H * qd
+        self.rows = (("dq" if self.q_rank else "q", self.q_rows),) + (
+            (("dkv", self.rank + self.rot_dim),) if own else ()) + ((("g", H),) if gate else ())
+        self.in_rows, self.out_cols = sum(n for _, n in self.rows), H * self.vdim
+        self.gate_at = self.in_rows - H if gate else None
+        self.dq_norm = w.ones(self.q_rank) if self.q_rank else None
+        self.wuq = w.matrix(H * qd, self.q_rank) if self.q_rank else None
+        self.dkv_norm = w.ones(self.rank) if own else None
         self.wuk = w.matrix(H * self.dim, self.rank)
         self.wuv = w.matrix(H * self.vdim, self.rank)
         self.wuv_t = w.zeros(H, self.rank, self.vdim)  # per head transposed: the decode form's right operand
-        self.wo = w.matrix(width, H * self.vdim)
+        self.sinks = w.zeros(H, dtype=torch.float32) if sink else None
         self.refresh()
 
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.w_in, self.wo = w_in, w_out
+
     def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
-        yield from split_rows(self.wproj, (("q", self.heads * (self.dim + self.rot_dim)),
-                                           ("dkv", self.rank + self.rot_dim)))
-        yield "dkv.norm", self.dkv_norm
-        yield "uk", self.wuk
-        yield "uv", self.wuv
-        yield "o", self.wo
+        yield from split_rows(self.w_in, self.rows)
+        for name, t in (("dq.norm", self.dq_norm), ("uq", self.wuq), ("dkv.norm", self.dkv_norm), ("uk", self.wuk),
+                        ("uv", self.wuv), ("sink", self.sinks), ("o", self.wo)):
+            if t is not None:
+                yield name, t
 
     def refresh(self) -> None:
         """Recompute derived tensors, in place, after the weights changed."""
@@ -289,12 +332,17 @@ class LatentAttention:
 
     # ---- cache
     def block_bytes(self) -> int:
+        if self.kv_from is not None:
+            return 0
         return BLOCK_SIZE * lk.latent_row(self.rank, self.rot_dim) * self.dtype.itemsize
 
     def row_bytes(self) -> int:
         return 0
 
-    def make_state(self, num_blocks: int, num_rows: int, device) -> torch.Tensor:
+    def make_state(self, num_blocks: int, num_rows: int, device, source=None) -> torch.Tensor:
+        """source: the state of the layer whose latents this one reads."""
+        if source is not None:
+            return source
         return torch.zeros((num_blocks, BLOCK_SIZE, lk.latent_row(self.rank, self.rot_dim)), dtype=self.dtype,
                            device=device)
 
@@ -314,7 +362,7 @@ class LatentAttention:
         return int(_ffi.query("skyrl_latent_attend_workspace_bytes", tokens, self.heads, self.rank, n)) if n > 1 else 0
 
     # ---- step
-    def _attend_rows(self, q, out, inp, a: int, b: int, cache, workspace):
+    def _attend_rows(self, q, gate, out, inp, a: int, b: int, cache, workspace):
         """Tokens [a, b) in the decode form."""
         H, D, R = self.heads, self.dim, self.rank
         n = b - a
@@ -322,29 +370,32 @@ class LatentAttention:
         qa = torch.bmm(q3[:, :, :D].transpose(0, 1), self.wuk.view(H, D, R))
         o = lk.latent_attend(qa, q3[:, :, D:], cache, R, self.rot_dim, inp.block_tables, inp.bt_row[a:b],
                              inp.positions[a:b], self.scale, self.window, nparts=self.nparts(n, inp.max_ctx),
-                             part_min=kernels.MIN_PARTITION, workspace=workspace)
+                             part_min=kernels.MIN_PARTITION, workspace=workspace, sinks=self.sinks,
+                             gate=None if gate is None else gate[a:b])
         out[a:b].view(n, H, self.vdim).copy_(torch.bmm(o, self.wuv_t).transpose(0, 1))
 
-    def forward(self, x: torch.Tensor, inp, cache: torch.Tensor, workspace) -> torch.Tensor:
-        H, T = self.heads, x.shape[0]
-        proj = F.linear(x, self.wproj)
-        lk.latent_write(proj, H, self.dim, self.rot_dim, self.rank, self.dkv_norm, self.eps, inp.positions, inp.slots,
-                        self.cos_sin, cache)
-        qw = H * (self.dim + self.rot_dim)
-        out = torch.empty((T, H * self.vdim), dtype=self.dtype, device=x.device)
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, cache: torch.Tensor, workspace) -> None:
+        H, T, qr = self.heads, proj.shape[0], self.q_rank
+        where = (self.rot_dim, inp.positions, inp.slots, self.cos_sin, cache, self.eps)
+        own = {} if self.kv_from is not None else {"rank": self.rank, "norm_weight": self.dkv_norm}
+        first = {"q_norm": self.dq_norm} if qr else {"heads": H, "dim": self.dim}
+        lk.latent_write(proj, *where, halves=self.halves, **first, **own)
+        q = proj[:, :self.q_rows]
+        if qr:
+            q = F.linear(q, self.wuq)
+            lk.latent_write(q, *where, heads=H, dim=self.dim, halves=self.halves)
+        gate = None if self.gate_at is None else proj[:, self.gate_at:]
         prompt = inp.plan is not None and self.window in inp.plan and lk.prefill_fits(self.dim, self.rot_dim, self.vdim, self.dtype)
         ts = inp.short_tokens if prompt else T
-        q = proj[:, :qw]
         for a in range(0, ts, 32768):  # the decode form's grid limit
-            self._attend_rows(q, out, inp, a, min(ts, a + 32768), cache, workspace)
+            self._attend_rows(q, gate, out, inp, a, min(ts, a + 32768), cache, workspace)
         if ts < T:
             seg, tiles, rows, longest = inp.plan[self.window]
             latent, k_rot = lk.latent_gather(cache, self.rank, self.rot_dim, inp.block_tables, seg, rows, longest)
             k = F.linear(latent, self.wuk)
             v_t = torch.mm(self.wuv, latent.t())
             lk.latent_prefill(q, k, k_rot, v_t, tiles, H, self.dim, self.rot_dim, self.vdim, self.scale, self.window,
-                              out)
-        return F.linear(out, self.wo)
+                              out, sinks=self.sinks, gate=gate)
 
 
 class GatedDelta:
@@ -426,6 +477,78 @@ class GatedDelta:
         return F.linear(out, self.wo)
 
 
+class GeneralDelta:
+    """Generalized delta rule: a decay per head and key channel from a low-rank projection, a removal along the unit key
+    at a rate of its own, output norm per head and elementwise gate. State per row (a running request): the f32 matrix
+    of every head."""
+
+    libraries = ("gdelta",)
+    paged = False
+    kv_from = None
+    in_bias = out_bias = False
+
+    @staticmethod
+    def prefix_cacheable(m: Dict[str, Any]) -> bool:
+        return False
+
+    @staticmethod
+    def complete(m: Dict[str, Any], shape_of) -> Dict[str, Any]:
+        """The mixer's entry with the size that only a checkpoint's tensors give; shape_of: a tensor's shape by name."""
+        return m if "decay_rank" in m or shape_of("w1") is None else dict(m, decay_rank=int(shape_of("w1")[0]))
+
+    def __init__(self, m: Dict[str, Any], width: int, eps: float, max_pos: int, w: Weights):
+        self.heads, self.dim = int(m["heads"]), int(m["dim"])
+        if not m.get("decay_rank"):
+            raise ValueError("the generalized delta rule needs decay_rank, from its entry or from a checkpoint's w1")
+        self.rank = int(m["decay_rank"])
+        self.shape = lk.gdelta_shape(self.heads, self.dim, eps)
+        self.dtype = w.dtype
+        HD = self.out_cols = self.heads * self.dim
+        self.rows = tuple((n, HD) for n in "rkvga") + (("w1", self.rank),)
+        self.in_rows = 5 * HD + self.rank
+        self.w2 = w.matrix(HD, self.rank)
+        self.w0, self.a_bias = w.zeros(HD, dtype=torch.float32), w.zeros(HD, dtype=torch.float32)
+        self.norm = w.ones(HD)
+
+    def bind(self, w_in, b_in, w_out, b_out) -> None:
+        self.w_in, self.wo = w_in, w_out
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        yield from split_rows(self.w_in, self.rows)
+        yield from (("w2", self.w2), ("w0", self.w0), ("a.b", self.a_bias), ("norm", self.norm), ("o", self.wo))
+
+    def refresh(self) -> None:
+        pass
+
+    # ---- state
+    def block_bytes(self) -> int:
+        return 0
+
+    def row_bytes(self) -> int:
+        return 4 * self.heads * self.dim * lk.gdelta_vpad(self.shape)
+
+    def make_state(self, num_blocks: int, num_rows: int, device) -> torch.Tensor:
+        return torch.zeros((num_rows, self.heads, self.dim, lk.gdelta_vpad(self.shape)), dtype=torch.float32, device=device)
+
+    def workspace_bytes(self, tokens: int, max_ctx: int) -> int:
+        return 0
+
+    def host_plans(self, seq_lens, starts, first_seq, first_token):
+        yield "chunks", lambda: chunk_plan(seq_lens, first_seq, first_token)
+
+    # ---- step
+    def inner(self, proj: torch.Tensor, out: torch.Tensor, inp, state: torch.Tensor, workspace) -> None:
+        wl = F.linear(lk.tanh(proj[:, 5 * self.out_cols:]), self.w2)
+        args = (proj, wl, self.w0, self.a_bias, self.norm)
+        n = inp.rows.shape[0]
+        prompt = inp.plan is not None and "chunks" in inp.plan
+        k = inp.n_short if prompt else n
+        if k:
+            lk.gdelta_scan(self.shape, *args, inp.cu[:k + 1], inp.rows[:k], inp.positions, state, out)
+        if k < n:
+            lk.gdelta_prompt(self.shape, *args, inp.cu, inp.rows, inp.positions, state, *inp.plan["chunks"], k, out)
+
+
 class DifferentialAttention:
     """Full causal attention in two softmax maps per head over the same values, their weighted difference
     normed per head and gated; short causal convolutions and partial interleaved rotation on its
@@ -435,6 +558,7 @@ class DifferentialAttention:
 
     libraries = ("diff",)
     paged = True
+    shared_keys = ("kv_heads", "dim", "vdim")
     in_bias, out_bias = True, False
 
     @staticmethod
@@ -892,7 +1016,36 @@ class PlainMLP:
         lk.xielu(proj, self.act, out=out)
 
 
-MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "attention": DifferentialAttention,
-          "rglru": GatedLinearRecurrence, "parallel": SideBySide}
+class RoutedExperts:
+    """Of many small silu-gated feed-forwards each token runs `top`, weighted by the sigmoid of their router logits;
+    they are chosen by those scores plus a learned correction, out of the best groups of neighbours. forward returns a
+    token's `top` weighted rows one after another, to be summed."""
+
+    libraries = ("moe",)
+    in_bias = out_bias = False
+
+    def __init__(self, m: Dict[str, Any], width: int, w: Weights):
+        ro = m["router"]
+        groups = ro.get("groups") or {"count": 1, "keep": 1}
+        self.ff, self.experts, self.rows_per_token = int(m["expert"]["ff"]), int(ro["experts"]), int(ro["top"])
+        self.shape = lk.moe_shape(width, self.ff, self.experts, self.rows_per_token, int(groups["count"]), int(groups["keep"]))
+        self.router = w.matrix(self.experts, width)
+        self.correction = w.zeros(self.experts, dtype=torch.float32)
+        self.gate_up = w.matrix(self.experts, 2, self.ff, width)
+        self.down = w.matrix(self.experts, width, self.ff)
+
+    def params(self) -> Iterator[Tuple[str, torch.Tensor]]:
+        for e in range(self.experts):
+            yield from ((f"e{e}.gate", self.gate_up[e, 0]), (f"e{e}.up", self.gate_up[e, 1]), (f"e{e}.down", self.down[e]))
+        yield from (("router", self.router), ("correction", self.correction))
+
+    def forward(self, x: torch.Tensor, inp, state, workspace) -> torch.Tensor:
+        idx, weight = lk.moe_route(self.shape, x, self.router, self.correction)
+        return lk.moe_experts(self.shape, x, idx, weight, self.gate_up, self.down)
+
+
+MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "general_delta": GeneralDelta,
+          "attention": DifferentialAttention, "rglru": GatedLinearRecurrence, "parallel": SideBySide}
 FEEDFORWARDS = {"dense": GatedMLP}
 PLAIN_FEEDFORWARDS = {"dense": PlainMLP}
+EXPERT_FEEDFORWARDS = {"moe": RoutedExperts}

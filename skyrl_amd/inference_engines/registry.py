@@ -30,7 +30,7 @@ def _hf_paged(config: Dict[str, Any], folder: str, device, dtype, max_model_len,
                         max_model_len=max_model_len)
 
 
-ARCHITECTURES: Dict[str, Callable] = {"Dovidra": _hybrid, "Lipedra": _hybrid, "Foduzen": _hybrid}
+ARCHITECTURES: Dict[str, Callable] = {"Dovidra": _hybrid, "Lipedra": _hybrid, "Foduzen": _hybrid, "Tativik": _hybrid}
 HF_MODEL_TYPES: Dict[str, Callable] = {t: _hf_paged for t in ("qwen2", "llama", "mistral", "qwen3")}
 
 
@@ -60,12 +60,16 @@ def kernel_libraries(config: Dict[str, Any]) -> Tuple[str, ...]:
     """The layer libraries (_ffi.LAYER_LIBS) that serving the checkpoint needs; none for the paged HF decoders."""
     if decoder_factory(config) is not _hybrid:
         return ()
+    from .hybrid import DESIGNS
     from .mixers import MIXERS
 
     unknown = sorted({e["type"] for e in config["layers"]} - set(MIXERS))
     if unknown:
         raise ValueError(f"unknown layer types {unknown} (known: {sorted(MIXERS)})")
-    return ("layers",) + tuple(sorted({lib for e in config["layers"] for lib in MIXERS[e["type"]].libraries}))
+    ffs = DESIGNS[config["architecture"]].feedforwards
+    kinds = [MIXERS[e["type"]] for e in config["layers"]] + [ffs[e["mlp"]["kind"]] for e in config["layers"]
+                                                             if e.get("mlp") and e["mlp"]["kind"] in ffs]
+    return ("layers",) + tuple(sorted({lib for k in kinds for lib in getattr(k, "libraries", ())}))
 
 
 def checkpoint_tensors(folder: str) -> Iterator[Tuple[str, torch.Tensor]]:
@@ -80,9 +84,35 @@ def checkpoint_tensors(folder: str) -> Iterator[Tuple[str, torch.Tensor]]:
                 yield name, f.get_tensor(name)
 
 
+def checkpoint_shapes(folder: str) -> Dict[str, Tuple[int, ...]]:
+    """Every tensor's shape, from the files' headers."""
+    from safetensors import safe_open
+
+    out: Dict[str, Tuple[int, ...]] = {}
+    for path in sorted(glob.glob(os.path.join(folder, "*.safetensors"))):
+        with safe_open(path, framework="pt", device="cpu") as f:
+            out.update((name, tuple(f.get_slice(name).get_shape())) for name in f.keys())
+    return out
+
+
+def complete_config(config: Dict[str, Any], folder: str) -> Dict[str, Any]:
+    """The config with the sizes that its mechanisms take from the checkpoint's tensors."""
+    if decoder_factory(config) is not _hybrid:
+        return config
+    from .mixers import MIXERS
+
+    shapes, layers = None, list(config["layers"])
+    for i, e in enumerate(layers):
+        complete = getattr(MIXERS.get(e["type"]), "complete", None)
+        if complete is not None:
+            shapes = checkpoint_shapes(folder) if shapes is None else shapes
+            layers[i] = dict(e, mixer=complete(e["mixer"], lambda name: shapes.get(f"l{i}.mix.{name}")))
+    return dict(config, layers=layers)
+
+
 def load_decoder(folder: str, device, dtype: torch.dtype = torch.bfloat16, max_model_len: Optional[int] = None):
     """The checkpoint's decoder with its weights loaded; a checkpoint that lacks a parameter is an error."""
-    config = read_config(folder)
+    config = complete_config(read_config(folder), folder)
     model = build_decoder(config, device, dtype, max_model_len, seed=None, folder=folder)
     seen = set()
 

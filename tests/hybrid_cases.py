@@ -280,3 +280,116 @@ def make_normed_weights(cfg, seed=0):
     number("final.norm")
     mat("head", cfg["vocab"], W, 3.0)
     return {k: v.to(torch.bfloat16) for k, v in w.items()}
+
+
+# ---------------------------------------------------------------- sublayers between two norms, routed experts
+def low_rank(heads=3, dim=20, rot_dim=12, vdim=28, kv_rank=40, q_rank=30, window=37, scale=None, base=5000.0, kv_from=None):
+    e = latent(heads, dim, rot_dim, vdim, kv_rank, window, scale, base, scaling=False)
+    e["mixer"]["q_rank"] = q_rank
+    if kv_from is not None:
+        e["mixer"]["kv_from"] = kv_from
+    return e
+
+
+def general(heads=3, dim=20, decay_rank=6):
+    return {"type": "general_delta", "mixer": {"heads": heads, "dim": dim, "decay_rank": decay_rank}}
+
+
+def routed(ff=28, experts=10, top=3, groups=None):
+    ro = {"experts": experts, "top": top}
+    if groups:
+        ro["groups"] = dict(zip(("count", "keep"), groups))
+    return {"kind": "moe", "expert": {"ff": ff}, "router": ro}
+
+
+def sandwich_config(layers, mlps, width=72, vocab=193, groups=3, eps=2e-5, mult=0.7):
+    layers = [dict(e, mlp=f) for e, f in zip(layers, mlps)]
+    return {"architecture": "Tativik", "layers": layers, "norm": {"eps": eps, "groups": groups}, "residual_mult": mult,
+            "vocab": vocab, "width": width}
+
+
+SANDWICH = {
+    # sizes no vector width divides; a layer on another's latents with its own heads, sizes, window and scale; one layer
+    # without a feed-forward; groups of two experts, of one, none
+    "odd": sandwich_config([low_rank(heads=3, dim=10, rot_dim=6, vdim=7, kv_rank=19, q_rank=13, window=21), general(heads=3, dim=18, decay_rank=5),
+                            low_rank(heads=5, dim=17, rot_dim=6, vdim=9, kv_rank=19, q_rank=11, window=None, kv_from=0), general(heads=2, dim=21)],
+                           [routed(ff=19, experts=6, top=2, groups=(3, 2)), None, routed(ff=22, experts=7, top=1),
+                            routed(ff=9, experts=5, top=3, groups=(5, 4))], width=70, groups=5, mult=0.4),
+    # shapes the matrix kernels take, one group, one kept group, the head gates and sinks of 16 heads
+    "wide": sandwich_config([general(heads=2, dim=64, decay_rank=16),
+                             low_rank(heads=16, dim=32, rot_dim=32, vdim=64, kv_rank=96, q_rank=64, window=50),
+                             low_rank(heads=8, dim=64, rot_dim=32, vdim=32, kv_rank=96, q_rank=40, window=50, kv_from=1)],
+                            [routed(ff=64, experts=32, top=4, groups=(8, 3)), routed(ff=48, experts=16, top=2, groups=(4, 1)),
+                             routed(ff=64, experts=16, top=8)], width=128, groups=1, mult=1.0),
+    # more than one slab of channels, a state of many columns, one token's window, shared latents twice over
+    "padded": sandwich_config([low_rank(heads=20, dim=24, rot_dim=8, vdim=40, kv_rank=136, q_rank=24, window=3), general(heads=2, dim=72),
+                               low_rank(heads=2, dim=130, rot_dim=8, vdim=24, kv_rank=136, q_rank=50, window=64, kv_from=0),
+                               general(heads=1, dim=136, decay_rank=40),
+                               low_rank(heads=4, dim=8, rot_dim=8, vdim=16, kv_rank=136, q_rank=88, window=1, kv_from=0)],
+                              [routed(ff=40, experts=12, top=4, groups=(2, 1)), routed(ff=24, experts=9, top=9), None, None, routed()],
+                              width=88, groups=2, mult=0.35),
+}
+
+
+def make_sandwich_weights(cfg, seed=0, steady=True):
+    """bf16 tensors by checkpoint name: decays from short to long memory, sinks and gates far from trivial. `steady`:
+    the corrections alone decide which experts run, so that rounding does not change the choice."""
+    g = torch.Generator().manual_seed(seed)
+    W, w = cfg["width"], {}
+
+    def rand(name, *shape, gain=1.0, mean=0.0):
+        w[name] = mean + torch.randn(*shape, generator=g) * gain
+
+    def mat(name, rows, cols, gain=1.0):
+        rand(name, rows, cols, gain=gain / math.sqrt(cols))
+
+    rand("embed", cfg["vocab"], W)
+    for n in ("embed.norm", "final.norm"):
+        rand(n, W, gain=0.3, mean=1.0)
+    for i, e in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        q = p + "mix."
+        H = m["heads"]
+        if e["type"] == "general_delta":
+            HD = H * m["dim"]
+            for n in "rkvga":
+                mat(q + n, HD, W, 1.2)
+            mat(q + "w1", m["decay_rank"], W, 1.2)
+            mat(q + "w2", HD, m["decay_rank"], 1.5)
+            rand(q + "w0", HD, gain=2.5, mean=-3.5)
+            rand(q + "a.b", HD, gain=1.5)
+            rand(q + "norm", HD, gain=0.3, mean=1.0)
+            mat(q + "o", W, HD, 1.5)
+        else:
+            C, R = m["kv_rank"], m["rot_dim"]
+            mat(q + "dq", m["q_rank"], W)
+            rand(q + "dq.norm", m["q_rank"], gain=0.3, mean=1.0)
+            mat(q + "uq", H * (m["dim"] + R), m["q_rank"], 1.6)
+            if m.get("kv_from") is None:
+                mat(q + "dkv", C + R, W, 1.5)
+                rand(q + "dkv.norm", C, gain=0.3, mean=1.0)
+            mat(q + "uk", H * m["dim"], C)
+            mat(q + "uv", H * m["vdim"], C)
+            rand(q + "sink", H, gain=1.5, mean=0.5)
+            mat(q + "g", H, W, 1.5)
+            mat(q + "o", W, H * m["vdim"], 1.5)
+        subs = [1]
+        if e.get("mlp"):
+            subs.append(2)
+            ro, ff, f = e["mlp"]["router"], e["mlp"]["expert"]["ff"], p + "mlp."
+            for k in range(ro["experts"]):
+                mat(f"{f}e{k}.gate", ff, W, 1.5)
+                mat(f"{f}e{k}.up", ff, W, 1.5)
+                mat(f"{f}e{k}.down", W, ff)
+            mat(f + "router", ro["experts"], W, 0.3 if steady else 1.5)
+            if steady:  # scores stay within 0.5 +- 0.25
+                w[f + "correction"] = torch.randperm(ro["experts"], generator=g) * 1.0 - 0.7 * ro["experts"]
+            else:
+                rand(f + "correction", ro["experts"], gain=0.3, mean=-0.8)
+        for k in subs:
+            rand(f"{p}norm{k}", W, gain=0.3, mean=1.0)
+            rand(f"{p}norm{k}b", W, gain=0.3, mean=1.0)
+            mat(f"{p}rg{k}", W, W, 1.5)
+            rand(f"{p}rg{k}.b", W, gain=0.8)
+    mat("head", cfg["vocab"], W, 3.0)
+    return {k: v.to(torch.bfloat16) for k, v in w.items()}

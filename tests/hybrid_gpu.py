@@ -4,7 +4,7 @@ import asyncio
 
 import torch
 
-from hybrid_cases import make_normed_weights, make_parallel_weights, make_weights
+from hybrid_cases import make_normed_weights, make_parallel_weights, make_sandwich_weights, make_weights
 from oracle import hybrid_ref as ref
 from skyrl_amd.inference_engines.engine import AMDInferenceEngine
 from skyrl_amd.inference_engines.hybrid import HybridDecoder
@@ -14,7 +14,8 @@ DTYPES = [torch.float32, torch.bfloat16]
 
 
 def weights_of(cfg, seed=0):
-    return {"Lipedra": make_parallel_weights, "Foduzen": make_normed_weights, "Dovidra": make_weights}[cfg["architecture"]](cfg, seed)
+    return {"Lipedra": make_parallel_weights, "Foduzen": make_normed_weights, "Dovidra": make_weights,
+            "Tativik": make_sandwich_weights}[cfg["architecture"]](cfg, seed)
 
 
 def rms(x):
@@ -36,8 +37,8 @@ def rnd(g, *shape, dtype=torch.float32, scale=1.0):
 LIMIT = {torch.float32: 2e-5, torch.bfloat16: 4e-2}
 
 
-def build(cfg, dtype, seed=0, max_len=512):
-    w = weights_of(cfg, seed)
+def build(cfg, dtype, seed=0, max_len=512, w=None):
+    w = weights_of(cfg, seed) if w is None else w
     m = HybridDecoder(cfg, DEV, dtype=dtype, seed=None, max_model_len=max_len)
     assert m.load_weights(w.items()) == len(w)
     return m, {k: v.double() for k, v in w.items()}

@@ -89,14 +89,18 @@ def test_layers_entries_validate_on_host():
             ("skyrl_gate_mul", (p, 15, 1, 8, 2, 1.0, 0.0, p, 8, _ffi.F32, None), "sizes"),
             ("skyrl_embed", (p, p, 1, 0, 1.0, None, None, p, None, _ffi.F32, None), "sizes"),
             ("skyrl_conv_save", (p, 7, 8, 3, p, p, p, 1, p, _ffi.F32, None), "sizes"),
-            ("skyrl_latent_write", (p, 10, 1, 1, 4, 4, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "proj_stride"),
-            ("skyrl_latent_write", (p, 100, 1, 1, 4, 4, 40, p, 1e-5, p, p, p, p, 40, _ffi.F32, None), "multiple of 32"),
-            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 8, 1, p, p, _ffi.BF16, None),
+            ("skyrl_latent_write", (p, 10, 1, 1, 4, 4, 0, 0, None, 8, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "proj_stride"),
+            ("skyrl_latent_write", (p, 100, 1, 1, 4, 4, 0, 0, None, 40, 8, p, 1e-5, p, p, p, p, 40, _ffi.F32, None), "multiple of 32"),
+            ("skyrl_latent_write", (p, 100, 1, 1, 4, 4, 1, 8, p, 8, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "not both"),
+            ("skyrl_latent_write", (p, 100, 1, 0, 0, 4, 1, 8, None, 8, 8, p, 1e-5, p, p, p, p, 32, _ffi.F32, None), "null"),
+            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 8, 1, None, None, 0, p, p, _ffi.BF16, None),
              "part_min"),
-            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 64, 2, p, None, _ffi.BF16, None),
+            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 1, 32, 16, 1.0, 0, 64, 2, None, None, 0, p, None, _ffi.BF16, None),
              "workspace"),
-            ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 65, p, 1, 1, 16, 16, 16, 1.0, 0, p, 16, None), "vt_stride"),
-            ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 64, p, 1, 1, 250, 16, 16, 1.0, 0, p, 16, None), "256"),
+            ("skyrl_latent_attend", (p, p, 8, 8, p, 64, p, 4, p, p, 1, 2, 32, 16, 1.0, 0, 64, 1, None, p, 1, p, None, _ffi.BF16, None),
+             "gate_stride"),
+            ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 65, p, 1, 1, 16, 16, 16, 1.0, 0, None, None, 0, p, 16, None), "vt_stride"),
+            ("skyrl_latent_prefill", (p, 8, p, 8, p, p, 64, p, 1, 1, 250, 16, 16, 1.0, 0, None, None, 0, p, 16, None), "256"),
             ("skyrl_delta_scan", (ctypes.byref(sh), p, 100, p, p, p, p, p, p, p, 1, p, p, 1, p, 24, _ffi.F32, None),
              "multiple of kv_heads"),
             ("skyrl_diff_write", (diff(3, 2, 8, 8, 4, 3, 1), p, 100, p, *rows, p, 0, 0, 1, p, p, p, _ffi.F32, None),
@@ -113,6 +117,33 @@ def test_layers_entries_validate_on_host():
             ("skyrl_diff_prefill", (good, p, p, 3, p, p, p, 8, p, 1, p, p, 32, None), "sizes")):
         with pytest.raises(_ffi.SkyrlHipError, match=msg):
             _ffi.call(name, *args)
+
+
+def test_routed_entries_validate_on_host():
+    p = ctypes.c_void_p(16)
+    gd = lambda *a: ctypes.byref(_ffi.GeneralDeltaShape(*a, 1e-5))  # noqa: E731
+    moe = lambda *a: ctypes.byref(_ffi.MoeShape(*a))  # noqa: E731
+    ok = moe(64, 32, 8, 2, 2, 1)
+    for name, args, msg in (
+            ("skyrl_gate_norm_add", (p, None, 1, None, 0, None, p, 1, 1e-5, 1.0, p, 0, p, 1, 9000, p, _ffi.BF16, None), "H must be"),
+            ("skyrl_gate_norm_add", (p, None, 1, None, 0, None, p, 3, 1e-5, 1.0, p, 0, p, 1, 64, p, _ffi.BF16, None), "multiple of groups"),
+            ("skyrl_gate_norm_add", (p, None, 1, p, 64, None, p, 4, 1e-5, 1.0, p, 0, p, 1, 64, p, _ffi.BF16, None), "bias"),
+            ("skyrl_tanh", (p, 7, 1, 8, p, _ffi.F32, None), "sizes"),
+            ("skyrl_gdelta_scan", (gd(2, 300), p, 9999, p, 9999, p, p, p, p, p, p, 1, p, p, 9999, _ffi.BF16, None), "256"),
+            ("skyrl_gdelta_scan", (gd(2, 8), p, 79, p, 16, p, p, p, p, p, p, 1, p, p, 16, _ffi.BF16, None), "strides"),
+            ("skyrl_gdelta_chunk", (gd(2, 8), p, 80, p, 15, p, p, p, 1, p, p, p, p, _ffi.F32, None), "strides"),
+            ("skyrl_gdelta_chain", (gd(2, 8), p, p, -1, 1, p, p, p, p, p, p, p, None), "sizes"),
+            ("skyrl_gdelta_out", (gd(2, 8), p, 1, p, p, p, p, 15, p, p, 16, _ffi.F32, None), "sizes"),
+            ("skyrl_moe_route", (moe(64, 32, 8, 2, 3, 1), p, 1, p, p, p, p, _ffi.F32, None), "multiple of groups"),
+            ("skyrl_moe_route", (moe(64, 32, 8, 5, 2, 1), p, 1, p, p, p, p, _ffi.F32, None), "top must be"),
+            ("skyrl_moe_route", (moe(64, 32, 2048, 2, 1, 1), p, 1, p, p, p, p, _ffi.F32, None), "1024"),
+            ("skyrl_moe_sort", (p, 20, 8, 16, 8, p, p, None), "too few tiles"),
+            ("skyrl_moe_sort", (p, 20, 8, 20, 99, p, p, None), "sizes"),
+            ("skyrl_moe_gate_up", (ok, p, p, p, p, 24, 4, p, _ffi.F32, None), "plain form"),
+            ("skyrl_moe_down", (ok, p, p, p, p, 16, 4, None, p, _ffi.F32, None), "null pointer")):
+        with pytest.raises(_ffi.SkyrlHipError, match=msg):
+            _ffi.call(name, *args)
+    assert [_ffi.query("skyrl_moe_tiles", *a) for a in ((8, 20, 16), (8, 3, 16), (8, 0, 16), (4, 1000, 128))] == [9, 3, 0, 11]
 
 
 def test_abi_version_and_error_path():

@@ -121,8 +121,8 @@ def test_latent_write(heads, dim, rot, rank, dtype):
     slots = torch.tensor([3, 40, 17, -1, 16, 15, 0, 63, 31])
     cache = torch.full((4, BS, lk.latent_row(rank, rot)), 7.0).to(dtype).to(DEV)
     pd = proj.to(DEV)
-    lk.latent_write(pd, heads, dim, rot, rank, w.to(DEV), 1e-4, pos.to(DEV), slots.to(DEV),
-                    mixers.rotary_table(r, 100).to(DEV), cache)
+    lk.latent_write(pd, rot, pos.to(DEV), slots.to(DEV), mixers.rotary_table(r, 100).to(DEV), cache, 1e-4, heads=heads,
+                    dim=dim, rank=rank, norm_weight=w.to(DEV))
     p = proj.double()
     q = p[:, :heads * (dim + rot)].view(T, heads, dim + rot)
     q = torch.cat([q[..., :dim], ref.rotate_pairs(q[..., dim:], pos, r)], -1)

@@ -7,8 +7,9 @@ import numpy as np
 import pytest
 import torch
 
-from hybrid_cases import (CONFIGS, NORMED, PARALLEL, attend, config, delta, diff_attention, latent, make_normed_weights,
-                          make_parallel_weights, make_weights, normed_config, parallel_config, rglru, side, ssd)
+from hybrid_cases import (CONFIGS, NORMED, PARALLEL, SANDWICH, attend, config, delta, diff_attention, general, latent, low_rank,
+                          make_normed_weights, make_parallel_weights, make_sandwich_weights, make_weights, normed_config,
+                          parallel_config, rglru, routed, sandwich_config, side, ssd)
 from oracle import hybrid_ref as ref
 from skyrl_amd.inference_engines import mixers
 from skyrl_amd.inference_engines.engine import BLOCK_SIZE, EngineCore, ModelRunner, RequestParams
@@ -329,7 +330,7 @@ def test_parallel_sizes_outside_the_design_are_refused():
     with pytest.raises(ValueError, match="kv_from"):  # not an owner
         build(good, diff_attention(kv_from=0), diff_attention(kv_from=1))
     with pytest.raises(ValueError, match="parallel"):
-        build(latent())
+        build(delta())
 
 
 def test_tile_and_run_plans_cover_every_token():
@@ -421,6 +422,118 @@ def test_kernel_libraries_of_a_checkpoint():
     assert kernel_libraries({"model_type": "qwen2"}) == ()
     with pytest.raises(ValueError, match="unknown layer"):
         kernel_libraries(normed_config([{"type": "none", "mixer": {}}]))
+
+
+@pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float32])
+@pytest.mark.parametrize("name", sorted(SANDWICH))
+def test_sandwich_weight_names_round_trip(name, dtype):
+    cfg = SANDWICH[name]
+    m = HybridDecoder(cfg, "cpu", dtype=dtype, seed=None, max_model_len=64)
+    w = make_sandwich_weights(cfg, 2)
+    assert m.load_weights(w.items()) == len(w)
+    ours = dict(m.hf_named_tensors())
+    assert sorted(ours) == sorted(w) and m.num_params() == sum(t.numel() for t in w.values())
+    for k in w:
+        assert ours[k].shape == w[k].shape and torch.equal(ours[k].float(), w[k].float()), k
+    for i, L in enumerate(m.layers):
+        p, x = f"l{i}.", L["mixer"]
+        if isinstance(x, mixers.LatentAttention):  # derived tensors follow the weights
+            uv = w[p + "mix.uv"].float().view(x.heads, x.vdim, x.rank)
+            assert torch.equal(x.wuv_t.float(), uv.transpose(1, 2)) and x.halves and x.sinks.dtype == torch.float32
+        sub = L["subs"][0][1].sub  # the result gate's rows follow the mixer's in one product
+        a, b = sub.beside
+        assert a % 8 == 0 and torch.equal(sub.w_in[a:b].float(), w[p + "rg1"].float())
+    with pytest.raises(KeyError):
+        m.load_weights([("l0.mix.none", w["final.norm"])])
+    with pytest.raises(ValueError):
+        m.load_weights([("final.norm", torch.ones(cfg["width"] + 1))])
+
+
+def test_sandwich_checkpoint_gives_the_decay_rank(tmp_path):
+    """The rank of the decay's projection is no part of a checkpoint's config: a tensor's shape gives it."""
+    from safetensors.torch import save_file
+
+    cfg, w = json.loads(json.dumps(SANDWICH["odd"])), make_sandwich_weights(SANDWICH["odd"], 3)
+    for e in cfg["layers"]:
+        e["mixer"].pop("decay_rank", None)
+    with pytest.raises(ValueError, match="decay_rank"):
+        HybridDecoder(cfg, "cpu", seed=None, max_model_len=64)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file(w, str(tmp_path / "model.safetensors"))
+    m = load_decoder(str(tmp_path), "cpu", max_model_len=64)
+    assert isinstance(m, HybridDecoder) and m.plain_lm_head and not m.prefix_cacheable and m.min_bucket == 1
+    assert [L["mixer"].rank for L in m.layers if isinstance(L["mixer"], mixers.GeneralDelta)] == [5, 6]
+    assert m.spec.norm_groups == cfg["norm"]["groups"] and m.spec.residual_mult == cfg["residual_mult"]
+    del w["l1.rg1.b"]
+    save_file(w, str(tmp_path / "model.safetensors"))
+    with pytest.raises(ValueError, match="l1.rg1.b"):
+        load_decoder(str(tmp_path), "cpu", max_model_len=64)
+
+
+def test_shared_latents_hold_one_cache():
+    cfg = SANDWICH["padded"]
+    m = HybridDecoder(cfg, "cpu", seed=None, max_model_len=64)
+    runs = HybridCache(m, 5, 3).runs
+    assert runs[2] is runs[0] and runs[4] is runs[0] and runs[0].shape == (5, BLOCK_SIZE, 160)
+    assert runs[1].shape == (3, 2, 72, 72) and runs[3].shape == (3, 1, 136, 136) and runs[1].dtype == torch.float32
+    assert m.block_bytes() == runs[0].numel() * 2 // 5 and m.row_bytes() == 4 * (2 * 72 * 72 + 136 * 136)
+    names = dict(m.hf_named_tensors())
+    assert "l0.mix.dkv" in names and "l2.mix.dkv" not in names and "l4.mix.dkv.norm" not in names
+
+
+def test_sandwich_sizes_outside_the_design_are_refused():
+    build = lambda layers, mlps=None, **kw: HybridDecoder(  # noqa: E731
+        dict(sandwich_config(layers, mlps or [None] * len(layers)), **kw), "cpu", seed=None, max_model_len=8)
+    one = low_rank()
+    for bad in (low_rank(kv_from=1), low_rank(kv_from=-1), low_rank(kv_from=0, kv_rank=44), low_rank(kv_from=0, rot_dim=8),
+                low_rank(kv_from=0, base=77.0)):
+        with pytest.raises(ValueError, match="kv_from"):
+            build([one, bad])
+    with pytest.raises(ValueError, match="kv_from"):
+        build([one, low_rank(kv_from=0), low_rank(kv_from=1)])
+    with pytest.raises(ValueError, match="kv_from"):  # a recurrent layer has nothing to share
+        build([general(), dict(general(), mixer=dict(general()["mixer"], kv_from=0))])
+    build([one, low_rank(heads=7, dim=9, vdim=5, q_rank=8, window=3, scale=0.5, kv_from=0)])  # all its own but the latents
+    for bad in (routed(experts=10, groups=(3, 1)), routed(experts=10, groups=(5, 6)), routed(experts=10, top=3, groups=(5, 1)),
+                routed(experts=10, top=0), routed(experts=2000)):
+        with pytest.raises(ValueError):
+            build([one], [bad])
+    for layer in (general(dim=300), low_rank(rot_dim=7)):
+        with pytest.raises(ValueError):
+            build([layer])
+    with pytest.raises(ValueError, match="norm.groups"):
+        build([one], norm={"eps": 1e-5, "groups": 5})
+    with pytest.raises(ValueError, match="looped"):
+        build([one], loop={"start": 0, "stop": 1, "times": 2})
+    with pytest.raises(ValueError, match="feed-forward"):
+        build([one], [{"kind": "dense", "ff": 8}])
+
+
+def test_sandwich_kernel_libraries_and_plans():
+    from skyrl_amd.inference_engines.registry import kernel_libraries
+
+    assert kernel_libraries(SANDWICH["odd"]) == ("layers", "gdelta", "latent", "moe")
+    assert kernel_libraries(sandwich_config([general()], [None])) == ("layers", "gdelta")
+    m = HybridDecoder(SANDWICH["odd"], "cpu", seed=None, max_model_len=64)
+    assert set(m.plan([3, 40], [0, 5], 1)) == {21, None, "chunks"} and m.plan([1, 3], [7, 0], 2) is None
+
+
+def test_experts_tiles_follow_the_mean_load():
+    sh = mixers.lk.moe_shape(64, 32, 64, 8, 8, 4)
+    assert [mixers.lk.moe_tile(sh, n) for n in (1, 64, 127, 128, 512, 767, 768, 8192)] == [16, 16, 16, 64, 64, 64, 128, 128]
+
+
+def test_oracle_grouped_norm_and_routing():
+    x, w = torch.randn(3, 12, dtype=torch.float64), torch.randn(12, dtype=torch.float64)
+    got = ref.grouped_rms_norm(x, w, 3, 1e-3)
+    for g in range(3):
+        part = x[:, 4 * g:4 * g + 4]
+        torch.testing.assert_close(got[:, 4 * g:4 * g + 4], part / (part.pow(2).mean(-1, keepdim=True) + 1e-3).sqrt() * w[4 * g:4 * g + 4])
+    s = torch.tensor([[0.9, 0.1, 0.7, 0.6, 0.2, 0.3]])
+    idx, weight = ref.route(s, torch.tensor([0.0, 0.0, 0.0, 0.0, -9.0, -9.0]), 2, 3, 1)
+    assert idx.tolist() == [[2, 3]] and weight.tolist() == [[s[0, 2].item(), s[0, 3].item()]]  # 0.7 + 0.6 beats 0.9 + 0.1
+    idx, _ = ref.route(s, torch.full((6,), -5.0), 3, 3, 2)
+    assert idx.tolist() == [[0, 2, 3]]  # corrected scores below zero: other groups' count as less than any
 
 
 def test_position_turns():
