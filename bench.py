@@ -1137,7 +1137,7 @@ def main():
     ap.add_argument("--hybrid", action="store_true",
                     help="instead: prefill and decode throughput of the hybrid decoders beside a dense one of equal size")
     ap.add_argument("--hybrid-size", default="2k,4k", help="of 2k, 4k (comma separated)")
-    ap.add_argument("--hybrid-model", choices=("dovidra", "lipedra", "foduzen", "qwen2"), default=None)
+    ap.add_argument("--hybrid-model", choices=("dovidra", "lipedra", "foduzen", "tativik", "qwen2"), default=None)
     ap.add_argument("--hybrid-phase", choices=("prefill", "decode"), default=None)
     ap.add_argument("--hybrid-prompts", default="", help="prompts x tokens, e.g. 1x8192,8x1024")
     ap.add_argument("--hybrid-decodes", default="", help="rows @ context, e.g. 64@2048")

@@ -371,9 +371,10 @@ int skyrl_gdelta_out(const skyrl_gdelta_shape* shape, const int32_t* chunk, int3
  * choice scores may be chosen from; the `top` largest of those are, ties to the lower index. Pair p = token * top + i.
  *   skyrl_moe_route    idx i32 [n, top], weight f32 [n, top] (the scores s of the chosen).
  *   skyrl_moe_tiles    the most tiles of tm rows that npairs pairs can fill.
- *   skyrl_moe_sort     pairs by expert: order i32 [ntiles, tm] (pair, or -1), tile_expert i32 [ntiles] (-1: unused).
- *   skyrl_moe_gate_up  act T [ntiles tm, ff], by sorted place = silu(gate x) * up x. tm a multiple of 16; 16, 64 and 128
- *                      have a matrix form (bf16, width and ff multiples of 8).
+ *   skyrl_moe_sort     pairs by expert: order i32 [ntiles, tm] (pair, or -1), tile_expert i32 [ntiles + 1] (-1: unused; the
+ *                      last: tiles in use). counts: scratch of skyrl_moe_counts(experts, npairs) i32 (0: NULL).
+ *   skyrl_moe_gate_up  act T [ntiles tm, ff], by sorted place = silu(gate x) * up x. tm a multiple of 16; 16, 64, 128 and
+ *                      256 have a matrix form (bf16, width and ff multiples of 8).
  *   skyrl_moe_down     out T [n top, width], by pair = weight * down act. */
 typedef struct {
     int32_t width, ff, experts, top, groups, keep;
@@ -381,8 +382,9 @@ typedef struct {
 int skyrl_moe_route(const skyrl_moe_shape* shape, const void* x, int32_t n, const void* router, const float* correction,
                     int32_t* idx, float* weight, int32_t dtype, void* stream);
 int32_t skyrl_moe_tiles(int32_t experts, int32_t npairs, int32_t tm);
-int skyrl_moe_sort(const int32_t* idx, int32_t npairs, int32_t experts, int32_t tm, int32_t ntiles, int32_t* order,
-                   int32_t* tile_expert, void* stream);
+int32_t skyrl_moe_counts(int32_t experts, int32_t npairs);
+int skyrl_moe_sort(const int32_t* idx, int32_t npairs, int32_t experts, int32_t tm, int32_t ntiles, int32_t* counts,
+                   int32_t* order, int32_t* tile_expert, void* stream);
 int skyrl_moe_gate_up(const skyrl_moe_shape* shape, const void* x, const void* w, const int32_t* order,
                       const int32_t* tile_expert, int32_t tm, int32_t ntiles, void* act, int32_t dtype, void* stream);
 int skyrl_moe_down(const skyrl_moe_shape* shape, const void* act, const void* w, const int32_t* order,

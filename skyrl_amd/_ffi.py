@@ -330,7 +330,8 @@ LAYERS_SIGNATURES = {
     "skyrl_gdelta_out": (_INT, [_GS, _P, _I32, _P, _P, _P, _P, _I64, _P, _P, _I64, _I32, _P]),
     "skyrl_moe_route": (_INT, [_MS, _P, _I32, _P, _P, _P, _P, _I32, _P]),
     "skyrl_moe_tiles": (_I32, [_I32, _I32, _I32]),
-    "skyrl_moe_sort": (_INT, [_P, _I32, _I32, _I32, _I32, _P, _P, _P]),
+    "skyrl_moe_counts": (_I32, [_I32, _I32]),
+    "skyrl_moe_sort": (_INT, [_P, _I32, _I32, _I32, _I32, _P, _P, _P, _P]),
     "skyrl_moe_gate_up": (_INT, [_MS, _P, _P, _P, _P, _I32, _I32, _P, _I32, _P]),
     "skyrl_moe_down": (_INT, [_MS, _P, _P, _P, _P, _I32, _I32, _P, _P, _I32, _P]),
 }

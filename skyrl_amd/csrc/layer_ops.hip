@@ -408,97 +408,114 @@ struct GateNormAdd {
     int H;
 };
 
-// 1 / root mean square of every group of `per` consecutive chunks into s_r, from the chunks' sums of squares s_p: teams
-// of up to 64 lanes. All threads of the block call it; s_p is written by them before.
-__device__ __forceinline__ void group_scales(const float* s_p, float* s_r, int groups, int per, float len, float eps) {
-    __syncthreads();
-    int L = kWave;
-    while (L > 1 && groups * L > kNT) L >>= 1;
-    const int sub = threadIdx.x & (L - 1);
-    for (int g = threadIdx.x / L; g < groups; g += kNT / L) {
-        float s = 0.f;
-        for (int i = sub; i < per; i += L) s += s_p[g * per + i];
-        for (int o = L >> 1; o > 0; o >>= 1) s += __shfl_xor(s, o, kWave);
-        if (sub == 0) s_r[g] = 1.f / sqrtf(s / len + eps);
-    }
-    __syncthreads();
-}
-
-// One block per row, the row in registers. Chunks of VEC elements lie in one group.
-template <typename T, int VEC, int kMaxV>
-__global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p) {
-    extern __shared__ float s_p[];  // a chunk's sum of squares; then the groups' scales
+// One block per row, the row in registers: chunks of VEC elements, chunk threadIdx + k kNT, each in one group of `per`
+// chunks. A group's sum: within L lanes (the power of two in per, at most a wave) by shuffles, then over per / L numbers
+// in LDS. PARTS: rows that are summed (0: any number).
+template <typename T, int VEC, int kMaxV, int PARTS>
+__global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, int L) {
+    extern __shared__ float s_p[];
     __shared__ float s_red[kNT / kWave];
-    const int nv = p.H / VEC, per = nv / p.groups;
-    float* s_r = s_p + nv;
+    const int nv = p.H / VEC, per = nv / p.groups, sums = per / L;
     const int64_t base = (int64_t)blockIdx.x * p.H;
     const int64_t row = p.rows ? p.rows[blockIdx.x] : blockIdx.x;
     const float len = (float)(p.H / p.groups);
-    float y[kMaxV][VEC], h[kMaxV][VEC];
-    float one = 0.f;
+    const int parts = PARTS ? PARTS : p.parts;
+    float y[kMaxV][VEC], h[kMaxV][VEC], r[kMaxV];
+    // r: 1 / root mean square of every chunk's group, from the chunks' sums of squares
+    auto scales = [&]() {
+        if (p.groups == 1) {
+            float one = 0.f;
+#pragma unroll
+            for (int k = 0; k < kMaxV; ++k) one += r[k];
+            one = 1.f / sqrtf(block_total<kNT>(one, s_red) / len + p.eps);
+#pragma unroll
+            for (int k = 0; k < kMaxV; ++k) r[k] = one;
+            return;
+        }
+#pragma unroll
+        for (int k = 0; k < kMaxV; ++k)
+            for (int o = 1; o < L; o <<= 1) r[k] += __shfl_xor(r[k], o, kWave);
+        if (sums > 1) {
+            __syncthreads();  // the sums before these are read
+#pragma unroll
+            for (int k = 0; k < kMaxV; ++k) {
+                const int v = threadIdx.x + k * kNT;
+                if (v < nv && v % L == 0) s_p[v / L] = r[k];
+            }
+            __syncthreads();
+#pragma unroll
+            for (int k = 0; k < kMaxV; ++k) {
+                const int v = threadIdx.x + k * kNT;
+                if (v >= nv) continue;
+                const float* q = s_p + v / per * sums;
+                float s = 0.f;
+                for (int i = 0; i < sums; ++i) s += q[i];
+                r[k] = s;
+            }
+        }
+#pragma unroll
+        for (int k = 0; k < kMaxV; ++k) r[k] = 1.f / sqrtf(r[k] / len + p.eps);
+    };
 #pragma unroll
     for (int k = 0; k < kMaxV; ++k) {
         const int v = threadIdx.x + k * kNT;
-        float ss = 0.f;
+        r[k] = 0.f;
 #pragma unroll
         for (int j = 0; j < VEC; ++j) y[k][j] = h[k][j] = 0.f;
         if (v < nv) {
-            const T* src = p.a + row * p.parts * p.H + VEC * v;
-            ldw<T, VEC>(src, y[k]);
-            if (!p.fresh) ldw<float, VEC>(p.h + base + VEC * v, h[k]);
-            for (int i = 1; i < p.parts; ++i) {
+            const T* src = p.a + row * parts * p.H + VEC * v;
+            ldv<T, VEC>(src, y[k]);
+            if (!p.fresh) ldv<float, VEC>(p.h + base + VEC * v, h[k]);
+            auto add = [&](int i) {
                 float x[VEC];
-                ldw<T, VEC>(src + (int64_t)i * p.H, x);
+                ldv<T, VEC>(src + (int64_t)i * p.H, x);
 #pragma unroll
                 for (int j = 0; j < VEC; ++j) y[k][j] += x[j];
+            };
+            if constexpr (PARTS > 0) {
+#pragma unroll
+                for (int i = 1; i < PARTS; ++i) add(i);
+            } else {
+                for (int i = 1; i < parts; ++i) add(i);
             }
             if (p.z) {
                 float z[VEC], b[VEC];
-                ldw<T, VEC>(p.z + blockIdx.x * p.z_stride + VEC * v, z);
-                ldw<float, VEC>(p.zb + VEC * v, b);
+                ldv<T, VEC>(p.z + blockIdx.x * p.z_stride + VEC * v, z);
+                ldv<float, VEC>(p.zb + VEC * v, b);
 #pragma unroll
                 for (int j = 0; j < VEC; ++j) y[k][j] *= sigmoid_<T>(z[j] + b[j]);
             }
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) ss += y[k][j] * y[k][j];
-            if (p.groups > 1) s_p[v] = ss;
+            for (int j = 0; j < VEC; ++j) r[k] += y[k][j] * y[k][j];
         }
-        one += ss;
     }
-    float r1 = 0.f;
-    if (p.groups == 1) r1 = 1.f / sqrtf(block_total<kNT>(one, s_red) / len + p.eps);
-    else group_scales(s_p, s_r, p.groups, per, len, p.eps);
-    one = 0.f;
+    scales();
 #pragma unroll
     for (int k = 0; k < kMaxV; ++k) {
         const int v = threadIdx.x + k * kNT;
-        float ss = 0.f;
+        const float rk = r[k];
+        r[k] = 0.f;
         if (v < nv) {
-            const float r = p.groups == 1 ? r1 : s_r[v / per];
             float w[VEC];
-            ldw<T, VEC>(p.w + VEC * v, w);
+            ldv<T, VEC>(p.w + VEC * v, w);
 #pragma unroll
             for (int j = 0; j < VEC; ++j) {
-                h[k][j] += p.mult * (y[k][j] * r * w[j]);
-                ss += h[k][j] * h[k][j];
+                h[k][j] += p.mult * (y[k][j] * rk * w[j]);
+                r[k] += h[k][j] * h[k][j];
             }
-            stw<float, VEC>(p.h + base + VEC * v, h[k]);
-            if (p.groups > 1) s_p[v] = ss;  // its own chunks only: the others' scales are not read again before the barrier
+            stv(p.h + base + VEC * v, h[k]);
         }
-        one += ss;
     }
-    if (p.groups == 1) r1 = 1.f / sqrtf(block_total<kNT>(one, s_red) / len + p.eps);
-    else group_scales(s_p, s_r, p.groups, per, len, p.eps);
+    scales();
 #pragma unroll
     for (int k = 0; k < kMaxV; ++k) {
         const int v = threadIdx.x + k * kNT;
         if (v < nv) {
-            const float r = p.groups == 1 ? r1 : s_r[v / per];
             float w[VEC];
-            ldw<T, VEC>(p.wn + VEC * v, w);
+            ldv<T, VEC>(p.wn + VEC * v, w);
 #pragma unroll
-            for (int j = 0; j < VEC; ++j) h[k][j] *= r * w[j];
-            stw<T, VEC>(p.out + base + VEC * v, h[k]);
+            for (int j = 0; j < VEC; ++j) h[k][j] *= r[k] * w[j];
+            stv(p.out + base + VEC * v, h[k]);
         }
     }
 }
@@ -650,8 +667,16 @@ extern "C" int skyrl_xielu(const void* x, int64_t stride, int64_t n, int32_t I, 
     return check_launch("xielu_kernel");
 }
 
-#define LAUNCH_GNA(V, K) \
-    hipLaunchKernelGGL((gate_norm_add_kernel<T, V, K>), dim3(n), dim3(kNT), lds(V), as_stream(stream), p)
+#define LAUNCH_GNA_(V, K, P) \
+    hipLaunchKernelGGL((gate_norm_add_kernel<T, V, K, P>), dim3(n), dim3(kNT), lds, as_stream(stream), p, L)
+#define LAUNCH_GNA(V, K)                     \
+    do {                                     \
+        if (parts == 1) LAUNCH_GNA_(V, K, 1); \
+        else if (parts == 2) LAUNCH_GNA_(V, K, 2); \
+        else if (parts == 4) LAUNCH_GNA_(V, K, 4); \
+        else if (parts == 8) LAUNCH_GNA_(V, K, 8); \
+        else LAUNCH_GNA_(V, K, 0);           \
+    } while (0)
 
 extern "C" int skyrl_gate_norm_add(const void* a, const int64_t* rows, int32_t parts, const void* gate,
                                    int64_t gate_stride, const float* gate_bias, const void* weight, int32_t groups,
@@ -663,22 +688,23 @@ extern "C" int skyrl_gate_norm_add(const void* a, const int64_t* rows, int32_t p
     SKYRL_REQUIRE(!gate || (gate_bias && gate_stride >= H), "gate_norm_add: gate needs a bias and a stride >= H");
     if (n == 0) return SKYRL_OK;
     SKYRL_REQUIRE(a && weight && hidden && next && out, "gate_norm_add: null pointer");
-    auto lds = [&](int V) { return groups > 1 ? (size_t)(H / V + groups) * sizeof(float) : (size_t)0; };
     SKYRL_DISPATCH_T(dtype, {
         auto t = [](const void* q) { return reinterpret_cast<const T*>(q); };
         const GateNormAdd<T> p{t(a), rows, parts, t(gate), gate_stride, gate_bias, t(weight), groups, eps, mult, hidden,
                                fresh, t(next), reinterpret_cast<T*>(out), H};
-        const bool wide = H / groups % 4 == 0 &&
-                          (!gate || (gate_stride % 4 == 0 && reinterpret_cast<uintptr_t>(gate) % (4 * sizeof(T)) == 0));
+        const bool wide = H / groups % 8 == 0 && (!gate || (gate_stride % 8 == 0 && aligned16(gate))) && aligned16(a) &&
+                          aligned16(hidden) && aligned16(weight) && aligned16(next) && aligned16(out);
+        const int V = wide ? 8 : 1;
+        int L = 1;
+        while (L < kWave && H / V / groups % (2 * L) == 0) L <<= 1;
+        const size_t lds = groups > 1 ? (size_t)(H / V / L) * sizeof(float) : 0;
         if (wide) {
-            if (H <= 4 * kNT) LAUNCH_GNA(4, 1);
-            else if (H <= 8 * kNT) LAUNCH_GNA(4, 2);
-            else if (H <= 16 * kNT) LAUNCH_GNA(4, 4);
-            else LAUNCH_GNA(4, 8);
+            if (H <= 8 * kNT) LAUNCH_GNA(8, 1);
+            else if (H <= 16 * kNT) LAUNCH_GNA(8, 2);
+            else LAUNCH_GNA(8, 4);
         } else {
-            SKYRL_REQUIRE(lds(1) <= 65536 - 64, "gate_norm_add: too many groups");
-            if (H <= 4 * kNT) LAUNCH_GNA(1, 4);
-            else LAUNCH_GNA(1, 32);
+            if (H <= 4 * kNT) LAUNCH_GNA_(1, 4, 0);
+            else LAUNCH_GNA_(1, 32, 0);
         }
     })
     return check_launch("gate_norm_add_kernel");

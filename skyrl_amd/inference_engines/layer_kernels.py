@@ -938,18 +938,21 @@ def moe_route(sh, x, router, correction):
 def moe_tile(sh, n: int) -> int:
     """Rows per tile of the experts' products for n tokens."""
     mean = n * sh.top / sh.experts
-    return 128 if mean >= 96 else 64 if mean >= 16 else 16
+    return 256 if mean >= 112 else 128 if mean >= 48 else 64 if mean >= 12 else 16
 
 
 def moe_sort(sh, idx, tm: int):
-    """(order int32 [tiles, tm], tile_expert int32 [tiles]): the (token, expert) pairs by expert."""
+    """(order int32 [tiles, tm], tile_expert int32 [tiles + 1]): the (token, expert) pairs by expert; the last entry is
+    the number of tiles in use."""
     dev = _require_gpu(idx)
     _check(idx, "idx", torch.int32, (idx.shape[0], sh.top))
     pairs = idx.numel()
     tiles = int(_ffi.query("skyrl_moe_tiles", sh.experts, pairs, tm))
     order = torch.empty((tiles, tm), dtype=torch.int32, device=dev)
-    tile_expert = torch.empty((tiles,), dtype=torch.int32, device=dev)
-    _ffi.call("skyrl_moe_sort", _ptr(idx), pairs, sh.experts, tm, tiles, _ptr(order), _ptr(tile_expert), _stream(dev))
+    tile_expert = torch.empty((tiles + 1,), dtype=torch.int32, device=dev)
+    scratch = int(_ffi.query("skyrl_moe_counts", sh.experts, pairs))
+    counts = torch.empty((scratch,), dtype=torch.int32, device=dev) if scratch else None
+    _ffi.call("skyrl_moe_sort", _ptr(idx), pairs, sh.experts, tm, tiles, _ptr(counts), _ptr(order), _ptr(tile_expert), _stream(dev))
     return order, tile_expert
 
 
@@ -968,7 +971,7 @@ def moe_experts(sh, x, idx, weight, gate_up, down, tm: Optional[int] = None) -> 
     if n == 0:
         return out
     order, tile_expert = moe_sort(sh, idx, tm)
-    tiles = tile_expert.shape[0]
+    tiles = order.shape[0]
     act = torch.empty((tiles * tm, sh.ff), dtype=x.dtype, device=dev)
     ref, st = ctypes.byref(sh), _stream(dev)
     _ffi.call("skyrl_moe_gate_up", ref, _ptr(x), _ptr(gate_up), _ptr(order), _ptr(tile_expert), tm, tiles, _ptr(act),

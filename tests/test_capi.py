@@ -137,8 +137,9 @@ def test_routed_entries_validate_on_host():
             ("skyrl_moe_route", (moe(64, 32, 8, 2, 3, 1), p, 1, p, p, p, p, _ffi.F32, None), "multiple of groups"),
             ("skyrl_moe_route", (moe(64, 32, 8, 5, 2, 1), p, 1, p, p, p, p, _ffi.F32, None), "top must be"),
             ("skyrl_moe_route", (moe(64, 32, 2048, 2, 1, 1), p, 1, p, p, p, p, _ffi.F32, None), "1024"),
-            ("skyrl_moe_sort", (p, 20, 8, 16, 8, p, p, None), "too few tiles"),
-            ("skyrl_moe_sort", (p, 20, 8, 20, 99, p, p, None), "sizes"),
+            ("skyrl_moe_sort", (p, 20, 8, 16, 8, None, p, p, None), "too few tiles"),
+            ("skyrl_moe_sort", (p, 20000, 8, 16, 9999, None, p, p, None), "counts"),
+            ("skyrl_moe_sort", (p, 20, 8, 20, 99, None, p, p, None), "sizes"),
             ("skyrl_moe_gate_up", (ok, p, p, p, p, 24, 4, p, _ffi.F32, None), "plain form"),
             ("skyrl_moe_down", (ok, p, p, p, p, 16, 4, None, p, _ffi.F32, None), "null pointer")):
         with pytest.raises(_ffi.SkyrlHipError, match=msg):

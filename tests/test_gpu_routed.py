@@ -290,7 +290,7 @@ def close_calls(choice, top, groups, keep):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("width,experts,top,groups,keep", [(72, 10, 3, 1, 1), (128, 64, 8, 8, 4), (70, 12, 2, 4, 3), (2048, 32, 4, 4, 1),
-                                                           (96, 256, 8, 8, 3), (64, 100, 5, 10, 2), (264, 600, 9, 6, 5), (40, 6, 4, 6, 4), (33, 1, 1, 1, 1)])
+                                                           (96, 256, 8, 8, 3), (64, 100, 5, 10, 2), (512, 128, 70, 2, 2), (264, 600, 9, 6, 5), (40, 6, 4, 6, 4), (33, 1, 1, 1, 1)])
 def test_route(width, experts, top, groups, keep, dtype):
     """Negative and positive choice scores, groups whose best expert alone would win."""
     g = torch.Generator().manual_seed(experts)
@@ -323,16 +323,16 @@ def test_group_scores_are_sums_of_two():
     assert idx.tolist() == [[4, 7]] and abs(float(w[0, 0]) - 0.7) < 1e-5
 
 
-@pytest.mark.parametrize("pairs,experts,tm", [(1, 1, 16), (37, 5, 16), (1000, 64, 64), (4096, 600, 128), (20000, 16, 128), (9, 1024, 16)])
+@pytest.mark.parametrize("pairs,experts,tm", [(1, 1, 16), (37, 5, 16), (1000, 64, 64), (4096, 600, 128), (20000, 16, 128), (9, 1024, 16), (70001, 130, 256), (4097, 3, 16)])
 def test_sort_lists_every_pair_once(pairs, experts, tm):
     g = torch.Generator().manual_seed(pairs)
     sh = lk.moe_shape(8, 8, experts, 1)
     idx = (torch.rand(pairs, 1, generator=g) ** 2 * experts).int().clamp(max=experts - 1)  # uneven, some without any
     order, tile_expert = (t.cpu() for t in lk.moe_sort(sh, dev(idx), tm))
-    used = tile_expert >= 0
-    assert int(used.sum()) == sum(-(-int(c) // tm) for c in idx.flatten().bincount()) and not bool(used[int(used.sum()):].any())
+    used = tile_expert[:-1] >= 0
+    assert int(tile_expert[-1]) == int(used.sum()) == sum(-(-int(c) // tm) for c in idx.flatten().bincount()) and not bool(used[int(used.sum()):].any())
     listed = order[used]
-    for e, row in zip(tile_expert[used].tolist(), listed):
+    for e, row in zip(tile_expert[:-1][used].tolist(), listed):
         assert bool((idx.flatten()[row[row >= 0].long()] == e).all())
     assert sorted(listed[listed >= 0].tolist()) == list(range(pairs))
 
@@ -355,8 +355,26 @@ def test_experts(width, ff, experts, top, n, dtype):
     X, G, D = x.double(), wgu.double(), wd.double()
     want = torch.stack([weight[t, i].double() * (D[e] @ (ref.silu(G[e, 0] @ X[t]) * (G[e, 1] @ X[t])))
                         for t in range(n) for i, e in enumerate(idx[t].tolist())])
-    for tm in (None, 16, 64, 128):
+    for tm in (None, 16, 64, 128, 256):
         close(lk.moe_experts(sh, dev(x), dev(idx), dev(weight), dev(wgu), dev(wd), tm=tm), want, dtype, f32=5e-6, bf16=8e-3)
+
+
+@pytest.mark.parametrize("width,ff,experts,top,n", [(2048, 768, 32, 8, 1500), (1024, 512, 64, 4, 300), (4096, 320, 8, 2, 90)])
+def test_tile_sizes_agree_bit_for_bit(width, ff, experts, top, n):
+    """A row's sums are formed in the same order whatever its tile: products of a real layer's size, over and over."""
+    g = torch.Generator(device=DEV).manual_seed(width)
+    sh = lk.moe_shape(width, ff, experts, top)
+    mk = lambda *s, scale=1.0: (torch.randn(s, generator=g, device=DEV) * scale).to(BF16)  # noqa: E731
+    x, wgu, wd = mk(n, width), mk(experts, 2, ff, width, scale=0.03), mk(experts, width, ff, scale=0.03)
+    idx, weight = lk.moe_route(sh, x, mk(experts, width, scale=0.03), torch.zeros(experts, device=DEV))
+    outs = [lk.moe_experts(sh, x, idx, weight, wgu, wd, tm=tm) for _ in range(4) for tm in (16, 64, 128, 256)]
+    rows = torch.randint(0, n * top, (8,), generator=torch.Generator().manual_seed(1))
+    for r in rows.tolist():
+        t, e = r // top, int(idx[r // top, r % top])
+        h = x[t].double().cpu()
+        a = ref.silu(wgu[e, 0].double().cpu() @ h) * (wgu[e, 1].double().cpu() @ h)
+        close(outs[0][r], float(weight[t, r % top]) * (wd[e].double().cpu() @ a), BF16, bf16=8e-3)
+    assert all(torch.equal(outs[0], o) for o in outs[1:])
 
 
 # ---------------------------------------------------------------- the model through the engine's steps

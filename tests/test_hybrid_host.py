@@ -520,7 +520,7 @@ def test_sandwich_kernel_libraries_and_plans():
 
 def test_experts_tiles_follow_the_mean_load():
     sh = mixers.lk.moe_shape(64, 32, 64, 8, 8, 4)
-    assert [mixers.lk.moe_tile(sh, n) for n in (1, 64, 127, 128, 512, 767, 768, 8192)] == [16, 16, 16, 64, 64, 64, 128, 128]
+    assert [mixers.lk.moe_tile(sh, n) for n in (1, 64, 95, 96, 383, 384, 895, 896, 8192)] == [16, 16, 16, 64, 64, 128, 128, 256, 256]
 
 
 def test_oracle_grouped_norm_and_routing():
