@@ -408,13 +408,13 @@ struct GateNormAdd {
     int H;
 };
 
-// One block per row, the row in registers: chunks of VEC elements, chunk threadIdx + k kNT, each in one group of `per`
+// One block per row, the row in registers: chunks of VEC elements, chunk threadIdx + k NT, each in one group of `per`
 // chunks. A group's sum: within L lanes (the power of two in per, at most a wave) by shuffles, then over per / L numbers
 // in LDS. PARTS: rows that are summed (0: any number).
-template <typename T, int VEC, int kMaxV, int PARTS>
-__global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, int L) {
+template <typename T, int NT, int VEC, int kMaxV, int PARTS>
+__global__ __launch_bounds__(NT) void gate_norm_add_kernel(GateNormAdd<T> p, int L) {
     extern __shared__ float s_p[];
-    __shared__ float s_red[kNT / kWave];
+    __shared__ float s_red[NT / kWave];
     const int nv = p.H / VEC, per = nv / p.groups, sums = per / L;
     const int64_t base = (int64_t)blockIdx.x * p.H;
     const int64_t row = p.rows ? p.rows[blockIdx.x] : blockIdx.x;
@@ -427,7 +427,7 @@ __global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, in
             float one = 0.f;
 #pragma unroll
             for (int k = 0; k < kMaxV; ++k) one += r[k];
-            one = 1.f / sqrtf(block_total<kNT>(one, s_red) / len + p.eps);
+            one = 1.f / sqrtf(block_total<NT>(one, s_red) / len + p.eps);
 #pragma unroll
             for (int k = 0; k < kMaxV; ++k) r[k] = one;
             return;
@@ -439,13 +439,13 @@ __global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, in
             __syncthreads();  // the sums before these are read
 #pragma unroll
             for (int k = 0; k < kMaxV; ++k) {
-                const int v = threadIdx.x + k * kNT;
+                const int v = threadIdx.x + k * NT;
                 if (v < nv && v % L == 0) s_p[v / L] = r[k];
             }
             __syncthreads();
 #pragma unroll
             for (int k = 0; k < kMaxV; ++k) {
-                const int v = threadIdx.x + k * kNT;
+                const int v = threadIdx.x + k * NT;
                 if (v >= nv) continue;
                 const float* q = s_p + v / per * sums;
                 float s = 0.f;
@@ -458,7 +458,7 @@ __global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, in
     };
 #pragma unroll
     for (int k = 0; k < kMaxV; ++k) {
-        const int v = threadIdx.x + k * kNT;
+        const int v = threadIdx.x + k * NT;
         r[k] = 0.f;
 #pragma unroll
         for (int j = 0; j < VEC; ++j) y[k][j] = h[k][j] = 0.f;
@@ -492,7 +492,7 @@ __global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, in
     scales();
 #pragma unroll
     for (int k = 0; k < kMaxV; ++k) {
-        const int v = threadIdx.x + k * kNT;
+        const int v = threadIdx.x + k * NT;
         const float rk = r[k];
         r[k] = 0.f;
         if (v < nv) {
@@ -509,7 +509,7 @@ __global__ __launch_bounds__(kNT) void gate_norm_add_kernel(GateNormAdd<T> p, in
     scales();
 #pragma unroll
     for (int k = 0; k < kMaxV; ++k) {
-        const int v = threadIdx.x + k * kNT;
+        const int v = threadIdx.x + k * NT;
         if (v < nv) {
             float w[VEC];
             ldv<T, VEC>(p.wn + VEC * v, w);
@@ -667,15 +667,15 @@ extern "C" int skyrl_xielu(const void* x, int64_t stride, int64_t n, int32_t I, 
     return check_launch("xielu_kernel");
 }
 
-#define LAUNCH_GNA_(V, K, P) \
-    hipLaunchKernelGGL((gate_norm_add_kernel<T, V, K, P>), dim3(n), dim3(kNT), lds, as_stream(stream), p, L)
-#define LAUNCH_GNA(V, K)                     \
-    do {                                     \
-        if (parts == 1) LAUNCH_GNA_(V, K, 1); \
-        else if (parts == 2) LAUNCH_GNA_(V, K, 2); \
-        else if (parts == 4) LAUNCH_GNA_(V, K, 4); \
-        else if (parts == 8) LAUNCH_GNA_(V, K, 8); \
-        else LAUNCH_GNA_(V, K, 0);           \
+#define LAUNCH_GNA_(NT, V, K, P) \
+    hipLaunchKernelGGL((gate_norm_add_kernel<T, NT, V, K, P>), dim3(n), dim3(NT), lds, as_stream(stream), p, L)
+#define LAUNCH_GNA(NT)                              \
+    do {                                            \
+        if (parts == 1) LAUNCH_GNA_(NT, 8, 1, 1);   \
+        else if (parts == 2) LAUNCH_GNA_(NT, 8, 1, 2); \
+        else if (parts == 4) LAUNCH_GNA_(NT, 8, 1, 4); \
+        else if (parts == 8) LAUNCH_GNA_(NT, 8, 1, 8); \
+        else LAUNCH_GNA_(NT, 8, 1, 0);              \
     } while (0)
 
 extern "C" int skyrl_gate_norm_add(const void* a, const int64_t* rows, int32_t parts, const void* gate,
@@ -699,12 +699,12 @@ extern "C" int skyrl_gate_norm_add(const void* a, const int64_t* rows, int32_t p
         while (L < kWave && H / V / groups % (2 * L) == 0) L <<= 1;
         const size_t lds = groups > 1 ? (size_t)(H / V / L) * sizeof(float) : 0;
         if (wide) {
-            if (H <= 8 * kNT) LAUNCH_GNA(8, 1);
-            else if (H <= 16 * kNT) LAUNCH_GNA(8, 2);
-            else LAUNCH_GNA(8, 4);
+            if (H <= 8 * 256) LAUNCH_GNA(256);
+            else if (H <= 8 * 512) LAUNCH_GNA(512);
+            else LAUNCH_GNA(1024);
         } else {
-            if (H <= 4 * kNT) LAUNCH_GNA_(1, 4, 0);
-            else LAUNCH_GNA_(1, 32, 0);
+            if (H <= 4 * kNT) LAUNCH_GNA_(kNT, 1, 4, 0);
+            else LAUNCH_GNA_(kNT, 1, 32, 0);
         }
     })
     return check_launch("gate_norm_add_kernel");
