@@ -382,8 +382,13 @@ def make_sandwich_weights(cfg, seed=0, steady=True):
                 mat(f"{f}e{k}.up", ff, W, 1.5)
                 mat(f"{f}e{k}.down", W, ff)
             mat(f + "router", ro["experts"], W, 0.3 if steady else 1.5)
-            if steady:  # scores stay within 0.5 +- 0.25
-                w[f + "correction"] = torch.randperm(ro["experts"], generator=g) * 1.0 - 0.7 * ro["experts"]
+            if steady:  # scores stay within 0.5 +- 0.25; where groups' sums tie, groups stand apart
+                E, count = ro["experts"], (ro.get("groups") or {"count": 1})["count"]
+                c = torch.randperm(E, generator=g) * 1.0 - 0.7 * E
+                sums = c.view(count, -1).topk(min(2, E // count)).values.sum(-1)
+                if len(set(sums.tolist())) < count:
+                    c = c + torch.arange(count).repeat_interleave(E // count) * E
+                w[f + "correction"] = c
             else:
                 rand(f + "correction", ro["experts"], gain=0.3, mean=-0.8)
         for k in subs:
