@@ -6,8 +6,8 @@
 //   sort     one workgroup counts the (token, expert) pairs by expert and lists them in tiles of TM rows that belong to
 //            one expert; the grids of the products are sized for the most tiles there can be, so that nothing comes
 //            back to the host and a step can be captured.
-//   gate_up  per tile and 64 hidden columns: both products of the gathered token rows and act(gate) * up.
-//   down     per tile and 128 output columns, scaled by the pair's weight, to the pair's own row: a token's rows are
+//   gate_up  per tile and 64 or 128 hidden columns: both products of the gathered token rows and act(gate) * up.
+//   down     per tile and 128 or 256 output columns, scaled by the pair's weight, to the pair's own row: a token's rows are
 //            consecutive and are summed where they are read (skyrl_gate_norm_add).
 //
 // The products stage pieces of the rows and of the weight rows through LDS (16-byte direct loads, chunk index
