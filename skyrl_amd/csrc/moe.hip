@@ -3,8 +3,8 @@
 //
 //   route    f32 logits (one workgroup per 16 tokens on the matrix instructions, bf16 products are exact in f32; any
 //            size and f32: a workgroup per token), then a wave per token picks groups and experts.
-//   sort     one workgroup counts the (token, expert) pairs by expert and lists them in tiles of TM rows that belong to
-//            one expert; the grids of the products are sized for the most tiles there can be, so that nothing comes
+//   sort     counts the (token, expert) pairs by expert (many pairs: in a launch of its own) and lists them in tiles of
+//            TM rows that belong to one expert; the grids of the products are sized for the most tiles there can be, so that nothing comes
 //            back to the host and a step can be captured.
 //   gate_up  per tile and 64 or 128 hidden columns: both products of the gathered token rows and act(gate) * up.
 //   down     per tile and 128 or 256 output columns, scaled by the pair's weight, to the pair's own row: a token's rows are
